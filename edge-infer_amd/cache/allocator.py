@@ -113,15 +113,19 @@ class SequencePages:
     that hold only positions no later query can see (position <= length - w)
     are given back; their table entries read -1.  `chunk` c: a query sees only keys of
     its own block of c positions (counted from the sequence's start), so pages that lie
-    wholly before the block of the next position are given back as well.  `stride` s: the
+    wholly before the block of the next position are given back as well.  `keep_first` k:
+    pages that hold one of the sequence's first k positions are never given back before the
+    sequence ends.  `stride` s: the
     group holds one entry for every complete block of s positions, so a sequence of n tokens
     needs pages for n // s entries (such a group has no window and no chunk).
     """
 
-    def __init__(self, pool: PagePool, n_slots: int, window=None, chunk=None, stride: int = 1):
+    def __init__(self, pool: PagePool, n_slots: int, window=None, chunk=None, stride: int = 1,
+                 keep_first: int = 0):
         self.pool = pool
         self.window = window
         self.chunk = chunk
+        self.kept_pages = pages_for(max(0, int(keep_first)))    # first pages that stay
         self.stride = max(1, int(stride))     # positions that share one entry of the group
         self._pages: Dict[int, List[int]] = {}
         self._version: Dict[int, int] = {}     # counts the changes of a slot's page list
@@ -164,7 +168,8 @@ class SequencePages:
         pages = self._pages[slot]
         dead = []
         for index, page in enumerate(pages):
-            if page >= 0 and (index + 1) * PAGE_TOKENS - 1 < first_visible:
+            if (page >= 0 and index >= self.kept_pages
+                    and (index + 1) * PAGE_TOKENS - 1 < first_visible):
                 dead.append(page)
                 pages[index] = -1
         if dead:

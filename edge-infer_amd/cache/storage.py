@@ -99,7 +99,8 @@ class SessionCache:
                             min(self.n_pages, self.n_pages // request.stride + self.n_slots + 1))
             self.kv_pools.append(pool)
             self.kv_pages.append(SequencePages(pool, self.n_slots, window=request.window,
-                                               chunk=request.chunk, stride=request.stride))
+                                               chunk=request.chunk, stride=request.stride,
+                                               keep_first=request.keep_first))
             shape = (len(entries), pool.n_pages, request.n_kv_heads, PAGE_TOKENS)
             value_dim = request.head_dim if request.value_dim is None else request.value_dim
             self.kv_k.append(torch.empty(shape + (request.head_dim,), dtype=dtype, device=device))

@@ -33,18 +33,32 @@ class FrequencyScaling:
 
 
 @dataclass(frozen=True)
+class YarnScaling:
+    """Pairs of a rotation are told apart by how often they turn within the original length: with
+    dim(t) = dims ln(original / (2 pi t)) / (2 ln theta), lo = max(floor(dim(fast)), 0),
+    hi = min(ceil(dim(slow)), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1),
+    the frequency of pair i becomes f_i / factor ramp_i + f_i (1 - ramp_i), and cosine and sine
+    are multiplied by 0.1 ln(factor) + 1."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
 class PositionSpec:
     """Position encoding of a mixer.  kind "rope": rotate-half pairs (i, i+dim/2)
     with angle = position / theta^(2i/dim), from a table of `max_positions` rows; kind
     "rope_pairs": neighbouring pairs (2i, 2i+1) with the same angles, worked out by the kernels
     from the frequencies theta^(-2i/dim), so no position is too far; kind "rope_half": the pairs
     of "rope" with the angles worked out by the kernels as for "rope_pairs", the frequencies
-    optionally rescaled (`scaling`); kind "none": no encoding."""
+    optionally rescaled (`scaling`: a `FrequencyScaling` or a `YarnScaling`); kind "none": no
+    encoding."""
     kind: str = "rope"
     theta: float = 10000.0
     dim: int = 0
     max_positions: int = 0
-    scaling: Optional[FrequencyScaling] = None      # kind "rope_half" only
+    scaling: Optional[object] = None                # kind "rope_half" only
 
 
 @dataclass(frozen=True)
@@ -56,7 +70,13 @@ class AttentionSpec:
     head_dim: int = 0
     qk_norm: bool = False          # per-head RMSNorm of q and k before the rotation
     qk_norm_eps: float = 1e-6
+    # q and k of every head are divided by their root mean square after the rotation (an RMS
+    # norm without a weight, eps `qk_norm_eps`)
+    qk_unit_norm: bool = False
     window: Optional[int] = None   # None: every earlier key; w: the last w keys
+    # with a window: the sequence's first `keep_first` positions stay visible however far back
+    # they lie, at their true positions
+    keep_first: int = 0
     scale: Optional[float] = None  # None: 1/sqrt(head_dim)
     position: PositionSpec = field(default_factory=PositionSpec)
     value_dim: Optional[int] = None     # None: values as wide as keys
@@ -151,6 +171,14 @@ class RoutedMLPSpec:
     down(silu(gate x) * up x) for every token, by the largest float32 logits W_router x, and
     adds their outputs weighted by the softmax over the chosen logits alone.
 
+    `scoring` "sigmoid": the scores are sigmoid(z), the choice is by the largest score, and the
+    weights are the chosen scores divided by their sum (+ 1e-20), times `weight_scale`.
+    `group_count` G > 1 (this scoring only): the experts form G equal groups of neighbours, a
+    group's score is the sum of its two largest scores, and only experts of the `group_keep`
+    best groups can be chosen.  `shared`: a gated feed-forward that runs for every token and is
+    added.  `activation`, `limit`, `alpha`: of an expert, as in `GatedMLPSpec` ("silu" or
+    "clamped_swish").
+
     `scoring` "softmax_all": the scores are the softmax over all router outputs, the choice is
     by the largest score (plus a learned per-output `correction` where the spec says so), and
     the weights are the chosen scores themselves, not renormalised.  `identity`: the router
@@ -163,6 +191,13 @@ class RoutedMLPSpec:
     scoring: str = "softmax_chosen"
     correction: bool = False
     identity: int = 0
+    weight_scale: float = 1.0
+    group_count: int = 1
+    group_keep: int = 1
+    activation: str = "silu"
+    limit: float = 0.0
+    alpha: float = 1.0
+    shared: Optional[GatedMLPSpec] = None
 
     @property
     def router_outputs(self) -> int:
@@ -331,10 +366,11 @@ class LoopSpec:
     """Layers start .. stop - 1 run `times` times in a row with the same weights, each pass
     with cache entries of its own.  Before a pass the stream x is made anew from itself and the
     embedding output x0: x <- W [x ; x0] + step[pass], with W [hidden, 2 hidden] and step
-    [times, hidden] parameters of the model."""
+    [times, hidden] parameters of the model; `remix` False: x <- x + step[pass] alone."""
     start: int
     stop: int
     times: int
+    remix: bool = True
 
 
 @dataclass(frozen=True)

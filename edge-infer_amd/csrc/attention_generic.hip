@@ -20,7 +20,9 @@
 // value for every block of `pool` positions, if b pool + pool - 1 <= p - w; tokens and blocks
 // share one softmax), `pool_only` (the tokens are left out: the kernel takes the pooled entries
 // alone and leaves every row's unnormalised sums, maximum and sum of weights in part_o and
-// part_ml, slice 0 of one, for a kernel that takes them in as one more slice of its own softmax).
+// part_ml, slice 0 of one, for a kernel that takes them in as one more slice of its own softmax),
+// `keep` (with a window: the keys of the sequence's first `keep` positions stay visible however
+// far back they lie; the walk takes their pages first and then the window's).
 // operators/src/cuda/execution.cu:137-179, runtime/src/qwen.cpp:374-402,
 // split merge: operators/src/cuda/kernels/gather_fa_variable.cu:14-118.
 #include "common.h"
@@ -46,7 +48,7 @@ attn_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pages,
                     float scale, int n_splits, int KH, int values_in_keys,
                     const float* __restrict__ gate, int pool, const T* __restrict__ pool_k,
                     const T* __restrict__ pool_v, const int32_t* __restrict__ pool_table,
-                    int pool_only) {
+                    int pool_only, int keep) {
   extern __shared__ float lds[];
   const int DQ = KH * D;                  // width of a query row and of a key as it is met
   float* Qs = lds;                        // [kRows][DQ]
@@ -129,7 +131,8 @@ attn_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pages,
           const int key = key0 + c;
           const bool visible =
               pooled ? (row_valid && key < blocks_r)
-                     : (row_valid && key <= pos_r && (window <= 0 || key > pos_r - window) &&
+                     : (row_valid && key <= pos_r &&
+                        (window <= 0 || key > pos_r - window || key < keep) &&
                         (chunk <= 0 || key / chunk == chunk_r));
           if (visible) {
             float dot = 0.f;
@@ -179,12 +182,14 @@ attn_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pages,
     int lo_key = window > 0 ? max(0, row_pos[row0] - window + 1) : 0;
     if (chunk > 0) lo_key = max(lo_key, row_pos[row0] / chunk * chunk);
     const int lo_page = lo_key / EI_PAGE, hi_page = hi_key / EI_PAGE;
-    const int total_pages = hi_page - lo_page + 1;
+    // pages before the window's that hold kept positions: they come first in the walk
+    const int kept_pages = min(lo_page, (keep + EI_PAGE - 1) / EI_PAGE);
+    const int total_pages = kept_pages + hi_page - lo_page + 1;
     const int per = (total_pages + n_splits - 1) / n_splits;
-    const int p_begin = lo_page + split * per;
-    const int p_end = min(lo_page + (split + 1) * per, hi_page + 1);
+    const int i_end = min((split + 1) * per, total_pages);
     const int chunks_per_page = EI_PAGE / BC;
-    for (int p = p_begin; p < p_end && !pool_only; ++p) {
+    for (int i = split * per; i < i_end && !pool_only; ++i) {
+      const int p = i < kept_pages ? i : lo_page + i - kept_pages;
       const int phys = page_table[static_cast<size_t>(seq) * table_width + p];
       if (phys < 0) continue;  // a page the window has released: every key in it is masked
       const T* kp = k_pages + (static_cast<size_t>(phys) * nkv + g) * EI_PAGE * D;
@@ -195,7 +200,7 @@ attn_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pages,
       for (int ch = 0; ch < chunks_per_page; ++ch) {
         const int key0 = p * EI_PAGE + ch * BC;
         if (key0 > hi_key) break;
-        if (key0 + BC <= lo_key) continue;   // wholly before what any row of the item sees
+        if (key0 + BC <= lo_key && key0 >= keep) continue;   // nothing that any row of the item sees
         walk(kp, vp, DVS, phys, ch, key0, hi_key, false);
       }
     }
@@ -302,7 +307,7 @@ extern "C" int ei_attention(const void* q, const void* k_pages, const void* v_pa
                             const float* sinks, float scale, int n_splits, int key_heads,
                             int values_in_keys, const float* gate, int pool, const void* pool_k,
                             const void* pool_v, const int32_t* pool_table, int pool_only,
-                            hipStream_t stream) {
+                            int keep, hipStream_t stream) {
   EI_REQUIRE(n_items > 0 && N > 0 && nq > 0 && nkv > 0, "attention: sizes must be positive");
   EI_REQUIRE(nq % nkv == 0, "attention: query heads must be a multiple of kv heads");
   EI_REQUIRE(key_heads == 1 || key_heads == nkv,
@@ -321,6 +326,7 @@ extern "C" int ei_attention(const void* q, const void* k_pages, const void* v_pa
   EI_REQUIRE(!pool_only || (pool > 0 && n_splits == 1 && !gate),
              "attention: the pooled entries alone are taken in one slice, without a gate");
   EI_REQUIRE(window >= 0, "attention: negative window");
+  EI_REQUIRE(keep >= 0 && (keep == 0 || chunk == 0), "attention: kept first positions with chunks");
   EI_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pool_k && pool_v && pool_table &&
                                          key_heads == 1 && !values_in_keys)),
              "attention: pooled blocks need a window, their cache and keys of one kv head");
@@ -354,14 +360,14 @@ extern "C" int ei_attention(const void* q, const void* k_pages, const void* v_pa
         static_cast<const float*>(v_pages), item_seq, item_row0, item_npos, row_pos, page_table,
         table_width, static_cast<float*>(out), part_o, part_ml, nq, nkv, D, DV, Gb, head_blocks,
         BC, window, chunk, slopes, sinks, scale, n_splits, key_heads, values_in_keys, gate, pool,
-        static_cast<const float*>(pool_k), static_cast<const float*>(pool_v), pool_table, pool_only);
+        static_cast<const float*>(pool_k), static_cast<const float*>(pool_v), pool_table, pool_only, keep);
   } else if (dtype == EI_BF16) {
     attn_generic_kernel<bf16_t><<<grid, kThreads, lds, stream>>>(
         static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
         static_cast<const bf16_t*>(v_pages), item_seq, item_row0, item_npos, row_pos, page_table,
         table_width, static_cast<bf16_t*>(out), part_o, part_ml, nq, nkv, D, DV, Gb, head_blocks,
         BC, window, chunk, slopes, sinks, scale, n_splits, key_heads, values_in_keys, gate, pool,
-        static_cast<const bf16_t*>(pool_k), static_cast<const bf16_t*>(pool_v), pool_table, pool_only);
+        static_cast<const bf16_t*>(pool_k), static_cast<const bf16_t*>(pool_v), pool_table, pool_only, keep);
   } else {
     EI_REQUIRE(false, "attention: unknown dtype");
   }

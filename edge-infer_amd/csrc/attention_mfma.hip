@@ -33,7 +33,11 @@ constexpr float kLowest = -1.0e30f;
 // of another source (the pooled blocks before a window): float32 sums of weighted values
 // [rows, nq, D] and (maximum, sum of weights) [rows, nq, 2] in natural units; they join the
 // row's softmax as one more slice.  `gate` (float32 [rows, nq], or null): the output of a row
-// and head is multiplied by sigmoid(gate).
+// and head is multiplied by sigmoid(gate).  `keep` > 0 (with a window): the keys of the sequence's
+// first `keep` positions stay visible however far back they lie; walks take what lies before the
+// window of them first.  `wide` (or null): one gate for every element of the output, the sums of
+// `wide_slices` slices of float32 or bfloat16 rows: element (row, head, d) is multiplied by
+// sigmoid of what lies at row * wide_row + head * D + d.
 struct AttnExtra {
   int chunk;
   const float* slopes;
@@ -41,7 +45,23 @@ struct AttnExtra {
   const float* pool_o;
   const float* pool_ml;
   const float* gate;
+  int keep;
+  const void* wide;
+  int wide_dtype, wide_slices;
+  size_t wide_slice, wide_row;
 };
+
+// The factor of output element `at` (row * wide_row + head * D + d) of `AttnExtra.wide`.
+__device__ __forceinline__ float wide_open(const AttnExtra& extra, size_t at) {
+  float z = 0.f;
+  if (extra.wide_dtype == EI_F32) {
+    const float* p = static_cast<const float*>(extra.wide) + at;
+    for (int s = 0; s < extra.wide_slices; ++s) z += p[s * extra.wide_slice];
+  } else {
+    z = ei::bf16_to_f32(static_cast<const bf16_t*>(extra.wide)[at]);
+  }
+  return 1.0f / (1.0f + expf(-z));
+}
 
 __device__ __forceinline__ float bf16_lo(uint32_t u) { return __uint_as_float(u << 16); }
 __device__ __forceinline__ float bf16_hi(uint32_t u) { return __uint_as_float(u & 0xffff0000u); }
@@ -226,6 +246,21 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   const int tile_end = split == n_splits - 1
                            ? last_tile + 1
                            : min(last_tile + 1, (lo_page + (split + 1) * per) * (EI_PAGE / kTile));
+  // (EXT) tiles of kept first positions before the window's: the walk is then over kept tiles and
+  // the window's tiles in a row, step v < kept being tile v and the others tile v + skipped, and
+  // slices are equal parts of it
+  int kept = 0, skipped = 0, step_begin = tile_begin, step_end = tile_end;
+  const int keep = EXT ? extra.keep : 0;
+  if constexpr (EXT) {
+    kept = min(first_tile, (keep + kTile - 1) / kTile);
+    if (kept > 0) {
+      skipped = first_tile - kept;
+      const int steps = kept + total_tiles;
+      const int share = (steps + n_splits - 1) / n_splits;
+      step_begin = split * share;
+      step_end = min(steps, (split + 1) * share);
+    }
+  }
   (void)total_tiles;
 
   float m_run = kLowest, l_run = 0.f;              // state of head r16 (same in all four c)
@@ -288,7 +323,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int key = key0 + 4 * c + r;
-      const bool visible = key <= pos && key >= lo_key;
+      const bool visible = key <= pos && (key >= lo_key || (EXT && key < keep));
       if constexpr (EXT)
         sc[r] = visible ? fmaf(-slope, static_cast<float>(pos - key), s[r] * scale) : -INFINITY;
       else
@@ -338,7 +373,8 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
   };
-  for (int tile = tile_begin + wave; tile < tile_end; tile += W) {
+  for (int step = step_begin + wave; step < step_end; step += W) {
+    const int tile = step < kept ? step : step + skipped;
     if (PREP && own_key && tile == last_tile)
       process(tile, std::integral_constant<bool, PREP>{});
     else
@@ -390,8 +426,12 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
       }
     }
     if (n_splits == 1) {
-      out[(static_cast<size_t>(row) * nq + head) * D + d] =
-          ei::from_f32<bf16_t>(l > 0.f ? o / l : 0.f);
+      float value = l > 0.f ? o / l : 0.f;
+      if constexpr (EXT)
+        if (extra.wide)
+          value *= wide_open(extra, static_cast<size_t>(row) * extra.wide_row +
+                                        static_cast<size_t>(head) * D + d);
+      out[(static_cast<size_t>(row) * nq + head) * D + d] = ei::from_f32<bf16_t>(value);
     } else {
       const size_t slot = (static_cast<size_t>(row) * nq + head) * n_splits + split;
       part_o[slot * D + d] = o;
@@ -610,6 +650,14 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
   }
   const int lo_key = lo_key_of;
   const int lo_page = lo_key / EI_PAGE, hi_page = last_pos / EI_PAGE;
+  // (EXT) pages of kept first positions before the window's come first: the walk is over visits
+  // first_visit .. hi_page, visit v >= lo_page being page v and the visits before it pages 0, 1, ...
+  const int keep = EXT ? extra.keep : 0;
+  const int kept_pages = EXT ? min(lo_page, (keep + EI_PAGE - 1) / EI_PAGE) : 0;
+  const int first_visit = lo_page - kept_pages;
+  auto page_of = [&](int visit) __attribute__((always_inline)) {
+    return (EXT && visit < lo_page) ? visit - first_visit : visit;
+  };
   const bool wave_rows_valid = pw * kWideRows + kWideRows <= npos;
   const int wave_min_pos = wave_rows_valid ? row_pos[row0 + pw * kWideRows] : -1;
   const int wave_max_pos = wave_rows_valid ? row_pos[row0 + pw * kWideRows + kWideRows - 1] : -1;
@@ -626,12 +674,12 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
 #pragma unroll
     for (int e = 0; e < 16; ++e) o_acc[db][e] = 0.f;
 
-  // Request page `page_index` of the sequence into buffer `buf` (nothing past the last page).
+  // Request the page of visit `page_index` into buffer `buf` (nothing past the last page).
   // A page that the window has given back (none of its keys is visible to any row: it only
   // lies in the walk) is cleared instead, by plain stores.
   auto fetch_page = [&](int page_index, int buf) __attribute__((always_inline)) {
     if (page_index > hi_page) return;
-    const int phys = page_table[static_cast<size_t>(seq) * table_width + page_index];
+    const int phys = page_table[static_cast<size_t>(seq) * table_width + page_of(page_index)];
     bf16_t* const to = page_lds + buf * 2 * PBUF;
     if (phys < 0) {
 #pragma unroll
@@ -726,7 +774,7 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int key = key_base + (kw * KBL + kb) * 32 + 8 * i + 4 * half + r;
-            bool visible = key <= pos_q && (window <= 0 || key > pos_q - window);
+            bool visible = key <= pos_q && (window <= 0 || key > pos_q - window || (EXT && key < keep));
             if constexpr (EXT) visible = visible && key >= chunk_lo;
             if (!visible) s[kb][4 * i + r] = -INFINITY;     // (pos_q = -1: a row that is not there)
           }
@@ -811,7 +859,8 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
   auto page_seen = [&](const int page) __attribute__((always_inline)) {
     const int key_lo = page * EI_PAGE + kw * KBL * 32, key_hi = key_lo + KBL * 32 - 1;
     bool seen = wave_has_rows && key_lo <= wave_last_pos &&
-                (window <= 0 || !wave_rows_valid || key_hi > wave_min_pos - window);
+                (window <= 0 || !wave_rows_valid || key_hi > wave_min_pos - window ||
+                 (EXT && key_lo < keep));
     if constexpr (EXT)     // wholly before the chunk of the wave's first row: no row sees it
       if (chunk > 0 && wave_rows_valid) seen = seen && key_hi >= wave_min_pos / chunk * chunk;
     return seen;
@@ -820,29 +869,30 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
     const int key_base = page * EI_PAGE;
     const int key_lo = key_base + kw * KBL * 32, key_hi = key_lo + KBL * 32 - 1;
     bool no_mask = wave_rows_valid && key_hi <= wave_min_pos &&
-                   (window <= 0 || key_lo > wave_max_pos - window);
+                   (window <= 0 || key_lo > wave_max_pos - window || (EXT && key_hi < keep));
     if constexpr (EXT)     // every key lies in the chunk of the wave's last row, so of all rows
       if (chunk > 0) no_mask = no_mask && key_lo >= wave_max_pos / chunk * chunk;
     scores(key_base, buf, !no_mask);
   };
   using Both = std::integral_constant<int, LOADS>;
   using None = std::integral_constant<int, 0>;
-  fetch_page(lo_page, 0);
-  fetch_page(lo_page + 1, 1);
-  if (lo_page + 1 <= hi_page) page_arrived(lo_page, 0, Both{});
-  else page_arrived(lo_page, 0, None{});
+  fetch_page(first_visit, 0);
+  fetch_page(first_visit + 1, 1);
+  if (first_visit + 1 <= hi_page) page_arrived(first_visit, 0, Both{});
+  else page_arrived(first_visit, 0, None{});
   int buf = 0;
-  for (int page = lo_page; page <= hi_page; ++page) {
+  for (int visit = first_visit; visit <= hi_page; ++visit) {
+    const int page = page_of(visit);
     const int next = buf == kPageBuffers - 1 ? 0 : buf + 1;
-    fetch_page(page + 2, next == kPageBuffers - 1 ? 0 : next + 1);
+    fetch_page(visit + 2, next == kPageBuffers - 1 ? 0 : next + 1);
     __builtin_amdgcn_sched_barrier(0);
     if (page_seen(page)) {
       scores_of(page, buf);
       values(buf);
     }
-    if (page < hi_page) {
-      if (page + 2 <= hi_page) page_arrived(page + 1, next, Both{});
-      else page_arrived(page + 1, next, None{});
+    if (visit < hi_page) {
+      if (visit + 2 <= hi_page) page_arrived(visit + 1, next, Both{});
+      else page_arrived(visit + 1, next, None{});
     }
     buf = next;
   }
@@ -963,6 +1013,9 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
             if (extra.pool_o && pooled[r] != 0.f)
               o = fmaf(extra.pool_o[(static_cast<size_t>(row0 + orow) * nq + head) * D + db * 32 + n32],
                        pooled[r], o);
+            if (extra.wide)
+              o *= wide_open(extra, static_cast<size_t>(row0 + orow) * extra.wide_row +
+                                        static_cast<size_t>(head) * D + db * 32 + n32);
           }
           dst[db * 32 + n32] = ei::from_f32<bf16_t>(o);
         }
@@ -983,7 +1036,7 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o,
                                   int nq, int D, int n_splits, int total,
                                   const float* __restrict__ pool_o,
                                   const float* __restrict__ pool_ml,
-                                  const float* __restrict__ gate) {
+                                  const float* __restrict__ gate, AttnExtra extra) {
   const int wave = (blockIdx.x * blockDim.x + threadIdx.x) / EI_WAVE;
   const int lane = threadIdx.x % EI_WAVE;
   if (wave >= total) return;
@@ -1032,8 +1085,16 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o,
       float inv = l > 0.f ? 1.f / l : 0.f;
       if (gate) inv *= 1.0f / (1.0f + expf(-gate[wave]));
       bf16_t* dst = out + static_cast<size_t>(wave) * D + d;
-      dst[0] = ei::from_f32<bf16_t>(o0 * inv);
-      dst[1] = ei::from_f32<bf16_t>(o1 * inv);
+      o0 *= inv;
+      o1 *= inv;
+      if (extra.wide) {
+        const size_t at = static_cast<size_t>(wave / nq) * extra.wide_row +
+                          static_cast<size_t>(wave % nq) * D + d;
+        o0 *= wide_open(extra, at);
+        o1 *= wide_open(extra, at + 1);
+      }
+      dst[0] = ei::from_f32<bf16_t>(o0);
+      dst[1] = ei::from_f32<bf16_t>(o1);
     }
   }
 }
@@ -1130,7 +1191,7 @@ static int prefill_launch(const void* q, const void* k_pages, const void* v_page
   const bf16_t* kk = static_cast<const bf16_t*>(k_pages);
   const bf16_t* vv = static_cast<const bf16_t*>(v_pages);
   bf16_t* oo = static_cast<bf16_t*>(out);
-  const AttnExtra none{0, nullptr, nullptr};
+  const AttnExtra none{};
 #define EI_PREFILL_KW(DD, HH, KK)                                                             \
   do {                                                                                        \
     if (extra)                                                                                \
@@ -1157,6 +1218,15 @@ static int prefill_launch(const void* q, const void* k_pages, const void* v_page
   EI_LAUNCH_CHECK();
 }
 
+// Whether the elements' gates of `AttnExtra` (null: none) are what the kernels assume: slices of
+// float32 rows or one bfloat16 row per row, each at least nq * D elements apart.
+static bool wide_fits(const void* wide, int dtype, int slices, long long slice, long long row,
+                      int nq, int D) {
+  if (!wide) return true;
+  return slices >= 1 && row >= static_cast<long long>(nq) * D && slice >= 0 &&
+         (dtype == EI_F32 || (dtype == EI_BF16 && slices == 1));
+}
+
 extern "C" int ei_attention_prefill_mfma(const void* q, const void* k_pages, const void* v_pages,
                                          const int32_t* item_seq, const int32_t* item_row0,
                                          const int32_t* item_npos, int n_items,
@@ -1170,19 +1240,25 @@ extern "C" int ei_attention_prefill_mfma(const void* q, const void* k_pages, con
 }
 
 // The same with the options of `AttnExtra`: chunk (0: none), slopes and sinks (float32 [nq] on
-// the device, or null).
+// the device, or null), another source's sums, the gates a head, kept first positions (0: none)
+// and the gates an element.
 extern "C" int ei_attention_prefill_mfma_ext(
     const void* q, const void* k_pages, const void* v_pages, const int32_t* item_seq,
     const int32_t* item_row0, const int32_t* item_npos, int n_items, const int32_t* row_pos,
     const int32_t* page_table, int table_width, void* out, int nq, int nkv, int D, int window,
     float scale, int key_ways, int pair_items, int chunk, const float* slopes,
-    const float* sinks, const float* pool_o, const float* pool_ml, const float* gate,
+    const float* sinks, const float* pool_o, const float* pool_ml, const float* gate, int keep,
+    const void* wide, int wide_dtype, int wide_slices, long long wide_slice, long long wide_row,
     hipStream_t stream) {
   EI_REQUIRE(chunk >= 0, "attention_prefill: negative chunk");
+  EI_REQUIRE(keep >= 0 && (keep == 0 || chunk == 0), "attention_prefill: kept first positions with chunks");
+  EI_REQUIRE(wide_fits(wide, wide_dtype, wide_slices, wide_slice, wide_row, nq, D),
+             "attention_prefill: the elements' gates have the wrong shape");
   EI_REQUIRE(scale > 0.f, "attention_prefill: the scale must be positive");
   EI_REQUIRE((pool_o == nullptr) == (pool_ml == nullptr),
              "attention_prefill: the other source's sums and their weights come together");
-  const AttnExtra extra{chunk, slopes, sinks, pool_o, pool_ml, gate};
+  const AttnExtra extra{chunk, slopes, sinks, pool_o, pool_ml, gate, keep, wide, wide_dtype,
+                        wide_slices, static_cast<size_t>(wide_slice), static_cast<size_t>(wide_row)};
   return prefill_launch(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_pos,
                         page_table, table_width, out, nq, nkv, D, window, scale, key_ways,
                         pair_items, &extra, stream);
@@ -1237,7 +1313,7 @@ static int decode_launch(const void* q, const void* k_pages, const void* v_pages
   const bf16_t* vv = static_cast<const bf16_t*>(v_pages);
   bf16_t* oo = static_cast<bf16_t*>(out);
   const DecodePrep none{};
-  const AttnExtra plain{0, nullptr, nullptr, nullptr, nullptr, nullptr};
+  const AttnExtra plain{};
 #define EI_DECODE(DD, GG)                                                                     \
   do {                                                                                        \
     if (prep)                                                                                 \
@@ -1282,7 +1358,7 @@ static int decode_launch(const void* q, const void* k_pages, const void* v_pages
     const int blocks = (total * EI_WAVE + threads - 1) / threads;
     attn_merge_kernel<<<blocks, threads, 0, stream>>>(
         part_o, part_ml, row_seq, oo, nq, D, n_splits, total, extra ? extra->pool_o : nullptr,
-        extra ? extra->pool_ml : nullptr, extra ? extra->gate : nullptr);
+        extra ? extra->pool_ml : nullptr, extra ? extra->gate : nullptr, extra ? *extra : plain);
   }
   EI_LAUNCH_CHECK();
 }
@@ -1307,7 +1383,8 @@ extern "C" int ei_attention_decode_mfma(const void* q, const void* k_pages, cons
 }
 
 // The same with the options of `AttnExtra`: chunk (0: none), slopes and sinks (float32 [nq] on
-// the device, or null).
+// the device, or null), another source's sums, the gates a head, kept first positions (0: none)
+// and the gates an element.
 extern "C" int ei_attention_decode_mfma_ext(const void* q, const void* k_pages,
                                             const void* v_pages, const int32_t* row_pos,
                                             const int32_t* row_seq, const int32_t* page_table,
@@ -1317,9 +1394,15 @@ extern "C" int ei_attention_decode_mfma_ext(const void* q, const void* k_pages,
                                             int heads, const int32_t* longest, int chunk,
                                             const float* slopes, const float* sinks,
                                             const float* pool_o, const float* pool_ml,
-                                            const float* gate, hipStream_t stream) {
+                                            const float* gate, int keep, const void* wide,
+                                            int wide_dtype, int wide_slices, long long wide_slice,
+                                            long long wide_row, hipStream_t stream) {
   EI_REQUIRE(chunk >= 0, "attention_decode: negative chunk");
-  const AttnExtra extra{chunk, slopes, sinks, pool_o, pool_ml, gate};
+  EI_REQUIRE(keep >= 0 && (keep == 0 || chunk == 0), "attention_decode: kept first positions with chunks");
+  EI_REQUIRE(wide_fits(wide, wide_dtype, wide_slices, wide_slice, wide_row, nq, D),
+             "attention_decode: the elements' gates have the wrong shape");
+  const AttnExtra extra{chunk, slopes, sinks, pool_o, pool_ml, gate, keep, wide, wide_dtype,
+                        wide_slices, static_cast<size_t>(wide_slice), static_cast<size_t>(wide_row)};
   return decode_launch(q, k_pages, v_pages, row_pos, row_seq, page_table, table_width, out,
                        part_o, part_ml, rows, nq, nkv, D, window, scale, n_splits, waves, heads,
                        longest, nullptr, stream, &extra);

@@ -56,7 +56,7 @@ _SIGNATURES = {
                           c_float, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                           c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int,
                           c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_longlong,
-                          c_void_p],
+                          c_void_p, c_float, c_int, c_void_p],
         "ei_projection_norm_store": [c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p, c_void_p,
                                      c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                                      c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
@@ -98,13 +98,15 @@ _SIGNATURES = {
     },
     "moe": {
         "ei_moe_route": [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
-                         c_int, c_int, c_int, c_void_p, c_void_p],
+                         c_int, c_int, c_int, c_void_p, c_int, c_int, c_float, c_void_p],
         "ei_moe_experts": [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
-                           c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+                           c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
+                           c_float, c_void_p, c_int, c_int, c_longlong, c_void_p],
         "ei_moe_grouped_supported": [c_int, c_int, c_int, c_int],
         "ei_moe_experts_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                    c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                                   c_int, c_int, c_int, c_int, c_int, c_void_p],
+                                   c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float,
+                                   c_void_p, c_int, c_int, c_longlong, c_void_p],
     },
     "delta_rule": {
         "ei_delta_conv": [c_void_p, c_int, c_int, c_longlong, c_int, c_void_p, c_int, c_void_p,
@@ -126,7 +128,8 @@ _SIGNATURES = {
         "ei_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                          c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                          c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float,
-                         c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
+                         c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
+                         c_int, c_void_p],
         "ei_pool_store": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                           c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
                           c_void_p],
@@ -175,11 +178,15 @@ _SIGNATURES = {
         "ei_attention_prefill_mfma_ext": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                           c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p,
                                           c_int, c_int, c_int, c_int, c_float, c_int, c_int,
-                                          c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p],
+                                          c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                          c_int, c_void_p, c_int, c_int, c_longlong, c_longlong,
+                                          c_void_p],
         "ei_attention_decode_mfma_ext": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                          c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                          c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int,
-                                         c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p],
+                                         c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                         c_int, c_void_p, c_int, c_int, c_longlong, c_longlong,
+                                         c_void_p],
         "ei_attention_decode_mfma_fused": [c_void_p, c_int, c_longlong, c_void_p, c_void_p, c_float,
                                            c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                                            c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
@@ -597,7 +604,7 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
               page_table, out, n_heads, n_kv_heads, head_dim, window=None, scale=None,
               n_splits=1, part_o=None, part_ml=None, value_dim=None, chunk=None, slopes=None,
               sinks=None, key_heads=1, values_in_keys=False, gate=None, pool=None,
-              pool_k=None, pool_v=None, pool_table=None, pool_only=False) -> None:
+              pool_k=None, pool_v=None, pool_table=None, pool_only=False, keep_first=0) -> None:
     """Generic causal attention over the paged cache (see attention_generic.hip).
     value_dim: head size of the values and of `out` (None: head_dim); chunk: a query sees only
     the keys of its own block of that many positions; slopes, sinks: float32 [n_heads], the
@@ -611,7 +618,8 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
     through `pool_table`) whose blocks of P positions lie wholly before its window.
     pool_only: the tokens are left out; `out` is not written, and part_o [rows, heads,
     value_dim] and part_ml [rows, heads, 2] receive every row's unnormalised sums over the
-    pooled entries, the largest score and the sum of weights (n_splits 1)."""
+    pooled entries, the largest score and the sum of weights (n_splits 1).  keep_first: with a
+    window, the keys of the sequence's first positions that stay visible however far back."""
     lib = library("attention_generic")
     n = q.shape[0]
     value_dim = head_dim if value_dim is None else int(value_dim)
@@ -641,6 +649,8 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
     for name, per_head in (("slopes", slopes), ("sinks", sinks)):
         if per_head is not None and per_head.numel() != n_heads:
             raise KernelError(f"attention: {name} must have one value per query head")
+    if keep_first < 0 or (keep_first and chunk):
+        raise KernelError("attention: kept first positions go with a window, not with chunks")
     if pool_only and (not pool or n_splits != 1 or gate is not None):
         raise KernelError("attention: the pooled entries alone are taken in one slice")
     if n_splits > 1 or pool_only:
@@ -672,7 +682,7 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
         None if gate is None else _gpu(gate, "gate", torch.float32), int(pool or 0),
         _gpu(pool_k, "pool_k") if pool else None, _gpu(pool_v, "pool_v") if pool else None,
         _gpu(pool_table, "pool_table", torch.int32) if pool else None, int(bool(pool_only)),
-        _stream())
+        int(keep_first) if window else 0, _stream())
     _check(lib, status, "attention")
 
 
@@ -978,7 +988,7 @@ def projection_norm_store(qkv, q_norm_w, k_norm_w, eps, row_pos, row_seq, page_t
 def head_store(proj, q_norm_w, k_norm_w, eps, frequencies, row_pos, row_seq, page_table, q_out,
                k_pages, v_pages, n_heads, n_kv_heads, head_dim, value_dim, write_cache=True,
                v_first=None, v_mode=0, v_lambda=None, query_temperature=None, gate_out=None,
-               gate_column=0) -> None:
+               gate_column=0, bias=None, turn_scale=1.0, unit_norm=False) -> None:
     """(query_temperature (coef, every): a query at position p is multiplied by
     1 + coef ln(floor((p + 1) / every) + 1); gate_out float32 [n, heads]: receives the rows'
     columns gate_column .. gate_column + heads - 1, summed over slices; n_kv_heads 0: the rows
@@ -990,7 +1000,9 @@ def head_store(proj, q_norm_w, k_norm_w, eps, frequencies, row_pos, row_seq, pag
     [*, kv heads, 64, head_dim] and values [*, kv heads, 64, value_dim] to their pages.
     v_mode 1: the values are also written to `v_first` (float32 [n, kv heads * value_dim]);
     v_mode 2: what is stored is (1 - lambda) v + lambda v_first, `v_lambda` one float32 on the
-    device."""
+    device.  bias: float32 [g] added to the sums of q, k and v.  turn_scale multiplies cosine and
+    sine; unit_norm: queries and keys are divided by the root of their mean square + eps after
+    the rotation."""
     lib = library("rope_store")
     n = q_out.shape[0]
     stride = proj.shape[-1]
@@ -1029,6 +1041,8 @@ def head_store(proj, q_norm_w, k_norm_w, eps, frequencies, row_pos, row_seq, pag
         raise KernelError("head_store: gate_out must be [rows, heads] and the rows hold its columns")
     if n_kv_heads == 0 and write_cache:
         raise KernelError("head_store: rows without keys cannot write the cache")
+    if bias is not None and bias.numel() != stride:
+        raise KernelError("head_store: the bias must be as wide as a row")
     status = lib.ei_head_store(
         _gpu(proj, "proj"), _code(proj, "proj"), nsplit, split_stride, stride,
         None if q_norm_w is None else _gpu(q_norm_w, "q_norm", torch.float32),
@@ -1042,7 +1056,8 @@ def head_store(proj, q_norm_w, k_norm_w, eps, frequencies, row_pos, row_seq, pag
         None if v_mode != 2 else _gpu(v_lambda, "v_lambda", torch.float32), n, n_heads,
         n_kv_heads, head_dim, value_dim, int(write_cache), float(temp[0]), int(temp[1]),
         None if gate_out is None else _gpu(gate_out, "gate_out", torch.float32), int(gate_column),
-        _stream())
+        None if bias is None else _gpu(bias, "bias", torch.float32), float(turn_scale),
+        int(bool(unit_norm)), _stream())
     _check(lib, status, "head_store")
 
 
@@ -1076,7 +1091,7 @@ def attention_prefill_mfma(q, k_pages, v_pages, item_seq, item_row0, item_npos, 
                            page_table, out, n_heads, n_kv_heads, head_dim, window=None,
                            scale=None, key_ways=1, pair_items=True, largest_item=None,
                            chunk=None, slopes=None, sinks=None, pool_o=None, pool_ml=None,
-                           gate=None) -> None:
+                           gate=None, keep_first=0, wide_gate=None) -> None:
     """bfloat16 prefill attention on the matrix cores; an item holds up to
     `attention_prefill_mfma_positions(group, key_ways)` positions of one sequence.
     pair_items: with enough items a block may take item i and then item n_items - 1 - i
@@ -1084,7 +1099,10 @@ def attention_prefill_mfma(q, k_pages, v_pages, item_seq, item_row0, item_npos, 
     largest_item: the most positions any item holds, from the host's copy of the list (the
     kernel gives a block's waves fixed rows of an item and would leave the rows of a larger
     one out); None: looked up from `item_npos` on the device, which waits for the device.
-    chunk, slopes, sinks: as for `attention` (any of them takes the kernel's extended form)."""
+    chunk, slopes, sinks, keep_first: as for `attention`; wide_gate (rows, first column): rows of
+    columns, of which those from `first column` on are the gates of the output's elements (the
+    output is multiplied by their sigmoid), as [n, w] or float32 slices [s, n, w].  Any of
+    these takes the kernel's extended form."""
     lib = library("attention_mfma")
     n = q.shape[0]
     capacity = attention_prefill_mfma_positions(n_heads // max(1, n_kv_heads), key_ways)
@@ -1113,20 +1131,24 @@ def attention_prefill_mfma(q, k_pages, v_pages, item_seq, item_row0, item_npos, 
         _gpu(page_table, "page_table", torch.int32), page_table.shape[-1],
         _gpu(out, "out", torch.bfloat16), n_heads, n_kv_heads, head_dim, int(window or 0),
         float(scale), int(key_ways), int(bool(pair_items)))
-    if chunk or slopes is not None or sinks is not None or pool_o is not None or gate is not None:
+    keep_first = keep_first if window else 0
+    if (chunk or slopes is not None or sinks is not None or pool_o is not None or gate is not None
+            or keep_first or wide_gate is not None):
         status = lib.ei_attention_prefill_mfma_ext(*common, *_attention_extras(
-            chunk, slopes, sinks, n_heads, n, head_dim, pool_o, pool_ml, gate), _stream())
+            chunk, slopes, sinks, n_heads, n, head_dim, pool_o, pool_ml, gate, keep_first,
+            wide_gate), _stream())
     else:
         status = lib.ei_attention_prefill_mfma(*common, _stream())
     _check(lib, status, "attention_prefill")
 
 
 def _attention_extras(chunk, slopes, sinks, n_heads, rows=0, head_dim=0, pool_o=None,
-                      pool_ml=None, gate=None):
-    """(chunk, slopes, sinks, pool_o, pool_ml, gate pointers) for the extended forms of the
-    matrix-core kernels.  pool_o float32 [rows * heads * head_dim] and pool_ml [rows * heads *
+                      pool_ml=None, gate=None, keep_first=0, wide_gate=None):
+    """The arguments of the extended forms of the matrix-core kernels from chunk on.  pool_o float32 [rows * heads * head_dim] and pool_ml [rows * heads *
     2]: what `attention(..., pool_only=True)` left for every row and head, taken in as one more
-    slice of the softmax; gate float32 [rows, heads]: the output is multiplied by its sigmoid."""
+    slice of the softmax; gate float32 [rows, heads]: the output is multiplied by its sigmoid;
+    wide_gate (rows [rows, w] or float32 slices of them, first column): so is every element of
+    the output, by the sigmoid of its own column."""
     for name, per_head in (("slopes", slopes), ("sinks", sinks)):
         if per_head is not None and per_head.numel() != n_heads:
             raise KernelError(f"attention: {name} must have one value per query head")
@@ -1140,8 +1162,19 @@ def _attention_extras(chunk, slopes, sinks, n_heads, rows=0, head_dim=0, pool_o=
 
     def f32(tensor, name):
         return None if tensor is None else _gpu(tensor, name, torch.float32)
+    if keep_first < 0 or (keep_first and chunk):
+        raise KernelError("attention: kept first positions go with a window, not with chunks")
+    wide = (None, F32, 1, 0, 0)
+    if wide_gate is not None:
+        columns, first = wide_gate
+        stride = columns.shape[-1]
+        slices, slice_stride = _splits(columns, rows, stride, "wide_gate")
+        if not 0 <= first <= stride - n_heads * head_dim:
+            raise KernelError("attention: the gate's columns lie outside its rows")
+        wide = (_gpu(columns, "wide_gate") + first * columns.element_size(),
+                _code(columns, "wide_gate"), slices, slice_stride, stride)
     return (int(chunk or 0), f32(slopes, "slopes"), f32(sinks, "sinks"), f32(pool_o, "pool_o"),
-            f32(pool_ml, "pool_ml"), f32(gate, "gate"))
+            f32(pool_ml, "pool_ml"), f32(gate, "gate"), int(keep_first), *wide)
 
 
 class DecodeProjection:
@@ -1159,7 +1192,8 @@ class DecodeProjection:
 def attention_decode_mfma(q, k_pages, v_pages, row_pos, row_seq, page_table, out, n_heads,
                           n_kv_heads, head_dim, window=None, scale=None, n_splits=1, part_o=None,
                           part_ml=None, waves=4, longest=None, heads=0, chunk=None, slopes=None,
-                          sinks=None, pool_o=None, pool_ml=None, gate=None) -> None:
+                          sinks=None, pool_o=None, pool_ml=None, gate=None, keep_first=0,
+                          wide_gate=None) -> None:
     """bfloat16 decode attention on the matrix cores: one query row per sequence.  `waves`
     (4, 8 or 16) of a block share its key range tile by tile; more suit fewer sequences (few
     blocks), whose ranges then need fewer slices or none.  `heads` (a power of two, or 0 for
@@ -1168,13 +1202,15 @@ def attention_decode_mfma(q, k_pages, v_pages, row_pos, row_seq, page_table, out
     device): the most tokens a sequence of the step holds; every sequence's range is then
     cut into slices of the longest one's share, so that unequal lengths give equal blocks.
     `q` is the queries [rows, heads * head_dim], or a `DecodeProjection`: the kernel then does
-    the work of `qk_norm_rope_store` for its rows as well.  chunk, slopes, sinks: as for
-    `attention` (any of them takes the kernel's extended form, which the fused one lacks)."""
+    the work of `qk_norm_rope_store` for its rows as well.  chunk, slopes, sinks,
+    keep_first: as for `attention`; wide_gate: as for `attention_prefill_mfma` (any of them takes
+    the kernel's extended form, which the fused one lacks)."""
     lib = library("attention_mfma")
     n = out.shape[0]
     fused = isinstance(q, DecodeProjection)
+    keep_first = keep_first if window else 0
     extended = (bool(chunk) or slopes is not None or sinks is not None or pool_o is not None
-                or gate is not None)
+                or gate is not None or keep_first != 0 or wide_gate is not None)
     if (pool_o is not None or gate is not None) and n_splits < 2:
         raise KernelError("attention_decode: pooled sums and the gate are taken in by the merge "
                           "of at least two slices")
@@ -1232,7 +1268,8 @@ def attention_decode_mfma(q, k_pages, v_pages, row_pos, row_seq, page_table, out
         None if longest is None else _gpu(longest, "longest", torch.int32))
     if extended:
         status = lib.ei_attention_decode_mfma_ext(*common, *_attention_extras(
-            chunk, slopes, sinks, n_heads, q.shape[0], head_dim, pool_o, pool_ml, gate), _stream())
+            chunk, slopes, sinks, n_heads, q.shape[0], head_dim, pool_o, pool_ml, gate, keep_first,
+            wide_gate), _stream())
     else:
         status = lib.ei_attention_decode_mfma(*common, _stream())
     _check(lib, status, "attention_decode")
@@ -1670,16 +1707,20 @@ def la_out(o_raw, proj, gate_column: int, norm_w, eps: float, row_seq, out) -> N
     _check(lib, status, "la_out")
 
 
-ROUTER_SCORINGS = {"softmax_chosen": 0, "softmax_all": 1}
+ROUTER_SCORINGS = {"softmax_chosen": 0, "softmax_all": 1, "sigmoid": 2}
+EXPERT_ACTIVATIONS = {"silu": 0, "clamped_swish": 1}
 
 
 def moe_route(x, router_w, row_seq, expert, weight, scoring: str = "softmax_chosen",
-              correction=None) -> None:
+              correction=None, groups: int = 1, keep: int = 1, weight_scale: float = 1.0) -> None:
     """For every row of x [n, w]: the `top` experts of largest float32 logit router_w [E, w] . x
     into `expert` (int32 [n, top], largest first), the softmax over their logits into `weight`
     (float32 [n, top]).  Rows with row_seq < 0 get weights of 0.  scoring "softmax_all": the
     scores are the softmax over all E logits, the choice is by score + correction [E] (None:
-    by the score), and the weights are the chosen scores themselves."""
+    by the score), and the weights are the chosen scores themselves.  scoring "sigmoid": the
+    scores are sigmoid(logit), only experts of the `keep` best of `groups` equal groups of
+    neighbours can be chosen (a group's score: the sum of its two largest), and the weights
+    are the chosen scores over their sum, times `weight_scale`."""
     lib = library("moe")
     if scoring not in ROUTER_SCORINGS:
         raise KernelError(f"moe_route: unknown scoring '{scoring}'")
@@ -1700,15 +1741,30 @@ def moe_route(x, router_w, row_seq, expert, weight, scoring: str = "softmax_chos
                               _gpu(weight, "weight", torch.float32), n, width, n_experts, top,
                               ROUTER_SCORINGS[scoring],
                               None if correction is None else _gpu(correction, "correction", torch.float32),
-                              _stream())
+                              int(groups), int(keep), float(weight_scale), _stream())
     _check(lib, status, "moe_route")
 
 
-def moe_experts(x, w_gate, w_up, w_down, expert, weight, act, out) -> None:
+def _expert_extras(activation, limit, alpha, extra, rows, width):
+    """(activation's code, limit, alpha, rows to add and how they lie) for the experts' kernels."""
+    if activation not in EXPERT_ACTIVATIONS:
+        raise KernelError(f"moe_experts: unknown activation '{activation}'; "
+                          f"known: {sorted(EXPERT_ACTIVATIONS)}")
+    how = (EXPERT_ACTIVATIONS[activation], float(limit), float(alpha))
+    if extra is None:
+        return (*how, None, F32, 1, 0)
+    slices, stride = _splits(extra, rows, width, "extra")
+    return (*how, _gpu(extra, "extra"), _code(extra, "extra"), slices, stride)
+
+
+def moe_experts(x, w_gate, w_up, w_down, expert, weight, act, out, activation="silu", limit=0.0,
+                alpha=1.0, extra=None) -> None:
     """out [n, w] float32 = sum over a row's choices k of weight[r, k] *
     w_down[e] (silu(w_gate[e] x_r) * (w_up[e] x_r)), e = expert[r, k]; w_gate and w_up
     [E, f, w], w_down [E, w, f], all of x's type; `act` [n * top, f] of that type is scratch.
-    A choice e >= E is an identity expert: it adds weight[r, k] * x_r."""
+    A choice e >= E is an identity expert: it adds weight[r, k] * x_r.  activation
+    "clamped_swish" (limit, alpha): as in `swiglu`.  extra: rows [n, w], or float32 slices of
+    them, that are added to the sums."""
     lib = library("moe")
     n, width = x.shape
     n_experts, inter = w_gate.shape[0], w_gate.shape[1]
@@ -1726,7 +1782,7 @@ def moe_experts(x, w_gate, w_up, w_down, expert, weight, act, out) -> None:
                                 _gpu(expert, "expert", torch.int32),
                                 _gpu(weight, "weight", torch.float32), _gpu(act, "act"),
                                 _gpu(out, "out", torch.float32), n, width, inter, n_experts, top,
-                                _stream())
+                                *_expert_extras(activation, limit, alpha, extra, n, width), _stream())
     _check(lib, status, "moe_experts")
 
 
@@ -1739,7 +1795,7 @@ def moe_grouped_supported(dtype, width: int, inter: int, n_experts: int) -> bool
 
 
 def moe_experts_grouped(x, w_gate, w_up, w_down, expert, weight, sorted_pairs, place, starts, act,
-                        sums, out) -> None:
+                        sums, out, activation="silu", limit=0.0, alpha=1.0, extra=None) -> None:
     """`moe_experts` as grouped matrix products on the matrix cores: the (row, choice) pairs are
     laid out by expert on the device, every expert's pairs meet its matrices in tiles, and the
     rows' weighted sums are taken last.  Scratch: sorted_pairs, place [n * top] and starts
@@ -1766,7 +1822,7 @@ def moe_experts_grouped(x, w_gate, w_up, w_down, expert, weight, sorted_pairs, p
         _gpu(sorted_pairs, "sorted_pairs", torch.int32), _gpu(place, "place", torch.int32),
         _gpu(starts, "starts", torch.int32), _gpu(act, "act", torch.bfloat16),
         _gpu(sums, "sums", torch.float32), _gpu(out, "out", torch.float32), n, width, inter,
-        n_experts, top, _stream())
+        n_experts, top, *_expert_extras(activation, limit, alpha, extra, n, width), _stream())
     _check(lib, status, "moe_experts_grouped")
 
 

@@ -6,6 +6,13 @@
 // router outputs, the `top` outputs of largest s + correction (a learned number per output,
 // null: none), and the weights s of the chosen, not renormalised.  Experts: for row r and its
 // choice k with expert e and weight p,  y_r += p W_down,e (silu(W_gate,e x_r) * (W_up,e x_r)).
+// `mode` 2: the scores s = sigmoid(z), the experts in `groups` equal groups of neighbours of which
+// the `keep` with the largest sums of their two largest scores take part (of equal sums the one of
+// lower index), the `top` largest scores among their experts, and the weights s / (sum of the
+// chosen s + 1e-20) * weight_scale.
+// The gated product of an expert is silu(gate) * up, or with the clamped swish (`ExpertAct`), with
+// g = min(gate, limit) and u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1).  The rows of
+// another product (an expert that every row takes) may be added to the sums: `extra`.
 // A router may have more outputs than there are experts: an output beyond the experts is an
 // identity expert, which adds p x_r and has no matrices.
 //
@@ -22,14 +29,84 @@ namespace {
 constexpr int kMaxTop = 64;
 constexpr int kRouteMax = 8;      // experts a lane holds: up to 512 experts
 
+struct ExpertAct {
+  int kind;                       // 0: silu(gate) * up, 1: the clamped swish
+  float limit, alpha;
+};
+
+__device__ __forceinline__ float expert_act(float gate, float up, const ExpertAct& act) {
+  if (act.kind == 0) return gate / (1.0f + expf(-gate)) * up;
+  const float g = fminf(gate, act.limit);
+  const float u = fminf(fmaxf(up, -act.limit), act.limit);
+  return g / (1.0f + expf(-act.alpha * g)) * (u + 1.0f);
+}
+
+// Rows [N, W] that are added to the experts' weighted sums: float32 slices or one bfloat16 tensor
+// (null: none).
+struct ExtraRows {
+  const void* rows;
+  int dtype, slices;
+  size_t slice;
+};
+
+__device__ __forceinline__ float extra_at(const ExtraRows& extra, size_t at) {
+  float sum = 0.f;
+  if (extra.dtype == EI_F32) {
+    const float* p = static_cast<const float*>(extra.rows) + at;
+    for (int s = 0; s < extra.slices; ++s) sum += p[s * extra.slice];
+  } else {
+    sum = ei::bf16_to_f32(static_cast<const bf16_t*>(extra.rows)[at]);
+  }
+  return sum;
+}
+
+// The grouped choice of mode 2 by one wave: lane l holds the scores z[j] of experts l + 64 j.  A
+// group that does not take part gets -1 for its experts' scores (all real ones are in [0, 1]).
+// `scores` is LDS for E numbers and `group_scores` for up to E.
+__device__ __forceinline__ void leave_groups_out(float (&z)[kRouteMax], float* scores,
+                                                 float* group_scores, int E, int groups, int keep) {
+  const int lane = threadIdx.x % EI_WAVE, size = E / groups;
+#pragma unroll
+  for (int j = 0; j < kRouteMax; ++j)
+    if (lane + j * EI_WAVE < E) scores[lane + j * EI_WAVE] = z[j];
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  for (int g = lane; g < groups; g += EI_WAVE) {
+    float first = 0.f, second = 0.f;            // (scores are not negative)
+    for (int i = 0; i < size; ++i) {
+      const float s = scores[g * size + i];
+      if (s > first) { second = first; first = s; }
+      else if (s > second) second = s;
+    }
+    group_scores[g] = first + second;
+  }
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+  for (int j = 0; j < kRouteMax; ++j) {
+    const int e = lane + j * EI_WAVE;
+    if (e >= E) continue;
+    const int g = e / size;
+    const float own = group_scores[g];
+    int ahead = 0;                              // groups that come before this expert's
+    for (int other = 0; other < groups; ++other) {
+      const float s = group_scores[other];
+      if (s > own || (s == own && other < g)) ++ahead;
+    }
+    if (ahead >= keep) z[j] = -1.0f;
+  }
+}
+
 // A block of four waves a row: the waves share the experts' logits out, the first wave chooses.
 template <typename TX>
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
                  const int32_t* __restrict__ row_seq, int32_t* __restrict__ expert,
                  float* __restrict__ weight, int N, int W, int E, int top, int mode,
-                 const float* __restrict__ correction) {
-  __shared__ float logits[kRouteMax * EI_WAVE];
+                 const float* __restrict__ correction, int groups, int keep, float weight_scale) {
+  __shared__ float logits[kRouteMax * EI_WAVE], group_scores[kRouteMax * EI_WAVE];
   const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
   const int row = blockIdx.x;
   int32_t* e_out = expert + static_cast<size_t>(row) * top;
@@ -86,6 +163,12 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
       z[j] = e < E ? score[j] + (correction ? correction[e] : 0.f) : -FLT_MAX;
     }
   }
+  if (mode == 2) {
+#pragma unroll
+    for (int j = 0; j < kRouteMax; ++j)
+      z[j] = lane + j * EI_WAVE < E ? 1.0f / (1.0f + expf(-z[j])) : -FLT_MAX;
+    if (groups > 1 && keep < groups) leave_groups_out(z, logits, group_scores, E, groups, keep);
+  }
   unsigned taken = 0;                            // bit j: this lane's expert lane + 64 j is chosen
   float total = 0.f, largest = 0.f;
   float mine = 0.f;                              // lane k keeps the k-th choice
@@ -114,12 +197,13 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
     }
     if (mode == 1) chosen_score = __shfl(chosen_score, best_e % EI_WAVE, EI_WAVE);
     if (k == 0) largest = best;
-    total += expf(best - largest);
+    total += mode == 2 ? best : expf(best - largest);
     if (lane == k) { mine = mode == 1 ? chosen_score : best; mine_e = best_e; }
   }
   if (lane < top) {
     e_out[lane] = mine_e;
-    w_out[lane] = mode == 1 ? mine : expf(mine - largest) / total;
+    w_out[lane] = mode == 2 ? mine / (total + 1e-20f) * weight_scale
+                            : mode == 1 ? mine : expf(mine - largest) / total;
   }
 }
 
@@ -129,7 +213,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ w_gate, const T* __restrict__ w_up,
                    const int32_t* __restrict__ expert, const float* __restrict__ weight,
-                   T* __restrict__ act, int W, int F, int top, int E) {
+                   T* __restrict__ act, int W, int F, int top, int E, ExpertAct how) {
   const int pair = blockIdx.x;
   if (weight[pair] == 0.f) return;              // a padding row's choice
   const int row = pair / top, e = expert[pair];
@@ -170,7 +254,7 @@ moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ w_gate, const 
   for (int q = 0; q < 4; ++q) {
     const float gate = ei::wave_sum(sg[q]), up = ei::wave_sum(su[q]);
     if (lane == 0 && q < nf)
-      act[static_cast<size_t>(pair) * F + f0 + q] = ei::from_f32<T>(gate / (1.0f + expf(-gate)) * up);
+      act[static_cast<size_t>(pair) * F + f0 + q] = ei::from_f32<T>(expert_act(gate, up, how));
   }
 }
 
@@ -180,7 +264,8 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 moe_down_kernel(const T* __restrict__ act, const T* __restrict__ w_down,
                 const int32_t* __restrict__ expert, const float* __restrict__ weight,
-                float* __restrict__ out, int W, int F, int top, int E, const T* __restrict__ x) {
+                float* __restrict__ out, int W, int F, int top, int E, const T* __restrict__ x,
+                ExtraRows extra) {
   const int row = blockIdx.x;
   const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
   const int c0 = blockIdx.y * 16 + wave * 4;
@@ -222,8 +307,12 @@ moe_down_kernel(const T* __restrict__ act, const T* __restrict__ w_down,
 #pragma unroll
     for (int q = 0; q < 4; ++q) total[q] += p * ei::wave_sum(s[q]);
   }
-  if (lane == 0)
-    for (int q = 0; q < nc; ++q) out[static_cast<size_t>(row) * W + c0 + q] = total[q];
+  if (lane < nc) {
+    float sum = lane == 0 ? total[0] : lane == 1 ? total[1] : lane == 2 ? total[2] : total[3];
+    const size_t at = static_cast<size_t>(row) * W + c0 + lane;
+    if (extra.rows) sum += extra_at(extra, at);
+    out[at] = sum;
+  }
 }
 
 
@@ -288,7 +377,7 @@ __global__ void __launch_bounds__(256)
 moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted,
                 const int32_t* __restrict__ starts, const bf16_t* __restrict__ w1,
                 const bf16_t* __restrict__ w2, bf16_t* __restrict__ out_act,
-                float* __restrict__ out_sum, int E, int N, int K, int top) {
+                float* __restrict__ out_sum, int E, int N, int K, int top, ExpertAct how) {
   constexpr int TM = MB * 16;
   constexpr int PER_THREAD = TM * (KT / 8) / 256 > 0 ? TM * (KT / 8) / 256 : 1;
   __shared__ __attribute__((aligned(16))) bf16_t xs[TM * KT];
@@ -383,8 +472,7 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
       const int n = n_wave + 4 * quarter + i;
       if (n >= N) continue;
       if (GATED) {
-        const float gate = acc1[mb][i], up = acc2[mb][i];
-        out_act[at + n] = ei::f32_to_bf16(gate / (1.0f + expf(-gate)) * up);
+        out_act[at + n] = ei::f32_to_bf16(expert_act(acc1[mb][i], acc2[mb][i], how));
       } else {
         out_sum[at + n] = acc1[mb][i];
       }
@@ -395,7 +483,8 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
 // out [rows, W] = sum over a row's choices of weight * the choice's product row.
 __global__ void moe_combine_kernel(const float* __restrict__ sums, const int32_t* __restrict__ place,
                                    const float* __restrict__ weight, float* __restrict__ out,
-                                   int W, int top, size_t total, const bf16_t* __restrict__ x) {
+                                   int W, int top, size_t total, const bf16_t* __restrict__ x,
+                                   ExtraRows extra) {
   const size_t start = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
   for (size_t idx = start; idx < total; idx += step) {
@@ -406,29 +495,40 @@ __global__ void moe_combine_kernel(const float* __restrict__ sums, const int32_t
       if (q >= 0) sum += weight[row * top + k] * sums[static_cast<size_t>(q) * W + col];
       else if (q == -2) sum += weight[row * top + k] * ei::bf16_to_f32(x[idx]);   // identity
     }
+    if (extra.rows) sum += extra_at(extra, idx);
     out[idx] = sum;
   }
+}
+
+bool known_act(int kind) { return kind == 0 || kind == 1; }
+
+bool extra_fits(const void* rows, int dtype, int slices, long long slice) {
+  return !rows || (slices >= 1 && slice >= 0 && (dtype == EI_F32 || (dtype == EI_BF16 && slices == 1)));
 }
 
 }  // namespace
 
 extern "C" int ei_moe_route(const void* x, int x_dtype, const float* w_router, const int32_t* row_seq,
                             int32_t* expert, float* weight, int N, int W, int E, int top,
-                            int mode, const float* correction, hipStream_t stream) {
+                            int mode, const float* correction, int groups, int keep,
+                            float weight_scale, hipStream_t stream) {
   EI_REQUIRE(x && w_router && expert && weight && N > 0 && W > 0, "moe_route: bad arguments");
   EI_REQUIRE(E >= 1 && E <= kRouteMax * EI_WAVE && top >= 1 && top <= E && top <= kMaxTop,
              "moe_route: up to 512 experts, of which 1 to 64 are chosen");
-  EI_REQUIRE(mode == 0 || mode == 1, "moe_route: unknown mode");
+  EI_REQUIRE(mode >= 0 && mode <= 2, "moe_route: unknown mode");
+  EI_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && (groups == 1 || mode == 2) &&
+                 top <= E / groups * keep,
+             "moe_route: equal groups of experts, enough of them kept for the choice");
   const int threads = 256;
   const unsigned blocks = static_cast<unsigned>(N);
   if (x_dtype == EI_F32)
     moe_route_kernel<float><<<blocks, threads, 0, stream>>>(static_cast<const float*>(x), w_router,
                                                             row_seq, expert, weight, N, W, E, top,
-                                                            mode, correction);
+                                                            mode, correction, groups, keep, weight_scale);
   else if (x_dtype == EI_BF16)
     moe_route_kernel<bf16_t><<<blocks, threads, 0, stream>>>(static_cast<const bf16_t*>(x), w_router,
                                                              row_seq, expert, weight, N, W, E, top,
-                                                            mode, correction);
+                                                            mode, correction, groups, keep, weight_scale);
   else
     EI_REQUIRE(false, "moe_route: unknown dtype");
   EI_LAUNCH_CHECK();
@@ -436,8 +536,15 @@ extern "C" int ei_moe_route(const void* x, int x_dtype, const float* w_router, c
 
 extern "C" int ei_moe_experts(const void* x, const void* w_gate, const void* w_up, const void* w_down,
                               int dtype, const int32_t* expert, const float* weight, void* act,
-                              float* out, int N, int W, int F, int E, int top, hipStream_t stream) {
+                              float* out, int N, int W, int F, int E, int top, int act_kind,
+                              float limit, float alpha, const void* extra_rows, int extra_dtype,
+                              int extra_slices, long long extra_slice, hipStream_t stream) {
   EI_REQUIRE(x && w_gate && w_up && w_down && expert && weight && act && out, "moe_experts: null pointer");
+  EI_REQUIRE(known_act(act_kind), "moe_experts: unknown activation");
+  EI_REQUIRE(extra_fits(extra_rows, extra_dtype, extra_slices, extra_slice),
+             "moe_experts: the rows to add have the wrong type");
+  const ExpertAct how{act_kind, limit, alpha};
+  const ExtraRows extra{extra_rows, extra_dtype, extra_slices, static_cast<size_t>(extra_slice)};
   EI_REQUIRE(N > 0 && W > 0 && F > 0 && top >= 1, "moe_experts: sizes must be positive");
   EI_REQUIRE(static_cast<long long>(N) * top <= 0x7fffffffLL && (F + 15) / 16 <= 65535 &&
                  (W + 15) / 16 <= 65535, "moe_experts: too large for one launch");
@@ -446,10 +553,10 @@ extern "C" int ei_moe_experts(const void* x, const void* w_gate, const void* w_u
   do {                                                                                         \
     moe_gate_up_kernel<T><<<grid_up, 256, 0, stream>>>(                                        \
         static_cast<const T*>(x), static_cast<const T*>(w_gate), static_cast<const T*>(w_up),  \
-        expert, weight, static_cast<T*>(act), W, F, top, E);                                   \
+        expert, weight, static_cast<T*>(act), W, F, top, E, how);                              \
     moe_down_kernel<T><<<grid_down, 256, 0, stream>>>(                                         \
         static_cast<const T*>(act), static_cast<const T*>(w_down), expert, weight, out, W, F, top, \
-        E, static_cast<const T*>(x));                                                          \
+        E, static_cast<const T*>(x), extra);                                                   \
   } while (0)
   if (dtype == EI_F32) EI_MOE(float);
   else if (dtype == EI_BF16) EI_MOE(bf16_t);
@@ -469,7 +576,14 @@ extern "C" int ei_moe_experts_grouped(const void* x, const void* w_gate, const v
                                       const void* w_down, const int32_t* expert, const float* weight,
                                       int32_t* sorted, int32_t* place, int32_t* starts, void* act,
                                       float* sums, float* out, int N, int W, int F, int E, int top,
-                                      hipStream_t stream) {
+                                      int act_kind, float limit, float alpha,
+                                      const void* extra_rows, int extra_dtype, int extra_slices,
+                                      long long extra_slice, hipStream_t stream) {
+  EI_REQUIRE(known_act(act_kind), "moe_experts_grouped: unknown activation");
+  EI_REQUIRE(extra_fits(extra_rows, extra_dtype, extra_slices, extra_slice),
+             "moe_experts_grouped: the rows to add have the wrong type");
+  const ExpertAct how{act_kind, limit, alpha};
+  const ExtraRows extra{extra_rows, extra_dtype, extra_slices, static_cast<size_t>(extra_slice)};
   EI_REQUIRE(x && w_gate && w_up && w_down && expert && weight && sorted && place && starts && act &&
                  sums && out, "moe_experts_grouped: null pointer");
   EI_REQUIRE(N > 0 && top >= 1 && E >= 1 && ei_moe_grouped_supported(EI_BF16, W, F, E),
@@ -491,23 +605,23 @@ extern "C" int ei_moe_experts_grouped(const void* x, const void* w_gate, const v
     // measured at 2, 16 and 128 pairs over 8 experts of 2,816 x 2,048)
     const bool few = P <= 4;
     if (few && W % 256 == 0)
-      moe_gemm_kernel<2, true, 256><<<grid_up, 256, 0, stream>>>(xb, sorted, starts, g, u, ab, nullptr, E, F, W, top);
+      moe_gemm_kernel<2, true, 256><<<grid_up, 256, 0, stream>>>(xb, sorted, starts, g, u, ab, nullptr, E, F, W, top, how);
     else
-      moe_gemm_kernel<2, true, 64><<<grid_up, 256, 0, stream>>>(xb, sorted, starts, g, u, ab, nullptr, E, F, W, top);
+      moe_gemm_kernel<2, true, 64><<<grid_up, 256, 0, stream>>>(xb, sorted, starts, g, u, ab, nullptr, E, F, W, top, how);
     if (few && F % 256 == 0)
-      moe_gemm_kernel<2, false, 256><<<grid_down, 256, 0, stream>>>(ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top);
+      moe_gemm_kernel<2, false, 256><<<grid_down, 256, 0, stream>>>(ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top, how);
     else
-      moe_gemm_kernel<2, false, 64><<<grid_down, 256, 0, stream>>>(ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top);
+      moe_gemm_kernel<2, false, 64><<<grid_down, 256, 0, stream>>>(ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top, how);
   } else {
     const unsigned tiles = static_cast<unsigned>((P + 127) / 128 + E);
     moe_gemm_kernel<8, true, 64><<<dim3(tiles, (F + kTileN - 1) / kTileN), 256, 0, stream>>>(
-        xb, sorted, starts, g, u, ab, nullptr, E, F, W, top);
+        xb, sorted, starts, g, u, ab, nullptr, E, F, W, top, how);
     moe_gemm_kernel<8, false, 64><<<dim3(tiles, (W + kTileN - 1) / kTileN), 256, 0, stream>>>(
-        ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top);
+        ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top, how);
   }
   const size_t total = static_cast<size_t>(N) * W;
   size_t blocks = (total + 255) / 256;
   if (blocks > static_cast<size_t>(ei_compute_units()) * 16) blocks = static_cast<size_t>(ei_compute_units()) * 16;
-  moe_combine_kernel<<<static_cast<unsigned>(blocks), 256, 0, stream>>>(sums, place, weight, out, W, top, total, xb);
+  moe_combine_kernel<<<static_cast<unsigned>(blocks), 256, 0, stream>>>(sums, place, weight, out, W, top, total, xb, extra);
   EI_LAUNCH_CHECK();
 }

@@ -631,6 +631,9 @@ extern "C" int ei_projection_norm_store(
 // part of (p + 1) / temp_every.  gate_out: the float32 sums of the nq columns from `gate_at` on
 // (one number a query head) go to gate_out [N, nq] for the attention kernel's output gate.
 // nkv may be 0 for rows that hold queries only (a layer that reads another layer's keys).
+// bias: float32 [row_stride] added to the sums of q, k and v, or null (what a product left to this
+// kernel).  turn_scale multiplies cosine and sine.  unit_norm: a query or key head is divided by
+// the root of its mean square + eps after the rotation (an RMS norm without a weight).
 namespace {
 
 constexpr int kHeadStoreMax = 8;  // elements a lane: head sizes up to 512
@@ -651,7 +654,8 @@ __global__ void head_store_kernel(
     TO* __restrict__ q_out, TO* __restrict__ k_pages, TO* __restrict__ v_pages,
     float* __restrict__ v_first, int v_mode, const float* __restrict__ v_lambda,
     int N, int nq, int nkv, int D, int DV, int write_cache, float temp_coef, int temp_every,
-    float* __restrict__ gate_out, size_t gate_at) {
+    float* __restrict__ gate_out, size_t gate_at, const float* __restrict__ bias,
+    float turn_scale, int unit_norm) {
   const int heads = nq + 2 * nkv;
   const int wave = (blockIdx.x * blockDim.x + threadIdx.x) / EI_WAVE;
   const int lane = threadIdx.x % EI_WAVE;
@@ -674,8 +678,10 @@ __global__ void head_store_kernel(
     TO* dst = write_cache
                   ? v_pages + ((page_slot * nkv + h) * EI_PAGE + pos % EI_PAGE) * static_cast<size_t>(DV)
                   : nullptr;
+    const float* b = bias ? bias + static_cast<size_t>(nq + nkv) * D + static_cast<size_t>(h) * DV : nullptr;
     for (int e = lane; e < DV; e += EI_WAVE) {
       float v = sliced(src + e, nsplit, split_stride);
+      if (b) v += b[e];
       if (v_mode == 1) first[e] = v;
       else if (v_mode == 2) v = (1.0f - lambda) * v + lambda * first[e];
       if (dst) dst[e] = ei::from_f32<TO>(v);
@@ -686,6 +692,7 @@ __global__ void head_store_kernel(
   if (!is_q && !write_cache) return;
   const TI* src = src_row + static_cast<size_t>(head) * D;
   const float* w = is_q ? q_norm_w : k_norm_w;
+  const float* b = bias ? bias + static_cast<size_t>(head) * D : nullptr;
   const int rhalf = R / 2;
   float x[kHeadStoreMax], y[kHeadStoreMax];   // a lane's elements and their partners in the rotation
   float sum = 0.f;
@@ -694,9 +701,14 @@ __global__ void head_store_kernel(
     const int e = lane + j * EI_WAVE;
     x[j] = y[j] = 0.f;
     if (e < D) {
+      const int partner = e < rhalf ? e + rhalf : e - rhalf;
       x[j] = sliced(src + e, nsplit, split_stride);
+      if (b) x[j] += b[e];
       sum += x[j] * x[j];
-      if (e < R) y[j] = sliced(src + (e < rhalf ? e + rhalf : e - rhalf), nsplit, split_stride);
+      if (e < R) {
+        y[j] = sliced(src + partner, nsplit, split_stride);
+        if (b) y[j] += b[partner];
+      }
     }
   }
   float inv = 1.0f;
@@ -707,6 +719,7 @@ __global__ void head_store_kernel(
     gate_out[static_cast<size_t>(row) * nq + head] = sliced(src_row + gate_at + head, nsplit, split_stride);
   TO* dst = is_q ? q_out + (static_cast<size_t>(row) * nq + head) * D
                  : k_pages + ((page_slot * nkv + (head - nq)) * EI_PAGE + pos % EI_PAGE) * static_cast<size_t>(D);
+  float turned = 0.f;                         // the lane's squares after the rotation
 #pragma unroll
   for (int j = 0; j < kHeadStoreMax; ++j) {
     const int e = lane + j * EI_WAVE;
@@ -720,9 +733,18 @@ __global__ void head_store_kernel(
       const float angle = static_cast<float>((turns - floor(turns)) * 6.283185307179586);
       float sn, cs;
       sincosf(angle, &sn, &cs);
+      cs *= turn_scale;
+      sn *= turn_scale;
       v = e < rhalf ? v * cs - p * sn : v * cs + p * sn;
     }
-    dst[e] = ei::from_f32<TO>(v * warm);
+    x[j] = v;
+    turned += v * v;
+  }
+  const float unit = unit_norm ? 1.0f / sqrtf(ei::wave_sum(turned) / static_cast<float>(D) + eps) : 1.0f;
+#pragma unroll
+  for (int j = 0; j < kHeadStoreMax; ++j) {
+    const int e = lane + j * EI_WAVE;
+    if (e < D) dst[e] = ei::from_f32<TO>(x[j] * unit * warm);
   }
 }
 
@@ -738,6 +760,13 @@ __device__ __forceinline__ void sliced8(const TI* p, int nsplit, size_t split_st
   }
 }
 
+__device__ __forceinline__ void add8(const float* p, float (&v)[8]) {
+  float more[8];
+  ei::VecN<float, 8>::load(p, more);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) v[i] += more[i];
+}
+
 // The same in 16-byte pieces, for head sizes, rotated halves and strides that are multiples of
 // 8: a lane takes 8 neighbouring elements, the G lanes of a head (G the power of two at or
 // above the widest head's eighth) add their squares by shuffles, and a wave takes 64 / G
@@ -751,7 +780,8 @@ __global__ void head_store_vec_kernel(
     TO* __restrict__ q_out, TO* __restrict__ k_pages, TO* __restrict__ v_pages,
     float* __restrict__ v_first, int v_mode, const float* __restrict__ v_lambda,
     int N, int nq, int nkv, int D, int DV, int write_cache, int G, float temp_coef, int temp_every,
-    float* __restrict__ gate_out, size_t gate_at) {
+    float* __restrict__ gate_out, size_t gate_at, const float* __restrict__ bias,
+    float turn_scale, int unit_norm) {
   const int heads = nq + 2 * nkv;
   const size_t thread = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
   const size_t item = thread / G;
@@ -773,8 +803,9 @@ __global__ void head_store_vec_kernel(
   if (is_v) {
     if (!live) return;          // (value heads take no part in any shuffle: whole groups leave)
     const int h = head - nq - nkv;
-    sliced8(src_row + static_cast<size_t>(nq + nkv) * D + static_cast<size_t>(h) * DV + j * 8, nsplit,
-            split_stride, x);
+    const size_t column = static_cast<size_t>(nq + nkv) * D + static_cast<size_t>(h) * DV + j * 8;
+    sliced8(src_row + column, nsplit, split_stride, x);
+    if (bias) add8(bias + column, x);
     if (v_mode) {
       float* first = v_first + static_cast<size_t>(row) * nkv * DV + static_cast<size_t>(h) * DV + j * 8;
       if (v_mode == 1) {
@@ -800,6 +831,10 @@ __global__ void head_store_vec_kernel(
   float y[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
   if (live) sliced8(src + e0, nsplit, split_stride, x);
   if (turns) sliced8(src + partner0, nsplit, split_stride, y);
+  if (bias && live) {
+    add8(bias + static_cast<size_t>(head) * D + e0, x);
+    if (turns) add8(bias + static_cast<size_t>(head) * D + partner0, y);
+  }
   float inv = 1.0f;
   if (w) {                      // (uniform: every lane of the wave takes the shuffles)
     float sum = 0.f;
@@ -808,8 +843,9 @@ __global__ void head_store_vec_kernel(
     for (int offset = G / 2; offset > 0; offset >>= 1) sum += __shfl_xor(sum, offset, EI_WAVE);
     inv = 1.0f / sqrtf(sum / static_cast<float>(D) + eps);
   }
-  if (!live) return;
-  if (w) {
+  // (uniform again: with a norm behind the rotation every lane stays for its shuffles)
+  if (!live && !unit_norm) return;
+  if (w && live) {
     float wx[8];
     ei::VecN<float, 8>::load(w + e0, wx);
 #pragma unroll
@@ -828,8 +864,20 @@ __global__ void head_store_vec_kernel(
       const float angle = static_cast<float>((whole - floor(whole)) * 6.283185307179586);
       float sn, cs;
       sincosf(angle, &sn, &cs);
+      cs *= turn_scale;
+      sn *= turn_scale;
       x[i] = e0 < rhalf ? x[i] * cs - y[i] * sn : x[i] * cs + y[i] * sn;
     }
+  }
+  if (unit_norm) {
+    float sum = 0.f;              // (lanes without elements hold zeros)
+#pragma unroll
+    for (int i = 0; i < 8; ++i) sum += x[i] * x[i];
+    for (int offset = G / 2; offset > 0; offset >>= 1) sum += __shfl_xor(sum, offset, EI_WAVE);
+    const float unit = 1.0f / sqrtf(sum / static_cast<float>(D) + eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] *= unit;
+    if (!live) return;
   }
   if (is_q && temp_every > 0) {
     const float warm = 1.0f + temp_coef * logf(static_cast<float>((pos + 1) / temp_every) + 1.0f);
@@ -851,7 +899,8 @@ extern "C" int ei_head_store(
     const int32_t* row_pos, const int32_t* row_seq, const int32_t* page_table, int table_width,
     void* q_out, void* k_pages, void* v_pages, int out_dtype, float* v_first, int v_mode,
     const float* v_lambda, int N, int nq, int nkv, int D, int DV, int write_cache,
-    float temp_coef, int temp_every, float* gate_out, long long gate_at, hipStream_t stream) {
+    float temp_coef, int temp_every, float* gate_out, long long gate_at, const float* bias,
+    float turn_scale, int unit_norm, hipStream_t stream) {
   EI_REQUIRE(N > 0 && nq > 0 && nkv >= 0 && D > 0 && DV > 0, "head_store: sizes must be positive");
   EI_REQUIRE(nkv > 0 || !write_cache, "head_store: rows without keys cannot write the cache");
   EI_REQUIRE(temp_every >= 0, "head_store: negative temperature step");
@@ -877,7 +926,7 @@ extern "C" int ei_head_store(
   const auto aligned16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
   const bool vec = D % 8 == 0 && DV % 8 == 0 && R % 16 == 0 && rs % 8 == 0 && (nsplit == 1 || ss % 8 == 0) &&
                    aligned16(proj) && aligned16(q_out) && aligned16(k_pages) && aligned16(v_pages) &&
-                   aligned16(v_first) && aligned16(q_norm_w) && aligned16(k_norm_w);
+                   aligned16(v_first) && aligned16(q_norm_w) && aligned16(k_norm_w) && aligned16(bias);
   if (vec) {
     int G = 1;
     while (G * 8 < (D > DV ? D : DV)) G *= 2;
@@ -888,7 +937,7 @@ extern "C" int ei_head_store(
       static_cast<const TI*>(proj), nsplit, ss, rs, q_norm_w, k_norm_w, eps, freqs, R, row_pos, \
       row_seq, page_table, table_width, static_cast<TO*>(q_out), static_cast<TO*>(k_pages),    \
       static_cast<TO*>(v_pages), v_first, v_mode, v_lambda, N, nq, nkv, D, DV, write_cache, G,  \
-      temp_coef, temp_every, gate_out, static_cast<size_t>(gate_at))
+      temp_coef, temp_every, gate_out, static_cast<size_t>(gate_at), bias, turn_scale, unit_norm)
     if (in_dtype == EI_F32 && out_dtype == EI_F32) EI_HSV(float, float);
     else if (in_dtype == EI_F32 && out_dtype == EI_BF16) EI_HSV(float, bf16_t);
     else if (in_dtype == EI_BF16 && out_dtype == EI_BF16) EI_HSV(bf16_t, bf16_t);
@@ -901,7 +950,7 @@ extern "C" int ei_head_store(
       static_cast<const TI*>(proj), nsplit, ss, rs, q_norm_w, k_norm_w, eps, freqs, R, row_pos, \
       row_seq, page_table, table_width, static_cast<TO*>(q_out), static_cast<TO*>(k_pages),    \
       static_cast<TO*>(v_pages), v_first, v_mode, v_lambda, N, nq, nkv, D, DV, write_cache,     \
-      temp_coef, temp_every, gate_out, static_cast<size_t>(gate_at))
+      temp_coef, temp_every, gate_out, static_cast<size_t>(gate_at), bias, turn_scale, unit_norm)
   if (in_dtype == EI_F32 && out_dtype == EI_F32) EI_HS(float, float);
   else if (in_dtype == EI_F32 && out_dtype == EI_BF16) EI_HS(float, bf16_t);
   else if (in_dtype == EI_BF16 && out_dtype == EI_BF16) EI_HS(bf16_t, bf16_t);

@@ -23,7 +23,8 @@ variations are options of the spec and need no subclass: `embedding_scale` multi
 embedding rows, `embedding_norm` norms them, `logit_scale` and `logit_softcap` scale and cap
 the logits, and `loop` (`config.specs.LoopSpec`) runs a span of layers several times, each
 pass with caches of its own, the stream being made anew before every pass from itself and the
-embedding output by a matrix [hidden, 2 hidden] and a vector per pass.  A subclass whose methods launch anything that a HIP graph
+embedding output by a matrix [hidden, 2 hidden] and a vector per pass, or only added the vector
+to (`remix` False).  A subclass whose methods launch anything that a HIP graph
 cannot hold says so with `seams_capture_safe = False`; decode then runs eagerly.
 """
 from __future__ import annotations
@@ -66,8 +67,9 @@ def model_parameters(spec: ModelSpec) -> Dict[str, ParamSpec]:
     params["head.weight"] = ParamSpec((spec.vocab_size, spec.hidden_size))
     params["head.bias"] = ParamSpec((spec.vocab_size,), optional=True)
     if spec.loop is not None:
-        params["loop.in.weight"] = ParamSpec((spec.hidden_size, 2 * spec.hidden_size),
-                                             scale=(2.0 * spec.hidden_size) ** -0.5)
+        if spec.loop.remix:
+            params["loop.in.weight"] = ParamSpec((spec.hidden_size, 2 * spec.hidden_size),
+                                                 scale=(2.0 * spec.hidden_size) ** -0.5)
         params["loop.step"] = ParamSpec((spec.loop.times, spec.hidden_size), scale=0.1)
     return params
 
@@ -173,7 +175,8 @@ class DecoderModel:
         self.loop_in = self.loop_step = None
         self._pass_starts = {}
         if spec.loop is not None:
-            self.loop_in = Linear(params["loop.in.weight"], self.dtype, self.device)
+            if spec.loop.remix:
+                self.loop_in = Linear(params["loop.in.weight"], self.dtype, self.device)
             self.loop_step = params["loop.step"].to(device=self.device,
                                                     dtype=torch.float32).contiguous()
             self._pass_starts = {run: turn for turn, run in
@@ -339,10 +342,13 @@ class DecoderModel:
 
     def enter_pass(self, ctx, residual, pending, embedded, turn: int):
         """Before pass `turn` of the loop: x <- W [x ; x0] + step[turn], with x0 the embedding
-        output.  The product reads both streams in the step's storage type; its float32 result
+        output (x <- x + step[turn] in a loop that does not remix).  The product reads both streams in the step's storage type; its float32 result
         takes the stream's place."""
         if pending is not None:
             raise ValueError("a pass of the loop starts after a block that left a delta pending")
+        if self.loop_in is None:
+            lib.bias_rows(self.loop_step[turn], residual, accumulate=True)
+            return None
         rows, hidden = residual.shape
         both = ctx.buffer("loop.both", (rows, 2 * hidden))
         lib.concat_cast(residual, embedded, both)

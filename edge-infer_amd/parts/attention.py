@@ -32,12 +32,19 @@ So do a rotation of neighbouring pairs (position kind "rope_pairs": a query and 
 the same score when both are permuted alike, so the rows of the q and k projections are
 reordered when the part is built, evens then odds within a head's rotated part, and the
 rotation of halves does the rest), `query_temperature` (queries grow with the position),
+`qk_unit_norm` (queries and keys brought to unit RMS after the rotation),
 `output_gate = "head"` (one gate a head, applied by the attention kernel), `shared_kv` (a part
 without key and value projections, whose runs read what another run cached) and `pool`
 (besides its window a query sees one key and value, the means, for every block of `pool`
 positions that lies wholly before the window: the part keeps them in a second paged cache of
 its own, one entry a block, which `lib.pool_store` fills from the cached tokens as blocks
-become complete, and the generic kernel walks after the window).
+become complete, and the generic kernel walks after the window).  Biases of these projections
+are added by the store kernel where the product leaves them to it.
+
+`keep_first`: with a window, the sequence's first positions stay visible however far back they
+lie; the cache never gives their pages back, and every kernel takes the pages (or tiles) of them
+that lie before the window first.  The matrix-core kernels take `output_gate = True` into their
+epilogue; beside the generic kernel it is a launch of its own.
 """
 from __future__ import annotations
 
@@ -141,7 +148,7 @@ class Attention:
             keep = None if spec.cache_span == 0 or keep is None else max(keep, spec.cache_span)
         return KVRequest(n_kv_heads=spec.n_kv_heads, head_dim=spec.head_dim, window=keep,
                          value_dim=None if spec.v_dim == spec.head_dim else spec.v_dim,
-                         chunk=spec.chunk)
+                         chunk=spec.chunk, keep_first=0 if keep is None else spec.keep_first)
 
     POOL = "pool"      # the name of the pooled cache under the run's own cache id
 
@@ -184,7 +191,7 @@ class Attention:
         """Whether the part norms, rotates and stores through `lib.head_store`."""
         return (spec.position.kind in ("rope_half", "rope_pairs")
                 or spec.value_mix in ("source", "mix") or bool(spec.output_gate)
-                or spec.query_temperature is not None or spec.shared_kv or spec.pool is not None)
+                or spec.qk_unit_norm or spec.query_temperature is not None or spec.shared_kv or spec.pool is not None)
 
     @classmethod
     def check(cls, spec):
@@ -201,8 +208,10 @@ class Attention:
                                  "with position kinds 'rope_half', 'rope_pairs' and 'none'")
             if spec.qk_norm and spec.qk_norm_scope != "head":
                 raise ValueError("attention: this store norms per head only")
-            if spec.talking_heads or spec.qkv_bias:
-                raise ValueError("attention: this store takes no biases and no mixed scores")
+            if spec.talking_heads:
+                raise ValueError("attention: this store takes no mixed scores")
+            if spec.shared_kv and spec.qkv_bias:
+                raise ValueError("attention: a part without keys of its own takes no biases")
             if not (1 <= spec.head_dim <= 256 and 1 <= spec.v_dim <= 256):
                 raise ValueError("attention: key and value head sizes must lie in 1..256, got "
                                  f"{spec.head_dim} and {spec.v_dim}")
@@ -231,6 +240,14 @@ class Attention:
             raise ValueError("attention: talking heads with a distance term are not implemented")
         if spec.window is not None and spec.window < 1:
             raise ValueError("attention: a window must be at least 1")
+        if spec.keep_first < 0:
+            raise ValueError("attention: a negative number of kept first positions")
+        if spec.keep_first and (spec.chunk is not None or spec.talking_heads):
+            raise ValueError("attention: kept first positions with chunks or mixed scores are not "
+                             "implemented")
+        if spec.keep_first and spec.pool is not None:
+            raise ValueError("attention: kept first positions beside pooled blocks are not "
+                             "implemented")
         if spec.output_gate not in (False, True, "head"):
             raise ValueError(f"attention: unknown output_gate {spec.output_gate!r}")
         if spec.pool is not None:
@@ -255,23 +272,30 @@ class Attention:
         q_weight = params["q_proj.weight"]
         k_weight = None if spec.shared_kv else params["k_proj.weight"]
         position_spec = spec.position
+        biases = {name: params[f"{name}.bias"] for name in ("q_proj", "k_proj", "v_proj")
+                  if f"{name}.bias" in params}
         if spec.position.kind == "rope_pairs":
             # neighbouring pairs (2i, 2i + 1) become the pairs (i, i + R/2) of permuted rows
             order = self._pairs_to_halves(spec.head_dim, spec.position.dim)
             q_weight = self._permute_heads(q_weight, spec.n_heads, order)
             if k_weight is not None:
                 k_weight = self._permute_heads(k_weight, spec.n_kv_heads, order)
+            for name, heads in (("q_proj", spec.n_heads), ("k_proj", spec.n_kv_heads)):
+                if name in biases:
+                    biases[name] = self._permute_heads(biases[name], heads, order)
             position_spec = dataclasses.replace(spec.position, kind="rope_half", scaling=None)
         fused = torch.cat([q_weight]
                           + ([] if spec.shared_kv else [k_weight, params["v_proj.weight"]])
                           + ([params["gate_proj.weight"]] if spec.output_gate else []), dim=0)
         names = ("q_proj",) if spec.shared_kv else ("q_proj", "k_proj", "v_proj")
         fused_bias = None
-        if any(f"{name}.bias" in params for name in names):   # absent ones count as zero
+        if any(name in biases for name in names):   # absent ones count as zero
             fused_bias = torch.cat([
-                params[f"{name}.bias"] if f"{name}.bias" in params
+                biases[name] if name in biases
                 else params[f"{name}.weight"].new_zeros(params[f"{name}.weight"].shape[0])
-                for name in names])
+                for name in names]
+                + ([params["gate_proj.weight"].new_zeros(params["gate_proj.weight"].shape[0])]
+                   if spec.output_gate else []))
         self.qkv = Linear(fused, dtype, device, bias=fused_bias)
         self.o = Linear(params["o_proj.weight"], dtype, device, bias=params.get("o_proj.bias"))
         self.q_norm = self.k_norm = None
@@ -313,10 +337,13 @@ class Attention:
         # beside the matrix-core kernels the pooled blocks are gathered by the generic kernel
         # (they are few: one for `pool` tokens) and taken in as one more slice of the softmax
         self.pooled_aside = self.matrix_cores and spec.pool is not None
-        # chunk, slopes, sink: what the kernels take beyond a window
+        # chunk, slopes, sink, kept first positions: what the kernels take beyond a window
         self.wide = self.wide_keys(spec, dtype)
-        self.extras = dict(chunk=spec.chunk, slopes=self.slopes, sinks=self.sinks)
-        self.has_extras = spec.chunk is not None or self.slopes is not None or self.sinks is not None
+        self.keep_first = spec.keep_first if spec.window is not None else 0
+        self.extras = dict(chunk=spec.chunk, slopes=self.slopes, sinks=self.sinks,
+                           keep_first=self.keep_first)
+        self.has_extras = (spec.chunk is not None or self.slopes is not None
+                           or self.sinks is not None or self.keep_first > 0)
         self.compute_units = lib.compute_units(device)     # the chip's size, for launch plans
         self._decode_launches = {}     # (sequences, pages of context) -> decode_launch's answer
 
@@ -429,7 +456,7 @@ class Attention:
         kernel: blocks of 4 waves and enough slices to put about two blocks on each compute
         unit, never more than there are pages."""
         if self.spec.window is not None:
-            context = min(context, self.spec.window + PAGE_TOKENS - 1)
+            context = min(context, self.spec.window + self.keep_first + PAGE_TOKENS - 1)
         if self.spec.chunk is not None:
             context = min(context, self.spec.chunk + PAGE_TOKENS - 1)
         pages = max(1, (context + PAGE_TOKENS - 1) // PAGE_TOKENS)
@@ -491,10 +518,14 @@ class Attention:
         meta = ctx.meta
         group_index, k_pages, v_pages = ctx.cache.kv(entry.cache)
         page_table = meta.page_table(group_index)
-        # (the kernel that norms and stores the whole projection adds its bias as well)
-        qkv, bias = (self.qkv.forward(ctx, x, "attn.qkv", bias_later=True) if self.whole_store
+        # (these store kernels add the projection's bias as well)
+        qkv, bias = (self.qkv.forward(ctx, x, "attn.qkv", bias_later=True)
+                     if self.whole_store or self.general
                      else (self.qkv.forward(ctx, x, "attn.qkv"), None))
         gate, pooled, aside = None, {}, {}
+        # a gate for every element of the heads: in the matrix-core kernels' epilogue
+        wide_gate = ((qkv, self.gate_column)
+                     if spec.output_gate is True and self.matrix_cores else None)
         if self.general:
             q = ctx.buffer("attn.q", (n, spec.q_width))
             v_first, v_mode = None, 0
@@ -520,7 +551,9 @@ class Attention:
                            self.own_kv_heads, spec.head_dim, spec.v_dim,
                            write_cache=entry.writes_cache, v_first=v_first, v_mode=v_mode,
                            v_lambda=self.value_lambda, query_temperature=spec.query_temperature,
-                           gate_out=gate, gate_column=self.gate_column)
+                           gate_out=gate, gate_column=self.gate_column, bias=bias,
+                           turn_scale=getattr(self.position, "magnitude", 1.0),
+                           unit_norm=spec.qk_unit_norm)
             if spec.pool is not None:
                 # the blocks that this step's rows complete, from the keys as the cache holds them
                 pool_group, pool_k, pool_v = ctx.cache.kv((entry.own_id, self.POOL))
@@ -587,7 +620,7 @@ class Attention:
                                           spec.head_dim, window=spec.window, scale=self.scale,
                                           n_splits=splits, part_o=part_o, part_ml=part_ml,
                                           waves=waves, longest=meta.longest, heads=heads,
-                                          gate=gate, **aside, **self.extras)
+                                          gate=gate, wide_gate=wide_gate, **aside, **self.extras)
             else:
                 item_seq, item_row0, item_npos, n_items = self._items(ctx, "attention.decode_items")
                 if self.wide:
@@ -618,7 +651,8 @@ class Attention:
                                            spec.n_kv_heads, spec.head_dim, window=spec.window,
                                            scale=self.scale, key_ways=key_ways,
                                            pair_items=len({(seq.start, seq.count) for seq in ctx.sequences}) == 1,
-                                           largest_item=largest, gate=gate, **aside, **self.extras)
+                                           largest_item=largest, gate=gate, wide_gate=wide_gate,
+                                           **aside, **self.extras)
             elif self.wide:
                 lib.attention_wide(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items,
                                    meta.row_pos, meta.row_seq, page_table, out, spec.n_heads,
@@ -630,7 +664,7 @@ class Attention:
                               meta.row_pos, meta.row_seq, page_table, out, spec.n_heads,
                               spec.n_kv_heads, spec.head_dim, window=spec.window,
                               scale=self.scale, **more)
-        if spec.output_gate and not self.head_gate:
+        if spec.output_gate and not self.head_gate and wide_gate is None:
             lib.gate_rows(qkv, self.gate_column, out)
         ctx.release(qkv, None if isinstance(q, lib.DecodeProjection) else q, part_o, part_ml, gate,
                     aside.get("pool_o"), aside.get("pool_ml"))

@@ -28,6 +28,7 @@ class KVRequest:
     [kv_heads, 64, head_dim] of keys and [kv_heads, 64, value_dim] of values (`value_dim`
     None: as wide as the keys).  `chunk`: a query sees only keys of its own block of that many
     positions, so pages that lie wholly before the block of the next position are given back.
+    `keep_first` k: the sequence's first k positions are kept whatever the window gives back.
     `stride` s > 1: the entry holds one key and value for every complete block of s positions
     (what a mixer derives from the tokens of the block), so a sequence of n tokens holds
     n // s of them, in pages of 64 like any other.
@@ -41,6 +42,7 @@ class KVRequest:
     value_dim: Optional[int] = None
     chunk: Optional[int] = None
     stride: int = 1
+    keep_first: int = 0
 
 
 @dataclass(frozen=True)

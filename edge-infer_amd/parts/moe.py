@@ -11,6 +11,12 @@ goes by score plus a learned `correction` per output (where the spec has one), a
 are the chosen scores themselves; with `identity = I` the router has I outputs beyond the
 experts, and one of them chosen adds p x itself.
 
+With `scoring = "sigmoid"` the scores are sigmoid(z); the experts form `group_count` equal groups
+of neighbours, of which the `group_keep` with the largest sums of their two largest scores take
+part, and the weights are the chosen scores over their sum, times `weight_scale`.  An expert's
+activation may be the clamped swish of `parts.mlp`; `shared` is a gated feed-forward of its own
+size that every row passes, whose rows the kernel that sums the experts' outputs adds.
+
 The experts' matrices are stacked when the part is built (gate and up [E, F, H], down
 [E, H, F]); routing stays on the device, so a step with this part is captured like any
 other.  In bfloat16 with widths that are multiples of 64 the experts run as grouped matrix
@@ -23,14 +29,24 @@ import torch
 
 from ..csrc import lib
 from ..weights.loader import ParamSpec
+from .mlp import GatedMLP
 
 
 class RoutedMLP:
-    capture_safe = True      # only this library's kernels, nothing read back, no allocation
+    @property
+    def capture_safe(self):
+        """Only this library's kernels, nothing read back, no allocation, as long as the shared
+        expert's products do the same."""
+        return self.shared is None or self.shared.capture_safe
+
+    @property
+    def capture_rows(self):
+        return (1 << 30) if self.shared is None else self.shared.capture_rows
 
     @classmethod
     def kernel_libraries(cls, spec, dtype):
-        return ("moe", "rowwise")
+        shared = getattr(spec, "shared", None)
+        return ("moe", "rowwise", *(() if shared is None else GatedMLP.kernel_libraries(shared, dtype)))
 
     @classmethod
     def parameters(cls, spec, hidden):
@@ -43,6 +59,9 @@ class RoutedMLP:
             params[prefix + "gate_proj.weight"] = ParamSpec((spec.intermediate_size, hidden))
             params[prefix + "up_proj.weight"] = ParamSpec((spec.intermediate_size, hidden))
             params[prefix + "down_proj.weight"] = ParamSpec((hidden, spec.intermediate_size))
+        if getattr(spec, "shared", None) is not None:
+            for name, param in GatedMLP.parameters(spec.shared, hidden).items():
+                params["shared." + name] = param
         return params
 
     @classmethod
@@ -58,6 +77,19 @@ class RoutedMLP:
             raise ValueError(f"routed_mlp: unknown scoring '{spec.scoring}'")
         if getattr(spec, "correction", False) and spec.scoring != "softmax_all":
             raise ValueError("routed_mlp: a correction belongs to the scoring 'softmax_all'")
+        groups, keep = getattr(spec, "group_count", 1), getattr(spec, "group_keep", 1)
+        if groups < 1 or not 1 <= keep <= groups or spec.n_experts % groups:
+            raise ValueError(f"routed_mlp: {groups} groups of which {keep} are kept do not fit "
+                             f"{spec.n_experts} experts")
+        if groups > 1 and spec.scoring != "sigmoid":
+            raise ValueError("routed_mlp: groups of experts belong to the scoring 'sigmoid'")
+        if getattr(spec, "scoring", None) == "sigmoid" and \
+                (identity or spec.top > spec.n_experts // groups * keep):
+            raise ValueError("routed_mlp: the scoring 'sigmoid' has no identity experts, and the "
+                             "kept groups must hold enough experts to choose from")
+        if getattr(spec, "activation", "silu") not in lib.EXPERT_ACTIVATIONS:
+            raise ValueError(f"routed_mlp: unknown activation '{spec.activation}'; "
+                             f"known: {sorted(lib.EXPERT_ACTIVATIONS)}")
         if spec.intermediate_size < 1:
             raise ValueError("routed_mlp: an expert's width must be positive")
 
@@ -76,16 +108,26 @@ class RoutedMLP:
         self.correction = None
         if getattr(spec, "correction", False):
             self.correction = params["router.correction"].to(device=device, dtype=torch.float32).contiguous()
+        self.routing = dict(scoring=self.scoring, correction=self.correction,
+                            groups=getattr(spec, "group_count", 1), keep=getattr(spec, "group_keep", 1),
+                            weight_scale=getattr(spec, "weight_scale", 1.0))
+        self.act = dict(activation=getattr(spec, "activation", "silu"),
+                        limit=getattr(spec, "limit", 0.0), alpha=getattr(spec, "alpha", 1.0))
+        self.shared = None
+        if getattr(spec, "shared", None) is not None:
+            self.shared = GatedMLP(spec.shared, hidden,
+                                   {name[len("shared."):]: tensor for name, tensor in params.items()
+                                    if name.startswith("shared.")}, dtype, device)
         self.grouped = lib.moe_grouped_supported(dtype, hidden, spec.intermediate_size,
                                                  spec.n_experts)
 
     def forward(self, ctx, x):
         spec = self.spec
         n = x.shape[0]
+        shared = None if self.shared is None else self.shared.forward(ctx, x)
         expert = ctx.buffer("moe.expert", (n, spec.top), torch.int32)
         weight = ctx.buffer("moe.weight", (n, spec.top), torch.float32)
-        lib.moe_route(x, self.router, ctx.meta.row_seq, expert, weight, scoring=self.scoring,
-                      correction=self.correction)
+        lib.moe_route(x, self.router, ctx.meta.row_seq, expert, weight, **self.routing)
         act = ctx.buffer("moe.act", (n * spec.top, spec.intermediate_size))
         out = ctx.buffer("moe.out", (n, self.hidden), torch.float32)
         if self.grouped:
@@ -94,9 +136,10 @@ class RoutedMLP:
             sums = ctx.buffer("moe.sums", (pairs, self.hidden), torch.float32)
             lib.moe_experts_grouped(x, self.w_gate, self.w_up, self.w_down, expert, weight,
                                     order[:pairs], order[pairs:2 * pairs], order[2 * pairs:], act,
-                                    sums, out)
+                                    sums, out, extra=shared, **self.act)
             ctx.release(order, sums)
         else:
-            lib.moe_experts(x, self.w_gate, self.w_up, self.w_down, expert, weight, act, out)
-        ctx.release(expert, weight, act)
+            lib.moe_experts(x, self.w_gate, self.w_up, self.w_down, expert, weight, act, out,
+                            extra=shared, **self.act)
+        ctx.release(shared, expert, weight, act)
         return out

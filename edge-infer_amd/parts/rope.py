@@ -15,6 +15,8 @@ import math
 
 import torch
 
+from ..config.specs import YarnScaling
+
 
 class RotaryTable:
     def __init__(self, spec, device):
@@ -61,12 +63,21 @@ class RotaryFrequencies:
 
 def scaled_frequencies(spec) -> torch.Tensor:
     """theta^(-2i / dim) for i < dim / 2 in float64, with the long wavelengths stretched as
-    `spec.scaling` says (see `config.specs.FrequencyScaling`)."""
+    `spec.scaling` says (see `config.specs.FrequencyScaling` and `config.specs.YarnScaling`)."""
     exponent = -2.0 * torch.arange(spec.dim // 2, dtype=torch.float64) / float(spec.dim)
     frequencies = torch.pow(torch.tensor(float(spec.theta), dtype=torch.float64), exponent)
     scaling = getattr(spec, "scaling", None)
     if scaling is None:
         return frequencies
+    if isinstance(scaling, YarnScaling):
+        def pair_of(turns):
+            return (spec.dim * math.log(scaling.original / (2.0 * math.pi * turns))
+                    / (2.0 * math.log(float(spec.theta))))
+        low = max(math.floor(pair_of(scaling.fast)), 0)
+        high = min(math.ceil(pair_of(scaling.slow)), spec.dim - 1)
+        index = torch.arange(spec.dim // 2, dtype=torch.float64)
+        ramp = ((index - low) / max(high - low, 0.001)).clamp(0.0, 1.0)
+        return frequencies / scaling.factor * ramp + frequencies * (1.0 - ramp)
     wavelength = 2.0 * math.pi / frequencies
     blend = (scaling.original / wavelength - scaling.low) / (scaling.high - scaling.low)
     between = (1.0 - blend) * frequencies / scaling.factor + blend * frequencies
@@ -75,17 +86,26 @@ def scaled_frequencies(spec) -> torch.Tensor:
                                    frequencies / scaling.factor, between))
 
 
+def rotation_magnitude(spec) -> float:
+    """What cosine and sine of the rotation are multiplied by."""
+    scaling = getattr(spec, "scaling", None)
+    if isinstance(scaling, YarnScaling):
+        return 0.1 * math.log(scaling.factor) + 1.0
+    return 1.0
+
+
 class RotaryHalfFrequencies:
     """Rotation of the pairs (i, i + dim/2) of a head's first `dim` elements by the angle
     position * f_i: the store kernel multiplies the position by the float64 frequency, takes
     the product modulo 2 pi, rounds it to float32 and takes cosine and sine itself, so there is
     no table, no position that is too far, and the float32 angle is the nearest one however
     far the position.  The frequencies are worked out in float64 (stretched where the spec
-    says)."""
+    says); `magnitude` is what cosine and sine are multiplied by."""
     def __init__(self, spec, device):
         if spec.dim % 2 or spec.dim < 2:
             raise ValueError("rotary dimension must be even and at least 2")
         self.spec = spec
+        self.magnitude = rotation_magnitude(spec)
         self.frequencies = scaled_frequencies(spec).to(device).contiguous()
         self.table = None
         self.max_positions = None
