@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers L]
                     [--shape 8b|0.6b|32b] [--only decode|prefill|generate] [--prompt P]
-                    [--with-32b] [--peaks] [--design tirurax|zadenex|vafepel|gopuzen [--design-shape 1k|2k|4k]]
+                    [--with-32b] [--peaks] [--design tirurax|zadenex|vafepel|gopuzen|dazapel [--design-shape 1k|2k|4k]]
 
 Prints one JSON line.  `value` is decoded tokens per second at the given batch after
 512-token prompts (one step = one decode step of the whole batch: the model, greedy
@@ -35,7 +35,9 @@ heads and parameters at work for a token.  `--design gopuzen` does the same for 
 blocks in turn, every second of the latter reading the keys and values of the one before it;
 layer norms on both sides of every sublayer, input convolutions, the feed-forwards in turn
 dense and routed over 8 experts and 2 identity experts) beside the Vafepel model of the same
-width, layers, heads and parameters at work for a token.
+width, layers, heads and parameters at work for a token.  `--design dazapel` does the same for a
+Dazapel model (window attention that keeps the first tokens, feed-forwards routed within groups
+of 16 experts beside a shared one) beside the Gopuzen model of the same width, layers and heads.
 Synthetic token ids, seeded random weights N(0, 0.02).  Peaks are the MI355X's published
 ones: HBM 8 TB/s, dense bf16 MFMA 2.5 PFLOP/s; `measured_peaks` (and `--peaks` alone) say what
 a plain read kernel and a loop of matrix-core products reach on the GPU at hand, and the
@@ -497,6 +499,34 @@ def gopuzen_configs(shape):
     return new, old
 
 
+def dazapel_configs(shape):
+    """(Dazapel configuration, Gopuzen configuration) of equal width, layers, heads and head size.
+    Dazapel: window attention that keeps the first 16 tokens, a rotation of the whole head with
+    stretched frequencies, queries and keys at unit RMS, a gate on every element; every layer
+    with a feed-forward of 16 experts in 4 groups (2 take part) of which a token takes 4, an
+    expert an eighth of the dense feed-forward's width, beside a shared one of half of it: as
+    many parameters at work for a token.  The last layers but the first two run in a loop of
+    one pass.  Gopuzen: `gopuzen_configs`."""
+    from edge_infer_amd.config import DazapelConfig
+    layers, width, d_heads, d_kv, a_heads, a_kv, dim, chunk, vocab = DESIGN_SHAPES[shape]
+    gated = (2 * 4 * width // 3 + 511) // 512 * 512
+    layer = {"type": "attention",
+             "mixer": {"heads": a_heads, "kv_heads": a_kv, "dim": dim, "vdim": dim,
+                       "scale": 1.5 * dim ** -0.5, "mask": {"size": chunk, "keep_first": 16},
+                       "rot": {"base": 500000.0, "dims": dim,
+                               "scaling": {"factor": 4.0, "original": 8192, "fast": 16.0, "slow": 1.0}}},
+             "mlp": {"kind": "moe", "expert": {"ff": gated // 8, "limit": 7.0},
+                     "router": {"experts": 16, "top": 4, "scale": 1.5,
+                                "groups": {"count": 4, "keep": 2}},
+                     "shared": {"ff": gated // 2, "limit": 7.0}}}
+    new = DazapelConfig.from_dict({"architecture": "Dazapel", "vocab": vocab, "width": width,
+                                   "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+                                   "loop": {"start": 2, "stop": layers, "times": 1},
+                                   "layers": [layer] * layers})
+    old, _ = gopuzen_configs(shape)
+    return new, old
+
+
 def measure_prompts(model, vocab, batch, tokens, repeats=3):
     """Best ms of one step over `batch` prompts of `tokens` tokens that start together."""
     import types
@@ -522,7 +552,8 @@ def measure_prompts(model, vocab, batch, tokens, repeats=3):
 
 def design_comparison(args):
     """Prefill and decode of the design's shape and of the closest other model of equal size
-    (Tirurax beside Qwen3, Zadenex and Vafepel beside Tirurax)."""
+    (Tirurax beside Qwen3, Zadenex and Vafepel beside Tirurax, Gopuzen beside Vafepel, Dazapel
+    beside Gopuzen)."""
     import types
     import torch
     import edge_infer_amd as ei
@@ -535,6 +566,9 @@ def design_comparison(args):
     elif args.design == "gopuzen":
         new, old = gopuzen_configs(args.design_shape)
         which = {"gopuzen": new, "vafepel": old}
+    elif args.design == "dazapel":
+        new, old = dazapel_configs(args.design_shape)
+        which = {"dazapel": new, "gopuzen": old}
     else:
         new, old = design_configs(args.design_shape)
         which = {"tirurax": new, "qwen3": old}
@@ -594,12 +628,14 @@ def main():
                         help="leave the 32B shape (decode at batch 1 and 16, prefill) out of `points`")
     parser.add_argument("--peaks", action="store_true",
                         help="measure the read and matrix-core yardsticks only")
-    parser.add_argument("--design", choices=["tirurax", "zadenex", "vafepel", "gopuzen"], default=None,
+    parser.add_argument("--design", choices=["tirurax", "zadenex", "vafepel", "gopuzen", "dazapel"],
+                        default=None,
                         help="measure this design beside the closest other model of equal size "
                              "(tirurax beside qwen3, zadenex beside tirurax) instead of the "
                              "default workload")
     parser.add_argument("--design-shape", choices=sorted(DESIGN_SHAPES), default="2k")
-    parser.add_argument("--design-only", choices=["gopuzen", "vafepel", "zadenex", "tirurax", "qwen3"], default=None,
+    parser.add_argument("--design-only", choices=["dazapel", "gopuzen", "vafepel", "zadenex", "tirurax", "qwen3"],
+                        default=None,
                         help="with --design: one of the two models only (for profiling)")
     args = parser.parse_args()
     if args.gpus != 1:
