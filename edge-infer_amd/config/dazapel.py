@@ -324,7 +324,7 @@ class DazapelConfig:
         norm = NormSpec(kind="rmsnorm", eps=self.norm_eps)
         layers = tuple(LayerSpec(block="sandwich", norm=norm, mixer=self._mixer_spec(layer.mixer),
                                  feed_forward=self._feed_forward_spec(layer.mlp),
-                                 residual_scale=self.residual_mult)
+                                 residual_scale=self.residual_mult, defer_output=True)
                        for layer in self.layers)
         loop = None if self.loop is None else LoopSpec(*self.loop, remix=False)
         schedule = (default_schedule(len(layers)) if loop is None

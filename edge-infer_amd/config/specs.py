@@ -359,6 +359,9 @@ class LayerSpec:
     input_conv: int = 0
     # the model's width, for arrangements that ask for state of that width (None: not needed)
     width: Optional[int] = None
+    # the norm on the last sublayer's output and its addition are left to the next layer's first
+    # kernel (arrangements that know it)
+    defer_output: bool = False
 
 
 @dataclass(frozen=True)

@@ -51,17 +51,23 @@ struct AttnExtra {
   size_t wide_slice, wide_row;
 };
 
-// The factor of output element `at` (row * wide_row + head * D + d) of `AttnExtra.wide`.
-__device__ __forceinline__ float wide_open(const AttnExtra& extra, size_t at) {
+// What goes into the sigmoid for output element `at` (row * wide_row + head * D + d) of
+// `AttnExtra.wide`: up to eight slices' loads travel together.
+__device__ __forceinline__ float wide_sum(const AttnExtra& extra, size_t at) {
+  if (extra.wide_dtype != EI_F32) return ei::bf16_to_f32(static_cast<const bf16_t*>(extra.wide)[at]);
+  const float* p = static_cast<const float*>(extra.wide) + at;
   float z = 0.f;
-  if (extra.wide_dtype == EI_F32) {
-    const float* p = static_cast<const float*>(extra.wide) + at;
-    for (int s = 0; s < extra.wide_slices; ++s) z += p[s * extra.wide_slice];
-  } else {
-    z = ei::bf16_to_f32(static_cast<const bf16_t*>(extra.wide)[at]);
+  for (int s0 = 0; s0 < extra.wide_slices; s0 += 8) {
+    float v[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) v[u] = s0 + u < extra.wide_slices ? p[(s0 + u) * extra.wide_slice] : 0.f;
+#pragma unroll
+    for (int u = 0; u < 8; ++u) z += v[u];
   }
-  return 1.0f / (1.0f + expf(-z));
+  return z;
 }
+
+__device__ __forceinline__ float opened(float z) { return 1.0f / (1.0f + expf(-z)); }
 
 __device__ __forceinline__ float bf16_lo(uint32_t u) { return __uint_as_float(u << 16); }
 __device__ __forceinline__ float bf16_hi(uint32_t u) { return __uint_as_float(u & 0xffff0000u); }
@@ -263,6 +269,13 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   }
   (void)total_tiles;
 
+  // (EXT) the gate of the first element that this thread will write, asked for ahead of the walk
+  const size_t wide_base = EXT ? static_cast<size_t>(row) * extra.wide_row +
+                                     static_cast<size_t>(head0) * D : 0;
+  float first_gate = 0.f;
+  if constexpr (EXT)
+    if (extra.wide && n_splits == 1 && t < heads_here * D) first_gate = wide_sum(extra, wide_base + t);
+
   float m_run = kLowest, l_run = 0.f;              // state of head r16 (same in all four c)
   float slope = 0.f;                               // of head r16
   if constexpr (EXT)
@@ -429,8 +442,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
       float value = l > 0.f ? o / l : 0.f;
       if constexpr (EXT)
         if (extra.wide)
-          value *= wide_open(extra, static_cast<size_t>(row) * extra.wide_row +
-                                        static_cast<size_t>(head) * D + d);
+          value *= opened(idx == t ? first_gate : wide_sum(extra, wide_base + idx));
       out[(static_cast<size_t>(row) * nq + head) * D + d] = ei::from_f32<bf16_t>(value);
     } else {
       const size_t slot = (static_cast<size_t>(row) * nq + head) * n_splits + split;
@@ -996,6 +1008,20 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
         const float4 p4 = *reinterpret_cast<const float4*>(&pool_lds[wave][8 * i + 4 * half]);
         pooled[0] = p4.x; pooled[1] = p4.y; pooled[2] = p4.z; pooled[3] = p4.w;
       }
+      // (EXT) the gates of the lane's elements of these four rows: their loads travel together
+      float open[EXT ? 4 : 1][EXT ? DB : 1];
+      if constexpr (EXT) {
+        if (extra.wide) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int db = 0; db < DB; ++db) {
+              const int orow = min(pw * kWideRows + 8 * i + 4 * half + r, npos - 1);
+              open[r][db] = wide_sum(extra, static_cast<size_t>(row0 + orow) * extra.wide_row +
+                                                static_cast<size_t>(head) * D + db * 32 + n32);
+            }
+        }
+      }
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int orow = pw * kWideRows + 8 * i + 4 * half + r;
@@ -1013,9 +1039,7 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
             if (extra.pool_o && pooled[r] != 0.f)
               o = fmaf(extra.pool_o[(static_cast<size_t>(row0 + orow) * nq + head) * D + db * 32 + n32],
                        pooled[r], o);
-            if (extra.wide)
-              o *= wide_open(extra, static_cast<size_t>(row0 + orow) * extra.wide_row +
-                                        static_cast<size_t>(head) * D + db * 32 + n32);
+            if (extra.wide) o *= opened(open[r][db]);
           }
           dst[db * 32 + n32] = ei::from_f32<bf16_t>(o);
         }
@@ -1090,8 +1114,9 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o,
       if (extra.wide) {
         const size_t at = static_cast<size_t>(wave / nq) * extra.wide_row +
                           static_cast<size_t>(wave % nq) * D + d;
-        o0 *= wide_open(extra, at);
-        o1 *= wide_open(extra, at + 1);
+        const float z0 = wide_sum(extra, at), z1 = wide_sum(extra, at + 1);
+        o0 *= opened(z0);
+        o1 *= opened(z1);
       }
       dst[0] = ei::from_f32<bf16_t>(o0);
       dst[1] = ei::from_f32<bf16_t>(o1);

@@ -105,6 +105,34 @@ template <> __device__ __forceinline__ float silu<bf16_t>(float x) {
   return x * __builtin_amdgcn_rcpf(1.0f + e);
 }
 
+// x / (1 + e^(-alpha x)), in the two precisions of `silu`.
+template <typename TO> __device__ __forceinline__ float swish(float x, float alpha);
+template <> __device__ __forceinline__ float swish<float>(float x, float alpha) {
+  return x / (1.0f + expf(-alpha * x));
+}
+template <> __device__ __forceinline__ float swish<bf16_t>(float x, float alpha) {
+  const float e = __builtin_amdgcn_exp2f(fmaxf(alpha * x, -80.f) * -1.44269504088896341f);
+  return x * __builtin_amdgcn_rcpf(1.0f + e);
+}
+
+// How a gated feed-forward joins its gate and up products.  kind (codes of the C interface): 0
+// silu(gate) up; 1 the tanh form of gelu for silu; 2 the clamped swish: with g = min(gate, limit)
+// and u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1).
+struct GateAct {
+  int kind;
+  float limit, alpha;
+};
+
+template <typename TO>
+__device__ __forceinline__ float gated_product(float gate, float up, const GateAct& act) {
+  if (act.kind == 0) return silu<TO>(gate) * up;
+  if (act.kind == 1)
+    return 0.5f * gate * (1.0f + tanhf(0.7978845608028654f * (gate + 0.044715f * gate * gate * gate))) * up;
+  const float g = fminf(gate, act.limit);
+  const float u = fminf(fmaxf(up, -act.limit), act.limit);
+  return swish<TO>(g, act.alpha) * (u + 1.0f);
+}
+
 // Reductions over the four 16-lane rows of a wave (lanes l, l^16, l^32, l^48), every lane
 // getting the result.  gfx950's row-swap instructions do each step in the vector ALU: with
 // both operands holding x, v_permlane32_swap leaves (x of the lower half, x of the upper

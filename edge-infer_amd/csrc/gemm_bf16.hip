@@ -43,13 +43,13 @@ constexpr int kPackedTile = 16 * 32;      // elements of one packed tile: 16 row
 //
 // GATED (one K slice only): the strips of W alternate between 16 gate rows and the 16 up rows
 // that belong to them; even waves hold gate sums, their odd neighbours the up sums (with two
-// strips a wave holds both), and the block writes silu(gate) * up as bfloat16 [M, N/2] to
-// `gated_out` instead of any sums.
+// strips a wave holds both), and the block writes their gated product (`act`) as bfloat16
+// [M, N/2] to `gated_out` instead of any sums.
 template <int MB, int WAVES, bool PACKED, bool GATED, int STRIPS, int KT>
 __global__ void __launch_bounds__(WAVES * EI_WAVE)
 skinny_gemm_kernel(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X,
                    float* __restrict__ out, bf16_t* __restrict__ gated_out, int M, int N, int K,
-                   int k_per_split, int row_groups) {
+                   int k_per_split, int row_groups, ei::GateAct act) {
   constexpr int JN = KT / 32;             // MFMA steps per K-tile
   static_assert(KT == 256 || (KT == 128 && PACKED), "K-tiles of 256, or 128 with packed weights");
   constexpr int ROWS_X = MB * 16;
@@ -339,8 +339,8 @@ skinny_gemm_kernel(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X,
         uint32_t packed[2];
 #pragma unroll
         for (int r = 0; r < 4; r += 2) {
-          const bf16_t lo = ei::f32_to_bf16(ei::silu<bf16_t>(acc[mb][0][r]) * acc[mb][1][r]);
-          const bf16_t hi = ei::f32_to_bf16(ei::silu<bf16_t>(acc[mb][0][r + 1]) * acc[mb][1][r + 1]);
+          const bf16_t lo = ei::f32_to_bf16(ei::gated_product<bf16_t>(acc[mb][0][r], acc[mb][1][r], act));
+          const bf16_t hi = ei::f32_to_bf16(ei::gated_product<bf16_t>(acc[mb][0][r + 1], acc[mb][1][r + 1], act));
           packed[r / 2] = static_cast<uint32_t>(lo) | (static_cast<uint32_t>(hi) << 16);
         }
         *reinterpret_cast<uint2*>(gated_out + static_cast<size_t>(m) * half + col) =
@@ -370,8 +370,8 @@ skinny_gemm_kernel(const bf16_t* __restrict__ W, const bf16_t* __restrict__ X,
         uint32_t packed[2];
 #pragma unroll
         for (int r = 0; r < 4; r += 2) {
-          const bf16_t lo = ei::f32_to_bf16(ei::silu<bf16_t>(acc[mb][0][r]) * up[r]);
-          const bf16_t hi = ei::f32_to_bf16(ei::silu<bf16_t>(acc[mb][0][r + 1]) * up[r + 1]);
+          const bf16_t lo = ei::f32_to_bf16(ei::gated_product<bf16_t>(acc[mb][0][r], up[r], act));
+          const bf16_t hi = ei::f32_to_bf16(ei::gated_product<bf16_t>(acc[mb][0][r + 1], up[r + 1], act));
           packed[r / 2] = static_cast<uint32_t>(lo) | (static_cast<uint32_t>(hi) << 16);
         }
         *reinterpret_cast<uint2*>(gated_out + static_cast<size_t>(m) * half + col) =
@@ -493,7 +493,8 @@ namespace {
 
 template <int MB, bool PACKED, bool GATED, int STRIPS, int KT = 256>
 void launch_tile_kernel(const bf16_t* w, const bf16_t* x, float* out, bf16_t* gated_out, int M,
-                        int N, int K, int k_per_split, int splits, hipStream_t stream) {
+                        int N, int K, int k_per_split, int splits, const ei::GateAct& act,
+                        hipStream_t stream) {
   const int n_strips = ((N + 15) / 16 + STRIPS - 1) / STRIPS;     // what a wave owns
   const int row_groups = (M + MB * 16 - 1) / (MB * 16);
   const int waves = tile_kernel_waves(n_strips, splits, row_groups,
@@ -503,18 +504,19 @@ void launch_tile_kernel(const bf16_t* w, const bf16_t* x, float* out, bf16_t* ga
   dim3 grid(strip_blocks * row_groups, splits);
   if (waves == 4)
     skinny_gemm_kernel<MB, 4, PACKED, GATED, STRIPS, KT><<<grid, 4 * EI_WAVE, 0, stream>>>(
-        w, x, out, gated_out, M, N, K, k_per_split, row_groups);
+        w, x, out, gated_out, M, N, K, k_per_split, row_groups, act);
   else if (waves == 6)
     skinny_gemm_kernel<MB, 6, PACKED, GATED, STRIPS, KT><<<grid, 6 * EI_WAVE, 0, stream>>>(
-        w, x, out, gated_out, M, N, K, k_per_split, row_groups);
+        w, x, out, gated_out, M, N, K, k_per_split, row_groups, act);
   else
     skinny_gemm_kernel<MB, 8, PACKED, GATED, STRIPS, KT><<<grid, 8 * EI_WAVE, 0, stream>>>(
-        w, x, out, gated_out, M, N, K, k_per_split, row_groups);
+        w, x, out, gated_out, M, N, K, k_per_split, row_groups, act);
 }
 
 template <bool PACKED, bool GATED>
 int launch_skinny(const void* X, const void* W, float* out, void* gated_out, int M, int N, int K,
-                  int splits, hipStream_t stream) {
+                  int splits, hipStream_t stream, const ei::GateAct& act = ei::GateAct{0, 0.f, 1.f}) {
+  EI_REQUIRE(act.kind >= 0 && act.kind <= 2, "gemm_bf16_skinny_gated: unknown activation");
   EI_REQUIRE(M >= 1 && M <= kMaxRows, "gemm_bf16_skinny: rows must lie in 1..256");
   EI_REQUIRE(N >= 1 && K >= 8 && K % 8 == 0, "gemm_bf16_skinny: K must be a multiple of 8");
   EI_REQUIRE(X && W && (GATED ? gated_out != nullptr : out != nullptr), "gemm_bf16_skinny: null pointer");
@@ -539,19 +541,19 @@ int launch_skinny(const void* X, const void* W, float* out, void* gated_out, int
   if (mode.strips == 2) {
     if constexpr (PACKED) {
       if (MB == 4)
-        launch_tile_kernel<4, PACKED, GATED, 2, 128>(w, x, out, g, M, N, K, k_per_split, splits, stream);
+        launch_tile_kernel<4, PACKED, GATED, 2, 128>(w, x, out, g, M, N, K, k_per_split, splits, act, stream);
       else
-        launch_tile_kernel<8, PACKED, GATED, 2, 128>(w, x, out, g, M, N, K, k_per_split, splits, stream);
+        launch_tile_kernel<8, PACKED, GATED, 2, 128>(w, x, out, g, M, N, K, k_per_split, splits, act, stream);
     }
   } else if (MB == 1) {
-    launch_tile_kernel<1, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, stream);
+    launch_tile_kernel<1, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, act, stream);
   } else if (MB == 2) {
-    launch_tile_kernel<2, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, stream);
+    launch_tile_kernel<2, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, act, stream);
   } else if (MB == 4) {
-    launch_tile_kernel<4, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, stream);
+    launch_tile_kernel<4, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, act, stream);
   } else {
     if constexpr (PACKED)
-      launch_tile_kernel<8, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, stream);
+      launch_tile_kernel<8, PACKED, GATED, 1>(w, x, out, g, M, N, K, k_per_split, splits, act, stream);
   }
   EI_LAUNCH_CHECK();
 }
@@ -580,10 +582,13 @@ extern "C" int ei_gemm_bf16_skinny_packed(const void* X, const void* Wp, float* 
 
 // Gated feed-forward in one pass: W [N, K] holds, in strips of 16 rows, the gate rows of 16
 // outputs followed by their up rows (N = 2 * outputs, a multiple of 32); act [M, N/2]
-// bfloat16 = silu(X . gate^T) * (X . up^T).  All of K in one slice.  `packed`: W is in the
+// bfloat16 = the gated product (`kind`, `limit`, `alpha` as in GateAct) of X . gate^T and
+// X . up^T.  All of K in one slice.  `packed`: W is in the
 // streaming layout of ei_gemm_bf16_skinny_packed.
 extern "C" int ei_gemm_bf16_skinny_gated(const void* X, const void* W, void* act, int M, int N,
-                                         int K, int packed, hipStream_t stream) {
-  if (packed) return launch_skinny<true, true>(X, W, nullptr, act, M, N, K, 1, stream);
-  return launch_skinny<false, true>(X, W, nullptr, act, M, N, K, 1, stream);
+                                         int K, int packed, int kind, float limit, float alpha,
+                                         hipStream_t stream) {
+  const ei::GateAct how{kind, limit, alpha};
+  if (packed) return launch_skinny<true, true>(X, W, nullptr, act, M, N, K, 1, stream, how);
+  return launch_skinny<false, true>(X, W, nullptr, act, M, N, K, 1, stream, how);
 }

@@ -35,7 +35,8 @@ _SIGNATURES = {
                          c_longlong, c_int, c_void_p],
         "ei_scale_cap": [c_void_p, c_float, c_float, c_longlong, c_void_p],
         "ei_norm_add_norm": [c_void_p, c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p,
-                             c_float, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p],
+                             c_float, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
+                             c_void_p],
         "ei_concat_cast": [c_void_p, c_void_p, c_void_p, c_int, c_longlong, c_int, c_void_p],
         "ei_set_rows": [c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p, c_longlong, c_int,
                         c_void_p],
@@ -103,6 +104,10 @@ _SIGNATURES = {
                            c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
                            c_float, c_void_p, c_int, c_int, c_longlong, c_void_p],
         "ei_moe_grouped_supported": [c_int, c_int, c_int, c_int],
+        "ei_moe_few_rows": [],
+        "ei_moe_experts_few": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                               c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                               c_float, c_float, c_void_p],
         "ei_moe_experts_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                    c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                    c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float,
@@ -204,7 +209,7 @@ _SIGNATURES = {
         "ei_gemm_bf16_skinny_packed": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                                        c_void_p],
         "ei_gemm_bf16_skinny_gated": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                                      c_void_p],
+                                      c_int, c_float, c_float, c_void_p],
     },
     "sampling": {
         "ei_argmax": [c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p, c_longlong, c_void_p],
@@ -477,9 +482,10 @@ def norm_add(residual: torch.Tensor, delta: torch.Tensor, weight: torch.Tensor, 
 
 def norm_add_norm(residual: torch.Tensor, delta: torch.Tensor, w_after: torch.Tensor,
                   w_next: torch.Tensor, eps: float, out: torch.Tensor,
-                  bias: Optional[torch.Tensor] = None) -> None:
-    """residual [R, H] float32 += rmsnorm(sum of delta's slices (+ bias [H])) * w_after, then
-    out [R, H] = rmsnorm(residual) * w_next in out's type: one pass over the rows."""
+                  bias: Optional[torch.Tensor] = None,
+                  vector: Optional[torch.Tensor] = None) -> None:
+    """residual [R, H] float32 += rmsnorm(sum of delta's slices (+ bias [H])) * w_after (+ vector
+    [H]), then out [R, H] = rmsnorm(residual) * w_next in out's type: one pass over the rows."""
     lib = library("rowwise")
     rows, hidden = residual.shape
     nsplit, stride = _splits(delta, rows, hidden, "delta")
@@ -492,7 +498,8 @@ def norm_add_norm(residual: torch.Tensor, delta: torch.Tensor, w_after: torch.Te
                                   _gpu(w_after, "w_after", torch.float32),
                                   _gpu(w_next, "w_next", torch.float32), float(eps),
                                   _gpu(out, "out"), _code(out, "out"), rows, hidden,
-                                  _row_bias(bias, hidden, "norm_add_norm"), _stream())
+                                  _row_bias(bias, hidden, "norm_add_norm"),
+                                  _row_bias(vector, hidden, "norm_add_norm"), _stream())
     _check(lib, status, "norm_add_norm")
 
 
@@ -1708,7 +1715,7 @@ def la_out(o_raw, proj, gate_column: int, norm_w, eps: float, row_seq, out) -> N
 
 
 ROUTER_SCORINGS = {"softmax_chosen": 0, "softmax_all": 1, "sigmoid": 2}
-EXPERT_ACTIVATIONS = {"silu": 0, "clamped_swish": 1}
+EXPERT_ACTIVATIONS = GATE_ACTIVATIONS
 
 
 def moe_route(x, router_w, row_seq, expert, weight, scoring: str = "softmax_chosen",
@@ -1792,6 +1799,43 @@ def moe_grouped_supported(dtype, width: int, inter: int, n_experts: int) -> bool
     if dtype != torch.bfloat16:
         return False
     return bool(library("moe").ei_moe_grouped_supported(BF16, width, inter, n_experts))
+
+
+MOE_FEW_ROWS = 64
+
+
+def moe_experts_few(x, w_gate, w_up, w_down, expert, weight, row_seq, act, out, activation="silu",
+                    limit=0.0, alpha=1.0) -> None:
+    """The experts of at most `MOE_FEW_ROWS` rows on the matrix cores (bfloat16, the sizes of
+    `moe_experts_grouped`), without a layout by expert first: out [top, n, w] float32, whose
+    slice k receives weight[r, k] times the product row of row r's k-th choice; the slices' sum
+    is what `moe_experts` gives.  Rows with row_seq < 0 are not written.  Every choice is an
+    expert (no identity ones).  `act` [n * top, f] bfloat16 is scratch."""
+    lib = library("moe")
+    n, width = x.shape
+    n_experts, inter = w_gate.shape[0], w_gate.shape[1]
+    top = expert.shape[1]
+    if tuple(w_gate.shape) != (n_experts, inter, width) or tuple(w_up.shape) != tuple(w_gate.shape) \
+            or tuple(w_down.shape) != (n_experts, width, inter):
+        raise KernelError("moe_experts_few: the stacked matrices have the wrong shapes")
+    if tuple(expert.shape) != (n, top) or tuple(weight.shape) != (n, top) \
+            or tuple(act.shape) != (n * top, inter) or tuple(out.shape) != (top, n, width):
+        raise KernelError("moe_experts_few: shapes do not fit")
+    if row_seq is not None and row_seq.numel() < n:
+        raise KernelError("moe_experts_few: row metadata shorter than the rows")
+    if n > MOE_FEW_ROWS or not moe_grouped_supported(x.dtype, width, inter, n_experts):
+        raise KernelError(f"moe_experts_few: bfloat16, at most {MOE_FEW_ROWS} rows and widths that "
+                          "are multiples of 64 only")
+    if activation not in EXPERT_ACTIVATIONS:
+        raise KernelError(f"moe_experts_few: unknown activation '{activation}'")
+    status = lib.ei_moe_experts_few(
+        _gpu(x, "x", torch.bfloat16), _gpu(w_gate, "w_gate", torch.bfloat16),
+        _gpu(w_up, "w_up", torch.bfloat16), _gpu(w_down, "w_down", torch.bfloat16),
+        _gpu(expert, "expert", torch.int32), _gpu(weight, "weight", torch.float32),
+        None if row_seq is None else _gpu(row_seq, "row_seq", torch.int32),
+        _gpu(act, "act", torch.bfloat16), _gpu(out, "out", torch.float32), n, width, inter,
+        n_experts, top, EXPERT_ACTIVATIONS[activation], float(limit), float(alpha), _stream())
+    _check(lib, status, "moe_experts_few")
 
 
 def moe_experts_grouped(x, w_gate, w_up, w_down, expert, weight, sorted_pairs, place, starts, act,
@@ -1979,13 +2023,16 @@ GATE_STRIP = 16     # gate rows and up rows alternate in strips of this many (on
 
 
 def gemm_bf16_skinny_gated(x: torch.Tensor, w: torch.Tensor, n: int, act: torch.Tensor,
-                           packed: bool) -> None:
-    """act[m, i] = silu(x[m] . gate_i) * (x[m] . up_i) for a weight [n, k] whose rows are, in
+                           packed: bool, activation: str = "silu", limit: float = 0.0,
+                           alpha: float = 1.0) -> None:
+    """act[m, i] = silu(x[m] . gate_i) * (x[m] . up_i) (or another `activation` of `swiglu`) for a weight [n, k] whose rows are, in
     strips of 16, the gate rows of 16 outputs followed by their up rows; `w` is that matrix or
     (packed) its `pack_weight` copy.  For at most 256 rows; K is not sliced, so it pays where
     `skinny_gemm_splits` is 1."""
     lib = library("gemm_bf16")
     m, k = x.shape
+    if activation not in GATE_ACTIVATIONS:
+        raise KernelError(f"gemm_bf16_skinny_gated: unknown activation '{activation}'")
     if tuple(act.shape) != (m, n // 2) or n % (2 * GATE_STRIP):
         raise KernelError(f"gemm_bf16_skinny_gated: {list(x.shape)} x [{n}, {k}] -> "
                           f"{list(act.shape)} do not agree")
@@ -1994,7 +2041,8 @@ def gemm_bf16_skinny_gated(x: torch.Tensor, w: torch.Tensor, n: int, act: torch.
         raise KernelError(f"gemm_bf16_skinny_gated: weight {list(w.shape)}, expected {list(expect)}")
     status = lib.ei_gemm_bf16_skinny_gated(_gpu(x, "x", torch.bfloat16), _gpu(w, "w", torch.bfloat16),
                                            _gpu(act, "act", torch.bfloat16), m, n, k, int(packed),
-                                           _stream())
+                                           GATE_ACTIVATIONS[activation], float(limit),
+                                           float(alpha), _stream())
     _check(lib, status, "gemm_bf16_skinny_gated")
 
 

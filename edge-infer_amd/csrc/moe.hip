@@ -10,16 +10,16 @@
 // the `keep` with the largest sums of their two largest scores take part (of equal sums the one of
 // lower index), the `top` largest scores among their experts, and the weights s / (sum of the
 // chosen s + 1e-20) * weight_scale.
-// The gated product of an expert is silu(gate) * up, or with the clamped swish (`ExpertAct`), with
-// g = min(gate, limit) and u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1).  The rows of
-// another product (an expert that every row takes) may be added to the sums: `extra`.
+// The gated product of an expert is silu(gate) * up or the clamped swish (`ei::GateAct`).  The rows
+// of another product (an expert that every row takes) may be added to the sums: `extra`.
 // A router may have more outputs than there are experts: an output beyond the experts is an
 // identity expert, which adds p x_r and has no matrices.
 //
-// Two forms of the experts.  One takes a (row, choice) pair at a time and streams the expert's
-// matrices for it: any type and any sizes.  The other (bfloat16, widths that are multiples of
-// 64) lays the pairs out by expert on the device and runs every expert's pairs against its
-// matrices as tiles on the matrix cores.  The matrices of all experts lie stacked: gate and up
+// Three forms of the experts.  One takes a (row, choice) pair at a time and streams the expert's
+// matrices for it: any type and any sizes.  The others (bfloat16, widths that are multiples of
+// 64) run every expert's pairs against its matrices as tiles on the matrix cores: for up to 64
+// rows a block finds its expert's pairs itself; for more the pairs are laid out by expert on the
+// device first.  The matrices of all experts lie stacked: gate and up
 // [E, F, W], down [E, W, F].
 #include "common.h"
 #include <float.h>
@@ -28,18 +28,6 @@ namespace {
 
 constexpr int kMaxTop = 64;
 constexpr int kRouteMax = 8;      // experts a lane holds: up to 512 experts
-
-struct ExpertAct {
-  int kind;                       // 0: silu(gate) * up, 1: the clamped swish
-  float limit, alpha;
-};
-
-__device__ __forceinline__ float expert_act(float gate, float up, const ExpertAct& act) {
-  if (act.kind == 0) return gate / (1.0f + expf(-gate)) * up;
-  const float g = fminf(gate, act.limit);
-  const float u = fminf(fmaxf(up, -act.limit), act.limit);
-  return g / (1.0f + expf(-act.alpha * g)) * (u + 1.0f);
-}
 
 // Rows [N, W] that are added to the experts' weighted sums: float32 slices or one bfloat16 tensor
 // (null: none).
@@ -99,49 +87,70 @@ __device__ __forceinline__ void leave_groups_out(float (&z)[kRouteMax], float* s
   }
 }
 
-// A block of four waves a row: the waves share the experts' logits out, the first wave chooses.
-template <typename TX>
-__global__ void __launch_bounds__(256)
+// A block R rows: its waves share the experts' logits out (a router row is read once for all R
+// rows), wave r then chooses for row r.
+template <typename TX, int R>
+__global__ void __launch_bounds__(1024)
 moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
                  const int32_t* __restrict__ row_seq, int32_t* __restrict__ expert,
                  float* __restrict__ weight, int N, int W, int E, int top, int mode,
                  const float* __restrict__ correction, int groups, int keep, float weight_scale) {
-  __shared__ float logits[kRouteMax * EI_WAVE], group_scores[kRouteMax * EI_WAVE];
-  const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
-  const int row = blockIdx.x;
-  int32_t* e_out = expert + static_cast<size_t>(row) * top;
-  float* w_out = weight + static_cast<size_t>(row) * top;
-  if (row_seq && row_seq[row] < 0) {            // a padding row: no expert has anything to add
-    for (int k = threadIdx.x; k < top; k += blockDim.x) { e_out[k] = 0; w_out[k] = 0.f; }
-    return;
+  __shared__ float logits[R][kRouteMax * EI_WAVE], group_scores[R][kRouteMax * EI_WAVE];
+  const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE, waves = blockDim.x / EI_WAVE;
+  const int row0 = blockIdx.x * R;
+  bool real[R];                                 // (rows beyond the last and padding rows: nothing to do)
+  bool any = false;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    real[r] = row0 + r < N && !(row_seq && row_seq[row0 + r] < 0);
+    any = any || real[r];
   }
-  const TX* xr = x + static_cast<size_t>(row) * W;
-  for (int e = wave; e < E; e += 4) {
+  for (int e = wave; e < E && any; e += waves) {
     const float* wr = w_router + static_cast<size_t>(e) * W;
-    float sum = 0.f;
+    float sum[R];
+#pragma unroll
+    for (int r = 0; r < R; ++r) sum[r] = 0.f;
     if (W % 4 == 0) {
 #pragma unroll 4
       for (int i = lane * 4; i < W; i += EI_WAVE * 4) {
-        float xv[4], wv[4];
-        ei::Vec4<TX>::load(xr + i, xv);
+        float wv[4];
         ei::Vec4<float>::load(wr + i, wv);
-        sum += xv[0] * wv[0];
-        sum += xv[1] * wv[1];
-        sum += xv[2] * wv[2];
-        sum += xv[3] * wv[3];
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+          if (!real[r]) continue;
+          float xv[4];
+          ei::Vec4<TX>::load(x + static_cast<size_t>(row0 + r) * W + i, xv);
+          sum[r] += xv[0] * wv[0];
+          sum[r] += xv[1] * wv[1];
+          sum[r] += xv[2] * wv[2];
+          sum[r] += xv[3] * wv[3];
+        }
       }
     } else {
-      for (int i = lane; i < W; i += EI_WAVE) sum += ei::to_f32<TX>(xr[i]) * wr[i];
+      for (int i = lane; i < W; i += EI_WAVE) {
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+          if (real[r]) sum[r] += ei::to_f32<TX>(x[static_cast<size_t>(row0 + r) * W + i]) * wr[i];
+      }
     }
-    sum = ei::wave_sum(sum);
-    if (!(sum > -FLT_MAX)) sum = -FLT_MAX;      // (a NaN chooses nothing ahead of a number)
-    if (lane == 0) logits[e] = sum;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      sum[r] = ei::wave_sum(sum[r]);
+      if (!(sum[r] > -FLT_MAX)) sum[r] = -FLT_MAX;      // (a NaN chooses nothing ahead of a number)
+      if (lane == 0) logits[r][e] = sum[r];
+    }
   }
   __syncthreads();
-  if (wave != 0) return;
+  if (wave >= R || row0 + wave >= N) return;
+  int32_t* e_out = expert + static_cast<size_t>(row0 + wave) * top;
+  float* w_out = weight + static_cast<size_t>(row0 + wave) * top;
+  if (row_seq && row_seq[row0 + wave] < 0) {    // a padding row: no expert has anything to add
+    for (int k = lane; k < top; k += EI_WAVE) { e_out[k] = 0; w_out[k] = 0.f; }
+    return;
+  }
   float z[kRouteMax];
 #pragma unroll
-  for (int j = 0; j < kRouteMax; ++j) z[j] = lane + j * EI_WAVE < E ? logits[lane + j * EI_WAVE] : -FLT_MAX;
+  for (int j = 0; j < kRouteMax; ++j) z[j] = lane + j * EI_WAVE < E ? logits[wave][lane + j * EI_WAVE] : -FLT_MAX;
   float score[kRouteMax];                        // mode 1: the softmax over all outputs
   if (mode == 1) {
     float top_z = -FLT_MAX;
@@ -167,7 +176,7 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
 #pragma unroll
     for (int j = 0; j < kRouteMax; ++j)
       z[j] = lane + j * EI_WAVE < E ? 1.0f / (1.0f + expf(-z[j])) : -FLT_MAX;
-    if (groups > 1 && keep < groups) leave_groups_out(z, logits, group_scores, E, groups, keep);
+    if (groups > 1 && keep < groups) leave_groups_out(z, logits[wave], group_scores[wave], E, groups, keep);
   }
   unsigned taken = 0;                            // bit j: this lane's expert lane + 64 j is chosen
   float total = 0.f, largest = 0.f;
@@ -213,7 +222,7 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ w_gate, const T* __restrict__ w_up,
                    const int32_t* __restrict__ expert, const float* __restrict__ weight,
-                   T* __restrict__ act, int W, int F, int top, int E, ExpertAct how) {
+                   T* __restrict__ act, int W, int F, int top, int E, ei::GateAct how) {
   const int pair = blockIdx.x;
   if (weight[pair] == 0.f) return;              // a padding row's choice
   const int row = pair / top, e = expert[pair];
@@ -254,7 +263,7 @@ moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ w_gate, const 
   for (int q = 0; q < 4; ++q) {
     const float gate = ei::wave_sum(sg[q]), up = ei::wave_sum(su[q]);
     if (lane == 0 && q < nf)
-      act[static_cast<size_t>(pair) * F + f0 + q] = ei::from_f32<T>(expert_act(gate, up, how));
+      act[static_cast<size_t>(pair) * F + f0 + q] = ei::from_f32<T>(ei::gated_product<T>(gate, up, how));
   }
 }
 
@@ -364,6 +373,32 @@ typedef float moe_f32x4 __attribute__((ext_vector_type(4)));
 
 constexpr int kTileN = 64, kTileK = 64;      // (kTileK: the least K-tile; K must be a multiple)
 
+// The tile `t` of TM places: its expert and its first place within the expert's span, or -1
+// beyond the last tile.  Every wave works it out for itself, an expert a lane.
+__device__ __forceinline__ int find_tile(const int32_t* __restrict__ starts, int E, int TM, int t,
+                                         int& m0) {
+  const int lane = threadIdx.x % EI_WAVE;
+  for (int base = 0; base < E; base += EI_WAVE) {
+    const int e = base + lane;
+    const int tiles = e < E ? (starts[e + 1] - starts[e] + TM - 1) / TM : 0;
+    int upto = tiles;                             // tiles of this and of the lanes before
+#pragma unroll
+    for (int offset = 1; offset < EI_WAVE; offset <<= 1) {
+      const int other = __shfl_up(upto, offset, EI_WAVE);
+      if (lane >= offset) upto += other;
+    }
+    const int total = __builtin_amdgcn_readfirstlane(__shfl(upto, EI_WAVE - 1, EI_WAVE));
+    if (t < total) {
+      const int found = __ffsll(static_cast<unsigned long long>(__ballot(upto > t))) - 1;
+      m0 = __builtin_amdgcn_readfirstlane((t - __shfl(upto - tiles, found, EI_WAVE)) * TM);
+      return __builtin_amdgcn_readfirstlane(base + found);
+    }
+    t -= total;
+  }
+  m0 = 0;
+  return -1;
+}
+
 // One tile of MB * 16 places of one expert against 64 rows of its matrix (GATED: of its gate
 // and of its up matrix).  GATED: the rows of `a` are gathered (row = pair / top) and
 // silu(gate) * up goes to `out_act` [P, N] at the pairs' places; else the rows of `a` are the
@@ -377,26 +412,14 @@ __global__ void __launch_bounds__(256)
 moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted,
                 const int32_t* __restrict__ starts, const bf16_t* __restrict__ w1,
                 const bf16_t* __restrict__ w2, bf16_t* __restrict__ out_act,
-                float* __restrict__ out_sum, int E, int N, int K, int top, ExpertAct how) {
+                float* __restrict__ out_sum, int E, int N, int K, int top, ei::GateAct how) {
   constexpr int TM = MB * 16;
   constexpr int PER_THREAD = TM * (KT / 8) / 256 > 0 ? TM * (KT / 8) / 256 : 1;
   __shared__ __attribute__((aligned(16))) bf16_t xs[TM * KT];
-  __shared__ int tile_info[2];
-  if (threadIdx.x == 0) {       // which expert's tile this block is
-    int t = blockIdx.x, found = -1, m0 = 0;
-    for (int e = 0; e < E; ++e) {
-      const int count = starts[e + 1] - starts[e];
-      const int tiles = (count + TM - 1) / TM;
-      if (t < tiles) { found = e; m0 = t * TM; break; }
-      t -= tiles;
-    }
-    tile_info[0] = found;
-    tile_info[1] = m0;
-  }
-  __syncthreads();
-  const int e = tile_info[0];
+  int m0;
+  const int e = find_tile(starts, E, TM, blockIdx.x, m0);      // which expert's tile this block is
   if (e < 0) return;
-  const int first = starts[e] + tile_info[1];                 // the tile's first place
+  const int first = starts[e] + m0;                           // the tile's first place
   const int valid = min(TM, starts[e + 1] - first);           // places of the tile that exist
   const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
   const int r16 = lane % 16, quarter = lane / 16;
@@ -472,7 +495,7 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
       const int n = n_wave + 4 * quarter + i;
       if (n >= N) continue;
       if (GATED) {
-        out_act[at + n] = ei::f32_to_bf16(expert_act(acc1[mb][i], acc2[mb][i], how));
+        out_act[at + n] = ei::f32_to_bf16(ei::gated_product<bf16_t>(acc1[mb][i], acc2[mb][i], how));
       } else {
         out_sum[at + n] = acc1[mb][i];
       }
@@ -480,27 +503,294 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
   }
 }
 
-// out [rows, W] = sum over a row's choices of weight * the choice's product row.
+// The experts of up to MB * 16 rows: a block an expert and 16 rows of its matrix (GATED: of its
+// gate and of its up matrix).  The block finds the pairs that chose its expert itself, in the
+// order of the pairs (padding rows left out), its WAVES waves share K out and meet in LDS.  Both
+// operands come from memory straight into operand registers, U steps of 32 at a time.  GATED: the
+// gated products go to out_act [pairs, N] at the pairs' own places; else the products times the
+// pairs' weights go to out_sum [top, rows, N], slice = the choice.
+template <int MB, bool GATED, int WAVES, int U>
+__global__ void __launch_bounds__(WAVES * EI_WAVE)
+moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
+               const float* __restrict__ weight, const int32_t* __restrict__ row_seq,
+               const bf16_t* __restrict__ w1, const bf16_t* __restrict__ w2,
+               bf16_t* __restrict__ out_act, float* __restrict__ out_sum, int rows, int N, int K,
+               int top, ei::GateAct how) {
+  constexpr int G = GATED ? 2 : 1;
+  __shared__ int places[MB * 16];
+  __shared__ int wave_counts[WAVES];
+  __shared__ float red[WAVES][MB][G][4][EI_WAVE];
+  const int e = blockIdx.y, n0 = blockIdx.x * 16, pairs = rows * top;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / EI_WAVE), lane = threadIdx.x % EI_WAVE;
+  int count = 0;
+  for (int base = 0; base < pairs; base += WAVES * EI_WAVE) {
+    const int p = base + threadIdx.x;
+    const bool mine = p < pairs && expert[p] == e && !(row_seq && row_seq[p / top] < 0);
+    const unsigned long long mask = __ballot(mine);
+    if (lane == 0) wave_counts[wave] = __popcll(mask);
+    __syncthreads();
+    int before = count, total = 0;
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) {
+      if (w < wave) before += wave_counts[w];
+      total += wave_counts[w];
+    }
+    const int at = before + __popcll(mask & ((1ull << lane) - 1ull));
+    if (mine && at < MB * 16) places[at] = p;    // (a row chooses an expert once at most)
+    count += total;
+    __syncthreads();
+  }
+  count = min(__builtin_amdgcn_readfirstlane(count), MB * 16);
+  if (count == 0) return;
+  const int r16 = lane % 16, quarter = lane / 16;
+  const bf16_t* w1_row = w1 + (static_cast<size_t>(e) * N + n0 + r16) * K + quarter * 8;
+  const bf16_t* w2_row = GATED ? w2 + (static_cast<size_t>(e) * N + n0 + r16) * K + quarter * 8 : nullptr;
+  const bf16_t* x_row[MB];
+#pragma unroll
+  for (int mb = 0; mb < MB; ++mb) {
+    const int p = places[min(mb * 16 + r16, count - 1)];      // (clamped: such rows are not stored)
+    x_row[mb] = a + static_cast<size_t>(GATED ? p / top : p) * K + quarter * 8;
+  }
+  moe_f32x4 acc[MB][G];
+#pragma unroll
+  for (int mb = 0; mb < MB; ++mb)
+#pragma unroll
+    for (int g = 0; g < G; ++g) acc[mb][g] = moe_f32x4{0.f, 0.f, 0.f, 0.f};
+  const int steps = K / 32, per = (steps + WAVES - 1) / WAVES;
+  const int s_end = min(steps, (wave + 1) * per);
+  for (int s0 = wave * per; s0 < s_end; s0 += U) {
+    moe_bf16x8 wa[U], wb[GATED ? U : 1], xf[U][MB];
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (s0 + u < s_end) {
+        wa[u] = *reinterpret_cast<const moe_bf16x8*>(w1_row + (s0 + u) * 32);
+        if (GATED) wb[u] = *reinterpret_cast<const moe_bf16x8*>(w2_row + (s0 + u) * 32);
+#pragma unroll
+        for (int mb = 0; mb < MB; ++mb)
+          if (mb * 16 < count) xf[u][mb] = *reinterpret_cast<const moe_bf16x8*>(x_row[mb] + (s0 + u) * 32);
+      }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (s0 + u < s_end) {
+#pragma unroll
+        for (int mb = 0; mb < MB; ++mb)
+          if (mb * 16 < count) {
+            acc[mb][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wa[u], xf[u][mb], acc[mb][0], 0, 0, 0);
+            if (GATED)
+              acc[mb][G - 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wb[u], xf[u][mb], acc[mb][G - 1], 0, 0, 0);
+          }
+      }
+  }
+#pragma unroll
+  for (int mb = 0; mb < MB; ++mb)
+#pragma unroll
+    for (int g = 0; g < G; ++g)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) red[wave][mb][g][i][lane] = acc[mb][g][i];
+  __syncthreads();
+  // lane (r16, quarter) of a wave held, of place mb * 16 + r16, the matrix rows n0 + 4 quarter + i
+  for (int o = threadIdx.x; o < count * 16; o += WAVES * EI_WAVE) {
+    const int index = o / 16, n = o % 16;
+    const int mb = index / 16, from = index % 16 + 16 * (n / 4), i = n % 4;
+    float sum[G];
+#pragma unroll
+    for (int g = 0; g < G; ++g) {
+      sum[g] = 0.f;
+#pragma unroll
+      for (int w = 0; w < WAVES; ++w) sum[g] += red[w][mb][g][i][from];
+    }
+    const int p = places[index];
+    if (GATED)
+      out_act[static_cast<size_t>(p) * N + n0 + n] =
+          ei::f32_to_bf16(ei::gated_product<bf16_t>(sum[0], sum[G - 1], how));
+    else
+      out_sum[(static_cast<size_t>(p % top) * rows + p / top) * N + n0 + n] = weight[p] * sum[0];
+  }
+}
+
+// The experts of a prompt: tiles of 128 places of one expert against 128 rows of its matrix
+// (GATED: 64 of its gate and the same 64 of its up matrix) on 32x32x16 products.  A block of four
+// waves, two by two; a wave holds 64 places against 64 matrix rows (GATED: 32 of each matrix, so
+// that a lane ends up with the gate and the up sum of the same element).  K goes by in tiles of 64
+// through two LDS buffers for both operands, moved from global memory straight into LDS (a wave
+// load is a kilobyte, lane l's 16 bytes at place l of it): tile k + 1 is asked for right after the
+// barrier that frees its buffer and arrives while tile k is multiplied; a second block on the
+// compute unit covers the rest of the wait.  The 16-byte pieces of a row are exchanged among
+// themselves (piece ^ (row / 2) % 8), so that 16 rows read at one place of a row meet every bank
+// once; a lane fetches the piece that belongs at its place.
+// Blocks are dealt to the 8 XCDs round robin; block ids are laid out so that an XCD works on
+// `group` tiles of places at a time against all rows of the matrix, whose operands its L2 then
+// holds.
+constexpr int kBig = 128, kBigK = 64;
+typedef float moe_f32x16 __attribute__((ext_vector_type(16)));
+
+template <bool GATED>
+__global__ void __launch_bounds__(256, 2)
+moe_tile_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted,
+                const int32_t* __restrict__ starts, const bf16_t* __restrict__ w1,
+                const bf16_t* __restrict__ w2, bf16_t* __restrict__ out_act,
+                float* __restrict__ out_sum, int E, int N, int K, int top, int n_tiles,
+                int place_tiles, int group, ei::GateAct how) {
+  __shared__ __attribute__((aligned(1024))) bf16_t lds[2][2][kBig * kBigK];   // [buffer][operand]
+  const int xcd = blockIdx.x & 7, slot = blockIdx.x >> 3;
+  const int per_group = group * n_tiles, rest = slot % per_group;
+  const int tile = (slot / per_group * 8 + xcd) * group + rest % group, n_tile = rest / group;
+  if (tile >= place_tiles) return;
+  int m0;
+  const int e = find_tile(starts, E, kBig, tile, m0);
+  if (e < 0) return;
+  const int first = starts[e] + m0;                           // the tile's first place
+  const int valid = min(kBig, starts[e + 1] - first);         // places of the tile that exist
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / EI_WAVE), lane = threadIdx.x % EI_WAVE;
+  const int l32 = lane & 31, half = lane >> 5, wm = wave >> 1, wn = wave & 1;
+  constexpr int LOADS = kBig * kBigK * 2 / 1024 / 4;          // wave loads of an operand's tile a wave
+  const bf16_t* from_a[LOADS];
+  const bf16_t* from_b[LOADS];
+#pragma unroll
+  for (int i = 0; i < LOADS; ++i) {
+    const int row = (wave * LOADS + i) * 8 + lane / 8, piece = (lane % 8) ^ ((row >> 1) & 7);
+    const int at = first + min(row, valid - 1);               // (clamped: such rows are not stored)
+    const size_t source = GATED ? static_cast<size_t>(sorted[at] / top) : static_cast<size_t>(at);
+    from_a[i] = a + source * K + piece * 8;
+    const bf16_t* matrix = GATED && row >= kBig / 2 ? w2 : w1;
+    const int n = GATED ? n_tile * (kBig / 2) + row % (kBig / 2) : n_tile * kBig + row;
+    from_b[i] = matrix + (static_cast<size_t>(e) * N + min(n, N - 1)) * K + piece * 8;
+  }
+  auto fetch = [&](int k0, int buffer) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < LOADS; ++i) {
+      const int at = (wave * LOADS + i) * 512;
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) void*)(from_a[i] + k0),
+          (__attribute__((address_space(3))) void*)(&lds[buffer][0][at]), 16, 0, 0);
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) void*)(from_b[i] + k0),
+          (__attribute__((address_space(3))) void*)(&lds[buffer][1][at]), 16, 0, 0);
+    }
+  };
+  int read_a[2], read_b[2], piece_at[4];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    read_a[j] = (wm * 64 + j * 32 + l32) * kBigK;
+    read_b[j] = (GATED ? j * 64 + wn * 32 + l32 : wn * 64 + j * 32 + l32) * kBigK;
+  }
+#pragma unroll
+  for (int s = 0; s < 4; ++s) piece_at[s] = ((2 * s + half) ^ ((l32 >> 1) & 7)) * 8;
+  moe_f32x16 acc[2][2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int v = 0; v < 16; ++v) acc[i][j][v] = 0.f;
+  fetch(0, 0);
+  const int k_tiles = K / kBigK;
+  for (int kt = 0; kt < k_tiles; ++kt) {
+    const int buffer = kt & 1;
+    // this tile has arrived (every wave waits for its own loads), the other buffer is free
+    __builtin_amdgcn_s_waitcnt(0x0F70);
+    __syncthreads();
+    if (kt + 1 < k_tiles) fetch((kt + 1) * kBigK, buffer ^ 1);
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int s = 0; s < 4; ++s) {
+      moe_bf16x8 fa[2], fb[2];
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        fa[j] = *reinterpret_cast<const moe_bf16x8*>(&lds[buffer][0][read_a[j] + piece_at[s]]);
+        fb[j] = *reinterpret_cast<const moe_bf16x8*>(&lds[buffer][1][read_b[j] + piece_at[s]]);
+      }
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+    }
+  }
+  // lane (matrix row l32, half) holds the places 8 (v / 4) + 4 half + v % 4 of a block of 32
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+#pragma unroll
+    for (int v = 0; v < 16; ++v) {
+      const int row = wm * 64 + i * 32 + 8 * (v / 4) + 4 * half + v % 4;
+      if (row >= valid) continue;
+      const size_t at = static_cast<size_t>(first + row) * N;
+      if (GATED) {
+        out_act[at + n_tile * (kBig / 2) + wn * 32 + l32] =
+            ei::f32_to_bf16(ei::gated_product<bf16_t>(acc[i][0][v], acc[i][1][v], how));
+      } else {
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+          const int n = n_tile * kBig + wn * 64 + j * 32 + l32;
+          if (n < N) out_sum[at + n] = acc[i][j][v];
+        }
+      }
+    }
+}
+
+template <bool GATED>
+void launch_tiles(const bf16_t* a, const int32_t* sorted, const int32_t* starts, const bf16_t* w1,
+                  const bf16_t* w2, bf16_t* act, float* sums, int P, int E, int N, int K, int top,
+                  const ei::GateAct& how, hipStream_t stream) {
+  const int n_tiles = (N + (GATED ? kBig / 2 : kBig) - 1) / (GATED ? kBig / 2 : kBig);
+  const int place_tiles = P / kBig + E;             // at most: whole tiles and one rest an expert
+  const int group = place_tiles >= 128 ? 4 : 2;
+  const int groups = (place_tiles + group - 1) / group;
+  const unsigned blocks = static_cast<unsigned>((groups + 7) / 8 * 8) * group * n_tiles;
+  moe_tile_kernel<GATED><<<blocks, 256, 0, stream>>>(a, sorted, starts, w1, w2, act, sums, E, N, K,
+                                                     top, n_tiles, place_tiles, group, how);
+}
+
+// out [rows, W] = sum over a row's choices of weight * the choice's product row, four columns a
+// thread.
 __global__ void moe_combine_kernel(const float* __restrict__ sums, const int32_t* __restrict__ place,
                                    const float* __restrict__ weight, float* __restrict__ out,
                                    int W, int top, size_t total, const bf16_t* __restrict__ x,
                                    ExtraRows extra) {
-  const size_t start = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
-  const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x;
+  const size_t start = (static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x) * 4;
+  const size_t step = static_cast<size_t>(gridDim.x) * blockDim.x * 4;
   for (size_t idx = start; idx < total; idx += step) {
     const size_t row = idx / W, col = idx % W;
-    float sum = 0.f;
-    for (int k = 0; k < top; ++k) {
-      const int q = place[row * top + k];
-      if (q >= 0) sum += weight[row * top + k] * sums[static_cast<size_t>(q) * W + col];
-      else if (q == -2) sum += weight[row * top + k] * ei::bf16_to_f32(x[idx]);   // identity
+    float sum[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < top; k0 += 4) {
+      int q[4];
+      float p[4], v[4][4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        q[u] = k0 + u < top ? place[row * top + k0 + u] : -1;
+        p[u] = k0 + u < top ? weight[row * top + k0 + u] : 0.f;
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        v[u][0] = v[u][1] = v[u][2] = v[u][3] = 0.f;
+        if (q[u] >= 0) ei::Vec4<float>::load(sums + static_cast<size_t>(q[u]) * W + col, v[u]);
+        else if (q[u] == -2) ei::Vec4<bf16_t>::load(x + idx, v[u]);            // identity
+      }
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) sum[i] += p[u] * v[u][i];
     }
-    if (extra.rows) sum += extra_at(extra, idx);
-    out[idx] = sum;
+    if (extra.rows) {
+      float more[4];
+      if (extra.dtype == EI_F32) {
+        const float* from = static_cast<const float*>(extra.rows) + idx;
+        for (int s = 0; s < extra.slices; ++s) {
+          ei::Vec4<float>::load(from + s * extra.slice, more);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) sum[i] += more[i];
+        }
+      } else {
+        ei::Vec4<bf16_t>::load(static_cast<const bf16_t*>(extra.rows) + idx, more);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) sum[i] += more[i];
+      }
+    }
+    ei::Vec4<float>::store(out + idx, sum);
   }
 }
 
-bool known_act(int kind) { return kind == 0 || kind == 1; }
+bool known_act(int kind) { return kind >= 0 && kind <= 2; }
 
 bool extra_fits(const void* rows, int dtype, int slices, long long slice) {
   return !rows || (slices >= 1 && slice >= 0 && (dtype == EI_F32 || (dtype == EI_BF16 && slices == 1)));
@@ -519,18 +809,24 @@ extern "C" int ei_moe_route(const void* x, int x_dtype, const float* w_router, c
   EI_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && (groups == 1 || mode == 2) &&
                  top <= E / groups * keep,
              "moe_route: equal groups of experts, enough of them kept for the choice");
-  const int threads = 256;
-  const unsigned blocks = static_cast<unsigned>(N);
-  if (x_dtype == EI_F32)
-    moe_route_kernel<float><<<blocks, threads, 0, stream>>>(static_cast<const float*>(x), w_router,
-                                                            row_seq, expert, weight, N, W, E, top,
-                                                            mode, correction, groups, keep, weight_scale);
-  else if (x_dtype == EI_BF16)
-    moe_route_kernel<bf16_t><<<blocks, threads, 0, stream>>>(static_cast<const bf16_t*>(x), w_router,
-                                                             row_seq, expert, weight, N, W, E, top,
-                                                            mode, correction, groups, keep, weight_scale);
-  else
-    EI_REQUIRE(false, "moe_route: unknown dtype");
+  // few rows: a block of up to 16 waves a row, an expert a wave where there are as many; many rows:
+  // four rows a block, which read the router's matrix together
+#define EI_ROUTE(TX)                                                                           \
+  do {                                                                                         \
+    const TX* xx = static_cast<const TX*>(x);                                                  \
+    if (N >= 512)                                                                              \
+      moe_route_kernel<TX, 4><<<(N + 3) / 4, 256, 0, stream>>>(                                \
+          xx, w_router, row_seq, expert, weight, N, W, E, top, mode, correction, groups, keep, \
+          weight_scale);                                                                       \
+    else                                                                                       \
+      moe_route_kernel<TX, 1><<<N, EI_WAVE * (E >= 16 ? 16 : E >= 8 ? 8 : 4), 0, stream>>>(    \
+          xx, w_router, row_seq, expert, weight, N, W, E, top, mode, correction, groups, keep, \
+          weight_scale);                                                                       \
+  } while (0)
+  if (x_dtype == EI_F32) EI_ROUTE(float);
+  else if (x_dtype == EI_BF16) EI_ROUTE(bf16_t);
+  else EI_REQUIRE(false, "moe_route: unknown dtype");
+#undef EI_ROUTE
   EI_LAUNCH_CHECK();
 }
 
@@ -543,7 +839,7 @@ extern "C" int ei_moe_experts(const void* x, const void* w_gate, const void* w_u
   EI_REQUIRE(known_act(act_kind), "moe_experts: unknown activation");
   EI_REQUIRE(extra_fits(extra_rows, extra_dtype, extra_slices, extra_slice),
              "moe_experts: the rows to add have the wrong type");
-  const ExpertAct how{act_kind, limit, alpha};
+  const ei::GateAct how{act_kind, limit, alpha};
   const ExtraRows extra{extra_rows, extra_dtype, extra_slices, static_cast<size_t>(extra_slice)};
   EI_REQUIRE(N > 0 && W > 0 && F > 0 && top >= 1, "moe_experts: sizes must be positive");
   EI_REQUIRE(static_cast<long long>(N) * top <= 0x7fffffffLL && (F + 15) / 16 <= 65535 &&
@@ -582,7 +878,7 @@ extern "C" int ei_moe_experts_grouped(const void* x, const void* w_gate, const v
   EI_REQUIRE(known_act(act_kind), "moe_experts_grouped: unknown activation");
   EI_REQUIRE(extra_fits(extra_rows, extra_dtype, extra_slices, extra_slice),
              "moe_experts_grouped: the rows to add have the wrong type");
-  const ExpertAct how{act_kind, limit, alpha};
+  const ei::GateAct how{act_kind, limit, alpha};
   const ExtraRows extra{extra_rows, extra_dtype, extra_slices, static_cast<size_t>(extra_slice)};
   EI_REQUIRE(x && w_gate && w_up && w_down && expert && weight && sorted && place && starts && act &&
                  sums && out, "moe_experts_grouped: null pointer");
@@ -613,15 +909,50 @@ extern "C" int ei_moe_experts_grouped(const void* x, const void* w_gate, const v
     else
       moe_gemm_kernel<2, false, 64><<<grid_down, 256, 0, stream>>>(ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top, how);
   } else {
-    const unsigned tiles = static_cast<unsigned>((P + 127) / 128 + E);
-    moe_gemm_kernel<8, true, 64><<<dim3(tiles, (F + kTileN - 1) / kTileN), 256, 0, stream>>>(
-        xb, sorted, starts, g, u, ab, nullptr, E, F, W, top, how);
-    moe_gemm_kernel<8, false, 64><<<dim3(tiles, (W + kTileN - 1) / kTileN), 256, 0, stream>>>(
-        ab, sorted, starts, d, nullptr, nullptr, sums, E, W, F, top, how);
+    launch_tiles<true>(xb, sorted, starts, g, u, ab, nullptr, P, E, F, W, top, how, stream);
+    launch_tiles<false>(ab, sorted, starts, d, nullptr, nullptr, sums, P, E, W, F, top, how, stream);
   }
   const size_t total = static_cast<size_t>(N) * W;
-  size_t blocks = (total + 255) / 256;
+  size_t blocks = (total / 4 + 255) / 256;
   if (blocks > static_cast<size_t>(ei_compute_units()) * 16) blocks = static_cast<size_t>(ei_compute_units()) * 16;
   moe_combine_kernel<<<static_cast<unsigned>(blocks), 256, 0, stream>>>(sums, place, weight, out, W, top, total, xb, extra);
+  EI_LAUNCH_CHECK();
+}
+
+// Most rows that `ei_moe_experts_few` takes.
+extern "C" int ei_moe_few_rows() { return 64; }
+
+// The experts of at most 64 rows: act [N * top, F] bfloat16 is scratch; slice k of out [top, N, W]
+// float32 receives every row's k-th choice's product row times its weight (a padding row, row_seq
+// < 0, is not written).  Every choice must be an expert (no identity ones), none twice in a row.
+extern "C" int ei_moe_experts_few(const void* x, const void* w_gate, const void* w_up,
+                                  const void* w_down, const int32_t* expert, const float* weight,
+                                  const int32_t* row_seq, void* act, float* out, int N, int W, int F,
+                                  int E, int top, int act_kind, float limit, float alpha,
+                                  hipStream_t stream) {
+  EI_REQUIRE(x && w_gate && w_up && w_down && expert && weight && act && out,
+             "moe_experts_few: null pointer");
+  EI_REQUIRE(N > 0 && N <= ei_moe_few_rows() && top >= 1 && E >= 1 && E <= 65535 &&
+                 ei_moe_grouped_supported(EI_BF16, W, F, E),
+             "moe_experts_few: sizes it does not take");
+  EI_REQUIRE(known_act(act_kind), "moe_experts_few: unknown activation");
+  const ei::GateAct how{act_kind, limit, alpha};
+  const bf16_t* xb = static_cast<const bf16_t*>(x);
+  const bf16_t* g = static_cast<const bf16_t*>(w_gate);
+  const bf16_t* u = static_cast<const bf16_t*>(w_up);
+  const bf16_t* d = static_cast<const bf16_t*>(w_down);
+  bf16_t* ab = static_cast<bf16_t*>(act);
+  const dim3 grid_up(F / 16, E), grid_down(W / 16, E);
+#define EI_FEW(MB, WAVES, U)                                                                   \
+  do {                                                                                         \
+    moe_few_kernel<MB, true, WAVES, U><<<grid_up, WAVES * EI_WAVE, 0, stream>>>(               \
+        xb, expert, weight, row_seq, g, u, ab, nullptr, N, F, W, top, how);                    \
+    moe_few_kernel<MB, false, WAVES, U><<<grid_down, WAVES * EI_WAVE, 0, stream>>>(            \
+        ab, expert, weight, row_seq, d, nullptr, nullptr, out, N, W, F, top, how);             \
+  } while (0)
+  if (N <= 16) EI_FEW(1, 8, 8);
+  else if (N <= 32) EI_FEW(2, 4, 8);
+  else EI_FEW(4, 4, 4);
+#undef EI_FEW
   EI_LAUNCH_CHECK();
 }

@@ -137,22 +137,6 @@ __global__ void add_rmsnorm_vec_kernel(float* __restrict__ residual, const TD* _
 
 // Where gate and up of output column `col` lie in a row of 2I: the halves [gate | up]
 // (strip = 0), or strips of `strip` gate columns followed by their `strip` up columns.
-// gate activations of the C interface: 0 silu, 1 the tanh form of gelu, 2 the clamped swish:
-// with g = min(gate, limit) and u = clamp(up, -limit, limit) the product is
-// g sigmoid(alpha g) (u + 1)
-template <typename TO> __device__ __forceinline__ float gate_act(float x, int act) {
-  if (act == 0) return ei::silu<TO>(x);
-  return 0.5f * x * (1.0f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
-}
-
-template <typename TO>
-__device__ __forceinline__ float gated_product(float gate, float up, int act, float limit, float alpha) {
-  if (act != 2) return gate_act<TO>(gate, act) * up;
-  const float g = fminf(gate, limit);
-  const float u = fminf(fmaxf(up, -limit), limit);
-  return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
-}
-
 __device__ __forceinline__ size_t gate_column(size_t col, int strip) {
   return strip ? (col / strip) * 2 * strip + col % strip : col;
 }
@@ -176,7 +160,7 @@ __global__ void swiglu_kernel(const TI* __restrict__ gate_up, int nsplit, size_t
       gate += bias[gate_column(col, strip)];
       up += bias[gate_column(col, strip) + up_offset];
     }
-    out[idx] = ei::from_f32<TO>(gated_product<TO>(gate, up, act, limit, alpha));
+    out[idx] = ei::from_f32<TO>(ei::gated_product<TO>(gate, up, ei::GateAct{act, limit, alpha}));
   }
 }
 
@@ -231,8 +215,8 @@ __global__ void swiglu_vec_kernel(const TI* __restrict__ gate_up, int nsplit, si
     float y0[4], y1[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      y0[i] = gated_product<TO>(gate[i], up[i], act, limit, alpha);
-      y1[i] = gated_product<TO>(gate[i + 4], up[i + 4], act, limit, alpha);
+      y0[i] = ei::gated_product<TO>(gate[i], up[i], ei::GateAct{act, limit, alpha});
+      y1[i] = ei::gated_product<TO>(gate[i + 4], up[i + 4], ei::GateAct{act, limit, alpha});
     }
     TO* dst = out + row * I + col;
     Vec4<TO>::store(dst, y0);
@@ -691,16 +675,17 @@ extern "C" int ei_activation(const void* in, int in_dtype, int nsplit, long long
 namespace {
 
 // One block per row.  x = sum over slices of delta[row]; y = residual[row] + x * rsqrt(mean(x^2)
-// + eps) * w_after (stored back); out[row] = y * rsqrt(mean(y^2) + eps) * w_next in the storage
-// type: the norm on a sublayer's output, the addition and the next sublayer's input norm in
-// one pass over the row.
+// + eps) * w_after (+ shift, a vector added to the stream; null: none) (stored back); out[row] =
+// y * rsqrt(mean(y^2) + eps) * w_next in the storage type: the norm on a sublayer's output, the
+// addition and the next sublayer's input norm in one pass over the row.
 template <typename TD, typename TO>
 __global__ void norm_add_norm_kernel(float* __restrict__ residual, const TD* __restrict__ delta,
                                      int nsplit, size_t split_stride,
                                      const float* __restrict__ w_after,
                                      const float* __restrict__ w_next, float eps,
                                      TO* __restrict__ out, int H,
-                                     const float* __restrict__ bias) {
+                                     const float* __restrict__ bias,
+                                     const float* __restrict__ shift) {
   extern __shared__ float row_values[];
   __shared__ float scratch[16];
   const size_t base = static_cast<size_t>(blockIdx.x) * H;
@@ -716,7 +701,8 @@ __global__ void norm_add_norm_kernel(float* __restrict__ residual, const TD* __r
   const float inv = 1.0f / sqrtf(ei::block_sum(sum, scratch) / static_cast<float>(H) + eps);
   float sum2 = 0.f;
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
-    const float y = residual[base + i] + (row_values[i] * inv) * w_after[i];
+    float y = residual[base + i] + (row_values[i] * inv) * w_after[i];
+    if (shift) y += shift[i];
     residual[base + i] = y;
     row_values[i] = y;
     sum2 += y * y;
@@ -734,7 +720,8 @@ __global__ void norm_add_norm_vec_kernel(float* __restrict__ residual, const TD*
                                          const float* __restrict__ w_after,
                                          const float* __restrict__ w_next, float eps,
                                          TO* __restrict__ out, int H,
-                                         const float* __restrict__ bias) {
+                                         const float* __restrict__ bias,
+                                         const float* __restrict__ shift) {
   __shared__ float scratch[16];
   const size_t base = static_cast<size_t>(blockIdx.x) * H;
   const int quads = H / 4;
@@ -784,10 +771,15 @@ __global__ void norm_add_norm_vec_kernel(float* __restrict__ residual, const TD*
     const int qd = threadIdx.x + k * blockDim.x;
     if (qd < quads) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        r[k][i] += (x[k][i] * inv) * wa[k][i];
-        sum2 += r[k][i] * r[k][i];
+      for (int i = 0; i < 4; ++i) r[k][i] += (x[k][i] * inv) * wa[k][i];
+      if (shift) {
+        float more[4];
+        Vec4<float>::load(shift + qd * 4, more);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) r[k][i] += more[i];
       }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) sum2 += r[k][i] * r[k][i];
       Vec4<float>::store(residual + base + qd * 4, r[k]);
     }
   }
@@ -839,7 +831,7 @@ __global__ void set_rows_kernel(const TD* __restrict__ x, int nsplit, size_t spl
 extern "C" int ei_norm_add_norm(float* residual, const void* delta, int delta_dtype, int nsplit,
                                 long long split_stride, const float* w_after, const float* w_next,
                                 float eps, void* out, int out_dtype, int N, int H,
-                                const float* bias, hipStream_t stream) {
+                                const float* bias, const float* shift, hipStream_t stream) {
   EI_REQUIRE(N > 0 && H > 0 && nsplit >= 1, "norm_add_norm: sizes must be positive");
   EI_REQUIRE(residual && delta && w_after && w_next && out, "norm_add_norm: null pointer");
   EI_REQUIRE(static_cast<size_t>(H) * sizeof(float) <= 60 * 1024, "norm_add_norm: row too wide");
@@ -856,7 +848,7 @@ extern "C" int ei_norm_add_norm(float* residual, const void* delta, int delta_dt
 #define EI_NAN_VEC(TD, TO, C)                                                                \
   norm_add_norm_vec_kernel<TD, TO, C><<<N, vthreads, 0, stream>>>(                           \
       residual, static_cast<const TD*>(delta), nsplit, ss, w_after, w_next, eps,             \
-      static_cast<TO*>(out), H, bias)
+      static_cast<TO*>(out), H, bias, shift)
 #define EI_NAN_CASE(TD, TO)                                                                  \
   do {                                                                                       \
     if (chunks == 1) EI_NAN_VEC(TD, TO, 1);                                                  \
@@ -865,7 +857,7 @@ extern "C" int ei_norm_add_norm(float* residual, const void* delta, int delta_dt
     else                                                                                     \
       norm_add_norm_kernel<TD, TO><<<N, threads, lds, stream>>>(                             \
           residual, static_cast<const TD*>(delta), nsplit, ss, w_after, w_next, eps,         \
-          static_cast<TO*>(out), H, bias);                                                   \
+          static_cast<TO*>(out), H, bias, shift);                                              \
   } while (0)
   if (delta_dtype == EI_F32 && out_dtype == EI_F32) EI_NAN_CASE(float, float);
   else if (delta_dtype == EI_F32 && out_dtype == EI_BF16) EI_NAN_CASE(float, bf16_t);

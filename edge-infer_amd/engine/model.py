@@ -35,6 +35,7 @@ import torch
 
 from ..config.specs import ModelSpec, pass_starts
 from ..csrc import lib
+from ..parts.block import PendingNorm
 from ..parts.linear import Linear
 from ..parts.registry import lookup
 from ..weights.loader import ParamSpec
@@ -338,12 +339,21 @@ class DecoderModel:
             if turn is not None:
                 pending = self.enter_pass(ctx, residual, pending, embedded, turn)
             pending = self.layers[entry.layer].forward(ctx, residual, pending, entry)
+        if isinstance(pending, PendingNorm):
+            pending.settle(ctx, residual)
+            pending = None
         return pending
 
     def enter_pass(self, ctx, residual, pending, embedded, turn: int):
         """Before pass `turn` of the loop: x <- W [x ; x0] + step[turn], with x0 the embedding
         output (x <- x + step[turn] in a loop that does not remix).  The product reads both streams in the step's storage type; its float32 result
         takes the stream's place."""
+        if isinstance(pending, PendingNorm):
+            if self.loop_in is None:
+                pending.vector = self.loop_step[turn]      # the kernel that adds it adds both
+                return pending
+            pending.settle(ctx, residual)
+            pending = None
         if pending is not None:
             raise ValueError("a pass of the loop starts after a block that left a delta pending")
         if self.loop_in is None:

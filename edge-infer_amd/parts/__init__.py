@@ -1,6 +1,6 @@
 from .attention import Attention
 from .base import KVRequest, StateRequest, StepContext, Workspace
-from .block import OutputNormBlock, PreNormBlock, SandwichBlock
+from .block import OutputNormBlock, PendingNorm, PreNormBlock, SandwichBlock
 from .delta import GatedDelta
 from .latent import LatentAttention
 from .linear_attention import LinearAttention
@@ -36,7 +36,7 @@ register_block("outnorm", OutputNormBlock)
 register_block("sandwich", SandwichBlock)
 
 __all__ = ["Attention", "KVRequest", "StateRequest", "StepContext", "Workspace", "PreNormBlock",
-           "OutputNormBlock", "SandwichBlock", "GatedDelta", "LatentAttention", "MatrixMemory", "RotaryFrequencies",
+           "OutputNormBlock", "PendingNorm", "SandwichBlock", "GatedDelta", "LatentAttention", "MatrixMemory", "RotaryFrequencies",
            "RotaryHalfFrequencies", "RoutedMLP", "LayerNorm", "LinearAttention", "ParallelMixer", "StateSpace", "DenseMLP", "Linear", "GatedMLP", "RMSNorm", "lookup", "register_block", "register_feed_forward",
            "register_mixer", "register_norm", "register_position", "unregister", "NoPosition",
            "RotaryTable"]

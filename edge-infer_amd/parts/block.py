@@ -201,6 +201,38 @@ class OutputNormBlock:
         return None
 
 
+class PendingNorm:
+    """What a layer has not yet added to the stream: stream += norm(delta (+ bias)) (+ vector), for
+    a plain RMS norm.  Whoever reads the stream next takes it in (`then`, one kernel with its own
+    norm) or adds it (`apply`); `vector` [width] may be set by whoever adds a vector in between."""
+
+    def __init__(self, delta, bias, norm):
+        self.delta, self.bias, self.norm = delta, bias, norm
+        self.vector = None
+
+    def apply(self, residual) -> None:
+        lib.norm_add(residual, self.delta, self.norm.weight, self.norm.eps, bias=self.bias)
+        if self.vector is not None:
+            lib.bias_rows(self.vector, residual, accumulate=True)
+
+    def settle(self, ctx, residual) -> None:
+        """Added to the stream; the delta's storage is free."""
+        self.apply(residual)
+        ctx.release(self.delta)
+
+    def then(self, ctx, residual, following, out_name):
+        """Added to the stream, and the rows of `following`, a plain RMS norm, in one pass where
+        the two have one eps."""
+        if following.eps != self.norm.eps:
+            self.settle(ctx, residual)
+            return following.add_norm(ctx, residual, None, out_name, write_residual=False)
+        out = ctx.buffer(out_name, tuple(residual.shape))
+        lib.norm_add_norm(residual, self.delta, self.norm.weight, following.weight, following.eps,
+                          out, bias=self.bias, vector=self.vector)
+        ctx.release(self.delta)
+        return out
+
+
 class SandwichBlock:
     """x += s * norm1b(mixer(norm1(x))); x += s * norm2b(feed_forward(norm2(x))): a norm before
     and a norm after every sublayer, and a multiplier s (`residual_scale`) on what is added.  A
@@ -216,8 +248,10 @@ class SandwichBlock:
 
     The multipliers are folded into the float32 weights (and biases) of the norms on the
     outputs when the block is built.  The norm on the mixer's output, the addition and the feed-forward's input
-    norm are one kernel; everything is added when the block returns, so it returns no pending
-    delta and follows only blocks that do the same."""
+    norm are one kernel.  Everything is added when the block returns, so it returns no pending
+    delta and follows only blocks that do the same; with `defer_output` (plain RMS norms only)
+    the norm on the last sublayer's output and its addition are returned as a `PendingNorm`, which
+    the next such block takes into the kernel of its first norm."""
 
     capture_safe = True      # nothing of its own besides its parts' kernels
 
@@ -339,6 +373,9 @@ class SandwichBlock:
                          for norm in (self.norm1b, self.norm2) if norm is not None)
         self.fused_own = (self.norm2 is not None and hasattr(self.norm1b, "norm_add_then")
                           and type(self.norm1b) is type(self.norm2))
+        self.defer = bool(getattr(layer_spec, "defer_output", False))
+        if self.defer and not (self.fused and not self.fused_own):
+            raise ValueError("sandwich: only plain RMS norms on a sublayer's output can be deferred")
         self.hidden = hidden
         self.taps = int(getattr(layer_spec, "input_conv", 0))
         self.conv1 = self.conv2 = None
@@ -376,12 +413,16 @@ class SandwichBlock:
         return out
 
     def forward(self, ctx, residual, pending, entry):
-        if pending is not None:
+        if pending is not None and not (isinstance(pending, PendingNorm) and self.defer):
             raise ValueError("sandwich: a delta of the block before is still pending; this "
                              "arrangement follows only blocks that add everything themselves")
-        conv = self._conv_in_norm(ctx, entry, 0, self.norm1)
-        h = self.norm1.add_norm(ctx, residual, None, "block.h", write_residual=False,
-                                **({} if conv is None else {"conv": conv}))
+        conv = None
+        if pending is not None:
+            h = pending.then(ctx, residual, self.norm1, "block.h")
+        else:
+            conv = self._conv_in_norm(ctx, entry, 0, self.norm1)
+            h = self.norm1.add_norm(ctx, residual, None, "block.h", write_residual=False,
+                                    **({} if conv is None else {"conv": conv}))
         if self.taps and conv is None:
             h = self._convolved(ctx, h, entry, 0)
         # a sublayer that can leave its last product's bias to the norm kernel behind it does
@@ -390,6 +431,8 @@ class SandwichBlock:
                      else (self.mixer.forward(ctx, h, entry), None))
         ctx.release(h)
         if self.ffn is None:
+            if self.defer:
+                return PendingNorm(a, a_bias, self.norm1b)
             self.norm1b.norm_add(ctx, residual, a, bias=a_bias)
             ctx.release(a)
             return None
@@ -415,6 +458,8 @@ class SandwichBlock:
                      if getattr(self.ffn, "bias_later", False)
                      else (self.ffn.forward(ctx, h2), None))
         ctx.release(h2)
+        if self.defer:
+            return PendingNorm(f, f_bias, self.norm2b)
         self.norm2b.norm_add(ctx, residual, f, bias=f_bias)
         ctx.release(f)
         return None

@@ -106,15 +106,29 @@ class Linear:
             return out, (self.bias_f32 if leave else None)
         return out
 
+    def slices_behind(self, ctx, x: torch.Tensor, out_name: str, leading: int):
+        """For a few-rows product without a bias: its float32 slices behind `leading` slices of
+        the same shape that the caller fills, as one buffer [leading + slices, N, out]; None where
+        that product does not apply."""
+        rows = x.shape[0]
+        if (self.dtype != torch.bfloat16 or self.bias is not None
+                or not lib.skinny_gemm_ok(rows, self.in_features)):
+            return None
+        splits = lib.skinny_gemm_splits(rows, self.out_features, self.in_features)
+        out = ctx.buffer(out_name + ".f32", (leading + splits, rows, self.out_features), torch.float32)
+        self._few_rows(x, out[leading:])
+        return out
+
     def _library(self, x: torch.Tensor, out: torch.Tensor) -> None:
         if self.bias is None:
             torch.matmul(x, self.weight.t(), out=out)
         else:
             torch.addmm(self.bias, x, self.weight.t(), out=out)
 
-    def forward_gated(self, ctx, x: torch.Tensor, out_name: str):
+    def forward_gated(self, ctx, x: torch.Tensor, out_name: str, **activation):
         """For a weight whose rows alternate, in strips of `lib.GATE_STRIP`, between gate rows
-        and their up rows: silu(gate) * up as [N, out/2] of the storage type straight from
+        and their up rows: silu(gate) * up (or another `activation` with its limit and alpha) as
+        [N, out/2] of the storage type straight from
         the few-rows kernel, or None where that kernel does not apply (float32, many rows, a
         bias, a large matrix whose K the planner would slice); the caller then takes
         `forward` and the activation kernel."""
@@ -127,7 +141,7 @@ class Linear:
         act = ctx.buffer(out_name, (rows, self.out_features // 2), torch.bfloat16)
         packed = self.packed is not None
         lib.gemm_bf16_skinny_gated(x, self.packed if packed else self.weight, self.out_features,
-                                   act, packed)
+                                   act, packed, **activation)
         return act
 
     def forward_f32(self, ctx, x: torch.Tensor, out_name: str) -> torch.Tensor:

@@ -79,23 +79,37 @@ class GatedMLP:
         self.down = Linear(params["down_proj.weight"], dtype, device,
                            bias=params.get("down_proj.bias"))
 
+    def _activated(self, ctx, x):
+        """The gated activations [N, intermediate] in the buffer "mlp.act"."""
+        how = dict(activation=self.spec.activation, limit=getattr(self.spec, "limit", 0.0),
+                   alpha=getattr(self.spec, "alpha", 1.0))
+        act = self.gate_up.forward_gated(ctx, x, "mlp.act", **how) if self.strip else None
+        if act is None:
+            # (the activation kernel adds the bias itself where the product left it to it)
+            gate_up, bias = self.gate_up.forward(ctx, x, "mlp.gate_up", bias_later=True)
+            act = ctx.buffer("mlp.act", (x.shape[0], self.spec.intermediate_size))
+            lib.swiglu(gate_up, act, self.strip, bias=bias, **how)
+            ctx.release(gate_up)
+        return act
+
+    def slices_behind(self, ctx, x, out_name, leading):
+        """The feed-forward's rows as float32 slices behind `leading` slices that the caller fills
+        (see `Linear.slices_behind`), or None where the few-rows product does not apply."""
+        if self.down.bias is not None or self.down.dtype != torch.bfloat16 \
+                or not lib.skinny_gemm_ok(x.shape[0], self.down.in_features):
+            return None
+        act = self._activated(ctx, x)
+        out = self.down.slices_behind(ctx, act, out_name, leading)
+        ctx.release(act)
+        return out
+
     bias_later = True      # forward(..., bias_later=True) hands the last product's bias on
 
     def forward(self, ctx, x, bias_later=False):
         """The feed-forward's rows; with `bias_later`, (rows, float32 bias of the down
         projection that is still to be added, or None): a caller whose next kernel reads the
         rows anyway adds it there and saves a launch."""
-        n = x.shape[0]
-        # (the few-rows product that applies the gate itself knows silu only)
-        act = (self.gate_up.forward_gated(ctx, x, "mlp.act")
-               if self.strip and self.spec.activation == "silu" else None)
-        if act is None:
-            # (the activation kernel adds the bias itself where the product left it to it)
-            gate_up, bias = self.gate_up.forward(ctx, x, "mlp.gate_up", bias_later=True)
-            act = ctx.buffer("mlp.act", (n, self.spec.intermediate_size))
-            lib.swiglu(gate_up, act, self.strip, self.spec.activation, bias=bias,
-                       limit=getattr(self.spec, "limit", 0.0), alpha=getattr(self.spec, "alpha", 1.0))
-            ctx.release(gate_up)
+        act = self._activated(ctx, x)
         out = self.down.forward(ctx, act, "mlp.down", bias_later=bias_later)
         ctx.release(act)
         return out

@@ -21,6 +21,7 @@ The experts' matrices are stacked when the part is built (gate and up [E, F, H],
 [E, H, F]); routing stays on the device, so a step with this part is captured like any
 other.  In bfloat16 with widths that are multiples of 64 the experts run as grouped matrix
 products on the matrix cores (the pairs of (row, choice) laid out by expert on the device);
+for few rows every expert's blocks find their pairs themselves and leave a slice a choice;
 otherwise, and in float32, a kernel takes one pair at a time.  Kernels: `csrc/moe.hip`.
 """
 from __future__ import annotations
@@ -120,10 +121,16 @@ class RoutedMLP:
                                     if name.startswith("shared.")}, dtype, device)
         self.grouped = lib.moe_grouped_supported(dtype, hidden, spec.intermediate_size,
                                                  spec.n_experts)
+        # (identity experts have no product whose rows could be a slice)
+        self.few = self.grouped and not getattr(spec, "identity", 0)
 
     def forward(self, ctx, x):
         spec = self.spec
         n = x.shape[0]
+        if self.few and n <= lib.MOE_FEW_ROWS:
+            slices = self._few_rows(ctx, x)
+            if slices is not None:
+                return slices
         shared = None if self.shared is None else self.shared.forward(ctx, x)
         expert = ctx.buffer("moe.expert", (n, spec.top), torch.int32)
         weight = ctx.buffer("moe.weight", (n, spec.top), torch.float32)
@@ -143,3 +150,24 @@ class RoutedMLP:
                             extra=shared, **self.act)
         ctx.release(shared, expert, weight, act)
         return out
+
+    def _few_rows(self, ctx, x):
+        """The rows of a step of few rows as float32 slices, one a choice, followed by those of the
+        shared expert's last product: whoever reads the rows adds them up (None where the shared
+        expert's product does not come in slices)."""
+        spec = self.spec
+        n = x.shape[0]
+        if self.shared is None:
+            slices = ctx.buffer("moe.slices.f32", (spec.top, n, self.hidden), torch.float32)
+        else:
+            slices = self.shared.slices_behind(ctx, x, "moe.slices", spec.top)
+            if slices is None:
+                return None
+        expert = ctx.buffer("moe.expert", (n, spec.top), torch.int32)
+        weight = ctx.buffer("moe.weight", (n, spec.top), torch.float32)
+        lib.moe_route(x, self.router, ctx.meta.row_seq, expert, weight, **self.routing)
+        act = ctx.buffer("moe.act", (n * spec.top, spec.intermediate_size))
+        lib.moe_experts_few(x, self.w_gate, self.w_up, self.w_down, expert, weight, ctx.meta.row_seq,
+                            act, slices[:spec.top], **self.act)
+        ctx.release(expert, weight, act)
+        return slices

@@ -191,11 +191,15 @@ def test_a_groups_score_is_the_sum_of_its_two_largest():
     (6, 3, 2, 2, 40, 56, 48, 9, "float32"), (5, 1, 1, 3, 13, 11, 50, 7, "float32"),
     (4, 2, 1, 2, 24, None, 48, 20, "float32"), (8, 4, 2, 2, 64, 96, 64, 1, "bfloat16"),
     (8, 4, 2, 2, 64, 96, 64, 50, "bfloat16"), (8, 4, 3, 3, 128, 64, 128, 300, "bfloat16"),
-    (4, 1, 1, 2, 256, 256, 256, 2, "bfloat16"), (5, 1, 1, 3, 24, 40, 48, 30, "bfloat16")])
+    (4, 1, 1, 2, 256, 256, 256, 2, "bfloat16"), (20, 4, 2, 4, 64, None, 192, 40, "bfloat16"),
+    (6, 2, 1, 2, 192, 40, 64, 16, "bfloat16"), (6, 2, 2, 3, 128, 33, 64, 30, "bfloat16"),
+    (70, 7, 3, 5, 64, 64, 128, 64, "bfloat16"), (33, 3, 2, 2, 64, None, 64, 200, "bfloat16"),
+    (3, 1, 1, 2, 192, 64, 64, 700, "bfloat16"), (5, 5, 4, 3, 64, None, 320, 1000, "bfloat16"),
+    (5, 1, 1, 3, 24, 40, 48, 30, "bfloat16")])
 def test_clamped_experts_beside_a_shared_one(experts, groups, keep, top, inter, shared, width, rows, dtype):
-    """The routed feed-forward part through the pair-at-a-time kernels and the grouped matrix-core
-    ones (small and large tiles, the long K-tile), the shared expert's rows as slices and as one
-    tensor; limits that clamp many activations on both sides."""
+    """The routed feed-forward part through the pair-at-a-time kernels, the matrix-core ones of few
+    rows (which leave a slice a choice) and the grouped ones (small and large tiles), the shared
+    expert's rows as slices and as one tensor; limits that clamp many activations on both sides."""
     from edge_infer_amd.config.specs import GatedMLPSpec, RoutedMLPSpec
     from edge_infer_amd.parts import RoutedMLP
     g = torch.Generator().manual_seed(inter + rows)
@@ -237,6 +241,9 @@ def test_clamped_experts_beside_a_shared_one(experts, groups, keep, top, inter, 
         def release(*buffers):
             pass
     got = part.forward(Context, x.to(DEV).to(part.w_gate.dtype))
+    if got.dim() == 3:              # (few rows: a slice a choice, then the shared product's)
+        assert part.grouped and rows <= 64
+        got = got.sum(0)
     assert clear.sum() >= 0.9 * rows
     got, want = got[clear.to(DEV)], want[clear]
     if dtype == "float32":
@@ -544,3 +551,35 @@ def test_a_vector_is_added_once_before_each_pass(start, stop, times):
             assert_close_f32(got, want, "stream after the passes")
         else:
             assert_close_bf16(got, want, "stream after the passes")
+
+
+def test_experts_of_few_rows_leave_padding_rows_out():
+    """A step padded to a fixed batch: padding rows (in between and at the end) take no expert and
+    do not disturb the others; a weight of exactly 0 still writes its slice."""
+    from edge_infer_amd.csrc import lib
+    g = torch.Generator().manual_seed(2)
+    rows, top, experts, inter, width = 24, 2, 4, 64, 128
+    x = exact((rows, width), g)
+    w = [exact((experts, inter, width), g, width ** -0.5), exact((experts, inter, width), g, width ** -0.5),
+         exact((experts, width, inter), g, inter ** -0.5)]
+    expert = torch.stack([torch.randperm(experts, generator=g)[:top] for _ in range(rows)]).to(torch.int32)
+    weight = torch.rand(rows, top, generator=g)
+    weight[5, 1] = 0.0
+    row_seq = torch.arange(rows, dtype=torch.int32)
+    dead = [3, 22, 23]
+    row_seq[dead] = -1
+    expert[dead], weight[dead] = 0, 0.0
+    act = torch.empty(rows * top, inter, device=DEV, dtype=torch.bfloat16)
+    out = torch.full((top, rows, width), 5.0, device=DEV)
+    dev = [m.to(DEV).to(torch.bfloat16) for m in w]
+    lib.moe_experts_few(x.to(DEV).to(torch.bfloat16), *dev, expert.to(DEV), weight.to(DEV),
+                        row_seq.to(DEV), act, out, activation="clamped_swish", limit=0.9, alpha=1.702)
+    for r in range(rows):
+        if r in dead:
+            assert bool((out[:, r] == 5.0).all())
+            continue
+        for k in range(top):
+            e = int(expert[r, k])
+            t = {"gate": w[0][e], "up": w[1][e], "down": w[2][e]}
+            want = weight[r, k].double() * plain.clamped_expert(x[r:r + 1], t, "", 0.9)[0]
+            assert torch.allclose(out[k, r].double().cpu(), want, atol=2e-2)
