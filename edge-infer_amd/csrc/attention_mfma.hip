@@ -25,19 +25,22 @@ namespace {
 constexpr int kTile = 16;          // keys per MFMA tile
 constexpr float kLowest = -1.0e30f;
 
-// Options beyond causal, windowed attention (the EXT instantiations of the kernels; the plain
-// ones are compiled without any of this): `chunk` > 0: a query at p sees key t only if
+// Options beyond causal, windowed attention, in two families that kernels are compiled with or
+// without (EXT: a sum of kExtOptions and kExtKept; 0: none of this; an option that is compiled
+// in costs scalar registers whether it is used or not).  kExtOptions: `chunk` > 0: a query at p sees key t only if
 // t / chunk == p / chunk; `slopes` (per query head, or null): slope * (p - t) is taken off the
 // scaled score; `sinks` (per query head, or null): exp(sink) joins the softmax's denominator.
 // `pool_o`, `pool_ml` (or null): what another kernel has gathered for every (row, head) from keys
 // of another source (the pooled blocks before a window): float32 sums of weighted values
 // [rows, nq, D] and (maximum, sum of weights) [rows, nq, 2] in natural units; they join the
 // row's softmax as one more slice.  `gate` (float32 [rows, nq], or null): the output of a row
-// and head is multiplied by sigmoid(gate).  `keep` > 0 (with a window): the keys of the sequence's
+// and head is multiplied by sigmoid(gate).  kExtKept: `keep` > 0 (with a window): the keys of the sequence's
 // first `keep` positions stay visible however far back they lie; walks take what lies before the
 // window of them first.  `wide` (or null): one gate for every element of the output, the sums of
 // `wide_slices` slices of float32 or bfloat16 rows: element (row, head, d) is multiplied by
 // sigmoid of what lies at row * wide_row + head * D + d.
+constexpr int kExtOptions = 1, kExtKept = 2;
+
 struct AttnExtra {
   int chunk;
   const float* slopes;
@@ -99,7 +102,7 @@ struct DecodePrep {
 // PREP: q is not read; the block forms its queries and the position's key and value itself
 // (the block of slice 0 and head block 0 stores them; the wave that meets the position in
 // its tile takes them from LDS, since the store of another block may not have landed).
-template <int D, int GB, int W, bool PREP, bool EXT>
+template <int D, int GB, int W, bool PREP, int EXT>
 __global__ void __launch_bounds__(W * EI_WAVE)
 attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pages,
                    const bf16_t* __restrict__ v_pages, const int32_t* __restrict__ row_pos,
@@ -116,6 +119,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   __shared__ float alpha_lds[W][16];
   __shared__ float m_lds[W][16], l_lds[W][16];
   __shared__ float o_lds[W][GB][D];
+  constexpr bool OPT = (EXT & kExtOptions) != 0, KEPT = (EXT & kExtKept) != 0;
 
   const int row = blockIdx.x;                      // packed row = sequence index in decode
   const int g = blockIdx.y / head_blocks, hb = blockIdx.y % head_blocks;
@@ -229,7 +233,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   }
 
   int lo_key_of = window > 0 ? max(0, pos - window + 1) : 0;
-  if constexpr (EXT)
+  if constexpr (OPT)
     if (extra.chunk > 0) lo_key_of = max(lo_key_of, pos / extra.chunk * extra.chunk);
   const int lo_key = lo_key_of;
   const int first_tile = lo_key / kTile, last_tile = pos / kTile;
@@ -243,7 +247,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   // the later slices of a short sequence are empty.  Without it (or with a window, where the
   // ranges start at different pages) every sequence is cut into n_splits equal parts.
   int per = (pages + n_splits - 1) / n_splits;
-  if (longest != nullptr && window <= 0 && !(EXT && extra.chunk > 0)) {
+  if (longest != nullptr && window <= 0 && !(OPT && extra.chunk > 0)) {
     const int most_pages = (*longest + EI_PAGE - 1) / EI_PAGE;
     per = max(1, (most_pages + n_splits - 1) / n_splits);
   }
@@ -252,12 +256,12 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   const int tile_end = split == n_splits - 1
                            ? last_tile + 1
                            : min(last_tile + 1, (lo_page + (split + 1) * per) * (EI_PAGE / kTile));
-  // (EXT) tiles of kept first positions before the window's: the walk is then over kept tiles and
+  // (KEPT) tiles of kept first positions before the window's: the walk is then over kept tiles and
   // the window's tiles in a row, step v < kept being tile v and the others tile v + skipped, and
   // slices are equal parts of it
   int kept = 0, skipped = 0, step_begin = tile_begin, step_end = tile_end;
-  const int keep = EXT ? extra.keep : 0;
-  if constexpr (EXT) {
+  const int keep = KEPT ? extra.keep : 0;
+  if constexpr (KEPT) {
     kept = min(first_tile, (keep + kTile - 1) / kTile);
     if (kept > 0) {
       skipped = first_tile - kept;
@@ -269,16 +273,16 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
   }
   (void)total_tiles;
 
-  // (EXT) the gate of the first element that this thread will write, asked for ahead of the walk
-  const size_t wide_base = EXT ? static_cast<size_t>(row) * extra.wide_row +
+  // (KEPT) the gate of the first element that this thread will write, asked for ahead of the walk
+  const size_t wide_base = KEPT ? static_cast<size_t>(row) * extra.wide_row +
                                      static_cast<size_t>(head0) * D : 0;
   float first_gate = 0.f;
-  if constexpr (EXT)
+  if constexpr (KEPT)
     if (extra.wide && n_splits == 1 && t < heads_here * D) first_gate = wide_sum(extra, wide_base + t);
 
   float m_run = kLowest, l_run = 0.f;              // state of head r16 (same in all four c)
   float slope = 0.f;                               // of head r16
-  if constexpr (EXT)
+  if constexpr (OPT)
     if (extra.slopes && r16 < heads_here) slope = extra.slopes[head0 + r16];
   float acc[GB][8];
 #pragma unroll
@@ -336,8 +340,8 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int key = key0 + 4 * c + r;
-      const bool visible = key <= pos && (key >= lo_key || (EXT && key < keep));
-      if constexpr (EXT)
+      const bool visible = key <= pos && (key >= lo_key || (KEPT && key < keep));
+      if constexpr (OPT)
         sc[r] = visible ? fmaf(-slope, static_cast<float>(pos - key), s[r] * scale) : -INFINITY;
       else
         sc[r] = visible ? s[r] * scale : -INFINITY;
@@ -429,7 +433,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
       o += o_lds[w][h][d] * f;
     }
     const int head = head0 + h;
-    if constexpr (EXT) {
+    if constexpr (OPT) {
       if (extra.sinks && split == 0) {     // one more term of the denominator, once a row
         const float sink = extra.sinks[head];
         const float m_all = fmaxf(m, sink), f = expf(m - m_all);
@@ -440,7 +444,7 @@ attn_decode_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pa
     }
     if (n_splits == 1) {
       float value = l > 0.f ? o / l : 0.f;
-      if constexpr (EXT)
+      if constexpr (KEPT)
         if (extra.wide)
           value *= opened(idx == t ? first_gate : wide_sum(extra, wide_base + idx));
       out[(static_cast<size_t>(row) * nq + head) * D + d] = ei::from_f32<bf16_t>(value);
@@ -524,7 +528,7 @@ constexpr int kPageBuffers = 3;
 // a lane and a trip through LDS) was a quarter of a page's vector work.
 constexpr float kLazyRise = 8.f;
 
-template <int D, int HB, int KW, bool EXT>
+template <int D, int HB, int KW, int EXT>
 __global__ void __launch_bounds__(kPrefillThreads, 2)
 attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_pages,
                          const bf16_t* __restrict__ v_pages, const int32_t* __restrict__ item_seq,
@@ -553,8 +557,9 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
   // running maximum and sum per row here, its output tile in the page buffers
   __shared__ float handed_lds[KW == 2 ? kPrefillWaves / 2 : 1][2][kWideRows];
   __shared__ __attribute__((aligned(16))) float other_lds[KW == 2 ? kPrefillWaves : 1][kWideRows];
-  // (EXT) what the other source's sums of a row are scaled by
-  __shared__ __attribute__((aligned(16))) float pool_lds[EXT ? kPrefillWaves : 1][kWideRows];
+  // (OPT) what the other source's sums of a row are scaled by
+  constexpr bool OPT = (EXT & kExtOptions) != 0, KEPT = (EXT & kExtKept) != 0;
+  __shared__ __attribute__((aligned(16))) float pool_lds[OPT ? kPrefillWaves : 1][kWideRows];
   static_assert(KW == 1 || (kPrefillWaves / 2) * (D / 32) * 16 * EI_WAVE * sizeof(float) <=
                                sizeof(bf16_t) * kPageBuffers * 2 * PBUF,
                 "the handed-over output tiles fit the page buffers");
@@ -648,12 +653,12 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
 
   const int first_pos = row_pos[row0], last_pos = row_pos[row0 + npos - 1];
   int lo_key_of = window > 0 ? max(0, first_pos - window + 1) : 0;
-  const int chunk = EXT ? extra.chunk : 0;
-  // (EXT) the first key of this lane's row's own chunk, and the slope of the wave's head in
+  const int chunk = OPT ? extra.chunk : 0;
+  // (OPT) the first key of this lane's row's own chunk, and the slope of the wave's head in
   // units of the raw score (the scale is positive)
   int chunk_lo = 0;
   float slope_raw = 0.f;
-  if constexpr (EXT) {
+  if constexpr (OPT) {
     if (chunk > 0) {
       lo_key_of = max(lo_key_of, first_pos / chunk * chunk);
       chunk_lo = pos_q >= 0 ? pos_q / chunk * chunk : 0;
@@ -662,13 +667,13 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
   }
   const int lo_key = lo_key_of;
   const int lo_page = lo_key / EI_PAGE, hi_page = last_pos / EI_PAGE;
-  // (EXT) pages of kept first positions before the window's come first: the walk is over visits
+  // (KEPT) pages of kept first positions before the window's come first: the walk is over visits
   // first_visit .. hi_page, visit v >= lo_page being page v and the visits before it pages 0, 1, ...
-  const int keep = EXT ? extra.keep : 0;
-  const int kept_pages = EXT ? min(lo_page, (keep + EI_PAGE - 1) / EI_PAGE) : 0;
+  const int keep = KEPT ? extra.keep : 0;
+  const int kept_pages = KEPT ? min(lo_page, (keep + EI_PAGE - 1) / EI_PAGE) : 0;
   const int first_visit = lo_page - kept_pages;
   auto page_of = [&](int visit) __attribute__((always_inline)) {
-    return (EXT && visit < lo_page) ? visit - first_visit : visit;
+    return (KEPT && visit < lo_page) ? visit - first_visit : visit;
   };
   const bool wave_rows_valid = pw * kWideRows + kWideRows <= npos;
   const int wave_min_pos = wave_rows_valid ? row_pos[row0 + pw * kWideRows] : -1;
@@ -762,7 +767,7 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
       __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
       __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
     }
-    if constexpr (EXT) {
+    if constexpr (OPT) {
       if (slope_raw != 0.f) {
 #pragma unroll
         for (int kb = 0; kb < KBL; ++kb)
@@ -786,8 +791,8 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int key = key_base + (kw * KBL + kb) * 32 + 8 * i + 4 * half + r;
-            bool visible = key <= pos_q && (window <= 0 || key > pos_q - window || (EXT && key < keep));
-            if constexpr (EXT) visible = visible && key >= chunk_lo;
+            bool visible = key <= pos_q && (window <= 0 || key > pos_q - window || (KEPT && key < keep));
+            if constexpr (OPT) visible = visible && key >= chunk_lo;
             if (!visible) s[kb][4 * i + r] = -INFINITY;     // (pos_q = -1: a row that is not there)
           }
     }
@@ -872,8 +877,8 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
     const int key_lo = page * EI_PAGE + kw * KBL * 32, key_hi = key_lo + KBL * 32 - 1;
     bool seen = wave_has_rows && key_lo <= wave_last_pos &&
                 (window <= 0 || !wave_rows_valid || key_hi > wave_min_pos - window ||
-                 (EXT && key_lo < keep));
-    if constexpr (EXT)     // wholly before the chunk of the wave's first row: no row sees it
+                 (KEPT && key_lo < keep));
+    if constexpr (OPT)     // wholly before the chunk of the wave's first row: no row sees it
       if (chunk > 0 && wave_rows_valid) seen = seen && key_hi >= wave_min_pos / chunk * chunk;
     return seen;
   };
@@ -881,8 +886,8 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
     const int key_base = page * EI_PAGE;
     const int key_lo = key_base + kw * KBL * 32, key_hi = key_lo + KBL * 32 - 1;
     bool no_mask = wave_rows_valid && key_hi <= wave_min_pos &&
-                   (window <= 0 || key_lo > wave_max_pos - window || (EXT && key_hi < keep));
-    if constexpr (EXT)     // every key lies in the chunk of the wave's last row, so of all rows
+                   (window <= 0 || key_lo > wave_max_pos - window || (KEPT && key_hi < keep));
+    if constexpr (OPT)     // every key lies in the chunk of the wave's last row, so of all rows
       if (chunk > 0) no_mask = no_mask && key_lo >= wave_max_pos / chunk * chunk;
     scores(key_base, buf, !no_mask);
   };
@@ -916,8 +921,8 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
                                                          __float_as_uint(l_run), false, false);
     l_wave = __uint_as_float(both.x) + __uint_as_float(both.y);
   }
-  float sink_fold = 1.f;       // (EXT) what taking the sink in rescales this wave's output by
-  if constexpr (EXT) {
+  float sink_fold = 1.f;       // (OPT) what taking the sink in rescales this wave's output by
+  if constexpr (OPT) {
     if (extra.sinks && kw == 0) {          // one more term of the denominator, once a row
       const float sink_l2 = extra.sinks[head] * 1.4426950408889634f;
       const float m_new = fmaxf(m_run, sink_l2);
@@ -926,8 +931,8 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
       m_run = m_new;
     }
   }
-  float pool_scale = 0.f;      // (EXT) what the other source's sums are scaled by, before 1 / l
-  if constexpr (EXT) {
+  float pool_scale = 0.f;      // (OPT) what the other source's sums are scaled by, before 1 / l
+  if constexpr (OPT) {
     if (extra.pool_ml && kw == 0 && pw * kWideRows + n32 < npos) {
       // the other source's slice of this lane's row: one more (maximum, sum) to take in
       const size_t slot = static_cast<size_t>(row0 + pw * kWideRows + n32) * nq + head;
@@ -976,7 +981,7 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
       pool_factor = pool_scale * f_own * inv;
     }
   }
-  if constexpr (EXT) {
+  if constexpr (OPT) {
     if (extra.gate && kw == 0 && pw * kWideRows + n32 < npos) {
       const float gate = extra.gate[static_cast<size_t>(row0 + pw * kWideRows + n32) * nq + head];
       const float open = 1.0f / (1.0f + expf(-gate));
@@ -988,7 +993,7 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
   if (half == 0) {
     factor_lds[wave][n32] = own_factor;
     if constexpr (KW == 2) other_lds[wave][n32] = other_factor;
-    if constexpr (EXT) pool_lds[wave][n32] = pool_factor;
+    if constexpr (OPT) pool_lds[wave][n32] = pool_factor;
   }
   __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
   __builtin_amdgcn_wave_barrier();
@@ -1004,22 +1009,44 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
         add[0] = add4.x; add[1] = add4.y; add[2] = add4.z; add[3] = add4.w;
       }
       float pooled[4] = {0.f, 0.f, 0.f, 0.f};
-      if constexpr (EXT) {
+      if constexpr (OPT) {
         const float4 p4 = *reinterpret_cast<const float4*>(&pool_lds[wave][8 * i + 4 * half]);
         pooled[0] = p4.x; pooled[1] = p4.y; pooled[2] = p4.z; pooled[3] = p4.w;
       }
-      // (EXT) the gates of the lane's elements of these four rows: their loads travel together
-      float open[EXT ? 4 : 1][EXT ? DB : 1];
-      if constexpr (EXT) {
+      // (KEPT) what goes into the gates of the lane's elements of these four rows: their loads
+      // travel together
+      float open[KEPT ? 4 : 1][KEPT ? DB : 1];
+      if constexpr (KEPT) {
         if (extra.wide) {
+          size_t at[4];
 #pragma unroll
           for (int r = 0; r < 4; ++r)
+            at[r] = static_cast<size_t>(row0 + min(pw * kWideRows + 8 * i + 4 * half + r, npos - 1)) *
+                        extra.wide_row + static_cast<size_t>(head) * D + n32;
+          if (extra.wide_dtype == EI_BF16) {
+            bf16_t raw[4][DB];
 #pragma unroll
-            for (int db = 0; db < DB; ++db) {
-              const int orow = min(pw * kWideRows + 8 * i + 4 * half + r, npos - 1);
-              open[r][db] = wide_sum(extra, static_cast<size_t>(row0 + orow) * extra.wide_row +
-                                                static_cast<size_t>(head) * D + db * 32 + n32);
+            for (int r = 0; r < 4; ++r)
+#pragma unroll
+              for (int db = 0; db < DB; ++db)
+                raw[r][db] = static_cast<const bf16_t*>(extra.wide)[at[r] + db * 32];
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+#pragma unroll
+              for (int db = 0; db < DB; ++db) open[r][db] = ei::bf16_to_f32(raw[r][db]);
+          } else {
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+#pragma unroll
+              for (int db = 0; db < DB; ++db) open[r][db] = 0.f;
+            const float* slice = static_cast<const float*>(extra.wide);
+            for (int s = 0; s < extra.wide_slices; ++s, slice += extra.wide_slice) {
+#pragma unroll
+              for (int r = 0; r < 4; ++r)
+#pragma unroll
+                for (int db = 0; db < DB; ++db) open[r][db] += slice[at[r] + db * 32];
             }
+          }
         }
       }
 #pragma unroll
@@ -1035,10 +1062,12 @@ attn_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ k_p
             o = fmaf(tile_lds[(((wave % (HB * NG)) * DB + db) * 16 + 4 * i + r) * EI_WAVE + lane],
                      add[r], o);
           }
-          if constexpr (EXT) {
+          if constexpr (OPT) {
             if (extra.pool_o && pooled[r] != 0.f)
               o = fmaf(extra.pool_o[(static_cast<size_t>(row0 + orow) * nq + head) * D + db * 32 + n32],
                        pooled[r], o);
+          }
+          if constexpr (KEPT) {
             if (extra.wide) o *= opened(open[r][db]);
           }
           dst[db * 32 + n32] = ei::from_f32<bf16_t>(o);
@@ -1124,7 +1153,15 @@ __global__ void attn_merge_kernel(const float* __restrict__ part_o,
   }
 }
 
-template <int D, int GB, bool PREP, bool EXT>
+// The families of options that `extra` uses.
+int families(const AttnExtra* extra) {
+  if (!extra) return 0;
+  return (extra->chunk > 0 || extra->slopes || extra->sinks || extra->pool_ml || extra->gate
+              ? kExtOptions : 0) |
+         (extra->keep > 0 || extra->wide ? kExtKept : 0);
+}
+
+template <int D, int GB, bool PREP, int EXT>
 void launch_decode(dim3 grid, hipStream_t stream, const bf16_t* q, const bf16_t* k,
                    const bf16_t* v, const int32_t* row_pos, const int32_t* row_seq,
                    const int32_t* page_table, int table_width, bf16_t* out, float* part_o,
@@ -1162,7 +1199,7 @@ extern "C" int ei_attn_prefill_mfma_positions(int G) {
   return kWideRows * (kPrefillWaves / HB);
 }
 
-template <int D, int HB, int KW, bool EXT>
+template <int D, int HB, int KW, int EXT>
 static void launch_prefill(int blocks, hipStream_t stream, const bf16_t* q, const bf16_t* k,
                                 const bf16_t* v, const int32_t* item_seq,
                                 const int32_t* item_row0, const int32_t* item_npos, int n_items,
@@ -1217,16 +1254,18 @@ static int prefill_launch(const void* q, const void* k_pages, const void* v_page
   const bf16_t* vv = static_cast<const bf16_t*>(v_pages);
   bf16_t* oo = static_cast<bf16_t*>(out);
   const AttnExtra none{};
+  const AttnExtra& given = extra ? *extra : none;
+  const int forms = families(extra);
+#define EI_PREFILL_FORM(DD, HH, KK, FORM)                                                     \
+  launch_prefill<DD, HH, KK, FORM>(static_cast<int>(blocks), stream, qq, kk, vv, item_seq,    \
+                                   item_row0, item_npos, n_items, row_pos, page_table,        \
+                                   table_width, oo, nq, nkv, window, scale, pair, given)
 #define EI_PREFILL_KW(DD, HH, KK)                                                             \
   do {                                                                                        \
-    if (extra)                                                                                \
-      launch_prefill<DD, HH, KK, true>(static_cast<int>(blocks), stream, qq, kk, vv, item_seq, \
-                                       item_row0, item_npos, n_items, row_pos, page_table,    \
-                                       table_width, oo, nq, nkv, window, scale, pair, *extra); \
-    else                                                                                      \
-      launch_prefill<DD, HH, KK, false>(static_cast<int>(blocks), stream, qq, kk, vv, item_seq, \
-                                        item_row0, item_npos, n_items, row_pos, page_table,   \
-                                        table_width, oo, nq, nkv, window, scale, pair, none); \
+    if (forms == 0) EI_PREFILL_FORM(DD, HH, KK, 0);                                           \
+    else if (forms == kExtOptions) EI_PREFILL_FORM(DD, HH, KK, kExtOptions);                  \
+    else if (forms == kExtKept) EI_PREFILL_FORM(DD, HH, KK, kExtKept);                        \
+    else EI_PREFILL_FORM(DD, HH, KK, kExtOptions | kExtKept);                                 \
   } while (0)
 #define EI_PREFILL(DD, HH)                                                                    \
   do {                                                                                        \
@@ -1240,6 +1279,7 @@ static int prefill_launch(const void* q, const void* k_pages, const void* v_page
   }
 #undef EI_PREFILL
 #undef EI_PREFILL_KW
+#undef EI_PREFILL_FORM
   EI_LAUNCH_CHECK();
 }
 
@@ -1339,23 +1379,19 @@ static int decode_launch(const void* q, const void* k_pages, const void* v_pages
   bf16_t* oo = static_cast<bf16_t*>(out);
   const DecodePrep none{};
   const AttnExtra plain{};
+  const AttnExtra& given = extra ? *extra : plain;
+  const int forms = families(extra);
+#define EI_DECODE_FORM(DD, GG, PREP, FORM, PP)                                                \
+  launch_decode<DD, GG, PREP, FORM>(grid, stream, qq, kk, vv, row_pos, row_seq, page_table,   \
+                                    table_width, oo, part_o, part_ml, nq, nkv, head_blocks,   \
+                                    window, scale, n_splits, waves, longest, PP, given)
 #define EI_DECODE(DD, GG)                                                                     \
   do {                                                                                        \
-    if (prep)                                                                                 \
-      launch_decode<DD, GG, true, false>(grid, stream, qq, kk, vv, row_pos, row_seq,          \
-                                         page_table, table_width, oo, part_o, part_ml, nq,    \
-                                         nkv, head_blocks, window, scale, n_splits, waves,    \
-                                         longest, *prep, plain);                              \
-    else if (extra)                                                                           \
-      launch_decode<DD, GG, false, true>(grid, stream, qq, kk, vv, row_pos, row_seq,          \
-                                         page_table, table_width, oo, part_o, part_ml, nq,    \
-                                         nkv, head_blocks, window, scale, n_splits, waves,    \
-                                         longest, none, *extra);                              \
-    else                                                                                      \
-      launch_decode<DD, GG, false, false>(grid, stream, qq, kk, vv, row_pos, row_seq,         \
-                                          page_table, table_width, oo, part_o, part_ml, nq,   \
-                                          nkv, head_blocks, window, scale, n_splits, waves,   \
-                                          longest, none, plain);                              \
+    if (prep) EI_DECODE_FORM(DD, GG, true, 0, *prep);                                         \
+    else if (forms == 0) EI_DECODE_FORM(DD, GG, false, 0, none);                              \
+    else if (forms == kExtOptions) EI_DECODE_FORM(DD, GG, false, kExtOptions, none);          \
+    else if (forms == kExtKept) EI_DECODE_FORM(DD, GG, false, kExtKept, none);                \
+    else EI_DECODE_FORM(DD, GG, false, kExtOptions | kExtKept, none);                         \
   } while (0)
 #define EI_DECODE_G(DD)            \
   switch (GB) {                    \
@@ -1372,6 +1408,7 @@ static int decode_launch(const void* q, const void* k_pages, const void* v_pages
   }
 #undef EI_DECODE_G
 #undef EI_DECODE
+#undef EI_DECODE_FORM
   hipError_t e = hipGetLastError();
   if (e != hipSuccess) {
     ei_set_error(hipGetErrorString(e));

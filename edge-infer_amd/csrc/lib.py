@@ -106,7 +106,7 @@ _SIGNATURES = {
         "ei_moe_grouped_supported": [c_int, c_int, c_int, c_int],
         "ei_moe_few_rows": [],
         "ei_moe_experts_few": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                               c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                               c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                c_float, c_float, c_void_p],
         "ei_moe_experts_grouped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                    c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
@@ -1804,20 +1804,42 @@ def moe_grouped_supported(dtype, width: int, inter: int, n_experts: int) -> bool
 MOE_FEW_ROWS = 64
 
 
+def pack_experts(w: torch.Tensor) -> torch.Tensor:
+    """Stacked matrices [E, n, k] (n a multiple of 16, k of 32) in the operand order of the
+    matrix-core forms of the experts, [E, n / 16, k / 32, 4, 16, 8]: tiles of 16 rows x 32 k, the
+    piece of row r and k = 8 c .. 8 c + 7 of a tile at [c, r]."""
+    experts, n, k = w.shape
+    if n % 16 or k % 32:
+        raise KernelError("pack_experts: rows must be a multiple of 16 and columns of 32")
+    tiles = w.view(experts, n // 16, 16, k // 32, 4, 8)
+    return tiles.permute(0, 1, 3, 4, 2, 5).contiguous()
+
+
+def _packed_shapes(w_gate, w_up, w_down, what):
+    """(experts, inter, width) of packed expert matrices."""
+    if w_gate.dim() != 6 or w_down.dim() != 6:
+        raise KernelError(f"{what}: the matrices come packed (`pack_experts`)")
+    n_experts, inter, width = w_gate.shape[0], 16 * w_gate.shape[1], 32 * w_gate.shape[2]
+    if tuple(w_gate.shape) != (n_experts, inter // 16, width // 32, 4, 16, 8) \
+            or tuple(w_up.shape) != tuple(w_gate.shape) \
+            or tuple(w_down.shape) != (n_experts, width // 16, inter // 32, 4, 16, 8):
+        raise KernelError(f"{what}: the packed matrices have the wrong shapes")
+    return n_experts, inter, width
+
+
 def moe_experts_few(x, w_gate, w_up, w_down, expert, weight, row_seq, act, out, activation="silu",
-                    limit=0.0, alpha=1.0) -> None:
-    """The experts of at most `MOE_FEW_ROWS` rows on the matrix cores (bfloat16, the sizes of
-    `moe_experts_grouped`), without a layout by expert first: out [top, n, w] float32, whose
+                    limit=0.0, alpha=1.0, identity=0) -> None:
+    """The experts of at most `MOE_FEW_ROWS` rows on the matrix cores (bfloat16, the sizes and
+    packed matrices of `moe_experts_grouped`), without a layout by expert first: out [top, n, w] float32, whose
     slice k receives weight[r, k] times the product row of row r's k-th choice; the slices' sum
-    is what `moe_experts` gives.  Rows with row_seq < 0 are not written.  Every choice is an
-    expert (no identity ones).  `act` [n * top, f] bfloat16 is scratch."""
+    is what `moe_experts` gives.  Rows with row_seq < 0 are not written.  `identity`: how many
+    outputs the router has beyond the experts.  `act` [n * top, f] bfloat16 is scratch."""
     lib = library("moe")
     n, width = x.shape
-    n_experts, inter = w_gate.shape[0], w_gate.shape[1]
+    n_experts, inter, packed_width = _packed_shapes(w_gate, w_up, w_down, "moe_experts_few")
     top = expert.shape[1]
-    if tuple(w_gate.shape) != (n_experts, inter, width) or tuple(w_up.shape) != tuple(w_gate.shape) \
-            or tuple(w_down.shape) != (n_experts, width, inter):
-        raise KernelError("moe_experts_few: the stacked matrices have the wrong shapes")
+    if packed_width != width:
+        raise KernelError("moe_experts_few: the matrices have another width than the rows")
     if tuple(expert.shape) != (n, top) or tuple(weight.shape) != (n, top) \
             or tuple(act.shape) != (n * top, inter) or tuple(out.shape) != (top, n, width):
         raise KernelError("moe_experts_few: shapes do not fit")
@@ -1834,24 +1856,24 @@ def moe_experts_few(x, w_gate, w_up, w_down, expert, weight, row_seq, act, out, 
         _gpu(expert, "expert", torch.int32), _gpu(weight, "weight", torch.float32),
         None if row_seq is None else _gpu(row_seq, "row_seq", torch.int32),
         _gpu(act, "act", torch.bfloat16), _gpu(out, "out", torch.float32), n, width, inter,
-        n_experts, top, EXPERT_ACTIVATIONS[activation], float(limit), float(alpha), _stream())
+        n_experts, top, int(identity), EXPERT_ACTIVATIONS[activation], float(limit), float(alpha), _stream())
     _check(lib, status, "moe_experts_few")
 
 
 def moe_experts_grouped(x, w_gate, w_up, w_down, expert, weight, sorted_pairs, place, starts, act,
                         sums, out, activation="silu", limit=0.0, alpha=1.0, extra=None) -> None:
-    """`moe_experts` as grouped matrix products on the matrix cores: the (row, choice) pairs are
+    """`moe_experts` as grouped matrix products on the matrix cores, over matrices in operand order
+    (`pack_experts`): the (row, choice) pairs are
     laid out by expert on the device, every expert's pairs meet its matrices in tiles, and the
     rows' weighted sums are taken last.  Scratch: sorted_pairs, place [n * top] and starts
     [E + 1] int32, act [n * top, f] bfloat16, sums [n * top, w] float32."""
     lib = library("moe")
     n, width = x.shape
-    n_experts, inter = w_gate.shape[0], w_gate.shape[1]
+    n_experts, inter, packed_width = _packed_shapes(w_gate, w_up, w_down, "moe_experts_grouped")
     top = expert.shape[1]
     pairs = n * top
-    if tuple(w_gate.shape) != (n_experts, inter, width) or tuple(w_up.shape) != tuple(w_gate.shape) \
-            or tuple(w_down.shape) != (n_experts, width, inter):
-        raise KernelError("moe_experts_grouped: the stacked matrices have the wrong shapes")
+    if packed_width != width:
+        raise KernelError("moe_experts_grouped: the matrices have another width than the rows")
     if tuple(expert.shape) != (n, top) or tuple(weight.shape) != (n, top) \
             or tuple(act.shape) != (pairs, inter) or tuple(sums.shape) != (pairs, width) \
             or tuple(out.shape) != (n, width) or sorted_pairs.numel() < pairs \

@@ -16,11 +16,14 @@
 // identity expert, which adds p x_r and has no matrices.
 //
 // Three forms of the experts.  One takes a (row, choice) pair at a time and streams the expert's
-// matrices for it: any type and any sizes.  The others (bfloat16, widths that are multiples of
+// matrices for it: any type and any sizes, matrices as stored, gate and up [E, F, W], down
+// [E, W, F], stacked.  The others (bfloat16, widths that are multiples of
 // 64) run every expert's pairs against its matrices as tiles on the matrix cores: for up to 64
 // rows a block finds its expert's pairs itself; for more the pairs are laid out by expert on the
-// device first.  The matrices of all experts lie stacked: gate and up
-// [E, F, W], down [E, W, F].
+// device first.  Those take the matrices in operand order: tiles of 16 rows x 32 k of one
+// kilobyte each, an expert's strip of 16 rows being its K / 32 tiles in a row, and inside a tile
+// the piece of row r and k = 8 c .. 8 c + 7 at (c * 16 + r) * 8 elements, so that a wave's load of
+// a tile is one contiguous kilobyte which holds lane l's operand at 16 l bytes.
 #include "common.h"
 #include <float.h>
 
@@ -28,6 +31,14 @@ namespace {
 
 constexpr int kMaxTop = 64;
 constexpr int kRouteMax = 8;      // experts a lane holds: up to 512 experts
+constexpr int kRanked = 2;        // up to so many a lane, the choice is made by ranks
+
+// What this wave has written to LDS, its lanes may read from here on.
+__device__ __forceinline__ void wave_lds_fence() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
 
 // Rows [N, W] that are added to the experts' weighted sums: float32 slices or one bfloat16 tensor
 // (null: none).
@@ -57,9 +68,7 @@ __device__ __forceinline__ void leave_groups_out(float (&z)[kRouteMax], float* s
 #pragma unroll
   for (int j = 0; j < kRouteMax; ++j)
     if (lane + j * EI_WAVE < E) scores[lane + j * EI_WAVE] = z[j];
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-  __builtin_amdgcn_wave_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  wave_lds_fence();
   for (int g = lane; g < groups; g += EI_WAVE) {
     float first = 0.f, second = 0.f;            // (scores are not negative)
     for (int i = 0; i < size; ++i) {
@@ -69,9 +78,7 @@ __device__ __forceinline__ void leave_groups_out(float (&z)[kRouteMax], float* s
     }
     group_scores[g] = first + second;
   }
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-  __builtin_amdgcn_wave_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+  wave_lds_fence();
 #pragma unroll
   for (int j = 0; j < kRouteMax; ++j) {
     const int e = lane + j * EI_WAVE;
@@ -96,16 +103,14 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
                  float* __restrict__ weight, int N, int W, int E, int top, int mode,
                  const float* __restrict__ correction, int groups, int keep, float weight_scale) {
   __shared__ float logits[R][kRouteMax * EI_WAVE], group_scores[R][kRouteMax * EI_WAVE];
+  __shared__ float ranked[R][kMaxTop];
+  __shared__ int ranked_e[R][kMaxTop];
   const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE, waves = blockDim.x / EI_WAVE;
   const int row0 = blockIdx.x * R;
-  bool real[R];                                 // (rows beyond the last and padding rows: nothing to do)
-  bool any = false;
+  const TX* x_row[R];                           // (rows beyond the last: the last row again)
 #pragma unroll
-  for (int r = 0; r < R; ++r) {
-    real[r] = row0 + r < N && !(row_seq && row_seq[row0 + r] < 0);
-    any = any || real[r];
-  }
-  for (int e = wave; e < E && any; e += waves) {
+  for (int r = 0; r < R; ++r) x_row[r] = x + static_cast<size_t>(min(row0 + r, N - 1)) * W;
+  for (int e = wave; e < E; e += waves) {
     const float* wr = w_router + static_cast<size_t>(e) * W;
     float sum[R];
 #pragma unroll
@@ -117,9 +122,8 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
         ei::Vec4<float>::load(wr + i, wv);
 #pragma unroll
         for (int r = 0; r < R; ++r) {
-          if (!real[r]) continue;
           float xv[4];
-          ei::Vec4<TX>::load(x + static_cast<size_t>(row0 + r) * W + i, xv);
+          ei::Vec4<TX>::load(x_row[r] + i, xv);
           sum[r] += xv[0] * wv[0];
           sum[r] += xv[1] * wv[1];
           sum[r] += xv[2] * wv[2];
@@ -129,8 +133,7 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
     } else {
       for (int i = lane; i < W; i += EI_WAVE) {
 #pragma unroll
-        for (int r = 0; r < R; ++r)
-          if (real[r]) sum[r] += ei::to_f32<TX>(x[static_cast<size_t>(row0 + r) * W + i]) * wr[i];
+        for (int r = 0; r < R; ++r) sum[r] += ei::to_f32<TX>(x_row[r][i]) * wr[i];
       }
     }
 #pragma unroll
@@ -177,6 +180,39 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
     for (int j = 0; j < kRouteMax; ++j)
       z[j] = lane + j * EI_WAVE < E ? 1.0f / (1.0f + expf(-z[j])) : -FLT_MAX;
     if (groups > 1 && keep < groups) leave_groups_out(z, logits[wave], group_scores[wave], E, groups, keep);
+  }
+  if (E <= kRanked * EI_WAVE) {
+    // a lane finds its outputs' places in the order by comparing them with all others
+    float* choice = logits[wave];
+#pragma unroll
+    for (int j = 0; j < kRanked; ++j)
+      if (lane + j * EI_WAVE < E) choice[lane + j * EI_WAVE] = z[j];
+    wave_lds_fence();
+#pragma unroll
+    for (int j = 0; j < kRanked; ++j) {
+      const int e = lane + j * EI_WAVE;
+      if (e >= E) continue;
+      int rank = 0;
+      for (int o = 0; o < E; ++o) {
+        const float other = choice[o];
+        rank += other > z[j] || (other == z[j] && o < e) ? 1 : 0;
+      }
+      if (rank < top) {
+        ranked_e[wave][rank] = e;
+        ranked[wave][rank] = mode == 1 ? score[j] : z[j];
+      }
+    }
+    wave_lds_fence();
+    const float largest = ranked[wave][0];
+    float total = 0.f;
+    for (int k = 0; k < top; ++k) total += mode == 2 ? ranked[wave][k] : expf(ranked[wave][k] - largest);
+    if (lane < top) {
+      const float mine = ranked[wave][lane];
+      e_out[lane] = ranked_e[wave][lane];
+      w_out[lane] = mode == 2 ? mine / (total + 1e-20f) * weight_scale
+                              : mode == 1 ? mine : expf(mine - largest) / total;
+    }
+    return;
   }
   unsigned taken = 0;                            // bit j: this lane's expert lane + 64 j is chosen
   float total = 0.f, largest = 0.f;
@@ -331,40 +367,85 @@ moe_down_kernel(const T* __restrict__ act, const T* __restrict__ w_down,
 // moe_group: the (row, choice) pairs counted and laid out by expert: `sorted` [P] holds the
 // pairs of expert 0, then those of expert 1, ...; `place` [P] is where a pair went (-1: a pair
 // of weight 0, which is left out; -2: a pair of an identity expert, an output of the router
-// beyond the E experts); `starts` [E + 1] are the experts' first places.  Which place
-// a pair gets inside its expert's span depends on the order of the atomics; every pair is
-// computed for itself, so no result depends on it.
+// beyond the E experts); `starts` [E + 1] are the experts' first places.  A block an expert: it
+// counts its own pairs and those of the experts before it, then lays its own out, in an order
+// that depends on the pairs alone.
 __global__ void __launch_bounds__(1024)
 moe_group_kernel(const int32_t* __restrict__ expert, const float* __restrict__ weight,
                  int32_t* __restrict__ sorted, int32_t* __restrict__ place,
                  int32_t* __restrict__ starts, int P, int E) {
-  __shared__ int counts[kRouteMax * EI_WAVE], cursor[kRouteMax * EI_WAVE];
-  for (int e = threadIdx.x; e < E; e += blockDim.x) counts[e] = 0;
-  __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x)
-    if (weight[p] != 0.f && expert[p] < E) atomicAdd(&counts[expert[p]], 1);
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    int at = 0;
-    for (int e = 0; e < E; ++e) {
-      starts[e] = at;
-      cursor[e] = at;
-      at += counts[e];
-    }
-    starts[E] = at;
-  }
-  __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x) {
-    int q = -1;
-    if (weight[p] != 0.f) {
-      if (expert[p] < E) {
-        q = atomicAdd(&cursor[expert[p]], 1);
-        sorted[q] = p;
-      } else {
-        q = -2;
+  constexpr int WAVES = 16, U = 4;
+  __shared__ int counts[2][WAVES];
+  const int e = blockIdx.x;
+  const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
+  int before = 0, own = 0;
+  for (int p0 = threadIdx.x; p0 < P; p0 += 1024 * U) {
+    int x[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int p = p0 + u * 1024;
+      x[u] = p < P && weight[p] != 0.f ? expert[p] : E;
+      if (e == 0 && p < P) {                       // (once: the pairs that are left out)
+        if (weight[p] == 0.f) place[p] = -1;
+        else if (x[u] >= E) place[p] = -2;
       }
     }
-    place[p] = q;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      before += x[u] < e ? 1 : 0;
+      own += x[u] == e ? 1 : 0;
+    }
+  }
+#pragma unroll
+  for (int offset = 1; offset < EI_WAVE; offset <<= 1) {
+    before += __shfl_xor(before, offset, EI_WAVE);
+    own += __shfl_xor(own, offset, EI_WAVE);
+  }
+  if (lane == 0) {
+    counts[0][wave] = before;
+    counts[1][wave] = own;
+  }
+  __syncthreads();
+  before = own = 0;
+#pragma unroll
+  for (int w = 0; w < WAVES; ++w) {
+    before += counts[0][w];
+    own += counts[1][w];
+  }
+  if (threadIdx.x == 0) {
+    starts[e] = before;
+    if (e == E - 1) starts[E] = before + own;
+  }
+  int at = before;
+  for (int p0 = 0; p0 < P && at < before + own; p0 += 1024 * U) {
+    unsigned long long mine[U];
+    int here = 0;
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int p = p0 + u * 1024 + threadIdx.x;
+      mine[u] = __ballot(p < P && expert[p] == e && weight[p] != 0.f);
+      here += __popcll(mine[u]);
+    }
+    __syncthreads();                               // the counts before have been read
+    if (lane == 0) counts[0][wave] = here;
+    __syncthreads();
+    int q = at, total = 0;
+#pragma unroll
+    for (int w = 0; w < WAVES; ++w) {
+      if (w < wave) q += counts[0][w];
+      total += counts[0][w];
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (mine[u] >> lane & 1ull) {
+        const int p = p0 + u * 1024 + threadIdx.x;
+        const int to = q + __popcll(mine[u] & ((1ull << lane) - 1ull));
+        sorted[to] = p;
+        place[p] = to;
+      }
+      q += __popcll(mine[u]);
+    }
+    at += total;
   }
 }
 
@@ -424,9 +505,9 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
   const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
   const int r16 = lane % 16, quarter = lane / 16;
   const int n_wave = blockIdx.y * kTileN + wave * 16;         // the wave's first matrix row
-  const int n_row = min(n_wave + r16, N - 1);                 // (clamped: rows beyond N are not stored)
-  const bf16_t* w1_row = w1 + (static_cast<size_t>(e) * N + n_row) * K + quarter * 8;
-  const bf16_t* w2_row = GATED ? w2 + (static_cast<size_t>(e) * N + n_row) * K + quarter * 8 : nullptr;
+  const size_t strip = (static_cast<size_t>(e) * (N / 16) + n_wave / 16) * (K / 32);   // (N is a multiple of 64)
+  const bf16_t* w1_strip = w1 + strip * 512 + lane * 8;
+  const bf16_t* w2_strip = GATED ? w2 + strip * 512 + lane * 8 : nullptr;
   // the chunks of the places' rows that this thread carries into LDS
   const bf16_t* src[PER_THREAD];
   int dst[PER_THREAD];
@@ -455,8 +536,8 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
       if (carries) x_next[i] = *reinterpret_cast<const uint4*>(src[i] + k0);
 #pragma unroll
     for (int s = 0; s < STEPS; ++s) {
-      wa_next[s] = *reinterpret_cast<const moe_bf16x8*>(w1_row + k0 + s * 32);
-      if (GATED) wb_next[s] = *reinterpret_cast<const moe_bf16x8*>(w2_row + k0 + s * 32);
+      wa_next[s] = *reinterpret_cast<const moe_bf16x8*>(w1_strip + (k0 / 32 + s) * 512);
+      if (GATED) wb_next[s] = *reinterpret_cast<const moe_bf16x8*>(w2_strip + (k0 / 32 + s) * 512);
     }
   };
   fetch(0);
@@ -508,20 +589,30 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
 // order of the pairs (padding rows left out), its WAVES waves share K out and meet in LDS.  Both
 // operands come from memory straight into operand registers, U steps of 32 at a time.  GATED: the
 // gated products go to out_act [pairs, N] at the pairs' own places; else the products times the
-// pairs' weights go to out_sum [top, rows, N], slice = the choice.
+// pairs' weights go to out_sum [top, rows, N], slice = the choice; the blocks of "expert" E, where
+// there are such, write the identity experts' slices, weight times the row itself.
 template <int MB, bool GATED, int WAVES, int U>
 __global__ void __launch_bounds__(WAVES * EI_WAVE)
 moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
                const float* __restrict__ weight, const int32_t* __restrict__ row_seq,
                const bf16_t* __restrict__ w1, const bf16_t* __restrict__ w2,
                bf16_t* __restrict__ out_act, float* __restrict__ out_sum, int rows, int N, int K,
-               int top, ei::GateAct how) {
+               int top, int E, const bf16_t* __restrict__ x, ei::GateAct how) {
   constexpr int G = GATED ? 2 : 1;
   __shared__ int places[MB * 16];
   __shared__ int wave_counts[WAVES];
   __shared__ float red[WAVES][MB][G][4][EI_WAVE];
   const int e = blockIdx.y, n0 = blockIdx.x * 16, pairs = rows * top;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / EI_WAVE), lane = threadIdx.x % EI_WAVE;
+  if (!GATED && e == E) {
+    for (int o = threadIdx.x; o < pairs * 16; o += WAVES * EI_WAVE) {
+      const int p = o / 16, row = p / top, n = n0 + o % 16;
+      if (expert[p] >= E && !(row_seq && row_seq[row] < 0))
+        out_sum[(static_cast<size_t>(p % top) * rows + row) * N + n] =
+            weight[p] * ei::bf16_to_f32(x[static_cast<size_t>(row) * N + n]);
+    }
+    return;
+  }
   int count = 0;
   for (int base = 0; base < pairs; base += WAVES * EI_WAVE) {
     const int p = base + threadIdx.x;
@@ -543,8 +634,9 @@ moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
   count = min(__builtin_amdgcn_readfirstlane(count), MB * 16);
   if (count == 0) return;
   const int r16 = lane % 16, quarter = lane / 16;
-  const bf16_t* w1_row = w1 + (static_cast<size_t>(e) * N + n0 + r16) * K + quarter * 8;
-  const bf16_t* w2_row = GATED ? w2 + (static_cast<size_t>(e) * N + n0 + r16) * K + quarter * 8 : nullptr;
+  const size_t strip = (static_cast<size_t>(e) * (N / 16) + blockIdx.x) * (K / 32);
+  const bf16_t* w1_strip = w1 + strip * 512 + lane * 8;
+  const bf16_t* w2_strip = GATED ? w2 + strip * 512 + lane * 8 : nullptr;
   const bf16_t* x_row[MB];
 #pragma unroll
   for (int mb = 0; mb < MB; ++mb) {
@@ -563,8 +655,8 @@ moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
 #pragma unroll
     for (int u = 0; u < U; ++u)
       if (s0 + u < s_end) {
-        wa[u] = *reinterpret_cast<const moe_bf16x8*>(w1_row + (s0 + u) * 32);
-        if (GATED) wb[u] = *reinterpret_cast<const moe_bf16x8*>(w2_row + (s0 + u) * 32);
+        wa[u] = *reinterpret_cast<const moe_bf16x8*>(w1_strip + (s0 + u) * 512);
+        if (GATED) wb[u] = *reinterpret_cast<const moe_bf16x8*>(w2_strip + (s0 + u) * 512);
 #pragma unroll
         for (int mb = 0; mb < MB; ++mb)
           if (mb * 16 < count) xf[u][mb] = *reinterpret_cast<const moe_bf16x8*>(x_row[mb] + (s0 + u) * 32);
@@ -615,9 +707,10 @@ moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
 // through two LDS buffers for both operands, moved from global memory straight into LDS (a wave
 // load is a kilobyte, lane l's 16 bytes at place l of it): tile k + 1 is asked for right after the
 // barrier that frees its buffer and arrives while tile k is multiplied; a second block on the
-// compute unit covers the rest of the wait.  The 16-byte pieces of a row are exchanged among
-// themselves (piece ^ (row / 2) % 8), so that 16 rows read at one place of a row meet every bank
-// once; a lane fetches the piece that belongs at its place.
+// compute unit covers the rest of the wait.  The matrix comes in operand order; of the places' rows
+// the 16-byte pieces are exchanged among themselves (piece ^ (row / 2) % 8), so that 16 rows read
+// at one place of a row meet every bank once, and a lane fetches the piece that belongs at its
+// place.
 // Blocks are dealt to the 8 XCDs round robin; block ids are laid out so that an XCD works on
 // `group` tiles of places at a time against all rows of the matrix, whose operands its L2 then
 // holds.
@@ -652,9 +745,13 @@ moe_tile_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
     const int at = first + min(row, valid - 1);               // (clamped: such rows are not stored)
     const size_t source = GATED ? static_cast<size_t>(sorted[at] / top) : static_cast<size_t>(at);
     from_a[i] = a + source * K + piece * 8;
-    const bf16_t* matrix = GATED && row >= kBig / 2 ? w2 : w1;
-    const int n = GATED ? n_tile * (kBig / 2) + row % (kBig / 2) : n_tile * kBig + row;
-    from_b[i] = matrix + (static_cast<size_t>(e) * N + min(n, N - 1)) * K + piece * 8;
+    // (a wave load of the matrix is one of its tiles: strip `load / 2` of the block's eight, the
+    // first or the second 32 of K)
+    const int load = wave * LOADS + i, strip = load / 2;
+    const bf16_t* matrix = GATED && strip >= 4 ? w2 : w1;
+    const int n_strip = GATED ? n_tile * 4 + strip % 4 : n_tile * 8 + strip;
+    from_b[i] = matrix + ((static_cast<size_t>(e) * (N / 16) + min(n_strip, N / 16 - 1)) * (K / 32) +
+                          load % 2) * 512 + lane * 8;
   }
   auto fetch = [&](int k0, int buffer) __attribute__((always_inline)) {
 #pragma unroll
@@ -664,7 +761,7 @@ moe_tile_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
           (const __attribute__((address_space(1))) void*)(from_a[i] + k0),
           (__attribute__((address_space(3))) void*)(&lds[buffer][0][at]), 16, 0, 0);
       __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) void*)(from_b[i] + k0),
+          (const __attribute__((address_space(1))) void*)(from_b[i] + k0 * 16),
           (__attribute__((address_space(3))) void*)(&lds[buffer][1][at]), 16, 0, 0);
     }
   };
@@ -672,7 +769,8 @@ moe_tile_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
 #pragma unroll
   for (int j = 0; j < 2; ++j) {
     read_a[j] = (wm * 64 + j * 32 + l32) * kBigK;
-    read_b[j] = (GATED ? j * 64 + wn * 32 + l32 : wn * 64 + j * 32 + l32) * kBigK;
+    const int row_b = GATED ? j * 64 + wn * 32 + l32 : wn * 64 + j * 32 + l32;
+    read_b[j] = row_b / 16 * 1024 + row_b % 16 * 8 + half * 128;
   }
 #pragma unroll
   for (int s = 0; s < 4; ++s) piece_at[s] = ((2 * s + half) ^ ((l32 >> 1) & 7)) * 8;
@@ -698,7 +796,7 @@ moe_tile_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         fa[j] = *reinterpret_cast<const moe_bf16x8*>(&lds[buffer][0][read_a[j] + piece_at[s]]);
-        fb[j] = *reinterpret_cast<const moe_bf16x8*>(&lds[buffer][1][read_b[j] + piece_at[s]]);
+        fb[j] = *reinterpret_cast<const moe_bf16x8*>(&lds[buffer][1][read_b[j] + s / 2 * 512 + s % 2 * 256]);
       }
 #pragma unroll
       for (int i = 0; i < 2; ++i)
@@ -815,7 +913,7 @@ extern "C" int ei_moe_route(const void* x, int x_dtype, const float* w_router, c
   do {                                                                                         \
     const TX* xx = static_cast<const TX*>(x);                                                  \
     if (N >= 512)                                                                              \
-      moe_route_kernel<TX, 4><<<(N + 3) / 4, 256, 0, stream>>>(                                \
+      moe_route_kernel<TX, 4><<<(N + 3) / 4, EI_WAVE * (E >= 8 ? 8 : 4), 0, stream>>>(         \
           xx, w_router, row_seq, expert, weight, N, W, E, top, mode, correction, groups, keep, \
           weight_scale);                                                                       \
     else                                                                                       \
@@ -887,7 +985,7 @@ extern "C" int ei_moe_experts_grouped(const void* x, const void* w_gate, const v
   const long long pairs = static_cast<long long>(N) * top;
   EI_REQUIRE(pairs <= 0x3fffffffLL, "moe_experts_grouped: too many rows for one launch");
   const int P = static_cast<int>(pairs);
-  moe_group_kernel<<<1, 1024, 0, stream>>>(expert, weight, sorted, place, starts, P, E);
+  moe_group_kernel<<<E, 1024, 0, stream>>>(expert, weight, sorted, place, starts, P, E);
   const bf16_t* xb = static_cast<const bf16_t*>(x);
   const bf16_t* g = static_cast<const bf16_t*>(w_gate);
   const bf16_t* u = static_cast<const bf16_t*>(w_up);
@@ -924,15 +1022,16 @@ extern "C" int ei_moe_few_rows() { return 64; }
 
 // The experts of at most 64 rows: act [N * top, F] bfloat16 is scratch; slice k of out [top, N, W]
 // float32 receives every row's k-th choice's product row times its weight (a padding row, row_seq
-// < 0, is not written).  Every choice must be an expert (no identity ones), none twice in a row.
+// < 0, is not written).  A row chooses an output of the router once at most; outputs from E on are
+// identity experts, which there are `identity` of.
 extern "C" int ei_moe_experts_few(const void* x, const void* w_gate, const void* w_up,
                                   const void* w_down, const int32_t* expert, const float* weight,
                                   const int32_t* row_seq, void* act, float* out, int N, int W, int F,
-                                  int E, int top, int act_kind, float limit, float alpha,
-                                  hipStream_t stream) {
-  EI_REQUIRE(x && w_gate && w_up && w_down && expert && weight && act && out,
+                                  int E, int top, int identity, int act_kind, float limit,
+                                  float alpha, hipStream_t stream) {
+  EI_REQUIRE(x && w_gate && w_up && w_down && expert && weight && act && out && identity >= 0,
              "moe_experts_few: null pointer");
-  EI_REQUIRE(N > 0 && N <= ei_moe_few_rows() && top >= 1 && E >= 1 && E <= 65535 &&
+  EI_REQUIRE(N > 0 && N <= ei_moe_few_rows() && top >= 1 && E >= 1 && E < 65535 &&
                  ei_moe_grouped_supported(EI_BF16, W, F, E),
              "moe_experts_few: sizes it does not take");
   EI_REQUIRE(known_act(act_kind), "moe_experts_few: unknown activation");
@@ -942,17 +1041,17 @@ extern "C" int ei_moe_experts_few(const void* x, const void* w_gate, const void*
   const bf16_t* u = static_cast<const bf16_t*>(w_up);
   const bf16_t* d = static_cast<const bf16_t*>(w_down);
   bf16_t* ab = static_cast<bf16_t*>(act);
-  const dim3 grid_up(F / 16, E), grid_down(W / 16, E);
+  const dim3 grid_up(F / 16, E), grid_down(W / 16, E + (identity > 0 ? 1 : 0));
 #define EI_FEW(MB, WAVES, U)                                                                   \
   do {                                                                                         \
     moe_few_kernel<MB, true, WAVES, U><<<grid_up, WAVES * EI_WAVE, 0, stream>>>(               \
-        xb, expert, weight, row_seq, g, u, ab, nullptr, N, F, W, top, how);                    \
+        xb, expert, weight, row_seq, g, u, ab, nullptr, N, F, W, top, E, xb, how);             \
     moe_few_kernel<MB, false, WAVES, U><<<grid_down, WAVES * EI_WAVE, 0, stream>>>(            \
-        ab, expert, weight, row_seq, d, nullptr, nullptr, out, N, W, F, top, how);             \
+        ab, expert, weight, row_seq, d, nullptr, nullptr, out, N, W, F, top, E, xb, how);      \
   } while (0)
   if (N <= 16) EI_FEW(1, 8, 8);
   else if (N <= 32) EI_FEW(2, 4, 8);
-  else EI_FEW(4, 4, 4);
+  else EI_FEW(4, 8, 4);
 #undef EI_FEW
   EI_LAUNCH_CHECK();
 }

@@ -121,13 +121,14 @@ class RoutedMLP:
                                     if name.startswith("shared.")}, dtype, device)
         self.grouped = lib.moe_grouped_supported(dtype, hidden, spec.intermediate_size,
                                                  spec.n_experts)
-        # (identity experts have no product whose rows could be a slice)
-        self.few = self.grouped and not getattr(spec, "identity", 0)
+        if self.grouped:       # (those forms take the matrices in operand order; no other copy is kept)
+            self.w_gate, self.w_up, self.w_down = (
+                lib.pack_experts(w) for w in (self.w_gate, self.w_up, self.w_down))
 
     def forward(self, ctx, x):
         spec = self.spec
         n = x.shape[0]
-        if self.few and n <= lib.MOE_FEW_ROWS:
+        if self.grouped and n <= lib.MOE_FEW_ROWS:
             slices = self._few_rows(ctx, x)
             if slices is not None:
                 return slices
@@ -168,6 +169,6 @@ class RoutedMLP:
         lib.moe_route(x, self.router, ctx.meta.row_seq, expert, weight, **self.routing)
         act = ctx.buffer("moe.act", (n * spec.top, spec.intermediate_size))
         lib.moe_experts_few(x, self.w_gate, self.w_up, self.w_down, expert, weight, ctx.meta.row_seq,
-                            act, slices[:spec.top], **self.act)
+                            act, slices[:spec.top], identity=getattr(spec, "identity", 0), **self.act)
         ctx.release(expert, weight, act)
         return slices

@@ -571,7 +571,7 @@ def test_experts_of_few_rows_leave_padding_rows_out():
     expert[dead], weight[dead] = 0, 0.0
     act = torch.empty(rows * top, inter, device=DEV, dtype=torch.bfloat16)
     out = torch.full((top, rows, width), 5.0, device=DEV)
-    dev = [m.to(DEV).to(torch.bfloat16) for m in w]
+    dev = [lib.pack_experts(m.to(DEV).to(torch.bfloat16)) for m in w]
     lib.moe_experts_few(x.to(DEV).to(torch.bfloat16), *dev, expert.to(DEV), weight.to(DEV),
                         row_seq.to(DEV), act, out, activation="clamped_swish", limit=0.9, alpha=1.702)
     for r in range(rows):

@@ -305,6 +305,9 @@ def test_identity_experts_add_the_row_itself(experts, identity, top, inter, widt
         def release(*buffers):
             pass
     got = part.forward(Context, x.to(DEV).to(part.w_gate.dtype))
+    if got.dim() == 3:              # (few rows: a slice a choice)
+        assert part.grouped and rows <= 64
+        got = got.sum(0)
     if dtype == "float32":
         assert_close_f32(got, want, "identity experts")
     else:

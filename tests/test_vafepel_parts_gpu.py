@@ -554,7 +554,8 @@ def test_the_experts_of_a_rows_choice(experts, top, inter, width, rows, dtype):
         pairs = rows * top
         order = torch.empty(2 * pairs + experts + 1, dtype=torch.int32, device=DEV)
         sums = torch.empty(pairs, width, device=DEV)
-        lib.moe_experts_grouped(xd, *matrices, expert, weight, order[:pairs], order[pairs:2 * pairs],
+        packed = [lib.pack_experts(m) for m in matrices]
+        lib.moe_experts_grouped(xd, *packed, expert, weight, order[:pairs], order[pairs:2 * pairs],
                                 order[2 * pairs:], act, sums, out)
         assert sorted(order[:pairs].tolist()) == list(range(pairs))
     else:
