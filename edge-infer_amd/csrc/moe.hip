@@ -110,13 +110,15 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
   const TX* x_row[R];                           // (rows beyond the last: the last row again)
 #pragma unroll
   for (int r = 0; r < R; ++r) x_row[r] = x + static_cast<size_t>(min(row0 + r, N - 1)) * W;
+  // (asked for now, looked at when the choice is made)
+  const int own_seq = row_seq && wave < R && row0 + wave < N ? row_seq[row0 + wave] : 0;
   for (int e = wave; e < E; e += waves) {
     const float* wr = w_router + static_cast<size_t>(e) * W;
     float sum[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) sum[r] = 0.f;
     if (W % 4 == 0) {
-#pragma unroll 4
+#pragma unroll(R == 1 ? 8 : 4)
       for (int i = lane * 4; i < W; i += EI_WAVE * 4) {
         float wv[4];
         ei::Vec4<float>::load(wr + i, wv);
@@ -147,7 +149,7 @@ moe_route_kernel(const TX* __restrict__ x, const float* __restrict__ w_router,
   if (wave >= R || row0 + wave >= N) return;
   int32_t* e_out = expert + static_cast<size_t>(row0 + wave) * top;
   float* w_out = weight + static_cast<size_t>(row0 + wave) * top;
-  if (row_seq && row_seq[row0 + wave] < 0) {    // a padding row: no expert has anything to add
+  if (own_seq < 0) {    // a padding row: no expert has anything to add
     for (int k = lane; k < top; k += EI_WAVE) { e_out[k] = 0; w_out[k] = 0.f; }
     return;
   }
@@ -374,7 +376,7 @@ __global__ void __launch_bounds__(1024)
 moe_group_kernel(const int32_t* __restrict__ expert, const float* __restrict__ weight,
                  int32_t* __restrict__ sorted, int32_t* __restrict__ place,
                  int32_t* __restrict__ starts, int P, int E) {
-  constexpr int WAVES = 16, U = 4;
+  constexpr int WAVES = 16, U = 8;
   __shared__ int counts[2][WAVES];
   const int e = blockIdx.x;
   const int wave = threadIdx.x / EI_WAVE, lane = threadIdx.x % EI_WAVE;
@@ -584,35 +586,42 @@ moe_gemm_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ sorted
   }
 }
 
-// The experts of up to MB * 16 rows: a block an expert and 16 rows of its matrix (GATED: of its
-// gate and of its up matrix).  The block finds the pairs that chose its expert itself, in the
-// order of the pairs (padding rows left out), its WAVES waves share K out and meet in LDS.  Both
-// operands come from memory straight into operand registers, U steps of 32 at a time.  GATED: the
+// The experts of up to MB * 16 rows: a block an expert and STRIPS strips of 16 rows of its matrix
+// (GATED: of its gate and of its up matrix).  The block finds the pairs that chose its expert
+// itself, in the order of the pairs (padding rows left out); KS waves share a strip's K out and
+// meet in LDS.  Both operands come from memory straight into operand registers, U steps of 32 at a
+// time.  GATED: the
 // gated products go to out_act [pairs, N] at the pairs' own places; else the products times the
 // pairs' weights go to out_sum [top, rows, N], slice = the choice; the blocks of "expert" E, where
 // there are such, write the identity experts' slices, weight times the row itself.
-template <int MB, bool GATED, int WAVES, int U>
-__global__ void __launch_bounds__(WAVES * EI_WAVE)
+template <int MB, bool GATED, int STRIPS, int KS, int U>
+__global__ void __launch_bounds__(STRIPS * KS * EI_WAVE)
 moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
                const float* __restrict__ weight, const int32_t* __restrict__ row_seq,
                const bf16_t* __restrict__ w1, const bf16_t* __restrict__ w2,
                bf16_t* __restrict__ out_act, float* __restrict__ out_sum, int rows, int N, int K,
                int top, int E, const bf16_t* __restrict__ x, ei::GateAct how) {
-  constexpr int G = GATED ? 2 : 1;
+  constexpr int G = GATED ? 2 : 1, WAVES = STRIPS * KS;
   __shared__ int places[MB * 16];
   __shared__ int wave_counts[WAVES];
   __shared__ float red[WAVES][MB][G][4][EI_WAVE];
-  const int e = blockIdx.y, n0 = blockIdx.x * 16, pairs = rows * top;
+  const int e = blockIdx.y, n0 = blockIdx.x * (STRIPS * 16), pairs = rows * top;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / EI_WAVE), lane = threadIdx.x % EI_WAVE;
   if (!GATED && e == E) {
-    for (int o = threadIdx.x; o < pairs * 16; o += WAVES * EI_WAVE) {
-      const int p = o / 16, row = p / top, n = n0 + o % 16;
+    for (int o = threadIdx.x; o < pairs * STRIPS * 16; o += WAVES * EI_WAVE) {
+      const int p = o / (STRIPS * 16), row = p / top, n = n0 + o % (STRIPS * 16);
       if (expert[p] >= E && !(row_seq && row_seq[row] < 0))
         out_sum[(static_cast<size_t>(p % top) * rows + row) * N + n] =
             weight[p] * ei::bf16_to_f32(x[static_cast<size_t>(row) * N + n]);
     }
     return;
   }
+  const int n_strip = wave / KS, slice = wave % KS;
+  const size_t strip = (static_cast<size_t>(e) * (N / 16) + n0 / 16 + n_strip) * (K / 32);
+  const bf16_t* w1_strip = w1 + strip * 512 + lane * 8;
+  const bf16_t* w2_strip = GATED ? w2 + strip * 512 + lane * 8 : nullptr;
+  const int steps = K / 32, per = (steps + KS - 1) / KS;
+  const int s_begin = slice * per, s_end = min(steps, (slice + 1) * per);
   int count = 0;
   for (int base = 0; base < pairs; base += WAVES * EI_WAVE) {
     const int p = base + threadIdx.x;
@@ -634,9 +643,6 @@ moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
   count = min(__builtin_amdgcn_readfirstlane(count), MB * 16);
   if (count == 0) return;
   const int r16 = lane % 16, quarter = lane / 16;
-  const size_t strip = (static_cast<size_t>(e) * (N / 16) + blockIdx.x) * (K / 32);
-  const bf16_t* w1_strip = w1 + strip * 512 + lane * 8;
-  const bf16_t* w2_strip = GATED ? w2 + strip * 512 + lane * 8 : nullptr;
   const bf16_t* x_row[MB];
 #pragma unroll
   for (int mb = 0; mb < MB; ++mb) {
@@ -648,9 +654,7 @@ moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
   for (int mb = 0; mb < MB; ++mb)
 #pragma unroll
     for (int g = 0; g < G; ++g) acc[mb][g] = moe_f32x4{0.f, 0.f, 0.f, 0.f};
-  const int steps = K / 32, per = (steps + WAVES - 1) / WAVES;
-  const int s_end = min(steps, (wave + 1) * per);
-  for (int s0 = wave * per; s0 < s_end; s0 += U) {
+  for (int s0 = s_begin; s0 < s_end; s0 += U) {
     moe_bf16x8 wa[U], wb[GATED ? U : 1], xf[U][MB];
 #pragma unroll
     for (int u = 0; u < U; ++u)
@@ -681,15 +685,15 @@ moe_few_kernel(const bf16_t* __restrict__ a, const int32_t* __restrict__ expert,
       for (int i = 0; i < 4; ++i) red[wave][mb][g][i][lane] = acc[mb][g][i];
   __syncthreads();
   // lane (r16, quarter) of a wave held, of place mb * 16 + r16, the matrix rows n0 + 4 quarter + i
-  for (int o = threadIdx.x; o < count * 16; o += WAVES * EI_WAVE) {
-    const int index = o / 16, n = o % 16;
-    const int mb = index / 16, from = index % 16 + 16 * (n / 4), i = n % 4;
+  for (int o = threadIdx.x; o < count * STRIPS * 16; o += WAVES * EI_WAVE) {
+    const int index = o / (STRIPS * 16), n = o % (STRIPS * 16);
+    const int mb = index / 16, from = index % 16 + 16 * (n % 16 / 4), i = n % 4, first = n / 16 * KS;
     float sum[G];
 #pragma unroll
     for (int g = 0; g < G; ++g) {
       sum[g] = 0.f;
 #pragma unroll
-      for (int w = 0; w < WAVES; ++w) sum[g] += red[w][mb][g][i][from];
+      for (int w = 0; w < KS; ++w) sum[g] += red[first + w][mb][g][i][from];
     }
     const int p = places[index];
     if (GATED)
@@ -1041,17 +1045,21 @@ extern "C" int ei_moe_experts_few(const void* x, const void* w_gate, const void*
   const bf16_t* u = static_cast<const bf16_t*>(w_up);
   const bf16_t* d = static_cast<const bf16_t*>(w_down);
   bf16_t* ab = static_cast<bf16_t*>(act);
-  const dim3 grid_up(F / 16, E), grid_down(W / 16, E + (identity > 0 ? 1 : 0));
-#define EI_FEW(MB, WAVES, U)                                                                   \
-  do {                                                                                         \
-    moe_few_kernel<MB, true, WAVES, U><<<grid_up, WAVES * EI_WAVE, 0, stream>>>(               \
-        xb, expert, weight, row_seq, g, u, ab, nullptr, N, F, W, top, E, xb, how);             \
-    moe_few_kernel<MB, false, WAVES, U><<<grid_down, WAVES * EI_WAVE, 0, stream>>>(            \
-        ab, expert, weight, row_seq, d, nullptr, nullptr, out, N, W, F, top, E, xb, how);      \
-  } while (0)
-  if (N <= 16) EI_FEW(1, 8, 8);
-  else if (N <= 32) EI_FEW(2, 4, 8);
-  else EI_FEW(4, 8, 4);
+  const int down_experts = E + (identity > 0 ? 1 : 0);
+#define EI_FEW(MB, GATED, STRIPS, KS, U, EXPERTS, A, W1, W2, ACT, OUT, ROWS, COLS)             \
+  moe_few_kernel<MB, GATED, STRIPS, KS, U>                                                     \
+      <<<dim3(ROWS / (STRIPS * 16), EXPERTS), STRIPS * KS * EI_WAVE, 0, stream>>>(             \
+          A, expert, weight, row_seq, W1, W2, ACT, OUT, N, ROWS, COLS, top, E, xb, how)
+  if (N <= 16) {
+    EI_FEW(1, true, 1, 8, 8, E, xb, g, u, ab, nullptr, F, W);
+    EI_FEW(1, false, 1, 8, 8, down_experts, ab, d, nullptr, nullptr, out, W, F);
+  } else if (N <= 32) {
+    EI_FEW(2, true, 1, 8, 8, E, xb, g, u, ab, nullptr, F, W);
+    EI_FEW(2, false, 1, 8, 8, down_experts, ab, d, nullptr, nullptr, out, W, F);
+  } else {
+    EI_FEW(4, true, 1, 8, 4, E, xb, g, u, ab, nullptr, F, W);
+    EI_FEW(4, false, 4, 2, 6, down_experts, ab, d, nullptr, nullptr, out, W, F);
+  }
 #undef EI_FEW
   EI_LAUNCH_CHECK();
 }

@@ -645,6 +645,19 @@ __device__ __forceinline__ float sliced(const TI* p, int nsplit, size_t split_st
   return v;
 }
 
+// Sine and cosine of an angle given in turns (of 2 pi): the whole turns are taken off in float64.
+// For float32 results the library's functions; for bfloat16 results the hardware's (which take
+// turns), good to about 1e-6 and swallowed by the rounding.
+template <typename TO> __device__ __forceinline__ void turn_of(double turns, float& sn, float& cs);
+template <> __device__ __forceinline__ void turn_of<float>(double turns, float& sn, float& cs) {
+  sincosf(static_cast<float>((turns - floor(turns)) * 6.283185307179586), &sn, &cs);
+}
+template <> __device__ __forceinline__ void turn_of<bf16_t>(double turns, float& sn, float& cs) {
+  const float part = static_cast<float>(turns - floor(turns));
+  sn = __builtin_amdgcn_sinf(part);
+  cs = __builtin_amdgcn_cosf(part);
+}
+
 template <typename TI, typename TO>
 __global__ void head_store_kernel(
     const TI* __restrict__ proj, int nsplit, size_t split_stride, size_t row_stride,
@@ -730,9 +743,8 @@ __global__ void head_store_kernel(
       const float p = w ? (y[j] * inv) * w[partner] : y[j];
       const double turns = static_cast<double>(pos) * freqs[e < rhalf ? e : e - rhalf] *
                            0.15915494309189535;       // in units of 2 pi
-      const float angle = static_cast<float>((turns - floor(turns)) * 6.283185307179586);
       float sn, cs;
-      sincosf(angle, &sn, &cs);
+      turn_of<TO>(turns, sn, cs);
       cs *= turn_scale;
       sn *= turn_scale;
       v = e < rhalf ? v * cs - p * sn : v * cs + p * sn;
@@ -861,9 +873,8 @@ __global__ void head_store_vec_kernel(
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const double whole = static_cast<double>(pos) * freqs[f0 + i] * 0.15915494309189535;
-      const float angle = static_cast<float>((whole - floor(whole)) * 6.283185307179586);
       float sn, cs;
-      sincosf(angle, &sn, &cs);
+      turn_of<TO>(whole, sn, cs);
       cs *= turn_scale;
       sn *= turn_scale;
       x[i] = e0 < rhalf ? x[i] * cs - y[i] * sn : x[i] * cs + y[i] * sn;

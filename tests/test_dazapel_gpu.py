@@ -133,6 +133,28 @@ def test_whole_prompts(models, references, name, dtype):
     session.cache.check()
 
 
+@pytest.mark.parametrize("name", NAMES)
+def test_prompts_of_more_rows_than_the_few_rows_product_takes(models, weights, name):
+    """A prompt of 420 tokens and one of 300 beside a short one (bfloat16: the library multiplies,
+    and adds the projections' biases itself), then tokens one by one together."""
+    import edge_infer_amd as ei
+    cfg = config_of(name, "bfloat16")
+    requests = [ids(cfg["vocab"], n, 60 + n) for n in (425, 305, 9)]
+    refs = [plain.forward(cfg, weights[name]["bfloat16"], r) for r in requests]
+    session = ei.Session(models(name, "bfloat16"), max_tokens=1024, max_seqs=3)
+    slots = [session.begin() for _ in requests]
+    cuts = [len(r) - 5 for r in requests]
+    logits = session.step([(s, r[:c], list(range(c))) for s, r, c in zip(slots, requests, cuts)])
+    at = 0
+    for ref, cut in zip(refs, cuts):
+        close("bfloat16", logits[at:at + cut], ref[:cut], f"{name} prompt of {cut} in a batch")
+        at += cut
+    for k in range(5):
+        logits = session.step([(s, r[c + k:c + k + 1], [0]) for s, r, c in zip(slots, requests, cuts)])
+        want = torch.stack([ref[cut + k] for ref, cut in zip(refs, cuts)])
+        close("bfloat16", logits, want, f"{name} token {k} after the prompts")
+
+
 @pytest.mark.parametrize("name", ["A", "C", "D"])
 def test_the_stream_after_every_run_of_a_layer(models, weights, name):
     """The float32 stream after each run of a layer (a looped layer counts each time), before
