@@ -1,5 +1,5 @@
-"""edge-infer for AMD MI355X: a small generation library for the Qwen3 dense, the Tirurax and
-the Zadenex decoders (the architecture is the one that a folder's config.json names).
+"""edge-infer for AMD MI355X: a small generation library for the Qwen3 dense, Tirurax, Zadenex,
+Vafepel, Gopuzen and Dazapel decoders (the architecture is the one that a folder's config.json names).
 
     model = load_model("/path/to/folder", dtype="bfloat16")     # config.json + safetensors
     session = Session(model, max_tokens=4096)

@@ -34,11 +34,12 @@ class FrequencyScaling:
 
 @dataclass(frozen=True)
 class YarnScaling:
-    """Pairs of a rotation are told apart by how often they turn within the original length: with
-    dim(t) = dims ln(original / (2 pi t)) / (2 ln theta), lo = max(floor(dim(fast)), 0),
-    hi = min(ceil(dim(slow)), dims - 1) and ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1),
-    the frequency of pair i becomes f_i / factor ramp_i + f_i (1 - ramp_i), and cosine and sine
-    are multiplied by 0.1 ln(factor) + 1."""
+    """Frequencies stretched by how often a pair turns within the original length L.  With
+    n(t) = R ln(L / (2 pi t)) / (2 ln theta), the pair (as a real number) that makes t turns of a
+    rotation of R elements, pairs up to a = floor(n(fast)), at least 0, keep their frequency,
+    pairs from b = ceil(n(slow)), at most R - 1, on have it divided by `factor`, and between them
+    the share of the divided one grows linearly with the pair's index (over a width of at least
+    1/1000).  Cosine and sine grow by 1 + ln(factor) / 10."""
     factor: float
     original: float
     fast: float
@@ -75,7 +76,7 @@ class AttentionSpec:
     qk_unit_norm: bool = False
     window: Optional[int] = None   # None: every earlier key; w: the last w keys
     # with a window: the sequence's first `keep_first` positions stay visible however far back
-    # they lie, at their true positions
+    # they lie
     keep_first: int = 0
     scale: Optional[float] = None  # None: 1/sqrt(head_dim)
     position: PositionSpec = field(default_factory=PositionSpec)
@@ -173,9 +174,9 @@ class RoutedMLPSpec:
 
     `scoring` "sigmoid": the scores are sigmoid(z), the choice is by the largest score, and the
     weights are the chosen scores divided by their sum (+ 1e-20), times `weight_scale`.
-    `group_count` G > 1 (this scoring only): the experts form G equal groups of neighbours, a
-    group's score is the sum of its two largest scores, and only experts of the `group_keep`
-    best groups can be chosen.  `shared`: a gated feed-forward that runs for every token and is
+    `group_count` G > 1 (this scoring only): the experts are cut into G runs of equal length,
+    ranked by what their two best scores add up to, and the choice is made among the members of
+    the first `group_keep` runs.  `shared`: a gated feed-forward that runs for every token and is
     added.  `activation`, `limit`, `alpha`: of an expert, as in `GatedMLPSpec` ("silu" or
     "clamped_swish").
 

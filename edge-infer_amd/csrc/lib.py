@@ -1725,9 +1725,8 @@ def moe_route(x, router_w, row_seq, expert, weight, scoring: str = "softmax_chos
     (float32 [n, top]).  Rows with row_seq < 0 get weights of 0.  scoring "softmax_all": the
     scores are the softmax over all E logits, the choice is by score + correction [E] (None:
     by the score), and the weights are the chosen scores themselves.  scoring "sigmoid": the
-    scores are sigmoid(logit), only experts of the `keep` best of `groups` equal groups of
-    neighbours can be chosen (a group's score: the sum of its two largest), and the weights
-    are the chosen scores over their sum, times `weight_scale`."""
+    scores are sigmoid(logit), the experts are cut into `groups` runs of equal length of which
+    the `keep` whose two best scores add up to most take part, and the weights are the chosen scores over their sum, times `weight_scale`."""
     lib = library("moe")
     if scoring not in ROUTER_SCORINGS:
         raise KernelError(f"moe_route: unknown scoring '{scoring}'")

@@ -6,9 +6,9 @@
 // router outputs, the `top` outputs of largest s + correction (a learned number per output,
 // null: none), and the weights s of the chosen, not renormalised.  Experts: for row r and its
 // choice k with expert e and weight p,  y_r += p W_down,e (silu(W_gate,e x_r) * (W_up,e x_r)).
-// `mode` 2: the scores s = sigmoid(z), the experts in `groups` equal groups of neighbours of which
-// the `keep` with the largest sums of their two largest scores take part (of equal sums the one of
-// lower index), the `top` largest scores among their experts, and the weights s / (sum of the
+// `mode` 2: the scores s = sigmoid(z), the experts cut into `groups` runs of equal length of which
+// the `keep` whose two best scores add up to most take part (of equal ones the one of lower
+// index), the `top` largest scores among their experts, and the weights s / (sum of the
 // chosen s + 1e-20) * weight_scale.
 // The gated product of an expert is silu(gate) * up or the clamped swish (`ei::GateAct`).  The rows
 // of another product (an expert that every row takes) may be added to the sums: `extra`.

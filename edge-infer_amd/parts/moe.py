@@ -11,9 +11,8 @@ goes by score plus a learned `correction` per output (where the spec has one), a
 are the chosen scores themselves; with `identity = I` the router has I outputs beyond the
 experts, and one of them chosen adds p x itself.
 
-With `scoring = "sigmoid"` the scores are sigmoid(z); the experts form `group_count` equal groups
-of neighbours, of which the `group_keep` with the largest sums of their two largest scores take
-part, and the weights are the chosen scores over their sum, times `weight_scale`.  An expert's
+With `scoring = "sigmoid"` the scores are sigmoid(z); the experts are cut into `group_count`
+runs of equal length, of which the `group_keep` whose two best scores add up to most take part, and the weights are the chosen scores over their sum, times `weight_scale`.  An expert's
 activation may be the clamped swish of `parts.mlp`; `shared` is a gated feed-forward of its own
 size that every row passes, whose rows the kernel that sums the experts' outputs adds.
 
