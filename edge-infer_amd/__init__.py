@@ -1,5 +1,5 @@
 """edge-infer for AMD MI355X: a small generation library for the Qwen3 dense, Tirurax, Zadenex,
-Vafepel, Gopuzen and Dazapel decoders (the architecture is the one that a folder's config.json names).
+Vafepel, Gopuzen, Dazapel and Lemotar decoders (the architecture is the one that a folder's config.json names).
 
     model = load_model("/path/to/folder", dtype="bfloat16")     # config.json + safetensors
     session = Session(model, max_tokens=4096)
@@ -33,6 +33,9 @@ def build_model(entry, cfg, tensors, dtype="bfloat16", device="cuda"):
     from .weights import match_parameters
 
     device = require_gpu(device)
+    sized_by = getattr(cfg, "sized_by", None)
+    if sized_by is not None:       # sizes that only the checkpoint's tensors tell
+        cfg = sized_by({name: tuple(tensor.shape) for name, tensor in tensors.items()})
     spec = cfg.model_spec()
     expected = expected_parameters(spec, cfg.checkpoint_name)
     optional = {"head.weight": "embed.weight"} if spec.tie_word_embeddings else {}

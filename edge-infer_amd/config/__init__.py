@@ -8,6 +8,7 @@ from .zadenex import ZadenexConfig
 from .vafepel import VafepelConfig
 from .gopuzen import GopuzenConfig
 from .dazapel import DazapelConfig
+from .lemotar import LemotarConfig
 from .registry import (Architecture, known_architectures, read_config, register_architecture,
                        resolve_architecture, unregister_architecture)
 
@@ -17,11 +18,12 @@ register_architecture(ZadenexConfig.architecture, ZadenexConfig, model_types=("z
 register_architecture(VafepelConfig.architecture, VafepelConfig, model_types=("vafepel",))
 register_architecture(GopuzenConfig.architecture, GopuzenConfig, model_types=("gopuzen",))
 register_architecture(DazapelConfig.architecture, DazapelConfig, model_types=("dazapel",))
+register_architecture(LemotarConfig.architecture, LemotarConfig, model_types=("lemotar",))
 
 __all__ = [
     "AttentionSpec", "DenseMLPSpec", "GatedDeltaSpec", "GatedMLPSpec", "LayerSpec", "ModelSpec", "NormSpec", "PositionSpec",
     "ScheduleEntry", "default_schedule", "ConfigError", "Qwen3Config", "TiruraxConfig", "ZadenexConfig",
-    "VafepelConfig", "GopuzenConfig", "DazapelConfig", "YarnScaling", "LinearAttentionSpec", "ParallelSpec", "FrequencyScaling", "RoutedMLPSpec", "StateSpaceSpec",
+    "VafepelConfig", "GopuzenConfig", "DazapelConfig", "LemotarConfig", "YarnScaling", "LinearAttentionSpec", "ParallelSpec", "FrequencyScaling", "RoutedMLPSpec", "StateSpaceSpec",
     "LatentAttentionSpec", "LoopSpec", "MatrixMemorySpec", "looped_schedule", "Architecture",
     "known_architectures", "read_config", "register_architecture", "resolve_architecture",
     "unregister_architecture",

@@ -16,9 +16,12 @@ from typing import Optional, Tuple
 @dataclass(frozen=True)
 class NormSpec:
     """kind "rmsnorm": x / sqrt(mean(x^2) + eps) * w; kind "layernorm":
-    (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b, with a weight and a bias."""
+    (x - mean) / sqrt(mean((x - mean)^2) + eps) * w + b, with a weight and a bias.
+    `weight_offset`: what the stored weight is added to (kind "rmsnorm"; 1: a weight stored
+    around zero)."""
     kind: str = "rmsnorm"
     eps: float = 1e-6
+    weight_offset: float = 0.0
 
 
 @dataclass(frozen=True)
@@ -129,6 +132,11 @@ class AttentionSpec:
     # positions behind the newest one that the cache keeps for other runs that read it with a
     # wider mask than this layer's own: None: what the own window and pool need; 0: all
     cache_span: Optional[int] = None
+    # the part has no value projection: its values are the keys as projected, before norm and
+    # rotation
+    values_from_keys: bool = False
+    # c: a scaled score s becomes c tanh(s / c) before a distance term is taken off it
+    softcap: Optional[float] = None
 
     @property
     def q_width(self) -> int:
@@ -270,20 +278,29 @@ class DenseMLPSpec:
 class LatentAttentionSpec:
     """Causal attention whose keys and values are up-projections of one latent vector a
     position, which is all the cache holds besides one rotated key part that every head
-    shares.  Queries pass a normed latent of their own.  A head's query and key are
-    [head_dim unrotated | rot_dim rotated].  See `parts.latent`."""
+    shares.  Queries pass a normed latent of their own, or (`q_rank` 0) are projected directly.  A
+    head's query and key are [head_dim unrotated | rot_dim rotated].  See `parts.latent`."""
     kind: str = "latent_attention"
     n_heads: int = 0
     head_dim: int = 0             # unrotated query/key elements of a head
     rot_dim: int = 0              # rotated elements of a head; the key's are shared by all heads
     value_dim: int = 0
     kv_rank: int = 0              # width of the cached latent
-    q_rank: int = 0               # width of the queries' latent
+    q_rank: int = 0               # width of the queries' latent; 0: queries have none
     scale: Optional[float] = None         # None: 1/sqrt(head_dim + rot_dim)
     norm_eps: float = 1e-6                # eps of the RMS norms of the two latents
     position: PositionSpec = field(default_factory=lambda: PositionSpec(kind="rope_pairs"))
     sink: bool = False            # a learned number per head in the softmax's denominator
-    output_gate: bool = False     # a head's output is multiplied by sigmoid(w_h . x), x the input
+    # True or "head": a head's output is multiplied by sigmoid(w_h . x), x the input; "element":
+    # every element of the concatenated heads by a sigmoid of its own (needs q_rank 0)
+    output_gate: object = False
+    window: Optional[int] = None   # None: every earlier position; w: the last w
+    # the part has no down-projection of keys: every run of it reads the latents and rotated key
+    # parts that another run has cached (its schedule entries never write the cache)
+    shared_kv: bool = False
+    # positions behind the newest one that the cache keeps for other runs that read it with a
+    # wider window than this layer's own: None: what the own window needs; 0: all
+    cache_span: Optional[int] = None
 
     @property
     def q_width(self) -> int:
@@ -332,6 +349,11 @@ class GatedDeltaSpec:
     conv_taps: int = 4            # taps of the causal convolution of q, k and v
     out_norm_eps: float = 1e-6    # eps of the RMS norm of each head's read-out
     unit_eps: float = 1e-6        # q and k become x / sqrt(sum(x^2) + unit_eps) per head
+    # r > 0: a decay per head and key channel from a product of rank r, W_2 (W_1 x), instead of one
+    # per head; the read-out's gate is then a product of rank `gate_rank` as well
+    decay_rank: int = 0
+    gate_rank: int = 0
+    gate_activation: str = "silu"      # of the read-out's gate: "silu" or "sigmoid"
 
     @property
     def qk_width(self) -> int:
@@ -363,6 +385,9 @@ class LayerSpec:
     # the norm on the last sublayer's output and its addition are left to the next layer's first
     # kernel (arrangements that know it)
     defer_output: bool = False
+    # the stream is multiplied by this where a sublayer's output is added to it (arrangements that
+    # know it)
+    stream_scale: float = 1.0
 
 
 @dataclass(frozen=True)

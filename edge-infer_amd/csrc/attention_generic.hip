@@ -22,7 +22,8 @@
 // alone and leaves every row's unnormalised sums, maximum and sum of weights in part_o and
 // part_ml, slice 0 of one, for a kernel that takes them in as one more slice of its own softmax),
 // `keep` (with a window: the keys of the sequence's first `keep` positions stay visible however
-// far back they lie; the walk takes their pages first and then the window's).
+// far back they lie; the walk takes their pages first and then the window's), `cap` (the scaled
+// score s becomes cap tanh(s / cap) before anything is added to it or compared).
 // operators/src/cuda/execution.cu:137-179, runtime/src/qwen.cpp:374-402,
 // split merge: operators/src/cuda/kernels/gather_fa_variable.cu:14-118.
 #include "common.h"
@@ -48,7 +49,7 @@ attn_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pages,
                     float scale, int n_splits, int KH, int values_in_keys,
                     const float* __restrict__ gate, int pool, const T* __restrict__ pool_k,
                     const T* __restrict__ pool_v, const int32_t* __restrict__ pool_table,
-                    int pool_only, int keep) {
+                    int pool_only, int keep, float cap) {
   extern __shared__ float lds[];
   const int DQ = KH * D;                  // width of a query row and of a key as it is met
   float* Qs = lds;                        // [kRows][DQ]
@@ -139,6 +140,7 @@ attn_generic_kernel(const T* __restrict__ q, const T* __restrict__ k_pages,
             const float* qr = Qs + r * DQ;
             const float* kr = Ks + c * (DQ + 1);
             for (int d = 0; d < DQ; ++d) dot += qr[d] * kr[d];
+            if (cap > 0.f) dot = cap * tanhf(dot / cap);
             if (!pooled) dot -= slope * static_cast<float>(pos_r - key);
             s[j] = dot;
             row_max = fmaxf(row_max, dot);
@@ -307,7 +309,7 @@ extern "C" int ei_attention(const void* q, const void* k_pages, const void* v_pa
                             const float* sinks, float scale, int n_splits, int key_heads,
                             int values_in_keys, const float* gate, int pool, const void* pool_k,
                             const void* pool_v, const int32_t* pool_table, int pool_only,
-                            int keep, hipStream_t stream) {
+                            int keep, float cap, hipStream_t stream) {
   EI_REQUIRE(n_items > 0 && N > 0 && nq > 0 && nkv > 0, "attention: sizes must be positive");
   EI_REQUIRE(nq % nkv == 0, "attention: query heads must be a multiple of kv heads");
   EI_REQUIRE(key_heads == 1 || key_heads == nkv,
@@ -326,6 +328,7 @@ extern "C" int ei_attention(const void* q, const void* k_pages, const void* v_pa
   EI_REQUIRE(!pool_only || (pool > 0 && n_splits == 1 && !gate),
              "attention: the pooled entries alone are taken in one slice, without a gate");
   EI_REQUIRE(window >= 0, "attention: negative window");
+  EI_REQUIRE(cap >= 0.f, "attention: negative cap");
   EI_REQUIRE(keep >= 0 && (keep == 0 || chunk == 0), "attention: kept first positions with chunks");
   EI_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pool_k && pool_v && pool_table &&
                                          key_heads == 1 && !values_in_keys)),
@@ -360,14 +363,16 @@ extern "C" int ei_attention(const void* q, const void* k_pages, const void* v_pa
         static_cast<const float*>(v_pages), item_seq, item_row0, item_npos, row_pos, page_table,
         table_width, static_cast<float*>(out), part_o, part_ml, nq, nkv, D, DV, Gb, head_blocks,
         BC, window, chunk, slopes, sinks, scale, n_splits, key_heads, values_in_keys, gate, pool,
-        static_cast<const float*>(pool_k), static_cast<const float*>(pool_v), pool_table, pool_only, keep);
+        static_cast<const float*>(pool_k), static_cast<const float*>(pool_v), pool_table, pool_only, keep,
+        cap);
   } else if (dtype == EI_BF16) {
     attn_generic_kernel<bf16_t><<<grid, kThreads, lds, stream>>>(
         static_cast<const bf16_t*>(q), static_cast<const bf16_t*>(k_pages),
         static_cast<const bf16_t*>(v_pages), item_seq, item_row0, item_npos, row_pos, page_table,
         table_width, static_cast<bf16_t*>(out), part_o, part_ml, nq, nkv, D, DV, Gb, head_blocks,
         BC, window, chunk, slopes, sinks, scale, n_splits, key_heads, values_in_keys, gate, pool,
-        static_cast<const bf16_t*>(pool_k), static_cast<const bf16_t*>(pool_v), pool_table, pool_only, keep);
+        static_cast<const bf16_t*>(pool_k), static_cast<const bf16_t*>(pool_v), pool_table, pool_only, keep,
+        cap);
   } else {
     EI_REQUIRE(false, "attention: unknown dtype");
   }

@@ -133,6 +133,31 @@ __device__ __forceinline__ float gated_product(float gate, float up, const GateA
   return swish<TO>(g, act.alpha) * (u + 1.0f);
 }
 
+// Sine and cosine of an angle given in turns (of 2 pi): the whole turns are taken off in float64.
+// For float32 results the library's functions; for bfloat16 results the hardware's (which take
+// turns), good to about 1e-6 and swallowed by the rounding.
+constexpr double kTurnsPerRadian = 0.15915494309189535;
+template <typename TO> __device__ __forceinline__ void turn_of(double turns, float& sn, float& cs);
+template <> __device__ __forceinline__ void turn_of<float>(double turns, float& sn, float& cs) {
+  sincosf(static_cast<float>((turns - floor(turns)) * 6.283185307179586), &sn, &cs);
+}
+template <> __device__ __forceinline__ void turn_of<bf16_t>(double turns, float& sn, float& cs) {
+  const float part = static_cast<float>(turns - floor(turns));
+  sn = __builtin_amdgcn_sinf(part);
+  cs = __builtin_amdgcn_cosf(part);
+}
+
+// Sine and cosine of position * frequency: for float64 frequencies as above; for float32 ones the
+// angle is the float32 product.
+template <typename TO>
+__device__ __forceinline__ void turn_at(int pos, double freq, float& sn, float& cs) {
+  turn_of<TO>(static_cast<double>(pos) * freq * kTurnsPerRadian, sn, cs);
+}
+template <typename TO>
+__device__ __forceinline__ void turn_at(int pos, float freq, float& sn, float& cs) {
+  sincosf(static_cast<float>(pos) * freq, &sn, &cs);
+}
+
 // Reductions over the four 16-lane rows of a wave (lanes l, l^16, l^32, l^48), every lane
 // getting the result.  gfx950's row-swap instructions do each step in the vector ALU: with
 // both operands holding x, v_permlane32_swap leaves (x of the lower half, x of the upper

@@ -8,14 +8,20 @@
 //   q, k   = x / sqrt(sum(x^2) + unit_eps)   per head; q also times q_scale
 //   beta   = sigmoid(b),  g = exp(-exp(A_log) * softplus(a + dt_bias))
 //   S     <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
-//   out    = o / sqrt(mean(o^2) + eps) * w * silu(gate)
+//   out    = o / sqrt(mean(o^2) + eps) * w * silu(gate)      (or sigmoid(gate))
+//
+// With a decay per key channel g is a vector [D] a head and acts on the rows of S:
+// g = exp(-exp(A_log) * softplus(z + dt_bias)), z [H, D] a product of low rank, z = W_2 (W_1 x),
+// as then are the gate's logits.
 //
 // Per sequence the cache keeps S (stored transposed, [H, DV, D], so that the D values a
 // thread owns are contiguous) and the last J - 1 inputs of every convolved channel.  One
 // set of kernels serves prompts (rows of a sequence are walked in order) and decoding (one
 // row a sequence):
 //
-//   delta_conv   convolution + silu of all q, k, v channels of every row
+//   delta_conv   convolution + silu of all q, k, v channels of every row; with a decay per key
+//                channel also the decays, from the logits of a product of many rows or, for few
+//                rows, from the low-rank part of the projection itself (delta_prepare: one launch)
 //   delta_tail   the new last J - 1 inputs of every sequence (after delta_conv has read the
 //                old ones)
 //   delta_rule   the recurrence; a thread owns 8 or 16 rows of one column of S, L lanes share a
@@ -51,6 +57,28 @@ __device__ __forceinline__ float softplus_f32(float x) {
   return x > 30.f ? x : log1pf(expf(x));
 }
 
+// What makes the decays of H heads x D key channels: rates and biases (float32 [H], [H D]) and the
+// logits z, rows z_row apart (TZ; null: no such decays).  A row's decays follow its C convolved
+// channels in the output.
+struct Decays {
+  const void* z;
+  int z_dtype;
+  size_t z_row;
+  const float* a_log;
+  const float* dt_bias;
+  int HD, D;
+};
+
+__device__ __forceinline__ float decay_of(float z, float a_log, float bias) {
+  return expf(-expf(a_log) * softplus_f32(z + bias));
+}
+
+__device__ __forceinline__ float decay_logit(const Decays& d, size_t row, int i) {
+  const size_t at = row * d.z_row + i;
+  return d.z_dtype == EI_BF16 ? ei::bf16_to_f32(static_cast<const bf16_t*>(d.z)[at])
+                              : static_cast<const float*>(d.z)[at];
+}
+
 // proj: [nsplit][N, WP]; the convolved channels are its first C columns.  conv_w: [C, J].
 // new_tail_state (the state again, or null): a step in which every sequence brings one row
 // may have the tails renewed here (up to kFewTaps taps), which saves the launch of delta_tail.
@@ -58,7 +86,7 @@ __device__ __forceinline__ float softplus_f32(float x) {
 // state + row * state_stride + tail_offset as [J - 1, C]; a sequence's state is read from row
 // seq_in[seq] and written to row seq_out[seq] (the same row, or the other of two versions).
 template <typename TI>
-__global__ void delta_conv_kernel(const TI* __restrict__ proj, int nsplit, size_t split_stride,
+__device__ __forceinline__ void conv_channel(size_t row, int c, const TI* __restrict__ proj, int nsplit, size_t split_stride,
                                   int WP, const float* __restrict__ conv_w, int J,
                                   const float* __restrict__ state, size_t state_stride,
                                   size_t tail_offset, const int32_t* __restrict__ row_pos,
@@ -66,9 +94,7 @@ __global__ void delta_conv_kernel(const TI* __restrict__ proj, int nsplit, size_
                                   const int32_t* __restrict__ seq_in,
                                   const int32_t* __restrict__ seq_out,
                                   const int32_t* __restrict__ seq_start, float* __restrict__ out,
-                                  int C, float* __restrict__ new_tail_state) {
-  const size_t row = blockIdx.x;
-  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+                                  int OW, int C, float* __restrict__ new_tail_state) {
   const int seq = row_seq[row];
   if (seq < 0 || c >= C) return;
   const int pos = row_pos[row], start = seq_start[seq];
@@ -99,14 +125,14 @@ __global__ void delta_conv_kernel(const TI* __restrict__ proj, int nsplit, size_
   } else {
     for (int j = 0; j < J; ++j) acc += conv_w[static_cast<size_t>(c) * J + j] * input(j);
   }
-  out[row * C + c] = silu_f32(acc);
+  out[row * OW + c] = silu_f32(acc);
 }
 
 // The same for four neighbouring channels a thread (channel counts, row widths and slice
 // strides that are multiples of 4, up to kFewTaps taps): 8- or 16-byte loads of the inputs, the
 // filters of four channels as J consecutive 16-byte pieces, one 16-byte store.
 template <typename TI>
-__global__ void delta_conv_vec_kernel(const TI* __restrict__ proj, int nsplit, size_t split_stride,
+__device__ __forceinline__ void conv_quad(size_t row, int c, const TI* __restrict__ proj, int nsplit, size_t split_stride,
                                       int WP, const float* __restrict__ conv_w, int J,
                                       const float* __restrict__ state, size_t state_stride,
                                       size_t tail_offset, const int32_t* __restrict__ row_pos,
@@ -114,10 +140,8 @@ __global__ void delta_conv_vec_kernel(const TI* __restrict__ proj, int nsplit, s
                                       const int32_t* __restrict__ seq_in,
                                       const int32_t* __restrict__ seq_out,
                                       const int32_t* __restrict__ seq_start,
-                                      float* __restrict__ out, int C,
+                                      float* __restrict__ out, int OW, int C,
                                       float* __restrict__ new_tail_state) {
-  const size_t row = blockIdx.x;
-  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
   const int seq = row_seq[row];
   if (seq < 0 || c >= C) return;
   const int pos = row_pos[row], start = seq_start[seq];
@@ -157,12 +181,165 @@ __global__ void delta_conv_vec_kernel(const TI* __restrict__ proj, int nsplit, s
     }
 #pragma unroll
   for (int e = 0; e < 4; ++e) acc[e] = silu_f32(acc[e]);
-  ei::Vec4<float>::store(out + row * C + c, acc);
+  ei::Vec4<float>::store(out + row * OW + c, acc);
   if (new_tail_state) {
     float* to = new_tail_state + static_cast<size_t>(seq_out[seq]) * state_stride + tail_offset;
 #pragma unroll
     for (int j = 1; j < kFewTaps; ++j)
       if (j < J) ei::Vec4<float>::store(to + static_cast<size_t>(j - 1) * C + c, x[j]);
+  }
+}
+
+// A thread a (row, channel), or four channels; channels C .. C + HD - 1 are decays made from their
+// logits.
+template <typename TI>
+__global__ void delta_conv_kernel(const TI* __restrict__ proj, int nsplit, size_t split_stride,
+                                  int WP, const float* __restrict__ conv_w, int J,
+                                  const float* __restrict__ state, size_t state_stride,
+                                  size_t tail_offset, const int32_t* __restrict__ row_pos,
+                                  const int32_t* __restrict__ row_seq,
+                                  const int32_t* __restrict__ seq_in,
+                                  const int32_t* __restrict__ seq_out,
+                                  const int32_t* __restrict__ seq_start, float* __restrict__ out,
+                                  int OW, int C, float* __restrict__ new_tail_state, Decays decays) {
+  const size_t row = blockIdx.x;
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c < C) {
+    conv_channel<TI>(row, c, proj, nsplit, split_stride, WP, conv_w, J, state, state_stride,
+                     tail_offset, row_pos, row_seq, seq_in, seq_out, seq_start, out, OW, C,
+                     new_tail_state);
+  } else if (decays.z && c < C + decays.HD && row_seq[row] >= 0) {
+    const int i = c - C;
+    out[row * OW + c] =
+        decay_of(decay_logit(decays, row, i), decays.a_log[i / decays.D], decays.dt_bias[i]);
+  }
+}
+
+template <typename TI>
+__global__ void delta_conv_vec_kernel(const TI* __restrict__ proj, int nsplit, size_t split_stride,
+                                      int WP, const float* __restrict__ conv_w, int J,
+                                      const float* __restrict__ state, size_t state_stride,
+                                      size_t tail_offset, const int32_t* __restrict__ row_pos,
+                                      const int32_t* __restrict__ row_seq,
+                                      const int32_t* __restrict__ seq_in,
+                                      const int32_t* __restrict__ seq_out,
+                                      const int32_t* __restrict__ seq_start,
+                                      float* __restrict__ out, int OW, int C,
+                                      float* __restrict__ new_tail_state, Decays decays) {
+  const size_t row = blockIdx.x;
+  const int c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
+  if (c < C) {
+    conv_quad<TI>(row, c, proj, nsplit, split_stride, WP, conv_w, J, state, state_stride,
+                  tail_offset, row_pos, row_seq, seq_in, seq_out, seq_start, out, OW, C,
+                  new_tail_state);
+  } else if (decays.z && c < C + decays.HD && row_seq[row] >= 0) {
+    const int i = c - C;
+    float g[4];
+    if (decays.z_dtype == EI_BF16)
+      ei::Vec4<bf16_t>::load(static_cast<const bf16_t*>(decays.z) + row * decays.z_row + i, g);
+    else
+      ei::Vec4<float>::load(static_cast<const float*>(decays.z) + row * decays.z_row + i, g);
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      g[e] = decay_of(g[e], decays.a_log[(i + e) / decays.D], decays.dt_bias[i + e]);
+    ei::Vec4<float>::store(out + row * OW + c, g);
+  }
+}
+
+// The low-rank products of few rows in the convolution's launch.  a_col, g_col: where the two
+// low-rank parts (ra and rg wide) begin in a projection row; wa [ra, HD], wg [rg, GW]: their second
+// matrices, transposed; the decays go behind the convolved channels of `out`, the gate's logits to
+// gate_out [N, GW].  Blocks 0 .. conv_blocks * N - 1 convolve 1,024 (four a thread) or 256 channels
+// of a row; the others make 64 columns of up to 16 rows each: four threads a column with a quarter
+// of every piece of 128 ranks, whose weights are all requested at once, added up through LDS.
+constexpr int kLowRows = 16, kLowK = 128, kLowCols = 64, kLowParts = 4;
+
+struct LowRank {
+  int a_col, ra, g_col, rg, GW;
+  const void* wa;
+  const void* wg;
+  float* gate_out;
+};
+
+template <typename TI, typename TW, bool VEC>
+__global__ void __launch_bounds__(kThreads)
+delta_prepare_kernel(const TI* __restrict__ proj, int nsplit, size_t split_stride, int WP,
+                     const float* __restrict__ conv_w, int J, const float* __restrict__ state,
+                     size_t state_stride, size_t tail_offset, const int32_t* __restrict__ row_pos,
+                     const int32_t* __restrict__ row_seq, const int32_t* __restrict__ seq_in,
+                     const int32_t* __restrict__ seq_out, const int32_t* __restrict__ seq_start,
+                     float* __restrict__ out, int OW, int N, int C,
+                     float* __restrict__ new_tail_state, Decays decays, LowRank low,
+                     int conv_blocks) {
+  __shared__ float xs[kLowRows][kLowK];
+  __shared__ float sums[kLowParts][kLowRows][kLowCols];
+  const int id = blockIdx.x;
+  if (id < conv_blocks * N) {
+    const size_t row = id / conv_blocks;
+    const int at = (id % conv_blocks) * kThreads + threadIdx.x;
+    if constexpr (VEC)
+      conv_quad<TI>(row, at * 4, proj, nsplit, split_stride, WP, conv_w, J, state, state_stride,
+                    tail_offset, row_pos, row_seq, seq_in, seq_out, seq_start, out, OW, C,
+                    new_tail_state);
+    else
+      conv_channel<TI>(row, at, proj, nsplit, split_stride, WP, conv_w, J, state, state_stride,
+                       tail_offset, row_pos, row_seq, seq_in, seq_out, seq_start, out, OW, C,
+                       new_tail_state);
+    return;
+  }
+  const int HD = decays.HD;
+  const int decay_blocks = (HD + kLowCols - 1) / kLowCols;
+  const int gate_blocks = (low.GW + kLowCols - 1) / kLowCols;
+  const int rest = id - conv_blocks * N;
+  const int row0 = rest / (decay_blocks + gate_blocks) * kLowRows;
+  int block = rest % (decay_blocks + gate_blocks);
+  const bool is_decay = block < decay_blocks;
+  if (!is_decay) block -= decay_blocks;
+  const int K = is_decay ? low.ra : low.rg, width = is_decay ? HD : low.GW;
+  const TI* x = proj + (is_decay ? low.a_col : low.g_col);
+  const TW* w = static_cast<const TW*>(is_decay ? low.wa : low.wg);
+  const int col = threadIdx.x % kLowCols, part = threadIdx.x / kLowCols;
+  const int j = block * kLowCols + col, j_safe = min(j, width - 1);
+  const int rows = min(kLowRows, N - row0);
+  constexpr int kQuarter = kLowK / kLowParts;
+  float acc[kLowRows];
+#pragma unroll
+  for (int r = 0; r < kLowRows; ++r) acc[r] = 0.f;
+  for (int k0 = 0; k0 < K; k0 += kLowK) {
+    const int kn = min(kLowK, K - k0);
+    // (every load from a clamped place, so that none waits behind a branch; beyond the tile's end
+    // x holds zeros)
+    TW wv[kQuarter];
+#pragma unroll
+    for (int u = 0; u < kQuarter; ++u)
+      wv[u] = w[static_cast<size_t>(min(k0 + part * kQuarter + u, K - 1)) * width + j_safe];
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < rows * kLowK; idx += kThreads) {
+      const int r = idx / kLowK, k = idx % kLowK;
+      xs[r][k] = k < kn ? slice_sum(x + static_cast<size_t>(row0 + r) * WP + k0 + k, nsplit, split_stride)
+                        : 0.f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < kQuarter; ++u) {
+      const float wu = ei::to_f32<TW>(wv[u]);
+#pragma unroll
+      for (int r = 0; r < kLowRows; ++r)
+        if (r < rows) acc[r] += xs[r][part * kQuarter + u] * wu;
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < kLowRows; ++r) sums[part][r][col] = acc[r];
+  __syncthreads();
+  if (j >= width) return;
+  for (int r = part; r < rows; r += kLowParts) {
+    const size_t row = row0 + r;
+    if (row_seq[row] < 0) continue;
+    const float z = (sums[0][r][col] + sums[1][r][col]) + (sums[2][r][col] + sums[3][r][col]);
+    if (is_decay)
+      out[row * OW + C + j] = decay_of(z, decays.a_log[j / decays.D], decays.dt_bias[j]);
+    else
+      low.gate_out[row * low.GW + j] = z;
   }
 }
 
@@ -229,9 +406,11 @@ __device__ __forceinline__ float group_sum(float v) {
 //   S[., col] <- g S[., col] + k u
 // (o = (g S + k u^T)^T q written out: both dot products are taken from the old S, so their
 // sums over the lanes run side by side and the update is off the read-out's path).
-template <typename TI, int L, int OWN>
+// KD: a decay per key channel, H D of them behind the C channels of a conv row (rows OW apart);
+// S is scaled by them first and both dot products are taken from the scaled S.
+template <typename TI, int L, int OWN, bool KD>
 __global__ void __launch_bounds__(kThreads)
-delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ proj, int nsplit,
+delta_rule_kernel(const float* __restrict__ conv, int OW, int C, const TI* __restrict__ proj, int nsplit,
                   size_t split_stride, int WP, int beta_col, int decay_col,
                   const float* __restrict__ a_log, const float* __restrict__ dt_bias,
                   float* __restrict__ state, size_t state_stride,
@@ -245,6 +424,7 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
   constexpr int PIECES = OWN / 4;         // 16-byte pieces of a thread's rows
   __shared__ __attribute__((aligned(16))) float q_s[TILE][DP];
   __shared__ __attribute__((aligned(16))) float k_s[TILE][DP];
+  __shared__ __attribute__((aligned(16))) float g_s[KD ? TILE : 1][KD ? DP : 4];
   __shared__ float v_s[TILE][CB];
   // per token: decay g, the factor kf that makes k a unit vector, beta kf, the factor qf of q
   // (unit vector times q_scale); and qf (k . q) of the raw vectors
@@ -286,7 +466,7 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
         if (i0 + m < D) s[m] = mine[m];
     }
   }
-  const float rate = expf(a_log[head]), shift = dt_bias[head];
+  const float rate = KD ? 0.f : expf(a_log[head]), shift = KD ? 0.f : dt_bias[head];
 
   // A tile's operands travel global memory -> registers -> LDS, and the registers are filled
   // for tile t + 1 while tile t is walked, so the walk does not wait for memory.  Rows of q, k
@@ -294,16 +474,31 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
   constexpr int QUADS = DP / 4;                          // 16-byte pieces of a padded q or k row
   constexpr int NQ = (TILE * QUADS + kThreads - 1) / kThreads;   // pieces a thread moves per tile
   constexpr int NV = (TILE * CB + kThreads - 1) / kThreads;      // values a thread moves per tile
-  const bool fast = D % 4 == 0 && C % 4 == 0;
-  float4 fq[NQ], fk[NQ];
+  const bool fast = D % 4 == 0 && C % 4 == 0 && OW % 4 == 0;
+  float4 fq[NQ], fk[NQ], fg[KD ? NQ : 1];
   float fv[NV], fb = 0.f, fa = 0.f;
   auto fetch = [&](int t0, int nt) __attribute__((always_inline)) {
 #pragma unroll
     for (int n = 0; n < NQ; ++n) {
       const int idx = tid + n * kThreads, tt = idx / QUADS, i = (idx % QUADS) * 4;
       fq[n] = fk[n] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if constexpr (KD) {
+        fg[n] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (tt < nt && i < D) {
+          const float* g = conv + static_cast<size_t>(row0 + t0 + tt) * OW + C + head * D + i;
+          if (fast) {
+            fg[n] = *reinterpret_cast<const float4*>(g);
+          } else {
+            float a[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int e = 0; e < 4; ++e)
+              if (i + e < D) a[e] = g[e];
+            fg[n] = make_float4(a[0], a[1], a[2], a[3]);
+          }
+        }
+      }
       if (tt < nt && i < D) {
-        const float* src = conv + static_cast<size_t>(row0 + t0 + tt) * C + shared_head * D + i;
+        const float* src = conv + static_cast<size_t>(row0 + t0 + tt) * OW + shared_head * D + i;
         if (fast) {
           fq[n] = *reinterpret_cast<const float4*>(src);
           fk[n] = *reinterpret_cast<const float4*>(src + QK);
@@ -324,12 +519,12 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
     for (int n = 0; n < NV; ++n) {
       const int idx = tid + n * kThreads, tt = idx / CB, cg = blockIdx.z * CB + idx % CB;
       fv[n] = (tt < nt && cg < DV)
-                  ? conv[static_cast<size_t>(row0 + t0 + tt) * C + 2 * QK + head * DV + cg] : 0.f;
+                  ? conv[static_cast<size_t>(row0 + t0 + tt) * OW + 2 * QK + head * DV + cg] : 0.f;
     }
     if (tid < nt) {
       const TI* src = proj + static_cast<size_t>(row0 + t0 + tid) * WP;
       fb = slice_sum(src + beta_col + head, nsplit, split_stride);
-      fa = slice_sum(src + decay_col + head, nsplit, split_stride);
+      if constexpr (!KD) fa = slice_sum(src + decay_col + head, nsplit, split_stride);
     }
   };
   auto commit = [&](int nt) __attribute__((always_inline)) {
@@ -339,6 +534,7 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
       if (tt < TILE) {
         *reinterpret_cast<float4*>(&q_s[tt][i]) = fq[n];
         *reinterpret_cast<float4*>(&k_s[tt][i]) = fk[n];
+        if constexpr (KD) *reinterpret_cast<float4*>(&g_s[tt][i]) = fg[n];
       }
     }
 #pragma unroll
@@ -348,7 +544,7 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
     }
     if (tid < nt) {
       beta_s[tid] = 1.0f / (1.0f + expf(-fb));
-      decay_s[tid] = expf(-rate * softplus_f32(fa + shift));
+      decay_s[tid] = KD ? 1.0f : expf(-rate * softplus_f32(fa + shift));
     }
   };
 
@@ -379,11 +575,12 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
     }
     __syncthreads();
     // the walk: what token tt + 1 needs is read from LDS while token tt is computed
-    float4 kn[PIECES], qn[PIECES];
+    float4 kn[PIECES], qn[PIECES], gn[KD ? PIECES : 1];
 #pragma unroll
     for (int pc = 0; pc < PIECES; ++pc) {
       kn[pc] = *reinterpret_cast<const float4*>(&k_s[0][i0 + 4 * pc]);
       qn[pc] = *reinterpret_cast<const float4*>(&q_s[0][i0 + 4 * pc]);
+      if constexpr (KD) gn[pc] = *reinterpret_cast<const float4*>(&g_s[0][i0 + 4 * pc]);
     }
     float4 cf = coef_s[0];
     float vv = v_s[0][col_in_block], kqv = kq_s[0];
@@ -394,12 +591,20 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
         kv[4 * pc] = kn[pc].x; kv[4 * pc + 1] = kn[pc].y; kv[4 * pc + 2] = kn[pc].z; kv[4 * pc + 3] = kn[pc].w;
         qv[4 * pc] = qn[pc].x; qv[4 * pc + 1] = qn[pc].y; qv[4 * pc + 2] = qn[pc].z; qv[4 * pc + 3] = qn[pc].w;
       }
+      if constexpr (KD) {
+#pragma unroll
+        for (int pc = 0; pc < PIECES; ++pc) {
+          s[4 * pc] *= gn[pc].x; s[4 * pc + 1] *= gn[pc].y;
+          s[4 * pc + 2] *= gn[pc].z; s[4 * pc + 3] *= gn[pc].w;
+        }
+      }
       const float g = cf.x, kf = cf.y, bk = cf.z, qf = cf.w, v_now = vv, kq_now = kqv;
       const int nx = tt + 1 < nt ? tt + 1 : tt;
 #pragma unroll
       for (int pc = 0; pc < PIECES; ++pc) {
         kn[pc] = *reinterpret_cast<const float4*>(&k_s[nx][i0 + 4 * pc]);
         qn[pc] = *reinterpret_cast<const float4*>(&q_s[nx][i0 + 4 * pc]);
+        if constexpr (KD) gn[pc] = *reinterpret_cast<const float4*>(&g_s[nx][i0 + 4 * pc]);
       }
       cf = coef_s[nx];
       vv = v_s[nx][col_in_block];
@@ -416,7 +621,7 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
       const float read = group_sum<L>(read0 + read1) * (g * qf);    // g (S^T q)[col]
       const float u = bk * (v_now - seen);                          // beta (v - seen), times k's factor
 #pragma unroll
-      for (int m = 0; m < OWN; ++m) s[m] = fmaf(s[m], g, kv[m] * u);
+      for (int m = 0; m < OWN; ++m) s[m] = KD ? fmaf(kv[m], u, s[m]) : fmaf(s[m], g, kv[m] * u);
       if (part == 0 && col_ok)
         o_raw[static_cast<size_t>(row0 + t0 + tt) * VW + head * DV + col] = fmaf(u, kq_now, read);
     }
@@ -436,11 +641,12 @@ delta_rule_kernel(const float* __restrict__ conv, int C, const TI* __restrict__ 
   }
 }
 
-// A wave a (row, head), four heads a block: out = o / sqrt(mean(o^2) + eps) * w * silu(gate).
+// A wave a (row, head), four heads a block: out = o / sqrt(mean(o^2) + eps) * w * silu(gate), or
+// sigmoid(gate) for silu.
 template <typename TI, typename TO>
 __global__ void delta_out_kernel(const float* __restrict__ o_raw, const TI* __restrict__ proj,
                                  int nsplit, size_t split_stride, int WP, int gate_col,
-                                 const float* __restrict__ norm_w, float eps,
+                                 int sigmoid_gate, const float* __restrict__ norm_w, float eps,
                                  const int32_t* __restrict__ row_seq, TO* __restrict__ out,
                                  int H, int DV) {
   const size_t row = blockIdx.x;
@@ -460,7 +666,9 @@ __global__ void delta_out_kernel(const float* __restrict__ o_raw, const TI* __re
     const float inv = 1.0f / sqrtf(sq / static_cast<float>(DV) + eps);
     for (int j = lane; j < DV; j += EI_WAVE) {
       const float gt = slice_sum(gate + j, nsplit, split_stride);
-      out[base + j] = ei::from_f32<TO>((o_raw[base + j] * inv) * norm_w[j] * silu_f32(gt));
+      const float open = 1.0f / (1.0f + expf(-gt));
+      out[base + j] = ei::from_f32<TO>((o_raw[base + j] * inv) * norm_w[j] *
+                                       (sigmoid_gate ? open : gt * open));
     }
   }
 }
@@ -473,54 +681,108 @@ int lanes_a_column(int D, int own) {
 
 }  // namespace
 
+// out: rows OW wide that begin with the C convolved channels.  z (or null): the logits of the
+// decays of H D key channels, rows z_row apart; the decays then follow the channels.
 extern "C" int ei_delta_conv(const void* proj, int in_dtype, int nsplit, long long split_stride,
                              int WP, const float* conv_w, int J, const float* state,
                              long long state_stride, long long tail_offset, const int32_t* row_pos,
                              const int32_t* row_seq, const int32_t* seq_in,
-                             const int32_t* seq_out, const int32_t* seq_start, float* out, int N,
-                             int C, int renew_tail, hipStream_t stream) {
+                             const int32_t* seq_out, const int32_t* seq_start, float* out, int OW,
+                             int N, int C, int renew_tail, const void* z, int z_dtype,
+                             long long z_row, const float* a_log, const float* dt_bias, int H, int D,
+                             hipStream_t stream) {
   EI_REQUIRE(proj && conv_w && state && row_pos && row_seq && seq_in && seq_out && seq_start && out,
              "delta_conv: null pointer");
   EI_REQUIRE(!renew_tail || J <= kFewTaps, "delta_conv: the tails are renewed here for up to 8 taps");
   float* renewed = renew_tail ? const_cast<float*>(state) : nullptr;
   EI_REQUIRE(N > 0 && C > 0 && C <= WP && nsplit >= 1, "delta_conv: sizes must be positive");
   EI_REQUIRE(J >= 1 && J <= kMaxTaps, "delta_conv: taps must lie between 1 and 32");
-  EI_REQUIRE((C + kThreads - 1) / kThreads <= 65535, "delta_conv: too many channels");
-  const dim3 grid(N, (C + kThreads - 1) / kThreads);
+  const int HD = z ? H * D : 0;
+  EI_REQUIRE(!z || (a_log && dt_bias && HD > 0 && z_row >= HD && (z_dtype == EI_F32 || z_dtype == EI_BF16)),
+             "delta_conv: decays need their logits, rates and biases");
+  EI_REQUIRE(OW >= C + HD, "delta_conv: the output's rows are too narrow");
+  EI_REQUIRE((C + HD + kThreads - 1) / kThreads <= 65535, "delta_conv: too many channels");
+  const Decays decays{z, z_dtype, static_cast<size_t>(z_row), a_log, dt_bias, HD, D};
+  const dim3 grid(N, (C + HD + kThreads - 1) / kThreads);
   const size_t ss = static_cast<size_t>(split_stride);
-  const bool vec = J <= kFewTaps && C % 4 == 0 && WP % 4 == 0 && ss % 4 == 0 &&
+  const bool vec = J <= kFewTaps && C % 4 == 0 && WP % 4 == 0 && ss % 4 == 0 && OW % 4 == 0 &&
+                   HD % 4 == 0 && (!z || (z_row % 4 == 0 && reinterpret_cast<uintptr_t>(z) % 16 == 0)) &&
                    state_stride % 4 == 0 && tail_offset % 4 == 0 &&
                    (reinterpret_cast<uintptr_t>(proj) | reinterpret_cast<uintptr_t>(out) |
                     reinterpret_cast<uintptr_t>(state)) % 16 == 0;
+#define EI_DCONV(KERNEL, TI, GRID, THREADS)                                                       \
+  KERNEL<TI><<<GRID, THREADS, 0, stream>>>(                                                       \
+      static_cast<const TI*>(proj), nsplit, ss, WP, conv_w, J, state,                             \
+      static_cast<size_t>(state_stride), static_cast<size_t>(tail_offset), row_pos, row_seq,      \
+      seq_in, seq_out, seq_start, out, OW, C, renewed, decays)
   if (vec) {
     const int threads = 64;         // four channels a thread: 256 channels a block
-    const dim3 vgrid(N, (C / 4 + threads - 1) / threads);
-    if (in_dtype == EI_F32)
-      delta_conv_vec_kernel<float><<<vgrid, threads, 0, stream>>>(
-          static_cast<const float*>(proj), nsplit, ss, WP, conv_w, J, state,
-          static_cast<size_t>(state_stride), static_cast<size_t>(tail_offset), row_pos, row_seq,
-          seq_in, seq_out, seq_start, out, C, renewed);
-    else if (in_dtype == EI_BF16)
-      delta_conv_vec_kernel<bf16_t><<<vgrid, threads, 0, stream>>>(
-          static_cast<const bf16_t*>(proj), nsplit, ss, WP, conv_w, J, state,
-          static_cast<size_t>(state_stride), static_cast<size_t>(tail_offset), row_pos, row_seq,
-          seq_in, seq_out, seq_start, out, C, renewed);
-    else
-      EI_REQUIRE(false, "delta_conv: unknown dtype");
+    const dim3 vgrid(N, ((C + HD) / 4 + threads - 1) / threads);
+    if (in_dtype == EI_F32) EI_DCONV(delta_conv_vec_kernel, float, vgrid, threads);
+    else if (in_dtype == EI_BF16) EI_DCONV(delta_conv_vec_kernel, bf16_t, vgrid, threads);
+    else EI_REQUIRE(false, "delta_conv: unknown dtype");
     EI_LAUNCH_CHECK();
   }
-  if (in_dtype == EI_F32)
-    delta_conv_kernel<float><<<grid, kThreads, 0, stream>>>(
-        static_cast<const float*>(proj), nsplit, ss, WP, conv_w, J, state,
-        static_cast<size_t>(state_stride), static_cast<size_t>(tail_offset), row_pos, row_seq,
-        seq_in, seq_out, seq_start, out, C, renewed);
-  else if (in_dtype == EI_BF16)
-    delta_conv_kernel<bf16_t><<<grid, kThreads, 0, stream>>>(
-        static_cast<const bf16_t*>(proj), nsplit, ss, WP, conv_w, J, state,
-        static_cast<size_t>(state_stride), static_cast<size_t>(tail_offset), row_pos, row_seq,
-        seq_in, seq_out, seq_start, out, C, renewed);
-  else
-    EI_REQUIRE(false, "delta_conv: unknown dtype");
+  if (in_dtype == EI_F32) EI_DCONV(delta_conv_kernel, float, grid, kThreads);
+  else if (in_dtype == EI_BF16) EI_DCONV(delta_conv_kernel, bf16_t, grid, kThreads);
+  else EI_REQUIRE(false, "delta_conv: unknown dtype");
+#undef EI_DCONV
+  EI_LAUNCH_CHECK();
+}
+
+// The convolution as above and, in the same launch, the decays [N, H D] behind its channels and the
+// gate's logits gate_out [N, GW], from the low-rank columns a_col .. a_col + ra - 1 and g_col ..
+// g_col + rg - 1 of the projection's float32 rows (or slices) and wa [ra, H D], wg [rg, GW] of
+// w_dtype.
+extern "C" int ei_delta_prepare(const float* proj, int nsplit, long long split_stride,
+                                int WP, const float* conv_w, int J, const float* state,
+                                long long state_stride, long long tail_offset,
+                                const int32_t* row_pos, const int32_t* row_seq,
+                                const int32_t* seq_in, const int32_t* seq_out,
+                                const int32_t* seq_start, float* out, int OW, int N, int C,
+                                int renew_tail, const float* a_log, const float* dt_bias, int H,
+                                int D, const void* wa, const void* wg, int w_dtype, int a_col,
+                                int ra, int g_col, int rg, int GW, float* gate_out,
+                                hipStream_t stream) {
+  EI_REQUIRE(proj && conv_w && state && row_pos && row_seq && seq_in && seq_out && seq_start && out &&
+                 a_log && dt_bias && wa && wg && gate_out,
+             "delta_prepare: null pointer");
+  EI_REQUIRE(!renew_tail || J <= kFewTaps, "delta_prepare: the tails are renewed here for up to 8 taps");
+  EI_REQUIRE(N > 0 && C > 0 && C <= WP && nsplit >= 1 && H > 0 && D > 0 && GW > 0 && ra > 0 && rg > 0,
+             "delta_prepare: sizes must be positive");
+  EI_REQUIRE(a_col >= 0 && g_col >= 0 && a_col + ra <= WP && g_col + rg <= WP,
+             "delta_prepare: low-rank columns outside the row");
+  EI_REQUIRE(J >= 1 && J <= kMaxTaps, "delta_prepare: taps must lie between 1 and 32");
+  EI_REQUIRE(OW >= C + H * D, "delta_prepare: the output's rows are too narrow");
+  float* renewed = renew_tail ? const_cast<float*>(state) : nullptr;
+  const size_t ss = static_cast<size_t>(split_stride);
+  const bool vec = J <= kFewTaps && C % 4 == 0 && WP % 4 == 0 && ss % 4 == 0 && OW % 4 == 0 &&
+                   state_stride % 4 == 0 && tail_offset % 4 == 0 &&
+                   (reinterpret_cast<uintptr_t>(proj) | reinterpret_cast<uintptr_t>(out) |
+                    reinterpret_cast<uintptr_t>(state)) % 16 == 0;
+  const int a_block = vec ? kThreads * 4 : kThreads;
+  const int conv_blocks = (C + a_block - 1) / a_block;
+  const Decays decays{nullptr, EI_F32, 0, a_log, dt_bias, H * D, D};
+  const LowRank low{a_col, ra, g_col, rg, GW, wa, wg, gate_out};
+  const long long low_blocks = static_cast<long long>((N + kLowRows - 1) / kLowRows) *
+                               ((H * D + kLowCols - 1) / kLowCols + (GW + kLowCols - 1) / kLowCols);
+  const long long blocks = static_cast<long long>(conv_blocks) * N + low_blocks;
+  EI_REQUIRE(blocks < (1ll << 31), "delta_prepare: too many rows");
+#define EI_DPREP(TW, VV)                                                                          \
+  delta_prepare_kernel<float, TW, VV><<<static_cast<unsigned>(blocks), kThreads, 0, stream>>>(    \
+      proj, nsplit, ss, WP, conv_w, J, state, static_cast<size_t>(state_stride),                  \
+      static_cast<size_t>(tail_offset), row_pos, row_seq, seq_in, seq_out, seq_start, out, OW, N, \
+      C, renewed, decays, low, conv_blocks)
+  if (w_dtype == EI_F32) {
+    if (vec) EI_DPREP(float, true);
+    else EI_DPREP(float, false);
+  } else if (w_dtype == EI_BF16) {
+    if (vec) EI_DPREP(bf16_t, true);
+    else EI_DPREP(bf16_t, false);
+  } else {
+    EI_REQUIRE(false, "delta_prepare: unknown dtype");
+  }
+#undef EI_DPREP
   EI_LAUNCH_CHECK();
 }
 
@@ -550,10 +812,12 @@ extern "C" int ei_delta_tail(const void* proj, int in_dtype, int nsplit, long lo
   EI_LAUNCH_CHECK();
 }
 
-// conv [N, 2 G D + H DV] float32; proj as above with the beta and decay projections (H
-// columns each) at beta_col and decay_col; o_raw [N, H DV] float32.  n_seqs blocks walk
+// conv [N, OW] float32, rows that begin with the 2 G D + H DV convolved channels; proj as above with
+// the beta and decay projections (H columns each) at beta_col and decay_col; key_decay: H D decays
+// follow the channels of a conv row instead (decay_col, a_log and dt_bias are then not read);
+// o_raw [N, H DV] float32.  n_seqs blocks walk
 // seq_count rows each from seq_row0.
-extern "C" int ei_delta_rule(const float* conv, const void* proj, int in_dtype, int nsplit,
+extern "C" int ei_delta_rule(const float* conv, int OW, int key_decay, const void* proj, int in_dtype, int nsplit,
                              long long split_stride, int WP, int beta_col, int decay_col,
                              const float* a_log, const float* dt_bias, float* state,
                              long long state_stride, const int32_t* seq_in,
@@ -561,11 +825,12 @@ extern "C" int ei_delta_rule(const float* conv, const void* proj, int in_dtype, 
                              const int32_t* seq_row0, float* o_raw,
                              int n_seqs, int H, int G, int D, int DV, float q_scale,
                              float unit_eps, hipStream_t stream) {
-  EI_REQUIRE(conv && proj && a_log && dt_bias && state && seq_in && seq_out && seq_count && seq_row0 && o_raw,
+  EI_REQUIRE(conv && proj && (key_decay || (a_log && dt_bias)) && state && seq_in && seq_out && seq_count && seq_row0 && o_raw,
              "delta_rule: null pointer");
   EI_REQUIRE(n_seqs > 0 && H > 0 && G > 0 && H % G == 0 && DV > 0, "delta_rule: bad head counts");
   EI_REQUIRE(D >= 1 && D <= 256, "delta_rule: the key size must lie between 1 and 256");
-  EI_REQUIRE(beta_col >= 0 && decay_col >= 0 && beta_col + H <= WP && decay_col + H <= WP,
+  EI_REQUIRE(beta_col >= 0 && beta_col + H <= WP &&
+                 (key_decay || (decay_col >= 0 && decay_col + H <= WP)),
              "delta_rule: projection columns outside the row");
   // Rows of a column that a thread owns: 8 or 16.  What a token costs a wave beside its FMAs
   // (two sums over the lanes, operand reads, the read-out's store) does not grow with them, so
@@ -589,19 +854,21 @@ extern "C" int ei_delta_rule(const float* conv, const void* proj, int in_dtype, 
   const int L = lanes_a_column(D, own);
   const int CB = kThreads / L;
   const int C = 2 * G * D + H * DV;
+  EI_REQUIRE(OW >= C + (key_decay ? H * D : 0), "delta_rule: conv rows too narrow");
   EI_REQUIRE(H <= 65535 && (DV + CB - 1) / CB <= 65535, "delta_rule: too many heads or columns");
   dim3 grid(n_seqs, H, (DV + CB - 1) / CB);
   const size_t ss = static_cast<size_t>(split_stride);
-#define EI_DELTA(TI, LL, OO)                                                                    \
-  delta_rule_kernel<TI, LL, OO><<<grid, kThreads, 0, stream>>>(                                 \
-      conv, C, static_cast<const TI*>(proj), nsplit, ss, WP, beta_col, decay_col, a_log, dt_bias, \
-      state, static_cast<size_t>(state_stride), seq_in, seq_out, seq_count, seq_row0, o_raw, H, \
-      G, D,                                                                                     \
-      DV, q_scale, unit_eps)
-#define EI_DELTA_O(TI, LL)                         \
-  do {                                             \
-    if (own == 8) EI_DELTA(TI, LL, 8);             \
-    else EI_DELTA(TI, LL, 16);                     \
+#define EI_DELTA(TI, LL, OO, KK)                                                                \
+  delta_rule_kernel<TI, LL, OO, KK><<<grid, kThreads, 0, stream>>>(                             \
+      conv, OW, C, static_cast<const TI*>(proj), nsplit, ss, WP, beta_col, decay_col, a_log,    \
+      dt_bias, state, static_cast<size_t>(state_stride), seq_in, seq_out, seq_count, seq_row0,  \
+      o_raw, H, G, D, DV, q_scale, unit_eps)
+#define EI_DELTA_O(TI, LL)                                  \
+  do {                                                      \
+    if (own == 8 && key_decay) EI_DELTA(TI, LL, 8, true);   \
+    else if (own == 8) EI_DELTA(TI, LL, 8, false);          \
+    else if (key_decay) EI_DELTA(TI, LL, 16, true);         \
+    else EI_DELTA(TI, LL, 16, false);                       \
   } while (0)
 #define EI_DELTA_L(TI)                                                  \
   do {                                                                  \
@@ -610,7 +877,8 @@ extern "C" int ei_delta_rule(const float* conv, const void* proj, int in_dtype, 
     else if (L == 4) EI_DELTA_O(TI, 4);                                 \
     else if (L == 8) EI_DELTA_O(TI, 8);                                 \
     else if (L == 16) EI_DELTA_O(TI, 16);                               \
-    else EI_DELTA(TI, 32, 8);                                           \
+    else if (key_decay) EI_DELTA(TI, 32, 8, true);                      \
+    else EI_DELTA(TI, 32, 8, false);                                    \
   } while (0)
   if (in_dtype == EI_F32) EI_DELTA_L(float);
   else if (in_dtype == EI_BF16) EI_DELTA_L(bf16_t);
@@ -621,9 +889,11 @@ extern "C" int ei_delta_rule(const float* conv, const void* proj, int in_dtype, 
   EI_LAUNCH_CHECK();
 }
 
+// proj: [nsplit] slices of rows WP wide whose gate logits begin at gate_col; sigmoid_gate: the gate
+// is their sigmoid, not their silu.
 extern "C" int ei_delta_out(const float* o_raw, const void* proj, int in_dtype, int nsplit,
-                            long long split_stride, int WP, int gate_col, const float* norm_w,
-                            float eps, const int32_t* row_seq, void* out, int out_dtype, int N,
+                            long long split_stride, int WP, int gate_col, int sigmoid_gate,
+                            const float* norm_w, float eps, const int32_t* row_seq, void* out, int out_dtype, int N,
                             int H, int DV, hipStream_t stream) {
   EI_REQUIRE(o_raw && proj && norm_w && row_seq && out, "delta_out: null pointer");
   EI_REQUIRE(N > 0 && H > 0 && DV > 0 && nsplit >= 1, "delta_out: sizes must be positive");
@@ -633,7 +903,7 @@ extern "C" int ei_delta_out(const float* o_raw, const void* proj, int in_dtype, 
   const size_t ss = static_cast<size_t>(split_stride);
 #define EI_DOUT(TI, TO)                                                                      \
   delta_out_kernel<TI, TO><<<dim3(N, (H + 3) / 4), kThreads, 0, stream>>>(                   \
-      o_raw, static_cast<const TI*>(proj), nsplit, ss, WP, gate_col, norm_w, eps, row_seq,   \
+      o_raw, static_cast<const TI*>(proj), nsplit, ss, WP, gate_col, sigmoid_gate, norm_w, eps, row_seq, \
       static_cast<TO*>(out), H, DV)
   if (in_dtype == EI_F32 && out_dtype == EI_F32) EI_DOUT(float, float);
   else if (in_dtype == EI_F32 && out_dtype == EI_BF16) EI_DOUT(float, bf16_t);

@@ -58,10 +58,11 @@ _SIGNATURES = {
                           c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int,
                           c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_longlong,
                           c_void_p, c_float, c_int, c_void_p],
-        "ei_projection_norm_store": [c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p, c_void_p,
-                                     c_float, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
-                                     c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                                     c_int, c_void_p],
+        "ei_projection_norm_store": [c_void_p, c_int, c_int, c_longlong, c_longlong, c_void_p,
+                                     c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
+                                     c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                                     c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_float,
+                                     c_void_p],
     },
     "ssm": {
         "ei_ssm_state_floats": [c_int, c_int, c_int, c_int, c_int],
@@ -82,6 +83,8 @@ _SIGNATURES = {
                            c_int, c_int, c_void_p],
         "ei_norm_mean": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_float,
                          c_void_p, c_int, c_int, c_void_p],
+        "ei_post_norm": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_float,
+                         c_float, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     },
     "input_conv": {
         "ei_input_conv": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p,
@@ -116,15 +119,21 @@ _SIGNATURES = {
     "delta_rule": {
         "ei_delta_conv": [c_void_p, c_int, c_int, c_longlong, c_int, c_void_p, c_int, c_void_p,
                           c_longlong, c_longlong, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                          c_void_p, c_int, c_int, c_int, c_void_p],
+                          c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_longlong,
+                          c_void_p, c_void_p, c_int, c_int, c_void_p],
+        "ei_delta_prepare": [c_void_p, c_int, c_longlong, c_int, c_void_p, c_int, c_void_p,
+                             c_longlong, c_longlong, c_void_p, c_void_p, c_void_p, c_void_p,
+                             c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p,
+                             c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                             c_int, c_void_p, c_void_p],
         "ei_delta_tail": [c_void_p, c_int, c_int, c_longlong, c_int, c_int, c_void_p, c_longlong,
                           c_longlong, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int,
                           c_void_p],
-        "ei_delta_rule": [c_void_p, c_void_p, c_int, c_int, c_longlong, c_int, c_int, c_int,
+        "ei_delta_rule": [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_longlong, c_int, c_int, c_int,
                           c_void_p, c_void_p, c_void_p, c_longlong, c_void_p, c_void_p, c_void_p,
                           c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_float,
                           c_void_p],
-        "ei_delta_out": [c_void_p, c_void_p, c_int, c_int, c_longlong, c_int, c_int, c_void_p,
+        "ei_delta_out": [c_void_p, c_void_p, c_int, c_int, c_longlong, c_int, c_int, c_int, c_void_p,
                          c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
     },
     "attention_generic": {
@@ -134,7 +143,7 @@ _SIGNATURES = {
                          c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                          c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float,
                          c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
-                         c_int, c_void_p],
+                         c_int, c_float, c_void_p],
         "ei_pool_store": [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                           c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
                           c_void_p],
@@ -148,15 +157,19 @@ _SIGNATURES = {
                               c_int, c_int, c_void_p, c_void_p],
     },
     "head_ops": {
-        "ei_latent_down_store": [c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p, c_float,
-                                 c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
-                                 c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                 c_void_p],
+        "ei_latent_down_store": [c_void_p, c_int, c_int, c_longlong, c_longlong, c_void_p, c_void_p,
+                                 c_float, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p,
+                                 c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
+                                 c_int, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_longlong,
+                                 c_int, c_void_p],
         "ei_head_matmul": [c_void_p, c_int, c_int, c_longlong, c_longlong, c_int, c_int, c_void_p,
                            c_int, c_void_p, c_int, c_longlong, c_int, c_int, c_int, c_int, c_int,
-                           c_int, c_void_p],
+                           c_int, c_void_p, c_int, c_int, c_longlong, c_longlong, c_void_p],
+        "ei_heads_to_rows": [c_void_p, c_int, c_void_p, c_longlong, c_int, c_int, c_int, c_int,
+                             c_void_p, c_longlong, c_void_p, c_longlong, c_int, c_int, c_void_p,
+                             c_float, c_void_p, c_void_p],
         "ei_rotate_pairs": [c_void_p, c_int, c_int, c_longlong, c_longlong, c_int, c_int, c_void_p,
-                            c_void_p, c_void_p, c_int, c_longlong, c_int, c_int, c_int, c_int,
+                            c_int, c_float, c_void_p, c_void_p, c_int, c_longlong, c_int, c_int, c_int, c_int,
                             c_int, c_void_p],
         "ei_mix_heads": [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int,
                          c_void_p],
@@ -197,6 +210,17 @@ _SIGNATURES = {
                                            c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                            c_int, c_int, c_int, c_int, c_float, c_int, c_int,
                                            c_int, c_void_p, c_void_p],
+    },
+    "attention_capped": {
+        "ei_attention_prefill_capped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                        c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int,
+                                        c_int, c_int, c_float, c_int, c_int, c_int, c_void_p,
+                                        c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_void_p],
+        "ei_attention_decode_capped": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                       c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
+                                       c_int, c_int, c_float, c_int, c_int, c_int, c_void_p, c_int,
+                                       c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float,
+                                       c_void_p],
     },
     "gemm_f32": {
         "ei_gemm_f32": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_longlong, c_longlong,
@@ -325,6 +349,48 @@ def _splits(tensor: torch.Tensor, rows: int, width: int, name: str):
         return tensor.shape[0], rows * width
     raise KernelError(f"{name} must be [{rows}, {width}] or [splits, {rows}, {width}], "
                       f"got {list(tensor.shape)}")
+
+
+class Columns:
+    """Columns first .. first + width - 1 of rows [rows, w] or of float32 slices [slices, rows, w]:
+    a part's share of a product that several parts read."""
+
+    def __init__(self, rows: torch.Tensor, first: int, width: int):
+        if not 0 <= first <= first + width <= rows.shape[-1]:
+            raise KernelError(f"columns {first} .. {first + width - 1} of rows of {rows.shape[-1]}")
+        self.rows, self.first, self.width = rows, int(first), int(width)
+
+    @property
+    def dtype(self):
+        return self.rows.dtype
+
+    def dim(self):
+        return self.rows.dim()
+
+
+def _columns(x, rows: int, width: int, name: str):
+    """(pointer, dtype code, nsplit, slice stride, row stride) of [rows, width], of float32 slices
+    of it, or of `Columns` of that width."""
+    if isinstance(x, Columns):
+        if x.width != width:
+            raise KernelError(f"{name} must be {width} columns, got {x.width}")
+        held = x.rows
+        nsplit, stride = _splits(held, rows, held.shape[-1], name)
+        return (_gpu(held, name) + x.first * held.element_size(), _code(held, name), nsplit, stride,
+                held.shape[-1])
+    nsplit, stride = _splits(x, rows, width, name)
+    return _gpu(x, name), _code(x, name), nsplit, stride, width
+
+
+def _frequencies(frequencies, pairs: int, name: str):
+    """(pointer, whether float64) of one frequency a rotated pair; (None, 0) without pairs."""
+    if not pairs:
+        return None, 0
+    if frequencies is None or frequencies.numel() != pairs:
+        raise KernelError(f"{name}: one frequency for every rotated pair")
+    if frequencies.dtype not in (torch.float32, torch.float64):
+        raise KernelError(f"{name}: frequencies must be float32 or float64")
+    return _gpu(frequencies, "frequencies"), int(frequencies.dtype == torch.float64)
 
 
 # ---------------------------------------------------------------------------
@@ -611,7 +677,8 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
               page_table, out, n_heads, n_kv_heads, head_dim, window=None, scale=None,
               n_splits=1, part_o=None, part_ml=None, value_dim=None, chunk=None, slopes=None,
               sinks=None, key_heads=1, values_in_keys=False, gate=None, pool=None,
-              pool_k=None, pool_v=None, pool_table=None, pool_only=False, keep_first=0) -> None:
+              pool_k=None, pool_v=None, pool_table=None, pool_only=False, keep_first=0,
+              softcap=None) -> None:
     """Generic causal attention over the paged cache (see attention_generic.hip).
     value_dim: head size of the values and of `out` (None: head_dim); chunk: a query sees only
     the keys of its own block of that many positions; slopes, sinks: float32 [n_heads], the
@@ -626,8 +693,11 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
     pool_only: the tokens are left out; `out` is not written, and part_o [rows, heads,
     value_dim] and part_ml [rows, heads, 2] receive every row's unnormalised sums over the
     pooled entries, the largest score and the sum of weights (n_splits 1).  keep_first: with a
-    window, the keys of the sequence's first positions that stay visible however far back."""
+    window, the keys of the sequence's first positions that stay visible however far back.
+    softcap c: a scaled score s becomes c tanh(s / c)."""
     lib = library("attention_generic")
+    if softcap is not None and not softcap > 0:
+        raise KernelError("attention: a cap on the scores must be positive")
     n = q.shape[0]
     value_dim = head_dim if value_dim is None else int(value_dim)
     key_heads = int(key_heads)
@@ -689,7 +759,7 @@ def attention(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_
         None if gate is None else _gpu(gate, "gate", torch.float32), int(pool or 0),
         _gpu(pool_k, "pool_k") if pool else None, _gpu(pool_v, "pool_v") if pool else None,
         _gpu(pool_table, "pool_table", torch.int32) if pool else None, int(bool(pool_only)),
-        int(keep_first) if window else 0, _stream())
+        int(keep_first) if window else 0, float(softcap or 0.0), _stream())
     _check(lib, status, "attention")
 
 
@@ -800,47 +870,77 @@ def _rows_of(x, name):
 
 def latent_down_store(proj, q_norm_w, c_norm_w, eps, frequencies, row_pos, row_seq, page_table,
                       q_latent, k_pages, gate_out, q_rank, kv_rank, rot_dim, n_gate,
-                      write_cache=True) -> None:
-    """One row of a fused down-projection [q_rank | kv_rank | rot_dim | n_gate]: the first two
+                      write_cache=True, turn_scale=1.0, turns=None) -> None:
+    """One row of a fused down-projection [q_rank | kv_rank | rot_dim | n_gate] (or those `Columns`
+    of a larger one): the first two
     parts are RMS-normed with their weights; the queries' latent goes to `q_latent` [rows,
     q_rank], the keys' latent and the rotated last part (neighbouring pairs, angle position *
-    frequencies[i]) to the row's cache page `k_pages` [pages, 1, 64, kv_rank + rot_dim], the gate
-    logits to `gate_out` float32 [rows, n_gate]."""
+    frequencies[i], cosine and sine times turn_scale) to the row's cache page `k_pages` [pages, 1,
+    64, kv_rank + rot_dim], the gate logits to `gate_out` float32 [rows, n_gate].  q_rank 0: the
+    queries have no latent.  turns (first column, heads, columns between heads, out [rows, w],
+    first place, places between heads): the queries' rotated parts lie in the same rows as `proj`
+    and go to `out` in the same launch; kv_rank 0: that is all the launch does (`rot_dim` is then
+    the width of a head's rotated part)."""
     lib = library("head_ops")
-    n, width, nsplit, stride = _rows_of(proj, "proj")
-    if width != q_rank + kv_rank + rot_dim + n_gate:
-        raise KernelError("latent_down_store: the projection's width does not fit its parts")
-    if tuple(q_latent.shape) != (n, q_rank):
-        raise KernelError("latent_down_store: q_latent must be [rows, q_rank]")
-    if q_norm_w.numel() != q_rank or c_norm_w.numel() != kv_rank:
+    width = (q_rank + kv_rank + rot_dim + n_gate) if kv_rank else 0
+    held = proj.rows if isinstance(proj, Columns) else proj
+    n = held.shape[-2]
+    if kv_rank:
+        pointer, code, nsplit, stride, row_stride = _columns(proj, n, width, "proj")
+    else:
+        if turns is None or q_rank or n_gate or write_cache:
+            raise KernelError("latent_down_store: without a latent there are only rotated queries")
+        nsplit, stride = _splits(held, n, held.shape[-1], "proj")
+        pointer, code, row_stride = _gpu(held, "proj"), _code(held, "proj"), held.shape[-1]
+    if q_rank and (tuple(q_latent.shape) != (n, q_rank) or q_norm_w.numel() != q_rank):
+        raise KernelError("latent_down_store: q_latent must be [rows, q_rank], its norm as wide")
+    if kv_rank and c_norm_w.numel() != kv_rank:
         raise KernelError("latent_down_store: norm weights must be as wide as the latents")
-    if rot_dim and (frequencies is None or frequencies.numel() != rot_dim // 2):
-        raise KernelError("latent_down_store: one frequency for every rotated pair")
+    freq, freq_double = _frequencies(frequencies, rot_dim // 2, "latent_down_store")
     if n_gate and (gate_out is None or gate_out.numel() < n * n_gate):
         raise KernelError("latent_down_store: gate_out must be float32 [rows, n_gate]")
     if row_pos.numel() < n or row_seq.numel() < n:
         raise KernelError("latent_down_store: row metadata shorter than the rows")
+    turn_args = (None, 0, 0, None, 0, 0)
+    out_code = None
+    if turns is not None:
+        first, heads, apart, out, place, places = turns
+        if not 0 <= first <= held.shape[-1] - ((heads - 1) * apart + rot_dim):
+            raise KernelError("latent_down_store: the queries' columns lie outside their rows")
+        if out.dim() != 2 or out.shape[0] != n or place < 0 or \
+                place + (heads - 1) * places + rot_dim > out.shape[1]:
+            raise KernelError("latent_down_store: the rotated queries lie outside their rows")
+        turn_args = (_gpu(held, "proj") + first * held.element_size(), int(heads), int(apart),
+                     _gpu(out, "turned") + place * out.element_size(), out.shape[1], int(places))
+        out_code = _code(out, "turned")
+    if q_rank:
+        out_code = _code(q_latent, "q_latent")
     if write_cache:
         if tuple(k_pages.shape[1:]) != (1, PAGE_TOKENS, kv_rank + rot_dim):
             raise KernelError("latent_down_store: pages must be [*, 1, 64, kv_rank + rot_dim]")
-        if k_pages.dtype != q_latent.dtype:
-            raise KernelError("latent_down_store: cache and q_latent dtypes differ")
+        if out_code is not None and _code(k_pages, "k_pages") != out_code:
+            raise KernelError("latent_down_store: the cache's and the queries' dtypes differ")
+        out_code = _code(k_pages, "k_pages")
+    if out_code is None:
+        raise KernelError("latent_down_store: nothing to write")
     status = lib.ei_latent_down_store(
-        _gpu(proj, "proj"), _code(proj, "proj"), nsplit, stride,
-        _gpu(q_norm_w, "q_norm_w", torch.float32), _gpu(c_norm_w, "c_norm_w", torch.float32),
-        float(eps), None if frequencies is None else _gpu(frequencies, "frequencies", torch.float32),
+        pointer, code, nsplit, stride, row_stride,
+        _gpu(q_norm_w, "q_norm_w", torch.float32) if q_rank else None,
+        _gpu(c_norm_w, "c_norm_w", torch.float32) if kv_rank else None,
+        float(eps), freq, freq_double, float(turn_scale),
         _gpu(row_pos, "row_pos", torch.int32), _gpu(row_seq, "row_seq", torch.int32),
         _gpu(page_table, "page_table", torch.int32), page_table.shape[-1],
-        _gpu(q_latent, "q_latent"), _gpu(k_pages, "k_pages") if write_cache else None,
+        _gpu(q_latent, "q_latent") if q_rank else None,
+        _gpu(k_pages, "k_pages") if write_cache else None,
         None if gate_out is None else _gpu(gate_out, "gate_out", torch.float32),
-        _code(q_latent, "q_latent"), n, q_rank, kv_rank, rot_dim, n_gate, int(write_cache),
-        _stream())
+        out_code, n, q_rank, kv_rank, rot_dim, n_gate, int(write_cache), *turn_args, _stream())
     _check(lib, status, "latent_down_store")
 
 
-def head_matmul(x, matrices, y, heads, x_head, x_first, y_head, y_first) -> None:
+def head_matmul(x, matrices, y, heads, x_head, x_first, y_head, y_first, gate=None) -> None:
     """y[n, h * y_head + y_first + j] = sum_i x[n, h * x_head + x_first + i] * matrices[h, i, j]
-    for matrices [heads, K, J] of the storage type; x [rows, width] or float32 slices of it."""
+    for matrices [heads, K, J] of the storage type; x [rows, width] or float32 slices of it.
+    gate: `Columns` [heads * J]; the element is multiplied by the sigmoid of its column h * J + j."""
     lib = library("head_ops")
     n, x_row, nsplit, stride = _rows_of(x, "x")
     if matrices.dim() != 3 or matrices.shape[0] != heads:
@@ -848,25 +948,65 @@ def head_matmul(x, matrices, y, heads, x_head, x_first, y_head, y_first) -> None
     if y.dim() != 2 or y.shape[0] != n:
         raise KernelError("head_matmul: y must be [rows, width]")
     _, k, j = matrices.shape
+    gate_args = (None, F32, 1, 0, 0)
+    if gate is not None:
+        gate_args = _columns(gate, n, heads * j, "gate")
     status = lib.ei_head_matmul(_gpu(x, "x"), _code(x, "x"), nsplit, stride, x_row, int(x_head),
                                 int(x_first), _gpu(matrices, "matrices"),
                                 _code(matrices, "matrices"), _gpu(y, "y"), _code(y, "y"),
-                                y.shape[1], int(y_head), int(y_first), n, heads, k, j, _stream())
+                                y.shape[1], int(y_head), int(y_first), n, heads, k, j, *gate_args,
+                                _stream())
     _check(lib, status, "head_matmul")
 
 
+def heads_to_rows(made, y, y_head, gate=None, turns=None, frequencies=None, turn_scale=1.0,
+                  row_pos=None) -> None:
+    """y[n, h * y_head + j] = made[h, n, j] for made [heads, rows, J] (J even) of y's type.  gate:
+    `Columns` [heads * J] of that type, whose sigmoid the elements are multiplied by.  turns (rows
+    [n, w] of that type, first column, columns between heads): every head's J elements are followed
+    by its rotated part, neighbouring pairs turned by row_pos[n] * frequencies[i] (float64)."""
+    lib = library("head_ops")
+    heads, n, j = made.shape
+    if y.dim() != 2 or y.shape[0] != n or y.dtype != made.dtype or j % 2:
+        raise KernelError("heads_to_rows: y must be [rows, width] of made's type, J even")
+    gate_args = (None, 0)
+    if gate is not None:
+        pointer, code, nsplit, _, row_stride = _columns(gate, n, heads * j, "gate")
+        if nsplit != 1 or code != _code(made, "made"):
+            raise KernelError("heads_to_rows: the gate must be one row of made's type a row")
+        gate_args = (pointer, row_stride)
+    turn_args = (None, 0, 0, 0, None, 1.0, None)
+    if turns is not None:
+        rows, first, apart = turns
+        rotated = 2 * frequencies.numel()
+        if rows.dim() != 2 or rows.shape[0] != n or rows.dtype != made.dtype or \
+                not 0 <= first <= rows.shape[1] - ((heads - 1) * apart + rotated):
+            raise KernelError("heads_to_rows: the rotated parts lie outside their rows")
+        if row_pos.numel() < n:
+            raise KernelError("heads_to_rows: one position a row")
+        # (the row's length from the first rotated element on)
+        turn_args = (_gpu(rows, "turns") + first * rows.element_size(), rows.shape[1], int(apart),
+                     rotated, _gpu(frequencies, "frequencies", torch.float64), float(turn_scale),
+                     _gpu(row_pos, "row_pos", torch.int32))
+    status = lib.ei_heads_to_rows(_gpu(made, "made"), _code(made, "made"), _gpu(y, "y"), y.shape[1],
+                                  int(y_head), n, heads, j, *gate_args, *turn_args, _stream())
+    _check(lib, status, "heads_to_rows")
+
+
 def rotate_pairs(x, frequencies, row_pos, y, heads, rot_dim, x_head, x_first, y_head,
-                 y_first) -> None:
+                 y_first, turn_scale=1.0) -> None:
     """Elements (2i, 2i + 1) of x[n, h * x_head + x_first + 0..rot_dim] turn by the angle
-    row_pos[n] * frequencies[i] and go to y[n, h * y_head + y_first + ...]."""
+    row_pos[n] * frequencies[i] (float32 or float64 frequencies; cosine and sine times turn_scale)
+    and go to y[n, h * y_head + y_first + ...]."""
     lib = library("head_ops")
     n, x_row, nsplit, stride = _rows_of(x, "x")
     if y.dim() != 2 or y.shape[0] != n:
         raise KernelError("rotate_pairs: y must be [rows, width]")
-    if frequencies.numel() != rot_dim // 2 or row_pos.numel() < n:
-        raise KernelError("rotate_pairs: one frequency a pair and one position a row")
+    if row_pos.numel() < n:
+        raise KernelError("rotate_pairs: one position a row")
+    freq, freq_double = _frequencies(frequencies, rot_dim // 2, "rotate_pairs")
     status = lib.ei_rotate_pairs(_gpu(x, "x"), _code(x, "x"), nsplit, stride, x_row, int(x_head),
-                                 int(x_first), _gpu(frequencies, "frequencies", torch.float32),
+                                 int(x_first), freq, freq_double, float(turn_scale),
                                  _gpu(row_pos, "row_pos", torch.int32), _gpu(y, "y"),
                                  _code(y, "y"), y.shape[1], int(y_head), int(y_first), n, heads,
                                  int(rot_dim), _stream())
@@ -953,17 +1093,26 @@ def mlstm_out(o_raw, proj, norm_w, eps, row_seq, out, heads, key_dim, value_dim)
 
 def projection_norm_store(qkv, q_norm_w, k_norm_w, eps, row_pos, row_seq, page_table, q_out,
                           k_pages, v_pages, n_heads, n_kv_heads, head_dim, value_dim,
-                          write_cache=True, bias=None) -> None:
+                          write_cache=True, bias=None, values_from_keys=False, frequencies=None,
+                          turn_scale=1.0) -> None:
     """One RMS norm over the whole query projection and one over the whole key projection
-    (weights [heads * head_dim] and [kv heads * head_dim], or None for no norm), no rotation;
+    (weights [heads * head_dim] and [kv heads * head_dim], or None for no norm), then, with
+    frequencies (float64 [R / 2]), the first R elements of every query and key head turned in
+    neighbouring pairs by position * frequencies[i] (cosine and sine times turn_scale);
     queries to `q_out`, keys [*, kv heads, 64, head_dim] and values [*, kv heads, 64, value_dim]
-    to their cache pages.  bias: float32 [q | k | v width], added to the projection first."""
+    to their cache pages.  bias: float32 [q | k | v width], added to the projection first.
+    values_from_keys: the rows are [q | k] and the values are the keys as projected, before norm
+    and rotation.  qkv: rows, float32 slices of them, or `Columns`."""
     lib = library("rope_store")
     n = q_out.shape[0]
-    width = n_heads * head_dim + n_kv_heads * (head_dim + value_dim)
+    if values_from_keys and value_dim != head_dim:
+        raise KernelError("projection_norm_store: values that are the keys are as wide as they are")
+    width = n_heads * head_dim + n_kv_heads * (head_dim + (0 if values_from_keys else value_dim))
+    if frequencies is not None and not 1 <= frequencies.numel() <= head_dim // 2:
+        raise KernelError("projection_norm_store: the rotation is wider than a head")
     if bias is not None and bias.numel() != width:
         raise KernelError("projection_norm_store: the bias must be as wide as the projection")
-    nsplit, stride = _splits(qkv, n, width, "qkv")
+    pointer, code, nsplit, stride, row_stride = _columns(qkv, n, width, "qkv")
     if tuple(q_out.shape) != (n, n_heads * head_dim):
         raise KernelError("projection_norm_store: q_out has the wrong shape")
     if row_pos.numel() < n or row_seq.numel() < n:
@@ -980,7 +1129,7 @@ def projection_norm_store(qkv, q_norm_w, k_norm_w, eps, row_pos, row_seq, page_t
         if k_pages.dtype != q_out.dtype or v_pages.dtype != q_out.dtype:
             raise KernelError("projection_norm_store: cache and q_out dtypes differ")
     status = lib.ei_projection_norm_store(
-        _gpu(qkv, "qkv"), _code(qkv, "qkv"), nsplit, stride,
+        pointer, code, nsplit, stride, row_stride,
         None if bias is None else _gpu(bias, "bias", torch.float32),
         None if q_norm_w is None else _gpu(q_norm_w, "q_norm", torch.float32),
         None if k_norm_w is None else _gpu(k_norm_w, "k_norm", torch.float32), float(eps),
@@ -988,7 +1137,9 @@ def projection_norm_store(qkv, q_norm_w, k_norm_w, eps, row_pos, row_seq, page_t
         _gpu(page_table, "page_table", torch.int32), page_table.shape[-1], _gpu(q_out, "q_out"),
         _gpu(k_pages, "k_pages") if write_cache else None,
         _gpu(v_pages, "v_pages") if write_cache else None, _code(q_out, "q_out"), n, n_heads,
-        n_kv_heads, head_dim, value_dim, int(write_cache), _stream())
+        n_kv_heads, head_dim, value_dim, int(write_cache), int(bool(values_from_keys)),
+        None if frequencies is None else _gpu(frequencies, "frequencies", torch.float64),
+        0 if frequencies is None else 2 * frequencies.numel(), float(turn_scale), _stream())
     _check(lib, status, "projection_norm_store")
 
 
@@ -1098,7 +1249,7 @@ def attention_prefill_mfma(q, k_pages, v_pages, item_seq, item_row0, item_npos, 
                            page_table, out, n_heads, n_kv_heads, head_dim, window=None,
                            scale=None, key_ways=1, pair_items=True, largest_item=None,
                            chunk=None, slopes=None, sinks=None, pool_o=None, pool_ml=None,
-                           gate=None, keep_first=0, wide_gate=None) -> None:
+                           gate=None, keep_first=0, wide_gate=None, softcap=None) -> None:
     """bfloat16 prefill attention on the matrix cores; an item holds up to
     `attention_prefill_mfma_positions(group, key_ways)` positions of one sequence.
     pair_items: with enough items a block may take item i and then item n_items - 1 - i
@@ -1109,8 +1260,9 @@ def attention_prefill_mfma(q, k_pages, v_pages, item_seq, item_row0, item_npos, 
     chunk, slopes, sinks, keep_first: as for `attention`; wide_gate (rows, first column): rows of
     columns, of which those from `first column` on are the gates of the output's elements (the
     output is multiplied by their sigmoid), as [n, w] or float32 slices [s, n, w].  Any of
-    these takes the kernel's extended form."""
-    lib = library("attention_mfma")
+    these takes the kernel's extended form.  softcap c: a scaled score s becomes c tanh(s / c)
+    (forms of their own, in a library of their own; not with keep_first or wide_gate)."""
+    lib = library("attention_mfma" if softcap is None else "attention_capped")
     n = q.shape[0]
     capacity = attention_prefill_mfma_positions(n_heads // max(1, n_kv_heads), key_ways)
     if capacity == 0:
@@ -1139,7 +1291,11 @@ def attention_prefill_mfma(q, k_pages, v_pages, item_seq, item_row0, item_npos, 
         _gpu(out, "out", torch.bfloat16), n_heads, n_kv_heads, head_dim, int(window or 0),
         float(scale), int(key_ways), int(bool(pair_items)))
     keep_first = keep_first if window else 0
-    if (chunk or slopes is not None or sinks is not None or pool_o is not None or gate is not None
+    if softcap is not None:
+        status = lib.ei_attention_prefill_capped(*common, *_capped_extras(
+            softcap, chunk, slopes, sinks, n_heads, n, head_dim, pool_o, pool_ml, gate, keep_first,
+            wide_gate), _stream())
+    elif (chunk or slopes is not None or sinks is not None or pool_o is not None or gate is not None
             or keep_first or wide_gate is not None):
         status = lib.ei_attention_prefill_mfma_ext(*common, *_attention_extras(
             chunk, slopes, sinks, n_heads, n, head_dim, pool_o, pool_ml, gate, keep_first,
@@ -1184,6 +1340,18 @@ def _attention_extras(chunk, slopes, sinks, n_heads, rows=0, head_dim=0, pool_o=
             f32(pool_ml, "pool_ml"), f32(gate, "gate"), int(keep_first), *wide)
 
 
+def _capped_extras(softcap, chunk, slopes, sinks, n_heads, rows, head_dim, pool_o, pool_ml, gate,
+                   keep_first, wide_gate):
+    """The arguments of the forms with a cap on the scores, from chunk on."""
+    if not softcap > 0:
+        raise KernelError("attention: a cap on the scores must be positive")
+    if keep_first or wide_gate is not None:
+        raise KernelError("attention: a cap on the scores with kept first positions or a gate an "
+                          "element is not implemented on the matrix cores")
+    return (*_attention_extras(chunk, slopes, sinks, n_heads, rows, head_dim, pool_o, pool_ml,
+                               gate)[:6], float(softcap))
+
+
 class DecodeProjection:
     """What `attention_decode_mfma` needs to make queries, key and value itself: the fused
     projection as float32 partial sums [slices, rows, (heads + 2 kv heads) * head_dim], the
@@ -1200,7 +1368,7 @@ def attention_decode_mfma(q, k_pages, v_pages, row_pos, row_seq, page_table, out
                           n_kv_heads, head_dim, window=None, scale=None, n_splits=1, part_o=None,
                           part_ml=None, waves=4, longest=None, heads=0, chunk=None, slopes=None,
                           sinks=None, pool_o=None, pool_ml=None, gate=None, keep_first=0,
-                          wide_gate=None) -> None:
+                          wide_gate=None, softcap=None) -> None:
     """bfloat16 decode attention on the matrix cores: one query row per sequence.  `waves`
     (4, 8 or 16) of a block share its key range tile by tile; more suit fewer sequences (few
     blocks), whose ranges then need fewer slices or none.  `heads` (a power of two, or 0 for
@@ -1211,13 +1379,15 @@ def attention_decode_mfma(q, k_pages, v_pages, row_pos, row_seq, page_table, out
     `q` is the queries [rows, heads * head_dim], or a `DecodeProjection`: the kernel then does
     the work of `qk_norm_rope_store` for its rows as well.  chunk, slopes, sinks,
     keep_first: as for `attention`; wide_gate: as for `attention_prefill_mfma` (any of them takes
-    the kernel's extended form, which the fused one lacks)."""
-    lib = library("attention_mfma")
+    the kernel's extended form, which the fused one lacks); softcap: as for
+    `attention_prefill_mfma`."""
+    lib = library("attention_mfma" if softcap is None else "attention_capped")
     n = out.shape[0]
     fused = isinstance(q, DecodeProjection)
     keep_first = keep_first if window else 0
     extended = (bool(chunk) or slopes is not None or sinks is not None or pool_o is not None
-                or gate is not None or keep_first != 0 or wide_gate is not None)
+                or gate is not None or keep_first != 0 or wide_gate is not None
+                or softcap is not None)
     if (pool_o is not None or gate is not None) and n_splits < 2:
         raise KernelError("attention_decode: pooled sums and the gate are taken in by the merge "
                           "of at least two slices")
@@ -1273,7 +1443,11 @@ def attention_decode_mfma(q, k_pages, v_pages, row_pos, row_seq, page_table, out
         None if part_ml is None else _gpu(part_ml, "part_ml", torch.float32), n, n_heads,
         n_kv_heads, head_dim, int(window or 0), float(scale), n_splits, int(waves), int(heads),
         None if longest is None else _gpu(longest, "longest", torch.int32))
-    if extended:
+    if softcap is not None:
+        status = lib.ei_attention_decode_capped(*common, *_capped_extras(
+            softcap, chunk, slopes, sinks, n_heads, q.shape[0], head_dim, pool_o, pool_ml, gate,
+            keep_first, wide_gate), _stream())
+    elif extended:
         status = lib.ei_attention_decode_mfma_ext(*common, *_attention_extras(
             chunk, slopes, sinks, n_heads, q.shape[0], head_dim, pool_o, pool_ml, gate, keep_first,
             wide_gate), _stream())
@@ -1293,26 +1467,41 @@ def delta_state_floats(n_heads: int, n_kv_heads: int, key_dim: int, value_dim: i
 
 
 class DeltaShape:
-    """Sizes of a gated-delta mixer and where its parts lie in a row of its fused projection
-    [q | k | v | beta | decay | gate]."""
+    """Sizes of a gated-delta mixer and where its parts lie in a row of its fused projection:
+    [q | k | v | beta | decay | gate], or, with a decay per key channel and a gate of low rank
+    (`decay_rank`, `gate_rank`), [q | k | v | . | low-rank decay | low-rank gate | beta | .] with
+    the low-rank part at a multiple of 8 columns and the row's width a multiple of 8."""
 
-    def __init__(self, n_heads, n_kv_heads, key_dim, value_dim, taps):
+    def __init__(self, n_heads, n_kv_heads, key_dim, value_dim, taps, decay_rank=0, gate_rank=0):
         self.n_heads, self.n_kv_heads = int(n_heads), int(n_kv_heads)
         self.key_dim, self.value_dim, self.taps = int(key_dim), int(value_dim), int(taps)
         self.qk_width = self.n_kv_heads * self.key_dim
         self.v_width = self.n_heads * self.value_dim
         self.channels = 2 * self.qk_width + self.v_width          # what the convolution covers
-        self.beta_col = self.channels
-        self.decay_col = self.beta_col + self.n_heads
-        self.gate_col = self.decay_col + self.n_heads
-        self.width = self.gate_col + self.v_width
+        self.decay_rank, self.gate_rank = int(decay_rank), int(gate_rank)
+        self.low_rank = self.decay_rank > 0
+        if self.low_rank != (self.gate_rank > 0):
+            raise KernelError("delta: decay and gate are both of low rank, or neither is")
+        self.decay_width = self.n_heads * self.key_dim if self.low_rank else 0
+        if self.low_rank:
+            self.low_col = (self.channels + 7) // 8 * 8
+            self.gate_low_col = self.low_col + self.decay_rank
+            self.beta_col = self.gate_low_col + self.gate_rank
+            self.width = (self.beta_col + self.n_heads + 7) // 8 * 8
+            self.decay_col = self.gate_col = -1
+        else:
+            self.beta_col = self.channels
+            self.decay_col = self.beta_col + self.n_heads
+            self.gate_col = self.decay_col + self.n_heads
+            self.width = self.gate_col + self.v_width
+        self.conv_width = self.channels + self.decay_width        # of a row of delta_conv's output
         self.tail_offset = self.n_heads * self.value_dim * self.key_dim
         self.state_floats = delta_state_floats(n_heads, n_kv_heads, key_dim, value_dim, taps)
 
 
 def _delta_proj(proj, rows, shape):
-    nsplit, stride = _splits(proj, rows, shape.width, "proj")
-    return _gpu(proj, "proj"), _code(proj, "proj"), nsplit, stride
+    """(pointer, dtype code, nsplit, slice stride, row stride) of the fused projection."""
+    return _columns(proj, rows, shape.width, "proj")
 
 
 def _delta_state(state, shape):
@@ -1333,31 +1522,82 @@ def _delta_rows(seq_in, seq_out, n_seqs):
 DELTA_FEW_TAPS = 8      # up to so many taps `delta_conv` can renew the tails itself
 
 
+def _delta_conv_args(conv_w, state, shape, row_pos, row_seq, seq_in, seq_out, seq_start, out, what):
+    rows = out.shape[0]
+    if tuple(out.shape) != (rows, shape.conv_width) or tuple(conv_w.shape) != (shape.channels, shape.taps):
+        raise KernelError(f"{what}: out must be [rows, channels (+ decays)] and conv_w [channels, taps]")
+    if row_pos.numel() < rows or row_seq.numel() < rows:
+        raise KernelError(f"{what}: row metadata shorter than the rows")
+    return (_gpu(conv_w, "conv_w", torch.float32), shape.taps, _delta_state(state, shape),
+            shape.state_floats, shape.tail_offset, _gpu(row_pos, "row_pos", torch.int32),
+            _gpu(row_seq, "row_seq", torch.int32),
+            *_delta_rows(seq_in, seq_out, seq_start.numel()),
+            _gpu(seq_start, "seq_start", torch.int32), _gpu(out, "out", torch.float32),
+            shape.conv_width, rows, shape.channels)
+
+
+def _delta_decays(a_log, dt_bias, shape, what):
+    if a_log.numel() != shape.n_heads or dt_bias.numel() != shape.decay_width:
+        raise KernelError(f"{what}: one decay rate a head and one bias a head and key channel")
+    return (_gpu(a_log, "a_log", torch.float32), _gpu(dt_bias, "dt_bias", torch.float32),
+            shape.n_heads, shape.key_dim)
+
+
 def delta_conv(proj, conv_w, state, shape: DeltaShape, row_pos, row_seq, seq_in, seq_out,
-               seq_start, out, renew_tail=False) -> None:
+               seq_start, out, renew_tail=False, decay_logits=None, a_log=None, dt_bias=None) -> None:
     """out [rows, channels] float32 = silu(causal convolution) of the q, k, v columns of
-    `proj` ([rows, width] or float32 slices of it); conv_w float32 [channels, taps]; inputs
-    from before this step come from the sequences' tails in `state` [rows, state_floats], row
+    `proj` ([rows, width], float32 slices of it, or `Columns`); conv_w float32 [channels, taps];
+    inputs from before this step come from the sequences' tails in `state` [rows, state_floats], row
     seq_in[s] for sequence s.  renew_tail: every sequence brings exactly one row (the caller vouches for it) and the
     tails become the last taps - 1 inputs here, written to row seq_out[s], so `delta_tail` is
-    not needed (at most `DELTA_FEW_TAPS` taps)."""
+    not needed (at most `DELTA_FEW_TAPS` taps).  With a decay per key channel: decay_logits
+    [rows, >= heads * key_dim], whose first columns become the decays behind the channels of
+    `out` [rows, channels + heads * key_dim] (a_log [heads], dt_bias [heads * key_dim])."""
     lib = library("delta_rule")
+    args = _delta_conv_args(conv_w, state, shape, row_pos, row_seq, seq_in, seq_out, seq_start, out,
+                            "delta_conv")
     rows = out.shape[0]
-    if tuple(out.shape) != (rows, shape.channels) or tuple(conv_w.shape) != (shape.channels, shape.taps):
-        raise KernelError("delta_conv: out must be [rows, channels] and conv_w [channels, taps]")
-    if row_pos.numel() < rows or row_seq.numel() < rows:
-        raise KernelError("delta_conv: row metadata shorter than the rows")
-    pointer, code, nsplit, stride = _delta_proj(proj, rows, shape)
-    status = lib.ei_delta_conv(pointer, code, nsplit, stride, shape.width,
-                               _gpu(conv_w, "conv_w", torch.float32), shape.taps,
-                               _delta_state(state, shape), shape.state_floats, shape.tail_offset,
-                               _gpu(row_pos, "row_pos", torch.int32),
-                               _gpu(row_seq, "row_seq", torch.int32),
-                               *_delta_rows(seq_in, seq_out, seq_start.numel()),
-                               _gpu(seq_start, "seq_start", torch.int32),
-                               _gpu(out, "out", torch.float32), rows, shape.channels,
-                               int(bool(renew_tail)), _stream())
+    if (decay_logits is not None) != shape.low_rank:
+        raise KernelError("delta_conv: decay logits go with a decay per key channel")
+    decays = (None, F32, 0, None, None, 0, 0)
+    if decay_logits is not None:
+        if decay_logits.dim() != 2 or decay_logits.shape[0] != rows \
+                or decay_logits.shape[1] < shape.decay_width:
+            raise KernelError("delta_conv: one decay logit a row, head and key channel")
+        decays = (_gpu(decay_logits, "decay_logits"), _code(decay_logits, "decay_logits"),
+                  decay_logits.shape[1], *_delta_decays(a_log, dt_bias, shape, "delta_conv"))
+    pointer, code, nsplit, stride, row_stride = _delta_proj(proj, rows, shape)
+    status = lib.ei_delta_conv(pointer, code, nsplit, stride, row_stride, *args,
+                               int(bool(renew_tail)), *decays, _stream())
     _check(lib, status, "delta_conv")
+
+
+def delta_prepare(proj, conv_w, state, shape: DeltaShape, row_pos, row_seq, seq_in, seq_out,
+                  seq_start, out, a_log, dt_bias, w_decay, w_gate, gate_out, renew_tail=False) -> None:
+    """`delta_conv` and, in the same launch, the low-rank products of few rows: w_decay
+    [decay_rank, heads * key_dim] on the projection's low-rank decay columns gives the decays
+    behind the channels of `out`, w_gate [gate_rank, heads * value_dim] the gate's logits, to
+    gate_out float32 [rows, heads * value_dim].  proj: float32 rows or slices."""
+    lib = library("delta_rule")
+    args = _delta_conv_args(conv_w, state, shape, row_pos, row_seq, seq_in, seq_out, seq_start, out,
+                            "delta_prepare")
+    rows = out.shape[0]
+    pointer, code, nsplit, stride, row_stride = _delta_proj(proj, rows, shape)
+    if code != F32 or not shape.low_rank:
+        raise KernelError("delta_prepare: float32 rows with a low-rank part")
+    if tuple(w_decay.shape) != (shape.decay_rank, shape.decay_width) or \
+            tuple(w_gate.shape) != (shape.gate_rank, shape.v_width) or w_decay.dtype != w_gate.dtype:
+        raise KernelError("delta_prepare: w_decay must be [decay_rank, heads * key_dim] and w_gate "
+                          "[gate_rank, heads * value_dim] of one type")
+    if tuple(gate_out.shape) != (rows, shape.v_width):
+        raise KernelError("delta_prepare: gate_out must be [rows, heads * value_dim]")
+    status = lib.ei_delta_prepare(
+        pointer, nsplit, stride, row_stride, *args, int(bool(renew_tail)),
+        *_delta_decays(a_log, dt_bias, shape, "delta_prepare"), _gpu(w_decay, "w_decay"),
+        _gpu(w_gate, "w_gate"), _code(w_decay, "w_decay"), shape.low_col, shape.decay_rank,
+        shape.gate_low_col, shape.gate_rank, shape.v_width,
+        _gpu(gate_out, "gate_out", torch.float32), _stream())
+    _check(lib, status, "delta_prepare")
 
 
 def delta_tail(proj, state, shape: DeltaShape, rows, seq_in, seq_out, seq_count, seq_row0) -> None:
@@ -1370,8 +1610,8 @@ def delta_tail(proj, state, shape: DeltaShape, rows, seq_in, seq_out, seq_count,
     n_seqs = seq_count.numel()
     if seq_row0.numel() < n_seqs:
         raise KernelError("delta_tail: sequence metadata shorter than the sequences")
-    pointer, code, nsplit, stride = _delta_proj(proj, rows, shape)
-    status = lib.ei_delta_tail(pointer, code, nsplit, stride, shape.width, shape.taps,
+    pointer, code, nsplit, stride, row_stride = _delta_proj(proj, rows, shape)
+    status = lib.ei_delta_tail(pointer, code, nsplit, stride, row_stride, shape.taps,
                                _delta_state(state, shape), shape.state_floats, shape.tail_offset,
                                *_delta_rows(seq_in, seq_out, n_seqs),
                                _gpu(seq_count, "seq_count", torch.int32),
@@ -1384,21 +1624,25 @@ def delta_rule(conv, proj, a_log, dt_bias, state, shape: DeltaShape, seq_in, seq
                seq_row0, o_raw, q_scale: float, unit_eps: float) -> None:
     """The recurrence over every sequence's rows of this step, in order; reads S from row
     seq_in[s] of `state` and writes it to row seq_out[s]; o_raw [rows, heads * value_dim]
-    float32 receives S^T q of every row."""
+    float32 receives S^T q of every row.  With a decay per key channel the decays come with the
+    rows of `conv` (a_log and dt_bias None)."""
     lib = library("delta_rule")
     rows = conv.shape[0]
     n_seqs = seq_count.numel()
-    if tuple(conv.shape) != (rows, shape.channels) or tuple(o_raw.shape) != (rows, shape.v_width):
-        raise KernelError("delta_rule: conv must be [rows, channels] and o_raw [rows, heads * value_dim]")
-    if a_log.numel() != shape.n_heads or dt_bias.numel() != shape.n_heads:
+    if tuple(conv.shape) != (rows, shape.conv_width) or tuple(o_raw.shape) != (rows, shape.v_width):
+        raise KernelError("delta_rule: conv must be [rows, channels (+ decays)] and o_raw [rows, "
+                          "heads * value_dim]")
+    if not shape.low_rank and (a_log.numel() != shape.n_heads or dt_bias.numel() != shape.n_heads):
         raise KernelError("delta_rule: one decay rate and bias per head")
     if seq_row0.numel() < n_seqs:
         raise KernelError("delta_rule: sequence metadata shorter than the sequences")
-    pointer, code, nsplit, stride = _delta_proj(proj, rows, shape)
-    status = lib.ei_delta_rule(_gpu(conv, "conv", torch.float32), pointer, code, nsplit, stride,
-                               shape.width, shape.beta_col, shape.decay_col,
-                               _gpu(a_log, "a_log", torch.float32),
-                               _gpu(dt_bias, "dt_bias", torch.float32), _delta_state(state, shape),
+    pointer, code, nsplit, stride, row_stride = _delta_proj(proj, rows, shape)
+    status = lib.ei_delta_rule(_gpu(conv, "conv", torch.float32), shape.conv_width,
+                               int(shape.low_rank), pointer, code, nsplit, stride,
+                               row_stride, shape.beta_col, shape.decay_col,
+                               None if shape.low_rank else _gpu(a_log, "a_log", torch.float32),
+                               None if shape.low_rank else _gpu(dt_bias, "dt_bias", torch.float32),
+                               _delta_state(state, shape),
                                shape.state_floats, *_delta_rows(seq_in, seq_out, n_seqs),
                                _gpu(seq_count, "seq_count", torch.int32),
                                _gpu(seq_row0, "seq_row0", torch.int32),
@@ -1408,17 +1652,29 @@ def delta_rule(conv, proj, a_log, dt_bias, state, shape: DeltaShape, seq_in, seq
     _check(lib, status, "delta_rule")
 
 
-def delta_out(o_raw, proj, norm_w, eps, shape: DeltaShape, row_seq, out) -> None:
-    """out [rows, heads * value_dim] = o / sqrt(mean(o^2) + eps) * norm_w * silu(gate) per head."""
+def delta_out(o_raw, proj, norm_w, eps, shape: DeltaShape, row_seq, out, sigmoid_gate=False,
+              gate_logits=None) -> None:
+    """out [rows, heads * value_dim] = o / sqrt(mean(o^2) + eps) * norm_w * silu(gate) per head
+    (sigmoid_gate: sigmoid for silu), the gate's logits being the projection's gate columns or
+    gate_logits (rows, float32 slices or `Columns` [heads * value_dim])."""
     lib = library("delta_rule")
     rows = o_raw.shape[0]
     if tuple(o_raw.shape) != (rows, shape.v_width) or tuple(out.shape) != tuple(o_raw.shape):
         raise KernelError("delta_out: o_raw and out must be [rows, heads * value_dim]")
     if norm_w.numel() != shape.value_dim:
         raise KernelError("delta_out: the norm weight must have value_dim elements")
-    pointer, code, nsplit, stride = _delta_proj(proj, rows, shape)
+    if gate_logits is None:
+        if shape.low_rank:
+            raise KernelError("delta_out: a gate of low rank comes as its logits")
+        pointer, code, nsplit, stride, row_stride = _delta_proj(proj, rows, shape)
+        gate_col = shape.gate_col
+    else:
+        pointer, code, nsplit, stride, row_stride = _columns(gate_logits, rows, shape.v_width,
+                                                             "gate_logits")
+        gate_col = 0
     status = lib.ei_delta_out(_gpu(o_raw, "o_raw", torch.float32), pointer, code, nsplit, stride,
-                              shape.width, shape.gate_col, _gpu(norm_w, "norm_w", torch.float32),
+                              row_stride, gate_col, int(bool(sigmoid_gate)),
+                              _gpu(norm_w, "norm_w", torch.float32),
                               float(eps), _gpu(row_seq, "row_seq", torch.int32), _gpu(out, "out"),
                               _code(out, "out"), rows, shape.n_heads, shape.value_dim, _stream())
     _check(lib, status, "delta_out")
@@ -1587,14 +1843,12 @@ def stream_norm(residual, delta, out, *, w_after=None, b_after=None, w_next=None
     _check(lib, status, "stream_norm")
 
 
-def norm_mean(branches, weights, eps: float, out: torch.Tensor) -> None:
-    """out [n, h] float32 = the mean over the branches b of rmsnorm(x_b) * w_b; every x_b is
-    [n, h] or float32 slices [s, n, h], of its own type."""
-    lib = library("norms")
-    rows, hidden = out.shape
+def _branch_arrays(branches, weights, rows, hidden, what):
+    """Arrays (pointers, slices, slice strides, dtype codes, weights) of rows [n, h] or float32
+    slices [s, n, h] side by side; a weight may be None."""
     count = len(branches)
     if not 1 <= count <= 4 or len(weights) != count:
-        raise KernelError("norm_mean: 1 to 4 branches, each with its weight")
+        raise KernelError(f"{what}: 1 to 4 branches, each with its weight")
     pointers = (c_void_p * count)()
     weight_pointers = (c_void_p * count)()
     nsplits = (c_int * count)()
@@ -1604,12 +1858,49 @@ def norm_mean(branches, weights, eps: float, out: torch.Tensor) -> None:
         nsplits[index], strides[index] = _splits(x, rows, hidden, "a branch")
         pointers[index] = _gpu(x, "a branch")
         codes[index] = _code(x, "a branch")
+        if w is None:
+            continue
         if w.numel() != hidden:
-            raise KernelError(f"norm_mean: a weight must have {hidden} elements")
+            raise KernelError(f"{what}: a weight must have {hidden} elements")
         weight_pointers[index] = _gpu(w, "weight", torch.float32)
-    status = lib.ei_norm_mean(pointers, nsplits, strides, codes, weight_pointers, count,
+    return pointers, nsplits, strides, codes, weight_pointers, count
+
+
+def norm_mean(branches, weights, eps: float, out: torch.Tensor) -> None:
+    """out [n, h] float32 = the mean over the branches b of rmsnorm(x_b) * w_b; every x_b is
+    [n, h] or float32 slices [s, n, h], of its own type."""
+    lib = library("norms")
+    rows, hidden = out.shape
+    status = lib.ei_norm_mean(*_branch_arrays(branches, weights, rows, hidden, "norm_mean"),
                               float(eps), _gpu(out, "out", torch.float32), rows, hidden, _stream())
     _check(lib, status, "norm_mean")
+
+
+def post_norm(residual: torch.Tensor, delta, alpha: float, weight: torch.Tensor, eps: float,
+              cast_out: Optional[torch.Tensor] = None, branch_weights=None,
+              branch_eps: float = 1.0) -> None:
+    """residual [n, h] float32 <- rmsnorm(alpha residual + d; eps) * weight, with d the sum of
+    `delta`'s slices ([n, h] or [s, n, h]); or, with branch_weights, the mean over the list
+    `delta` of rmsnorm(x_b; branch_eps) * branch_weights[b].  cast_out [n, h] (optional) receives
+    the new rows in its own type."""
+    lib = library("norms")
+    rows, hidden = residual.shape
+    if weight.numel() != hidden:
+        raise KernelError(f"post_norm: the weight must have {hidden} elements")
+    if cast_out is not None and tuple(cast_out.shape) != (rows, hidden):
+        raise KernelError("post_norm: cast_out must have the residual's shape")
+    if branch_weights is None:
+        arrays = _branch_arrays([delta], [None], rows, hidden, "post_norm")
+    else:
+        if any(w is None for w in branch_weights):
+            raise KernelError("post_norm: every branch has a weight")
+        arrays = _branch_arrays(delta, branch_weights, rows, hidden, "post_norm")
+    status = lib.ei_post_norm(_gpu(residual, "residual", torch.float32), *arrays, float(branch_eps),
+                              float(alpha), _gpu(weight, "weight", torch.float32), float(eps),
+                              None if cast_out is None else _gpu(cast_out, "cast_out"),
+                              F32 if cast_out is None else _code(cast_out, "cast_out"), rows, hidden,
+                              _stream())
+    _check(lib, status, "post_norm")
 
 
 def input_conv(h, weight, state, part: int, parts: int, row_pos, row_seq, seq_in, seq_out,

@@ -364,6 +364,137 @@ __global__ void norm_mean_vec_kernel(Branches branches, int n, float eps, float*
   }
 }
 
+// A norm over the scaled stream and what a sublayer adds: y = alpha residual[row] + d, then
+// residual[row] = y / sqrt(mean(y^2) + eps) * w, also written to `cast` in its own type (or null).
+// d is the plain sum of one branch's slices (its weight null), or the mean over the branches of
+// rmsnorm(sum of slices; inner_eps) * w_b.
+template <typename TO>
+__global__ void post_norm_kernel(float* __restrict__ residual, Branches branches, int n,
+                                 float inner_eps, float alpha, const float* __restrict__ w,
+                                 float eps, TO* __restrict__ cast, int H) {
+  extern __shared__ float values[];      // [2][H]: the branch at hand, the running sum
+  __shared__ float scratch[16];
+  float* current = values;
+  float* total = values + H;
+  const size_t base = static_cast<size_t>(blockIdx.x) * H;
+  for (int b = 0; b < n; ++b) {
+    const bool narrow = branches.dtype[b] == EI_BF16;
+    const float* x32 = static_cast<const float*>(branches.rows[b]) + base;
+    const bf16_t* x16 = static_cast<const bf16_t*>(branches.rows[b]) + base;
+    const float* wb = branches.weight[b];
+    float squares = 0.f;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      float v = 0.f;
+      for (int s = 0; s < branches.nsplit[b]; ++s) {
+        const size_t at = static_cast<size_t>(s) * branches.split_stride[b] + i;
+        v += narrow ? ei::bf16_to_f32(x16[at]) : x32[at];
+      }
+      current[i] = v;
+      squares += v * v;
+    }
+    const float inv =
+        wb ? 1.0f / sqrtf(ei::block_sum(squares, scratch) / static_cast<float>(H) + inner_eps) : 1.0f;
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      const float y = wb ? (current[i] * inv) * wb[i] : current[i];
+      total[i] = b == 0 ? y : total[i] + y;
+    }
+  }
+  const float share = 1.0f / static_cast<float>(n);
+  float squares = 0.f;
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    const float y = fmaf(alpha, residual[base + i], total[i] * share);
+    total[i] = y;
+    squares += y * y;
+  }
+  const float inv = 1.0f / sqrtf(ei::block_sum(squares, scratch) / static_cast<float>(H) + eps);
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    const float y = (total[i] * inv) * w[i];
+    residual[base + i] = y;
+    if (cast) cast[base + i] = ei::from_f32<TO>(y);
+  }
+}
+
+// The same for widths that are a multiple of 4: 16-byte accesses, everything in registers.
+template <typename TO, int CHUNKS>
+__global__ void post_norm_vec_kernel(float* __restrict__ residual, Branches branches, int n,
+                                     float inner_eps, float alpha, const float* __restrict__ w,
+                                     float eps, TO* __restrict__ cast, int H) {
+  __shared__ float scratch[16];
+  const size_t base = static_cast<size_t>(blockIdx.x) * H;
+  const int quads = H / 4;
+  float y[CHUNKS][4], total[CHUNKS][4];
+#pragma unroll
+  for (int k = 0; k < CHUNKS; ++k) {
+    const int qd = threadIdx.x + k * blockDim.x;
+    total[k][0] = total[k][1] = total[k][2] = total[k][3] = 0.f;
+    y[k][0] = y[k][1] = y[k][2] = y[k][3] = 0.f;
+    if (qd < quads) Vec4<float>::load(residual + base + qd * 4, y[k]);
+  }
+  for (int b = 0; b < n; ++b) {
+    const bool narrow = branches.dtype[b] == EI_BF16;
+    const size_t stride = static_cast<size_t>(branches.split_stride[b]);
+    const float* wb = branches.weight[b];
+    float x[CHUNKS][4];
+    float squares = 0.f;
+#pragma unroll
+    for (int k = 0; k < CHUNKS; ++k) {
+      const int qd = threadIdx.x + k * blockDim.x;
+      x[k][0] = x[k][1] = x[k][2] = x[k][3] = 0.f;
+      if (qd < quads) {
+        if (narrow)
+          sliced4(static_cast<const bf16_t*>(branches.rows[b]) + base + qd * 4, branches.nsplit[b],
+                  stride, x[k]);
+        else
+          sliced4(static_cast<const float*>(branches.rows[b]) + base + qd * 4, branches.nsplit[b],
+                  stride, x[k]);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) squares += x[k][i] * x[k][i];
+      }
+    }
+    if (wb) {                            // (uniform: every thread takes the sum's barriers)
+      const float inv =
+          1.0f / sqrtf(ei::block_sum(squares, scratch) / static_cast<float>(H) + inner_eps);
+#pragma unroll
+      for (int k = 0; k < CHUNKS; ++k) {
+        const int qd = threadIdx.x + k * blockDim.x;
+        if (qd < quads) {
+          float v[4];
+          Vec4<float>::load(wb + qd * 4, v);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) total[k][i] += (x[k][i] * inv) * v[i];
+        }
+      }
+    } else {
+#pragma unroll
+      for (int k = 0; k < CHUNKS; ++k)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) total[k][i] += x[k][i];
+    }
+  }
+  const float share = 1.0f / static_cast<float>(n);
+  float squares = 0.f;
+#pragma unroll
+  for (int k = 0; k < CHUNKS; ++k)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {        // (quads beyond the row hold zeros)
+      y[k][i] = fmaf(alpha, y[k][i], total[k][i] * share);
+      squares += y[k][i] * y[k][i];
+    }
+  const float inv = 1.0f / sqrtf(ei::block_sum(squares, scratch) / static_cast<float>(H) + eps);
+#pragma unroll
+  for (int k = 0; k < CHUNKS; ++k) {
+    const int qd = threadIdx.x + k * blockDim.x;
+    if (qd < quads) {
+      float v[4];
+      Vec4<float>::load(w + qd * 4, v);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) y[k][i] = (y[k][i] * inv) * v[i];
+      Vec4<float>::store(residual + base + qd * 4, y[k]);
+      if (cast) Vec4<TO>::store(cast + base + qd * 4, y[k]);
+    }
+  }
+}
+
 // Threads a row of the register-held forms: up to 1024 for few rows, so that many loads are in
 // flight; 256 for many rows, so that several rows share a compute unit.
 int vec_threads(int N, int quads) {
@@ -432,6 +563,31 @@ extern "C" int ei_stream_norm(float* residual, const void* delta, int delta_dtyp
   EI_LAUNCH_CHECK();
 }
 
+// The branches as the kernels take them; false where an argument is missing or unknown.
+static bool gather_branches(const void* const* x, const int* nsplit, const long long* split_stride,
+                            const int* dtype, const float* const* weight, int n, bool weights,
+                            Branches* branches) {
+  for (int b = 0; b < kMaxBranches; ++b) {
+    branches->rows[b] = b < n ? x[b] : nullptr;
+    branches->weight[b] = b < n ? weight[b] : nullptr;
+    branches->nsplit[b] = b < n ? nsplit[b] : 0;
+    branches->split_stride[b] = b < n ? split_stride[b] : 0;
+    branches->dtype[b] = b < n ? dtype[b] : EI_F32;
+    if (b < n && (!x[b] || (weights && !weight[b]) || nsplit[b] < 1 ||
+                  (dtype[b] != EI_F32 && dtype[b] != EI_BF16)))
+      return false;
+  }
+  return true;
+}
+
+static bool branches_vec(const Branches& branches, int n, int H) {
+  bool vec = H % 4 == 0 && H <= 16384;
+  for (int b = 0; b < n; ++b)
+    vec = vec && branches.split_stride[b] % 4 == 0 &&
+          reinterpret_cast<uintptr_t>(branches.rows[b]) % 16 == 0;
+  return vec;
+}
+
 // out [N, H] float32 = mean over the n branches of rmsnorm(x_b) * w_b; x_b [nsplit_b][N, H] of
 // the type dtype[b].
 extern "C" int ei_norm_mean(const void* const* x, const int* nsplit, const long long* split_stride,
@@ -442,20 +598,11 @@ extern "C" int ei_norm_mean(const void* const* x, const int* nsplit, const long 
              "norm_mean: bad arguments");
   EI_REQUIRE(static_cast<size_t>(H) * 2 * sizeof(float) <= 64 * 1024, "norm_mean: row too wide");
   Branches branches;
-  for (int b = 0; b < kMaxBranches; ++b) {
-    branches.rows[b] = b < n ? x[b] : nullptr;
-    branches.weight[b] = b < n ? weight[b] : nullptr;
-    branches.nsplit[b] = b < n ? nsplit[b] : 0;
-    branches.split_stride[b] = b < n ? split_stride[b] : 0;
-    branches.dtype[b] = b < n ? dtype[b] : EI_F32;
-    EI_REQUIRE(b >= n || (x[b] && weight[b] && nsplit[b] >= 1), "norm_mean: null pointer");
-    EI_REQUIRE(b >= n || dtype[b] == EI_F32 || dtype[b] == EI_BF16, "norm_mean: unknown dtype");
-  }
+  EI_REQUIRE(gather_branches(x, nsplit, split_stride, dtype, weight, n, true, &branches),
+             "norm_mean: null pointer or unknown dtype");
   const int threads = row_threads(H);
   const size_t lds = static_cast<size_t>(H) * 2 * sizeof(float);
-  bool vec = H % 4 == 0 && H <= 16384;
-  for (int b = 0; b < n; ++b)
-    vec = vec && split_stride[b] % 4 == 0 && reinterpret_cast<uintptr_t>(x[b]) % 16 == 0;
+  const bool vec = branches_vec(branches, n, H);
   const int vthreads = vec_threads(N, H / 4);
   const int chunks = vec ? (H / 4 + vthreads - 1) / vthreads : 0;
   if (chunks == 1) norm_mean_vec_kernel<1><<<N, vthreads, 0, stream>>>(branches, n, eps, out, H);
@@ -464,5 +611,46 @@ extern "C" int ei_norm_mean(const void* const* x, const int* nsplit, const long 
     norm_mean_vec_kernel<4><<<N, vthreads, 0, stream>>>(branches, n, eps, out, H);
   else
     norm_mean_kernel<<<N, threads, lds, stream>>>(branches, n, eps, out, H);
+  EI_LAUNCH_CHECK();
+}
+
+// residual [N, H] float32 <- rmsnorm(alpha residual + d; eps) * w, d the plain sum of one branch's
+// slices (weight[0] null) or the mean over the n branches of rmsnorm(x_b; inner_eps) * weight[b];
+// cast [N, H] of cast_dtype, or null, receives the new rows as well.
+extern "C" int ei_post_norm(float* residual, const void* const* x, const int* nsplit,
+                            const long long* split_stride, const int* dtype,
+                            const float* const* weight, int n, float inner_eps, float alpha,
+                            const float* w, float eps, void* cast, int cast_dtype, int N, int H,
+                            hipStream_t stream) {
+  EI_REQUIRE(n >= 1 && n <= kMaxBranches, "post_norm: 1 to 4 branches");
+  EI_REQUIRE(residual && x && nsplit && split_stride && dtype && weight && w && N > 0 && H > 0,
+             "post_norm: bad arguments");
+  EI_REQUIRE(eps > 0.f && inner_eps > 0.f, "post_norm: eps must be positive");
+  EI_REQUIRE(static_cast<size_t>(H) * 2 * sizeof(float) <= 64 * 1024, "post_norm: row too wide");
+  Branches branches;
+  EI_REQUIRE(gather_branches(x, nsplit, split_stride, dtype, weight, n, n > 1, &branches),
+             "post_norm: null pointer or unknown dtype");
+  const int threads = row_threads(H);
+  const size_t lds = static_cast<size_t>(H) * 2 * sizeof(float);
+  const bool vec = branches_vec(branches, n, H);
+  const int vthreads = vec_threads(N, H / 4);
+  const int chunks = vec ? (H / 4 + vthreads - 1) / vthreads : 0;
+#define EI_PN_VEC(TO, C)                                                                      \
+  post_norm_vec_kernel<TO, C><<<N, vthreads, 0, stream>>>(residual, branches, n, inner_eps,   \
+                                                          alpha, w, eps, static_cast<TO*>(cast), H)
+#define EI_PN(TO)                                                                             \
+  do {                                                                                        \
+    if (chunks == 1) EI_PN_VEC(TO, 1);                                                        \
+    else if (chunks == 2) EI_PN_VEC(TO, 2);                                                   \
+    else if (chunks == 3 || chunks == 4) EI_PN_VEC(TO, 4);                                    \
+    else                                                                                      \
+      post_norm_kernel<TO><<<N, threads, lds, stream>>>(residual, branches, n, inner_eps,     \
+                                                        alpha, w, eps, static_cast<TO*>(cast), H); \
+  } while (0)
+  if (!cast || cast_dtype == EI_F32) EI_PN(float);
+  else if (cast_dtype == EI_BF16) EI_PN(bf16_t);
+  else EI_REQUIRE(false, "post_norm: unknown dtype");
+#undef EI_PN
+#undef EI_PN_VEC
   EI_LAUNCH_CHECK();
 }

@@ -352,28 +352,50 @@ extern "C" int ei_qk_norm_rope_store(
 
 // ---------------------------------------------------------------------------------------
 // Queries and keys normed over the whole projection (one RMS norm over all heads of q, one
-// over all heads of k, weights of those widths; or no norm), no rotation, and values whose
-// head size may differ from the keys'.  One block a row; sums in float32, one rounding.
+// over all heads of k, weights of those widths; or no norm), then, with frequencies, neighbouring
+// elements (2i, 2i + 1) of the first R of every query and key head turned by position * f_i
+// (cosine and sine times turn_scale), and values whose head size may differ from the keys'.
+// VK: the rows hold no values of their own, the values are the keys as projected, before norm and
+// rotation.  Rows lie row_stride apart and begin with [q | k | v].  One block a row; sums in
+// float32, one rounding.
 namespace {
+
+// Elements d .. d + 3 of a head (d a multiple of 4).
+template <typename TO>
+__device__ __forceinline__ void turn_quad(float (&x)[4], int d, int R, int pos,
+                                          const double* __restrict__ freqs, float turn_scale) {
+#pragma unroll
+  for (int p = 0; p < 2; ++p) {
+    if (d + 2 * p >= R) continue;
+    float sn, cs;
+    ei::turn_at<TO>(pos, freqs[d / 2 + p], sn, cs);
+    cs *= turn_scale;
+    sn *= turn_scale;
+    const float u = x[2 * p], v = x[2 * p + 1];
+    x[2 * p] = u * cs - v * sn;
+    x[2 * p + 1] = v * cs + u * sn;
+  }
+}
 
 // The same for rows of at most 4 x 256 16-byte pieces whose widths are all multiples of 4: a
 // thread keeps its pieces in registers between the sums of squares and the stores, and the two
 // sums cross the block together.
-template <typename TI, typename TO, int CH>
+template <typename TI, typename TO, int CH, bool VK>
 __global__ void __launch_bounds__(256)
 projection_norm_store_reg_kernel(
-    const TI* __restrict__ qkv, int nsplit, size_t split_stride, const float* __restrict__ bias,
+    const TI* __restrict__ qkv, int nsplit, size_t split_stride, size_t row_stride,
+    const float* __restrict__ bias,
     const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, float eps,
     const int32_t* __restrict__ row_pos, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ page_table, int table_width, TO* __restrict__ q_out,
     TO* __restrict__ k_pages, TO* __restrict__ v_pages, int nq, int nkv, int D, int DV,
-    int write_cache) {
+    int write_cache, const double* __restrict__ freqs, int R, float turn_scale) {
   __shared__ float sums[2][4];
   const int row = blockIdx.x;
   const int seq = row_seq[row];
   if (seq < 0) return;                      // padding row of a fixed-size batch
-  const int QW = nq * D, KW = nkv * D, VW = nkv * DV, W = QW + KW + VW;
-  const TI* src = qkv + static_cast<size_t>(row) * W;
+  const int QW = nq * D, KW = nkv * D, VW = VK ? 0 : nkv * DV, W = QW + KW + VW;
+  const TI* src = qkv + static_cast<size_t>(row) * row_stride;
   float x[CH][4];
   float q_sq = 0.f, k_sq = 0.f;
 #pragma unroll
@@ -424,14 +446,19 @@ projection_norm_store_reg_kernel(
 #pragma unroll
         for (int e = 0; e < 4; ++e) x[c][e] = (x[c][e] * q_inv) * w[e];
       }
+      if (R > 0) turn_quad<TO>(x[c], i % D, R, pos, freqs, turn_scale);
       ei::Vec4<TO>::store(q_out + static_cast<size_t>(row) * QW + i, x[c]);
     } else if (phys >= 0 && i < QW + KW) {
       const int at = i - QW, head = at / D, d = at % D;
+      if constexpr (VK)
+        ei::Vec4<TO>::store(
+            v_pages + ((static_cast<size_t>(phys) * nkv + head) * EI_PAGE + in_page) * D + d, x[c]);
       if (k_norm_w) {
         ei::Vec4<float>::load(k_norm_w + at, w);
 #pragma unroll
         for (int e = 0; e < 4; ++e) x[c][e] = (x[c][e] * k_inv) * w[e];
       }
+      if (R > 0) turn_quad<TO>(x[c], d, R, pos, freqs, turn_scale);
       ei::Vec4<TO>::store(
           k_pages + ((static_cast<size_t>(phys) * nkv + head) * EI_PAGE + in_page) * D + d, x[c]);
     } else if (phys >= 0) {
@@ -442,21 +469,22 @@ projection_norm_store_reg_kernel(
   }
 }
 
-template <typename TI, typename TO, bool VEC>
+template <typename TI, typename TO, bool VEC, bool VK>
 __global__ void projection_norm_store_kernel(
-    const TI* __restrict__ qkv, int nsplit, size_t split_stride, const float* __restrict__ bias,
+    const TI* __restrict__ qkv, int nsplit, size_t split_stride, size_t row_stride,
+    const float* __restrict__ bias,
     const float* __restrict__ q_norm_w, const float* __restrict__ k_norm_w, float eps,
     const int32_t* __restrict__ row_pos, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ page_table, int table_width, TO* __restrict__ q_out,
     TO* __restrict__ k_pages, TO* __restrict__ v_pages, int nq, int nkv, int D, int DV,
-    int write_cache) {
+    int write_cache, const double* __restrict__ freqs, int R, float turn_scale) {
   extern __shared__ __attribute__((aligned(16))) float row_values[];     // the row's q, k and v sums
   __shared__ float scratch[16];
   const int row = blockIdx.x;
   const int seq = row_seq[row];
   if (seq < 0) return;                      // padding row of a fixed-size batch
-  const int QW = nq * D, KW = nkv * D, VW = nkv * DV, W = QW + KW + VW;
-  const TI* src = qkv + static_cast<size_t>(row) * W;
+  const int QW = nq * D, KW = nkv * D, VW = VK ? 0 : nkv * DV, W = QW + KW + VW;
+  const TI* src = qkv + static_cast<size_t>(row) * row_stride;
   float q_sq = 0.f, k_sq = 0.f;
   if constexpr (VEC) {      // every width a multiple of 4: 16-byte pieces, 8 slices per trip
     for (int i = threadIdx.x * 4; i < W; i += blockDim.x * 4) {
@@ -513,14 +541,19 @@ __global__ void projection_norm_store_kernel(
 #pragma unroll
           for (int e = 0; e < 4; ++e) x[e] = (x[e] * q_inv) * w[e];
         }
+        if (R > 0) turn_quad<TO>(x, i % D, R, pos, freqs, turn_scale);
         ei::Vec4<TO>::store(q_out + static_cast<size_t>(row) * QW + i, x);
       } else if (phys >= 0 && i < QW + KW) {
         const int at = i - QW, head = at / D, d = at % D;
+        if constexpr (VK)
+          ei::Vec4<TO>::store(
+              v_pages + ((static_cast<size_t>(phys) * nkv + head) * EI_PAGE + in_page) * D + d, x);
         if (k_norm_w) {
           ei::Vec4<float>::load(k_norm_w + at, w);
 #pragma unroll
           for (int e = 0; e < 4; ++e) x[e] = (x[e] * k_inv) * w[e];
         }
+        if (R > 0) turn_quad<TO>(x, d, R, pos, freqs, turn_scale);
         ei::Vec4<TO>::store(
             k_pages + ((static_cast<size_t>(phys) * nkv + head) * EI_PAGE + in_page) * D + d, x);
       } else if (phys >= 0) {
@@ -531,15 +564,30 @@ __global__ void projection_norm_store_kernel(
     }
     return;
   }
-  for (int i = threadIdx.x; i < QW; i += blockDim.x) {
-    const float y = q_norm_w ? (row_values[i] * q_inv) * q_norm_w[i] : row_values[i];
-    q_out[static_cast<size_t>(row) * QW + i] = ei::from_f32<TO>(y);
-  }
+  // element i of a projection whose values lie from `at` on, normed and turned
+  auto made = [&](int at, int i, float inv, const float* w) {
+    float y = w ? (row_values[at + i] * inv) * w[i] : row_values[at + i];
+    const int d = i % D;
+    if (d < R) {
+      const int j = d % 2 == 0 ? i + 1 : i - 1;              // its partner in the rotation
+      const float z = w ? (row_values[at + j] * inv) * w[j] : row_values[at + j];
+      float sn, cs;
+      ei::turn_at<TO>(pos, freqs[d / 2], sn, cs);
+      cs *= turn_scale;
+      sn *= turn_scale;
+      y = d % 2 == 0 ? y * cs - z * sn : y * cs + z * sn;
+    }
+    return y;
+  };
+  for (int i = threadIdx.x; i < QW; i += blockDim.x)
+    q_out[static_cast<size_t>(row) * QW + i] = ei::from_f32<TO>(made(0, i, q_inv, q_norm_w));
   if (phys < 0) return;
   for (int i = threadIdx.x; i < KW; i += blockDim.x) {
     const int head = i / D, d = i % D;
-    const float x = row_values[QW + i];
-    const float y = k_norm_w ? (x * k_inv) * k_norm_w[i] : x;
+    if constexpr (VK)
+      v_pages[((static_cast<size_t>(phys) * nkv + head) * EI_PAGE + in_page) * D + d] =
+          ei::from_f32<TO>(row_values[QW + i]);
+    const float y = made(QW, i, k_inv, k_norm_w);
     k_pages[((static_cast<size_t>(phys) * nkv + head) * EI_PAGE + in_page) * D + d] =
         ei::from_f32<TO>(y);
   }
@@ -552,16 +600,18 @@ __global__ void projection_norm_store_kernel(
 
 }  // namespace
 
-// qkv: [nsplit][N, nq * D + nkv * D + nkv * DV] of in_dtype; q_out: [N, nq * D]; key pages
+// qkv: [nsplit][N, row_stride] of in_dtype, rows that begin with nq * D + nkv * D (+ nkv * DV
+// unless values_from_keys, which needs DV = D) columns; q_out: [N, nq * D]; key pages
 // [n_pages, nkv, 64, D], value pages [n_pages, nkv, 64, DV] of out_dtype; q_norm_w [nq * D] and
 // k_norm_w [nkv * D] float32, or both null (no norm); bias: float32 [row width] added to the
-// sums, or null.
+// sums, or null; freqs: float64 [rot_dim / 2], or null for no rotation.
 extern "C" int ei_projection_norm_store(
-    const void* qkv, int in_dtype, int nsplit, long long split_stride, const float* bias,
-    const float* q_norm_w,
+    const void* qkv, int in_dtype, int nsplit, long long split_stride, long long row_stride,
+    const float* bias, const float* q_norm_w,
     const float* k_norm_w, float eps, const int32_t* row_pos, const int32_t* row_seq,
     const int32_t* page_table, int table_width, void* q_out, void* k_pages, void* v_pages,
-    int out_dtype, int N, int nq, int nkv, int D, int DV, int write_cache, hipStream_t stream) {
+    int out_dtype, int N, int nq, int nkv, int D, int DV, int write_cache,
+    int values_from_keys, const double* freqs, int rot_dim, float turn_scale, hipStream_t stream) {
   EI_REQUIRE(N > 0 && nq > 0 && nkv > 0 && D > 0 && DV > 0,
              "projection_norm_store: sizes must be positive");
   EI_REQUIRE(qkv && row_pos && row_seq && q_out, "projection_norm_store: null pointer");
@@ -570,7 +620,14 @@ extern "C" int ei_projection_norm_store(
   EI_REQUIRE(!write_cache || (k_pages && v_pages && page_table && table_width > 0),
              "projection_norm_store: cache pointers missing");
   EI_REQUIRE(nsplit >= 1, "projection_norm_store: nsplit must be at least 1");
-  const long long width = static_cast<long long>(nq) * D + static_cast<long long>(nkv) * (D + DV);
+  EI_REQUIRE(!values_from_keys || DV == D,
+             "projection_norm_store: values that are the keys are as wide as they are");
+  const int R = freqs ? rot_dim : 0;
+  EI_REQUIRE(R >= 0 && R % 2 == 0 && R <= D,
+             "projection_norm_store: the rotated width must be even and at most head_dim");
+  const long long width = static_cast<long long>(nq) * D +
+                          static_cast<long long>(nkv) * (values_from_keys ? D : D + DV);
+  EI_REQUIRE(row_stride >= width, "projection_norm_store: rows narrower than the projections");
   EI_REQUIRE(width * 4 <= 160 * 1024 - 1024, "projection_norm_store: the row does not fit in LDS");
   const size_t lds = static_cast<size_t>(width) * sizeof(float);
   const int threads = width >= 2048 ? 512 : 256;
@@ -579,36 +636,43 @@ extern "C" int ei_projection_norm_store(
                         reinterpret_cast<uintptr_t>(k_pages) | reinterpret_cast<uintptr_t>(v_pages) |
                         reinterpret_cast<uintptr_t>(q_norm_w) | reinterpret_cast<uintptr_t>(k_norm_w) |
                         reinterpret_cast<uintptr_t>(bias)) % 16 == 0;
-  const bool vec = D % 4 == 0 && DV % 4 == 0 && ss % 4 == 0 && aligned;
-#define EI_PNS_V(TI, TO, VV)                                                                    \
+  const size_t rs = static_cast<size_t>(row_stride);
+  const bool vec = D % 4 == 0 && DV % 4 == 0 && ss % 4 == 0 && rs % 4 == 0 && aligned;
+#define EI_PNS_V(TI, TO, VV, VK)                                                                   \
   do {                                                                                          \
     if (lds > 64 * 1024)                                                                        \
       (void)hipFuncSetAttribute(                                                                \
-          reinterpret_cast<const void*>(&projection_norm_store_kernel<TI, TO, VV>),             \
+          reinterpret_cast<const void*>(&projection_norm_store_kernel<TI, TO, VV, VK>),             \
           hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds));                   \
-    projection_norm_store_kernel<TI, TO, VV><<<N, threads, lds, stream>>>(                      \
-        static_cast<const TI*>(qkv), nsplit, ss, bias, q_norm_w, k_norm_w, eps, row_pos,        \
+    projection_norm_store_kernel<TI, TO, VV, VK><<<N, threads, lds, stream>>>(                      \
+        static_cast<const TI*>(qkv), nsplit, ss, rs, bias, q_norm_w, k_norm_w, eps, row_pos,        \
         row_seq, page_table, table_width, static_cast<TO*>(q_out), static_cast<TO*>(k_pages),   \
-        static_cast<TO*>(v_pages), nq, nkv, D, DV, write_cache);                                \
+        static_cast<TO*>(v_pages), nq, nkv, D, DV, write_cache, freqs, R, turn_scale);                            \
   } while (0)
-#define EI_PNS_R(TI, TO, CC)                                                                    \
-  projection_norm_store_reg_kernel<TI, TO, CC><<<N, 256, 0, stream>>>(                          \
-      static_cast<const TI*>(qkv), nsplit, ss, bias, q_norm_w, k_norm_w, eps, row_pos, row_seq, \
+#define EI_PNS_R(TI, TO, CC, VK)                                                                   \
+  projection_norm_store_reg_kernel<TI, TO, CC, VK><<<N, 256, 0, stream>>>(                          \
+      static_cast<const TI*>(qkv), nsplit, ss, rs, bias, q_norm_w, k_norm_w, eps, row_pos, row_seq, \
       page_table, table_width, static_cast<TO*>(q_out), static_cast<TO*>(k_pages),              \
-      static_cast<TO*>(v_pages), nq, nkv, D, DV, write_cache)
-#define EI_PNS(TI, TO)                                   \
-  do {                                                   \
-    if (vec && width <= 1024) EI_PNS_R(TI, TO, 1);       \
-    else if (vec && width <= 2048) EI_PNS_R(TI, TO, 2);  \
-    else if (vec && width <= 4096) EI_PNS_R(TI, TO, 4);  \
-    else if (vec) EI_PNS_V(TI, TO, true);                \
-    else EI_PNS_V(TI, TO, false);                        \
+      static_cast<TO*>(v_pages), nq, nkv, D, DV, write_cache, freqs, R, turn_scale)
+#define EI_PNS_K(TI, TO, VK)                                 \
+  do {                                                       \
+    if (vec && width <= 1024) EI_PNS_R(TI, TO, 1, VK);       \
+    else if (vec && width <= 2048) EI_PNS_R(TI, TO, 2, VK);  \
+    else if (vec && width <= 4096) EI_PNS_R(TI, TO, 4, VK);  \
+    else if (vec) EI_PNS_V(TI, TO, true, VK);                \
+    else EI_PNS_V(TI, TO, false, VK);                        \
+  } while (0)
+#define EI_PNS(TI, TO)                            \
+  do {                                            \
+    if (values_from_keys) EI_PNS_K(TI, TO, true); \
+    else EI_PNS_K(TI, TO, false);                 \
   } while (0)
   if (in_dtype == EI_F32 && out_dtype == EI_F32) EI_PNS(float, float);
   else if (in_dtype == EI_F32 && out_dtype == EI_BF16) EI_PNS(float, bf16_t);
   else if (in_dtype == EI_BF16 && out_dtype == EI_BF16) EI_PNS(bf16_t, bf16_t);
   else EI_REQUIRE(false, "projection_norm_store: unsupported dtype combination");
 #undef EI_PNS
+#undef EI_PNS_K
 #undef EI_PNS_R
 #undef EI_PNS_V
   EI_LAUNCH_CHECK();
@@ -643,19 +707,6 @@ __device__ __forceinline__ float sliced(const TI* p, int nsplit, size_t split_st
   float v = 0.f;
   for (int s = 0; s < nsplit; ++s) v += ei::to_f32<TI>(p[s * split_stride]);
   return v;
-}
-
-// Sine and cosine of an angle given in turns (of 2 pi): the whole turns are taken off in float64.
-// For float32 results the library's functions; for bfloat16 results the hardware's (which take
-// turns), good to about 1e-6 and swallowed by the rounding.
-template <typename TO> __device__ __forceinline__ void turn_of(double turns, float& sn, float& cs);
-template <> __device__ __forceinline__ void turn_of<float>(double turns, float& sn, float& cs) {
-  sincosf(static_cast<float>((turns - floor(turns)) * 6.283185307179586), &sn, &cs);
-}
-template <> __device__ __forceinline__ void turn_of<bf16_t>(double turns, float& sn, float& cs) {
-  const float part = static_cast<float>(turns - floor(turns));
-  sn = __builtin_amdgcn_sinf(part);
-  cs = __builtin_amdgcn_cosf(part);
 }
 
 template <typename TI, typename TO>
@@ -741,10 +792,8 @@ __global__ void head_store_kernel(
     if (e < R) {
       const int partner = e < rhalf ? e + rhalf : e - rhalf;
       const float p = w ? (y[j] * inv) * w[partner] : y[j];
-      const double turns = static_cast<double>(pos) * freqs[e < rhalf ? e : e - rhalf] *
-                           0.15915494309189535;       // in units of 2 pi
       float sn, cs;
-      turn_of<TO>(turns, sn, cs);
+      ei::turn_at<TO>(pos, freqs[e < rhalf ? e : e - rhalf], sn, cs);
       cs *= turn_scale;
       sn *= turn_scale;
       v = e < rhalf ? v * cs - p * sn : v * cs + p * sn;
@@ -872,9 +921,8 @@ __global__ void head_store_vec_kernel(
     const int f0 = e0 < rhalf ? e0 : e0 - rhalf;
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      const double whole = static_cast<double>(pos) * freqs[f0 + i] * 0.15915494309189535;
       float sn, cs;
-      turn_of<TO>(whole, sn, cs);
+      ei::turn_at<TO>(pos, freqs[f0 + i], sn, cs);
       cs *= turn_scale;
       sn *= turn_scale;
       x[i] = e0 < rhalf ? x[i] * cs - y[i] * sn : x[i] * cs + y[i] * sn;

@@ -1,6 +1,6 @@
 from .attention import Attention
 from .base import KVRequest, StateRequest, StepContext, Workspace
-from .block import OutputNormBlock, PendingNorm, PreNormBlock, SandwichBlock
+from .block import OutputNormBlock, PendingNorm, PostNormBlock, PreNormBlock, SandwichBlock
 from .delta import GatedDelta
 from .latent import LatentAttention
 from .linear_attention import LinearAttention
@@ -33,10 +33,11 @@ register_position("rope_pairs", RotaryFrequencies)
 register_position("rope_half", RotaryHalfFrequencies)
 register_block("prenorm", PreNormBlock)
 register_block("outnorm", OutputNormBlock)
+register_block("postnorm", PostNormBlock)
 register_block("sandwich", SandwichBlock)
 
 __all__ = ["Attention", "KVRequest", "StateRequest", "StepContext", "Workspace", "PreNormBlock",
-           "OutputNormBlock", "PendingNorm", "SandwichBlock", "GatedDelta", "LatentAttention", "MatrixMemory", "RotaryFrequencies",
+           "OutputNormBlock", "PostNormBlock", "PendingNorm", "SandwichBlock", "GatedDelta", "LatentAttention", "MatrixMemory", "RotaryFrequencies",
            "RotaryHalfFrequencies", "RoutedMLP", "LayerNorm", "LinearAttention", "ParallelMixer", "StateSpace", "DenseMLP", "Linear", "GatedMLP", "RMSNorm", "lookup", "register_block", "register_feed_forward",
            "register_mixer", "register_norm", "register_position", "unregister", "NoPosition",
            "RotaryTable"]

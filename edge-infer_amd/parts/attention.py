@@ -41,6 +41,12 @@ its own, one entry a block, which `lib.pool_store` fills from the cached tokens 
 become complete, and the generic kernel walks after the window).  Biases of these projections
 are added by the store kernel where the product leaves them to it.
 
+`values_from_keys`: there is no value projection, a position's values are its keys as projected,
+before norm and rotation; with a norm over the whole projection and a rotation of neighbouring
+pairs the store kernel of the whole projection (`lib.projection_norm_store`) norms, turns and
+stores.  `softcap` c: a scaled score s becomes c tanh(s / c) (forms of their own of the
+matrix-core kernels).
+
 `keep_first`: with a window, the sequence's first positions stay visible however far back they
 lie; the cache never gives their pages back, and every kernel takes the pages (or tiles) of them
 that lie before the window first.  The matrix-core kernels take `output_gate = True` into their
@@ -108,7 +114,8 @@ class Attention:
         params = {"q_proj.weight": ParamSpec((spec.q_width, hidden))}
         if not spec.shared_kv:
             params["k_proj.weight"] = ParamSpec((spec.kv_width, hidden))
-            params["v_proj.weight"] = ParamSpec((spec.v_width, hidden))
+            if not spec.values_from_keys:
+                params["v_proj.weight"] = ParamSpec((spec.v_width, hidden))
         params["o_proj.weight"] = ParamSpec((hidden, spec.out_width))
         if spec.o_bias is not False:
             params["o_proj.bias"] = ParamSpec((hidden,), optional=spec.o_bias is not True)
@@ -119,7 +126,8 @@ class Attention:
             required = spec.qkv_bias is True
             params["q_proj.bias"] = ParamSpec((spec.q_width,), optional=not required)
             params["k_proj.bias"] = ParamSpec((spec.kv_width,), optional=not required)
-            params["v_proj.bias"] = ParamSpec((spec.v_width,), optional=not required)
+            if not spec.values_from_keys:
+                params["v_proj.bias"] = ParamSpec((spec.v_width,), optional=not required)
         if spec.qk_norm:
             whole = spec.qk_norm_scope == "projection"
             params["q_norm.weight"] = ParamSpec((spec.q_width if whole else spec.head_dim,),
@@ -166,17 +174,25 @@ class Attention:
     def kernel_libraries(cls, spec, dtype):
         """What this part will run, so that a model can have it compiled ahead of its first
         step."""
-        group = spec.n_heads // max(1, spec.n_kv_heads)
-        fast = (dtype == torch.bfloat16 and spec.v_dim == spec.head_dim and MATRIX_CORE_ATTENTION
-                and not spec.talking_heads
-                and lib.attention_decode_mfma_supported(spec.head_dim, group))
-        kernels = "attention_mfma" if fast else "attention_generic"
+        kernels = "attention_generic"
+        if cls.on_matrix_cores(spec, dtype):
+            kernels = "attention_mfma" if spec.softcap is None else "attention_capped"
         if cls.wide_keys(spec, dtype):
             kernels = "attention_wide"
         # (the pooled blocks are stored, and beside the matrix-core kernels also gathered, by
         # kernels of the generic library)
         return ("rope_store", kernels, *(("attention_generic",) if spec.pool is not None else ()),
                 *(("head_ops",) if spec.talking_heads else ()), *Linear.kernel_libraries(dtype))
+
+    @classmethod
+    def on_matrix_cores(cls, spec, dtype) -> bool:
+        """Whether this part runs the matrix-core kernels: bfloat16 with head sizes 64 and 128 and
+        values as wide as the keys; every other case runs the generic kernel."""
+        group = spec.n_heads // max(1, spec.n_kv_heads)
+        return (dtype == torch.bfloat16 and spec.v_dim == spec.head_dim and MATRIX_CORE_ATTENTION
+                and not spec.talking_heads
+                and (spec.softcap is None or not (spec.keep_first or spec.output_gate is True))
+                and lib.attention_decode_mfma_supported(spec.head_dim, group))
 
     @classmethod
     def wide_keys(cls, spec, dtype) -> bool:
@@ -189,9 +205,16 @@ class Attention:
     @classmethod
     def general_store(cls, spec) -> bool:
         """Whether the part norms, rotates and stores through `lib.head_store`."""
-        return (spec.position.kind in ("rope_half", "rope_pairs")
+        return (spec.position.kind == "rope_half"
+                or (spec.position.kind == "rope_pairs" and not cls.whole_rotation(spec))
                 or spec.value_mix in ("source", "mix") or bool(spec.output_gate)
                 or spec.qk_unit_norm or spec.query_temperature is not None or spec.shared_kv or spec.pool is not None)
+
+    @staticmethod
+    def whole_rotation(spec) -> bool:
+        """Whether the store kernel of the whole projection turns neighbouring pairs as well."""
+        return spec.position.kind == "rope_pairs" and (
+            spec.qk_norm_scope == "projection" if spec.qk_norm else spec.values_from_keys)
 
     @classmethod
     def check(cls, spec):
@@ -215,7 +238,7 @@ class Attention:
             if not (1 <= spec.head_dim <= 256 and 1 <= spec.v_dim <= 256):
                 raise ValueError("attention: key and value head sizes must lie in 1..256, got "
                                  f"{spec.head_dim} and {spec.v_dim}")
-        elif whole and spec.position.kind == "none":
+        elif whole and (spec.position.kind == "none" or cls.whole_rotation(spec)):
             # the store kernel without a rotation takes any sizes the attention kernel takes
             if not (1 <= spec.head_dim <= 256 and 1 <= spec.v_dim <= 256):
                 raise ValueError("attention: key and value head sizes must lie in 1..256, got "
@@ -223,13 +246,21 @@ class Attention:
         else:
             if spec.qk_norm_scope == "projection" and spec.qk_norm:
                 raise ValueError("attention: a norm over the whole projection is implemented "
-                                 "only without a rotation")
+                                 "without a rotation or with one of neighbouring pairs")
             if spec.v_dim != spec.head_dim:
                 raise ValueError("attention: values of another width than the keys are "
                                  "implemented only without a rotation and per-head norms")
             if spec.head_dim % 16 or not 16 <= spec.head_dim <= 256:
                 raise ValueError("attention: head_dim must be a multiple of 16 between 16 and "
                                  f"256, got {spec.head_dim}")
+        if spec.values_from_keys and (spec.v_dim != spec.head_dim or spec.shared_kv
+                                      or cls.general_store(spec) or not whole
+                                      or spec.position.kind not in ("none", "rope_pairs")):
+            raise ValueError("attention: values that are the keys as projected are as wide as them "
+                             "and implemented with the store of the whole projection only")
+        if spec.softcap is not None and (not spec.softcap > 0 or spec.talking_heads):
+            raise ValueError("attention: a cap on the scores must be positive and goes with no "
+                             "mixed scores")
         if spec.sink and spec.unit_sink:
             raise ValueError("attention: a learned sink and a sink of 1 exclude each other")
         if spec.talking_heads and spec.n_kv_heads * spec.head_dim > 1024:
@@ -271,10 +302,14 @@ class Attention:
         self.dtype = dtype
         q_weight = params["q_proj.weight"]
         k_weight = None if spec.shared_kv else params["k_proj.weight"]
+        names = ("q_proj",) if spec.shared_kv else \
+            ("q_proj", "k_proj") if spec.values_from_keys else ("q_proj", "k_proj", "v_proj")
         position_spec = spec.position
         biases = {name: params[f"{name}.bias"] for name in ("q_proj", "k_proj", "v_proj")
                   if f"{name}.bias" in params}
-        if spec.position.kind == "rope_pairs":
+        if self.whole_rotation(spec):      # the store kernel turns neighbours, by float64 frequencies
+            position_spec = dataclasses.replace(spec.position, kind="rope_half", scaling=None)
+        elif spec.position.kind == "rope_pairs":
             # neighbouring pairs (2i, 2i + 1) become the pairs (i, i + R/2) of permuted rows
             order = self._pairs_to_halves(spec.head_dim, spec.position.dim)
             q_weight = self._permute_heads(q_weight, spec.n_heads, order)
@@ -285,9 +320,9 @@ class Attention:
                     biases[name] = self._permute_heads(biases[name], heads, order)
             position_spec = dataclasses.replace(spec.position, kind="rope_half", scaling=None)
         fused = torch.cat([q_weight]
-                          + ([] if spec.shared_kv else [k_weight, params["v_proj.weight"]])
+                          + ([] if spec.shared_kv else [k_weight])
+                          + ([params["v_proj.weight"]] if "v_proj" in names else [])
                           + ([params["gate_proj.weight"]] if spec.output_gate else []), dim=0)
-        names = ("q_proj",) if spec.shared_kv else ("q_proj", "k_proj", "v_proj")
         fused_bias = None
         if any(name in biases for name in names):   # absent ones count as zero
             fused_bias = torch.cat([
@@ -307,7 +342,8 @@ class Attention:
         self.scale = spec.scale if spec.scale is not None else spec.head_dim ** -0.5
         # without a rotation and without per-head norms, one kernel norms (or not) and stores
         self.general = self.general_store(spec)
-        self.whole_store = (not self.general and spec.position.kind == "none"
+        self.whole_store = (not self.general
+                            and (spec.position.kind == "none" or self.whole_rotation(spec))
                             and (spec.qk_norm_scope == "projection" or not spec.qk_norm))
         self.value_lambda = None
         if spec.value_mix == "mix":
@@ -329,21 +365,18 @@ class Attention:
         self.talk = None
         if spec.talking_heads:
             self.talk = params["talk"].to(device=device, dtype=torch.float32).contiguous()
-        # the matrix-core kernels take bfloat16 with head sizes 64 and 128 and values as wide
-        # as the keys; every other case runs the generic kernel
-        self.matrix_cores = (dtype == torch.bfloat16 and spec.v_dim == spec.head_dim and
-                            MATRIX_CORE_ATTENTION and self.talk is None and
-                            lib.attention_decode_mfma_supported(spec.head_dim, self.group))
+        self.matrix_cores = self.on_matrix_cores(spec, dtype)
         # beside the matrix-core kernels the pooled blocks are gathered by the generic kernel
         # (they are few: one for `pool` tokens) and taken in as one more slice of the softmax
         self.pooled_aside = self.matrix_cores and spec.pool is not None
-        # chunk, slopes, sink, kept first positions: what the kernels take beyond a window
+        # chunk, slopes, sink, kept first positions, cap: what the kernels take beyond a window
         self.wide = self.wide_keys(spec, dtype)
         self.keep_first = spec.keep_first if spec.window is not None else 0
         self.extras = dict(chunk=spec.chunk, slopes=self.slopes, sinks=self.sinks,
-                           keep_first=self.keep_first)
+                           keep_first=self.keep_first, softcap=spec.softcap)
         self.has_extras = (spec.chunk is not None or self.slopes is not None
-                           or self.sinks is not None or self.keep_first > 0)
+                           or self.sinks is not None or self.keep_first > 0
+                           or spec.softcap is not None)
         self.compute_units = lib.compute_units(device)     # the chip's size, for launch plans
         self._decode_launches = {}     # (sequences, pages of context) -> decode_launch's answer
 
@@ -576,7 +609,8 @@ class Attention:
                                   meta.row_pos, meta.row_seq, page_table, q, spec.n_heads,
                                   spec.n_kv_heads, spec.head_dim, window=spec.window,
                                   scale=self.scale, part_o=pool_o, part_ml=pool_ml,
-                                  value_dim=spec.v_dim, pool_only=True, **pooled)
+                                  value_dim=spec.v_dim, pool_only=True, softcap=spec.softcap,
+                                  **pooled)
                     aside = dict(pool_o=pool_o, pool_ml=pool_ml)
         elif (ctx.decode and self.matrix_cores and FUSED_DECODE and qkv.dim() == 3
                 and qkv.dtype == torch.float32 and not self.whole_store and not self.has_extras):
@@ -588,7 +622,10 @@ class Attention:
             lib.projection_norm_store(
                 qkv, self.q_norm, self.k_norm, spec.qk_norm_eps, meta.row_pos, meta.row_seq,
                 page_table, q, k_pages, v_pages, spec.n_heads, spec.n_kv_heads, spec.head_dim,
-                spec.v_dim, write_cache=entry.writes_cache, bias=bias)
+                spec.v_dim, write_cache=entry.writes_cache, bias=bias,
+                values_from_keys=spec.values_from_keys,
+                frequencies=getattr(self.position, "frequencies", None),
+                turn_scale=getattr(self.position, "magnitude", 1.0))
         else:
             q = ctx.buffer("attn.q", (n, spec.q_width))
             lib.qk_norm_rope_store(

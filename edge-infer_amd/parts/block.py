@@ -105,6 +105,7 @@ class OutputNormBlock:
     added when it returns."""
 
     capture_safe = True      # nothing of its own besides its parts' kernels and the cast
+    needs = "norm_add"       # what its norms must be able to do
     CAST_NOTE = "outnorm.cast"     # ctx.notes: (stream rows in the storage type, index of its buffer)
 
     def members(self):
@@ -154,7 +155,7 @@ class OutputNormBlock:
             return {name[len(prefix) + 1:]: tensor for name, tensor in params.items()
                     if name.startswith(prefix + ".")}
         norm_cls = lookup("norm", layer_spec.norm.kind)
-        if not hasattr(norm_cls, "norm_add"):
+        if not hasattr(norm_cls, self.needs):
             raise ValueError(f"norm kind '{layer_spec.norm.kind}' cannot sit on a sublayer's output")
         self.mixer = lookup("mixer", layer_spec.mixer.kind)(
             layer_spec.mixer, hidden, sub("mixer"), dtype, device, positions=positions)
@@ -179,26 +180,65 @@ class OutputNormBlock:
 
     def forward(self, ctx, residual, pending, entry):
         if pending is not None:
-            raise ValueError("outnorm: a delta of the block before is still pending; this "
-                             "arrangement follows only blocks that add everything themselves")
+            raise ValueError("a delta of the block before is still pending; this arrangement "
+                             "follows only blocks that add everything themselves")
         x, index = self._stream_rows(ctx, residual)
-        a = self.mixer.forward(ctx, x, entry)
+        a = self._mixed(ctx, x, entry)
         if self.narrow:
             ctx.release(x)
-        x = self.norm1.norm_add(ctx, residual, a, f"outnorm.x{1 - index}" if self.narrow else None)
-        ctx.release(a)
+        x = self._add(self.norm1, ctx, residual, a, f"outnorm.x{1 - index}" if self.narrow else None)
+        self._release(ctx, a)
         index = 1 - index
         if self.ffn is not None:
             f = self.ffn.forward(ctx, residual if x is None else x)
             if self.narrow:
                 ctx.release(x)
-            x = self.norm2.norm_add(ctx, residual, f,
-                                    f"outnorm.x{1 - index}" if self.narrow else None)
+            x = self._add(self.norm2, ctx, residual, f,
+                          f"outnorm.x{1 - index}" if self.narrow else None)
             ctx.release(f)
             index = 1 - index
         if self.narrow:
             ctx.notes[self.CAST_NOTE] = (x, index)
         return None
+
+    def _mixed(self, ctx, x, entry):
+        return self.mixer.forward(ctx, x, entry)
+
+    def _add(self, norm, ctx, residual, delta, cast_name):
+        """The sublayer's output joins the stream; the stream's rounded rows, where asked for."""
+        return norm.norm_add(ctx, residual, delta, cast_name)
+
+    def _release(self, ctx, delta):
+        ctx.release(delta)
+
+
+class PostNormBlock(OutputNormBlock):
+    """x <- norm1(alpha x + mixer(x)); x <- norm2(alpha x + feed_forward(x)), alpha the spec's
+    `stream_scale`: as in `OutputNormBlock` the sublayers read the stream itself, but the norm is
+    taken over the scaled stream and the sublayer's output together and its result is the new
+    stream.  One kernel a sublayer does the sum, the norm and the rounded rows for the next
+    reader; with mixers side by side (`parts.parallel`) their norms and their mean as well."""
+
+    needs = "norm_sum"
+
+    @classmethod
+    def kernel_libraries(cls, layer_spec, dtype):
+        return ("norms", *super().kernel_libraries(layer_spec, dtype))
+
+    def __init__(self, layer_spec, hidden, params, dtype, device, positions):
+        super().__init__(layer_spec, hidden, params, dtype, device, positions)
+        self.alpha = float(layer_spec.stream_scale)
+
+    def _mixed(self, ctx, x, entry):
+        if getattr(self.mixer, "join_later", False):
+            return self.mixer.forward(ctx, x, entry, join_later=True)
+        return self.mixer.forward(ctx, x, entry)
+
+    def _add(self, norm, ctx, residual, delta, cast_name):
+        return norm.norm_sum(ctx, residual, delta, self.alpha, cast_name)
+
+    def _release(self, ctx, delta):
+        ctx.release(*getattr(delta, "outputs", (delta,)))
 
 
 class PendingNorm:

@@ -3,7 +3,8 @@
 y = x * rsqrt(mean(x^2) + eps) * w, all in float32, rounded once to the storage
 type (the reference's float32 path, operators/src/cuda/rms_norm_cuda.cu:99-100;
 its bfloat16 path rounds twice, :91-98, which this implementation does not copy).
-The weight is kept in float32 whatever it was stored in.
+The weight is kept in float32 whatever it was stored in; the spec may name a number that it
+is stored without (`weight_offset`).
 """
 from __future__ import annotations
 
@@ -22,12 +23,18 @@ class RMSNorm:
 
     @classmethod
     def parameters(cls, spec, width):
+        offset = getattr(spec, "weight_offset", 0.0)
+        if offset:
+            return {"weight": ParamSpec((width,), init="uniform", low=0.9 - offset, high=1.1 - offset)}
         return {"weight": ParamSpec((width,), init="norm")}
 
     def __init__(self, spec, width, params, dtype, device):
         self.eps = float(spec.eps)
         self.width = width
         self.weight = params["weight"].to(device=device, dtype=torch.float32).contiguous()
+        offset = getattr(spec, "weight_offset", 0.0)
+        if offset:
+            self.weight = self.weight + float(offset)
 
     def add_norm(self, ctx, residual, delta, out_name, rows=None, write_residual=True):
         """residual += delta (all splits); returns rmsnorm(residual)[rows] * weight in
@@ -47,6 +54,20 @@ class RMSNorm:
         if cast_name is not None:
             cast = ctx.buffer(cast_name, tuple(residual.shape))
         lib.norm_add(residual, delta, self.weight, self.eps, cast_out=cast, bias=bias)
+        return cast
+
+    def norm_sum(self, ctx, residual, delta, alpha, cast_name=None):
+        """residual <- rmsnorm(alpha residual + delta) * weight: the norm over the sum.  `delta`:
+        what a sublayer returned, or `parts.parallel.Branches`, whose norms and mean are then
+        part of the same kernel.  With `cast_name` as for `norm_add`."""
+        cast = None
+        if cast_name is not None:
+            cast = ctx.buffer(cast_name, tuple(residual.shape))
+        more = {}
+        if hasattr(delta, "weights"):
+            more = dict(branch_weights=delta.weights, branch_eps=delta.eps)
+            delta = delta.outputs
+        lib.post_norm(residual, delta, alpha, self.weight, self.eps, cast_out=cast, **more)
         return cast
 
 

@@ -20,6 +20,15 @@ from .registry import lookup
 
 
 @dataclass(frozen=True)
+class Branches:
+    """The branches' outputs before their norms and their mean, for a caller whose next kernel
+    takes those in."""
+    outputs: tuple
+    weights: tuple
+    eps: float
+
+
+@dataclass(frozen=True)
 class BranchEntry:
     """A branch's view of the layer's schedule entry: its own part of the cache entry."""
     layer: int
@@ -109,12 +118,17 @@ class ParallelMixer:
                 sections.update(branch.plan_step(plan))
         return sections
 
-    def forward(self, ctx, x, entry):
+    join_later = True      # forward(..., join_later=True) hands the branches' outputs on
+
+    def forward(self, ctx, x, entry, join_later=False):
+        """The mean of the normed branches; with `join_later`, the `Branches` themselves."""
         outputs = []
         for name, branch in zip(self.names, self.branches):
             outputs.append(branch.forward(ctx, x, BranchEntry(
                 layer=entry.layer, cache=(entry.cache, name), writes_cache=entry.writes_cache,
                 own_id=(entry.own_id, name))))
+        if join_later:
+            return Branches(tuple(outputs), tuple(self.out_norms), self.spec.norm_eps)
         out = ctx.buffer("parallel.out", (x.shape[0], self.hidden), torch.float32)
         lib.norm_mean(outputs, self.out_norms, self.spec.norm_eps, out)
         ctx.release(*outputs)
