@@ -2,7 +2,7 @@
 
     python bench.py [--gpus 1] [--steps K] [--warmup W] [--batch 8] [--layers L]
                     [--shape 8b|0.6b|32b] [--only decode|prefill|generate] [--prompt P]
-                    [--with-32b] [--peaks] [--design tirurax|zadenex|vafepel|gopuzen|dazapel [--design-shape 1k|2k|4k]]
+                    [--with-32b] [--peaks] [--design tirurax|zadenex|vafepel|gopuzen|dazapel|lemotar [--design-shape 1k|2k|4k]]
 
 Prints one JSON line.  `value` is decoded tokens per second at the given batch after
 512-token prompts (one step = one decode step of the whole batch: the model, greedy
@@ -38,6 +38,10 @@ dense and routed over 8 experts and 2 identity experts) beside the Vafepel model
 width, layers, heads and parameters at work for a token.  `--design dazapel` does the same for a
 Dazapel model (window attention that keeps the first tokens, feed-forwards routed within groups
 of 16 experts beside a shared one) beside the Gopuzen model of the same width, layers and heads.
+`--design lemotar` does the same for a Lemotar model (layers of window attention whose values are
+its keys beside the delta rule with a decay per key channel, and of latent attention with a window,
+every second of the latter reading the latents of the one before it; norms over the sum of stream
+and sublayer) beside the Zadenex model of the same width, layers, heads and feed-forward.
 Synthetic token ids, seeded random weights N(0, 0.02).  Peaks are the MI355X's published
 ones: HBM 8 TB/s, dense bf16 MFMA 2.5 PFLOP/s; `measured_peaks` (and `--peaks` alone) say what
 a plain read kernel and a loop of matrix-core products reach on the GPU at hand, and the
@@ -527,6 +531,45 @@ def dazapel_configs(shape):
     return new, old
 
 
+def lemotar_configs(shape):
+    """(Lemotar configuration, Zadenex configuration) of equal width, layers, heads, head size and
+    feed-forward.  Lemotar: window attention with values that are the keys, a rotation of a quarter
+    of the head and capped scores, beside the delta rule with a decay per key channel (ranks of
+    one head size), in turn with latent attention (a latent four head sizes wide, a rotated part
+    of half a head size with stretched frequencies, the same window), every second of the latter
+    reading the latents of the one before it.  Zadenex: `zadenex_configs`."""
+    from edge_infer_amd.config import LemotarConfig
+    layers, width, d_heads, d_kv, a_heads, a_kv, dim, chunk, vocab = DESIGN_SHAPES[shape]
+    mlp = {"kind": "dense", "ff": (2 * 4 * width // 3 + 255) // 256 * 256}
+    parallel = {"type": "parallel",
+                "mixer": {"left": {"heads": a_heads, "kv_heads": a_kv, "dim": dim, "vdim": dim,
+                                   "scale": dim ** -0.5, "softcap": 30.0, "mask": {"size": chunk},
+                                   "rot": {"base": 500000.0, "dims": dim // 4}},
+                          "right": {"heads": d_heads, "kv_heads": d_kv, "dim": dim, "vdim": dim,
+                                    "conv": 4}}, "mlp": mlp}
+    latent = {"heads": a_heads, "dim": dim, "rot_dim": dim // 2, "vdim": dim, "kv_rank": 4 * dim,
+              "scale": (1.5 * dim) ** -0.5, "mask": {"size": chunk},
+              "rot": {"base": 500000.0, "dims": dim // 2,
+                      "scaling": {"factor": 4.0, "original": 8192, "fast": 16.0, "slow": 1.0}}}
+    order, last_latent = [], None
+    for i in range(layers):
+        if i % 2 == 0:
+            order.append(parallel)
+            continue
+        mixer = dict(latent)
+        if last_latent is not None:
+            mixer["kv_from"] = last_latent
+            last_latent = None
+        else:
+            last_latent = i
+        order.append({"type": "latent_attention", "mixer": mixer, "mlp": mlp})
+    new = LemotarConfig.from_dict({"architecture": "Lemotar", "vocab": vocab, "width": width,
+                                   "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+                                   "postln_alpha": 2.0, "layers": order})
+    old, _ = zadenex_configs(shape)
+    return new, old
+
+
 def measure_prompts(model, vocab, batch, tokens, repeats=3):
     """Best ms of one step over `batch` prompts of `tokens` tokens that start together."""
     import types
@@ -553,7 +596,7 @@ def measure_prompts(model, vocab, batch, tokens, repeats=3):
 def design_comparison(args):
     """Prefill and decode of the design's shape and of the closest other model of equal size
     (Tirurax beside Qwen3, Zadenex and Vafepel beside Tirurax, Gopuzen beside Vafepel, Dazapel
-    beside Gopuzen)."""
+    beside Gopuzen, Lemotar beside Zadenex)."""
     import types
     import torch
     import edge_infer_amd as ei
@@ -569,6 +612,9 @@ def design_comparison(args):
     elif args.design == "dazapel":
         new, old = dazapel_configs(args.design_shape)
         which = {"dazapel": new, "gopuzen": old}
+    elif args.design == "lemotar":
+        new, old = lemotar_configs(args.design_shape)
+        which = {"lemotar": new, "zadenex": old}
     else:
         new, old = design_configs(args.design_shape)
         which = {"tirurax": new, "qwen3": old}
@@ -628,13 +674,13 @@ def main():
                         help="leave the 32B shape (decode at batch 1 and 16, prefill) out of `points`")
     parser.add_argument("--peaks", action="store_true",
                         help="measure the read and matrix-core yardsticks only")
-    parser.add_argument("--design", choices=["tirurax", "zadenex", "vafepel", "gopuzen", "dazapel"],
+    parser.add_argument("--design", choices=["tirurax", "zadenex", "vafepel", "gopuzen", "dazapel", "lemotar"],
                         default=None,
                         help="measure this design beside the closest other model of equal size "
                              "(tirurax beside qwen3, zadenex beside tirurax) instead of the "
                              "default workload")
     parser.add_argument("--design-shape", choices=sorted(DESIGN_SHAPES), default="2k")
-    parser.add_argument("--design-only", choices=["dazapel", "gopuzen", "vafepel", "zadenex", "tirurax", "qwen3"],
+    parser.add_argument("--design-only", choices=["lemotar", "dazapel", "gopuzen", "vafepel", "zadenex", "tirurax", "qwen3"],
                         default=None,
                         help="with --design: one of the two models only (for profiling)")
     args = parser.parse_args()
