@@ -325,7 +325,8 @@ extern "C" int ei_attn_wide_positions(int G) {
 // q: [N, nq, key_heads * D]; key pages [pages, nkv, 64, D]; value pages [pages, nkv, 64, DV] (not
 // read with values_in_keys); out [N, nq, DV]; all bfloat16.  Items as in ei_attention, with at
 // most ei_attn_wide_positions positions each.  n_splits > 1: items of one position, scratch
-// part_o [N, nq, n_splits, DV] and part_ml [N, nq, n_splits, 2], merged here.
+// part_o [N, nq, n_splits, DV] and part_ml [N, nq, n_splits, 2], merged here unless merge is 0 (the
+// caller's next kernel then reads the slices, and `out` is not written).
 extern "C" int ei_attention_wide(const void* q, const void* k_pages, const void* v_pages,
                                  const int32_t* item_seq, const int32_t* item_row0,
                                  const int32_t* item_npos, int n_items, const int32_t* row_pos,
@@ -333,7 +334,8 @@ extern "C" int ei_attention_wide(const void* q, const void* k_pages, const void*
                                  int table_width, void* out, float* part_o, float* part_ml, int N,
                                  int nq, int nkv, int D, int DV, int window, const float* sinks,
                                  float scale, int n_splits, int key_heads, int values_in_keys,
-                                 const float* gate, hipStream_t stream) {
+                                 const float* gate, int merge, hipStream_t stream) {
+  EI_REQUIRE(merge || (n_splits > 1 && !gate), "attention_wide: nothing to merge later");
   EI_REQUIRE(n_items > 0 && N > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention_wide: bad sizes");
   EI_REQUIRE(key_heads == 1 || key_heads == nkv,
              "attention_wide: a query meets the keys of its own kv head or of all of them");
@@ -392,7 +394,7 @@ extern "C" int ei_attention_wide(const void* q, const void* k_pages, const void*
     ei_set_error(hipGetErrorString(e));
     return static_cast<int>(e);
   }
-  if (n_splits > 1) {
+  if (n_splits > 1 && merge) {
     const int total = N * nq;
     const int threads = 256;
     const int blocks = (total * EI_WAVE + threads - 1) / threads;

@@ -28,6 +28,7 @@
 //                column; tokens come in tiles through LDS
 //   delta_out    the read-out's norm and gate
 #include "common.h"
+#include "few_rows.h"
 
 namespace {
 
@@ -250,10 +251,7 @@ __global__ void delta_conv_vec_kernel(const TI* __restrict__ proj, int nsplit, s
 // low-rank parts (ra and rg wide) begin in a projection row; wa [ra, HD], wg [rg, GW]: their second
 // matrices, transposed; the decays go behind the convolved channels of `out`, the gate's logits to
 // gate_out [N, GW].  Blocks 0 .. conv_blocks * N - 1 convolve 1,024 (four a thread) or 256 channels
-// of a row; the others make 64 columns of up to 16 rows each: four threads a column with a quarter
-// of every piece of 128 ranks, whose weights are all requested at once, added up through LDS.
-constexpr int kLowRows = 16, kLowK = 128, kLowCols = 64, kLowParts = 4;
-
+// of a row; the others make 64 columns of R rows each.
 struct LowRank {
   int a_col, ra, g_col, rg, GW;
   const void* wa;
@@ -261,7 +259,7 @@ struct LowRank {
   float* gate_out;
 };
 
-template <typename TI, typename TW, bool VEC>
+template <typename TI, typename TW, bool VEC, int R>
 __global__ void __launch_bounds__(kThreads)
 delta_prepare_kernel(const TI* __restrict__ proj, int nsplit, size_t split_stride, int WP,
                      const float* __restrict__ conv_w, int J, const float* __restrict__ state,
@@ -271,8 +269,8 @@ delta_prepare_kernel(const TI* __restrict__ proj, int nsplit, size_t split_strid
                      float* __restrict__ out, int OW, int N, int C,
                      float* __restrict__ new_tail_state, Decays decays, LowRank low,
                      int conv_blocks) {
-  __shared__ float xs[kLowRows][kLowK];
-  __shared__ float sums[kLowParts][kLowRows][kLowCols];
+  constexpr int kParts = kThreads / ei::kFewCols;
+  __shared__ ei::FewRows<R, kParts> few;
   const int id = blockIdx.x;
   if (id < conv_blocks * N) {
     const size_t row = id / conv_blocks;
@@ -288,54 +286,28 @@ delta_prepare_kernel(const TI* __restrict__ proj, int nsplit, size_t split_strid
     return;
   }
   const int HD = decays.HD;
-  const int decay_blocks = (HD + kLowCols - 1) / kLowCols;
-  const int gate_blocks = (low.GW + kLowCols - 1) / kLowCols;
+  const int decay_blocks = (HD + ei::kFewCols - 1) / ei::kFewCols;
+  const int gate_blocks = (low.GW + ei::kFewCols - 1) / ei::kFewCols;
   const int rest = id - conv_blocks * N;
-  const int row0 = rest / (decay_blocks + gate_blocks) * kLowRows;
+  const int row0 = rest / (decay_blocks + gate_blocks) * R;
   int block = rest % (decay_blocks + gate_blocks);
   const bool is_decay = block < decay_blocks;
   if (!is_decay) block -= decay_blocks;
-  const int K = is_decay ? low.ra : low.rg, width = is_decay ? HD : low.GW;
+  const int width = is_decay ? HD : low.GW;
   const TI* x = proj + (is_decay ? low.a_col : low.g_col);
-  const TW* w = static_cast<const TW*>(is_decay ? low.wa : low.wg);
-  const int col = threadIdx.x % kLowCols, part = threadIdx.x / kLowCols;
-  const int j = block * kLowCols + col, j_safe = min(j, width - 1);
-  const int rows = min(kLowRows, N - row0);
-  constexpr int kQuarter = kLowK / kLowParts;
-  float acc[kLowRows];
-#pragma unroll
-  for (int r = 0; r < kLowRows; ++r) acc[r] = 0.f;
-  for (int k0 = 0; k0 < K; k0 += kLowK) {
-    const int kn = min(kLowK, K - k0);
-    // (every load from a clamped place, so that none waits behind a branch; beyond the tile's end
-    // x holds zeros)
-    TW wv[kQuarter];
-#pragma unroll
-    for (int u = 0; u < kQuarter; ++u)
-      wv[u] = w[static_cast<size_t>(min(k0 + part * kQuarter + u, K - 1)) * width + j_safe];
-    __syncthreads();
-    for (int idx = threadIdx.x; idx < rows * kLowK; idx += kThreads) {
-      const int r = idx / kLowK, k = idx % kLowK;
-      xs[r][k] = k < kn ? slice_sum(x + static_cast<size_t>(row0 + r) * WP + k0 + k, nsplit, split_stride)
-                        : 0.f;
-    }
-    __syncthreads();
-#pragma unroll
-    for (int u = 0; u < kQuarter; ++u) {
-      const float wu = ei::to_f32<TW>(wv[u]);
-#pragma unroll
-      for (int r = 0; r < kLowRows; ++r)
-        if (r < rows) acc[r] += xs[r][part * kQuarter + u] * wu;
-    }
-  }
-#pragma unroll
-  for (int r = 0; r < kLowRows; ++r) sums[part][r][col] = acc[r];
-  __syncthreads();
+  const int col = threadIdx.x % ei::kFewCols;
+  const int j = block * ei::kFewCols + col;
+  few.product(static_cast<const TW*>(is_decay ? low.wa : low.wg), width, is_decay ? low.ra : low.rg,
+              j, width - 1, [&](int r, int k) {
+                return row0 + r < N ? slice_sum(x + static_cast<size_t>(row0 + r) * WP + k, nsplit,
+                                                split_stride)
+                                    : 0.f;
+              });
   if (j >= width) return;
-  for (int r = part; r < rows; r += kLowParts) {
+  for (int r = threadIdx.x / ei::kFewCols; r < R && row0 + r < N; r += kParts) {
     const size_t row = row0 + r;
     if (row_seq[row] < 0) continue;
-    const float z = (sums[0][r][col] + sums[1][r][col]) + (sums[2][r][col] + sums[3][r][col]);
+    const float z = few.total(r, col);
     if (is_decay)
       out[row * OW + C + j] = decay_of(z, decays.a_log[j / decays.D], decays.dt_bias[j]);
     else
@@ -764,15 +736,23 @@ extern "C" int ei_delta_prepare(const float* proj, int nsplit, long long split_s
   const int conv_blocks = (C + a_block - 1) / a_block;
   const Decays decays{nullptr, EI_F32, 0, a_log, dt_bias, H * D, D};
   const LowRank low{a_col, ra, g_col, rg, GW, wa, wg, gate_out};
-  const long long low_blocks = static_cast<long long>((N + kLowRows - 1) / kLowRows) *
-                               ((H * D + kLowCols - 1) / kLowCols + (GW + kLowCols - 1) / kLowCols);
+  const int rows = N == 1 ? 1 : (N <= 64 ? 8 : 16);       // rows a block of the products takes
+  const long long low_blocks =
+      static_cast<long long>((N + rows - 1) / rows) *
+      ((H * D + ei::kFewCols - 1) / ei::kFewCols + (GW + ei::kFewCols - 1) / ei::kFewCols);
   const long long blocks = static_cast<long long>(conv_blocks) * N + low_blocks;
   EI_REQUIRE(blocks < (1ll << 31), "delta_prepare: too many rows");
-#define EI_DPREP(TW, VV)                                                                          \
-  delta_prepare_kernel<float, TW, VV><<<static_cast<unsigned>(blocks), kThreads, 0, stream>>>(    \
+#define EI_DPREP_R(TW, VV, RR)                                                                    \
+  delta_prepare_kernel<float, TW, VV, RR><<<static_cast<unsigned>(blocks), kThreads, 0, stream>>>(    \
       proj, nsplit, ss, WP, conv_w, J, state, static_cast<size_t>(state_stride),                  \
       static_cast<size_t>(tail_offset), row_pos, row_seq, seq_in, seq_out, seq_start, out, OW, N, \
       C, renewed, decays, low, conv_blocks)
+#define EI_DPREP(TW, VV)                      \
+  do {                                        \
+    if (rows == 1) EI_DPREP_R(TW, VV, 1);     \
+    else if (rows == 8) EI_DPREP_R(TW, VV, 8); \
+    else EI_DPREP_R(TW, VV, 16);              \
+  } while (0)
   if (w_dtype == EI_F32) {
     if (vec) EI_DPREP(float, true);
     else EI_DPREP(float, false);
@@ -783,6 +763,7 @@ extern "C" int ei_delta_prepare(const float* proj, int nsplit, long long split_s
     EI_REQUIRE(false, "delta_prepare: unknown dtype");
   }
 #undef EI_DPREP
+#undef EI_DPREP_R
   EI_LAUNCH_CHECK();
 }
 

@@ -9,7 +9,8 @@
 //                      kv_rank + rot_dim elements a position), the gate logits out as float32;
 //                      where the queries lie in the same projection, their rotated parts as well
 //   head_matmul        Y[n, h, :] = X[n, h, :] . M[h] for one matrix [in, out] a head; the result
-//                      may be multiplied by the sigmoid of a gate an element
+//                      may be multiplied by the sigmoid of a gate an element, and X may be the merge of
+//                      the slices that attention over a cut key range has left
 //   heads_to_rows      rows of heads out of a product made head by head ([heads, N, J]): gated, or
 //                      with every head's rotated part behind it
 //   rotate_pairs       neighbouring elements (2i, 2i + 1) of a part of every head turn by
@@ -18,6 +19,7 @@
 //                      the kv head they meet: out[n, h, c, :] = sum over heads g of kv head c of
 //                      T[h, g] q[n, g, :]
 #include "common.h"
+#include "few_rows.h"
 
 namespace {
 
@@ -101,76 +103,75 @@ __global__ void latent_down_store_kernel(
   }
 }
 
-constexpr int kTileRows = 16;
-constexpr int kTileK = 128;
-constexpr int kCols = 64;            // output columns of a block
-constexpr int kParts = 4;            // threads that share a column, each a quarter of a K tile
+constexpr int kMaxSlices = 64;
 
-// Block: head blockIdx.y, rows blockIdx.x * 16 .., output columns blockIdx.z * 64 + t % 64; the
-// four threads of a column take a quarter of every K tile each (all its weights requested at
-// once, so that a step of few rows is not a chain of trips to memory) and add up through LDS.
-template <typename TI, typename TW, typename TO, typename TG>
-__global__ void __launch_bounds__(256)
+// What stands for x where attention has left a row's output in slices of the key range: unnormalised
+// sums part_o [N, heads, slices, K], and per slice a maximum and a sum of weights part_ml [.., 2].
+struct Slices {
+  const float* part_o;
+  const float* part_ml;
+  int n;
+};
+
+// Block: head blockIdx.y, rows blockIdx.x * R .., output columns blockIdx.z * 64 + t % 64.
+template <typename TI, typename TW, typename TO, typename TG, int R, int PARTS>
+__global__ void __launch_bounds__(ei::kFewCols * PARTS)
 head_matmul_kernel(const TI* __restrict__ x, int nsplit, size_t split_stride, long long x_row,
                    int x_head, int x_first, const TW* __restrict__ m, TO* __restrict__ y,
                    long long y_row, int y_head, int y_first, int N, int K, int J,
-                   const TG* __restrict__ gate, int gate_slices, size_t gate_stride, size_t gate_row) {
-  __shared__ float xs[kTileRows][kTileK];
-  __shared__ float sums[kParts][kTileRows][kCols];
-  const int h = blockIdx.y;
-  const int row0 = blockIdx.x * kTileRows;
-  const int col = threadIdx.x % kCols, part = threadIdx.x / kCols;
-  const int j = blockIdx.z * kCols + col;
+                   const TG* __restrict__ gate, int gate_slices, size_t gate_stride, size_t gate_row,
+                   Slices slices) {
+  __shared__ ei::FewRows<R, PARTS> few;
+  __shared__ float weight[R][kMaxSlices];
+  const int h = blockIdx.y, heads = gridDim.y;
+  const int row0 = blockIdx.x * R;
+  const int col = threadIdx.x % ei::kFewCols;
+  const int j = blockIdx.z * ei::kFewCols + col;
   const TW* mh = m + static_cast<size_t>(h) * K * J;
-  float acc[kTileRows];
-#pragma unroll
-  for (int r = 0; r < kTileRows; ++r) acc[r] = 0.f;
-  constexpr int kQuarter = kTileK / kParts;
-  for (int k0 = 0; k0 < K; k0 += kTileK) {
-    const int kn = min(kTileK, K - k0);
+  if (slices.part_o) {
+    // a wave a row: what each slice of it counts for, over the sum of all
+    const int lane = threadIdx.x % EI_WAVE;
+    for (int r = threadIdx.x / EI_WAVE; r < R; r += PARTS) {
+      if (row0 + r >= N) break;
+      const float* ml = slices.part_ml +
+                        (static_cast<size_t>(row0 + r) * heads + h) * slices.n * 2;
+      const bool mine = lane < slices.n;
+      const float m_own = mine ? ml[2 * lane] : -1.0e30f, l_own = mine ? ml[2 * lane + 1] : 0.f;
+      const float m_all = ei::wave_max(m_own);
+      const float f = mine ? expf(m_own - m_all) : 0.f;
+      const float l = ei::wave_sum(l_own * f);
+      weight[r][lane] = l > 0.f ? f / l : 0.f;
+    }
     __syncthreads();
-    for (int idx = threadIdx.x; idx < kTileRows * kTileK; idx += 256) {
-      const int r = idx / kTileK, k = idx % kTileK;
+    few.product(mh, J, K, j, J - 1, [&](int r, int k) {
+      if (row0 + r >= N) return 0.f;
+      const float* po = slices.part_o +
+                        (static_cast<size_t>(row0 + r) * heads + h) * slices.n * K + k;
       float v = 0.f;
-      if (row0 + r < N && k < kn)
-        v = sliced<TI>(x + static_cast<size_t>(row0 + r) * x_row + h * x_head + x_first + k0 + k,
-                       nsplit, split_stride);
-      xs[r][k] = v;
-    }
-    __syncthreads();
-    if (j < J) {
-      const int k_lo = part * kQuarter, k_hi = min(kn, k_lo + kQuarter);
-      // the thread's whole quarter of the tile is requested before any of it is used
-      // (every load is unconditional, from a clamped place, so that none waits for a branch;
-      // beyond the tile's end x holds zeros)
-      TW w[kQuarter];
-      const int last = K - 1 - k0;
+      for (int s0 = 0; s0 < slices.n; s0 += 8) {            // eight slices per trip to memory
+        float p[8];
 #pragma unroll
-      for (int u = 0; u < kQuarter; ++u)
-        w[u] = mh[static_cast<size_t>(k0 + min(k_lo + u, last)) * J + j];
+        for (int u = 0; u < 8; ++u) p[u] = s0 + u < slices.n ? po[static_cast<size_t>(s0 + u) * K] : 0.f;
 #pragma unroll
-      for (int u = 0; u < kQuarter; ++u) {
-        const float wu = ei::to_f32<TW>(w[u]);
-#pragma unroll
-        for (int r = 0; r < kTileRows; ++r) acc[r] += xs[r][k_lo + u] * wu;
+        for (int u = 0; u < 8; ++u)
+          if (s0 + u < slices.n) v = fmaf(p[u], weight[r][s0 + u], v);
       }
-      (void)k_hi;
-    }
+      return v;
+    });
+  } else {
+    few.product(mh, J, K, j, J - 1, [&](int r, int k) {
+      return row0 + r < N ? sliced<TI>(x + static_cast<size_t>(row0 + r) * x_row + h * x_head + x_first + k,
+                                       nsplit, split_stride)
+                          : 0.f;
+    });
   }
-#pragma unroll
-  for (int r = 0; r < kTileRows; ++r) sums[part][r][col] = acc[r];
-  __syncthreads();
-  // thread (part, col) finishes rows part, part + 4, ...
-  if (j < J) {
-    for (int r = part; r < kTileRows; r += kParts) {
-      if (row0 + r < N) {
-        float total = (sums[0][r][col] + sums[1][r][col]) + (sums[2][r][col] + sums[3][r][col]);
-        if (gate)      // (element j of head h has column h J + j)
-          total *= opened(sliced<TG>(gate + (row0 + r) * gate_row + static_cast<size_t>(h) * J + j,
-                                     gate_slices, gate_stride));
-        y[static_cast<size_t>(row0 + r) * y_row + h * y_head + y_first + j] = ei::from_f32<TO>(total);
-      }
-    }
+  if (j >= J) return;
+  for (int r = threadIdx.x / ei::kFewCols; r < R && row0 + r < N; r += PARTS) {
+    float total = few.total(r, col);
+    if (gate)      // (element j of head h has column h J + j)
+      total *= opened(sliced<TG>(gate + (row0 + r) * gate_row + static_cast<size_t>(h) * J + j,
+                                 gate_slices, gate_stride));
+    y[static_cast<size_t>(row0 + r) * y_row + h * y_head + y_first + j] = ei::from_f32<TO>(total);
   }
 }
 
@@ -384,30 +385,49 @@ extern "C" int ei_latent_down_store(const void* proj, int in_dtype, int nsplit,
 // x: [nsplit][N, x_row] read at x_head * h + x_first + 0..K; m: [heads, K, J] of the storage
 // type; y: [N, y_row] written at y_head * h + y_first + 0..J.  gate (or null): gate_slices slices
 // of rows gate_row apart; element j of head h is multiplied by the sigmoid of column h J + j.
+// n_slices > 0: x is not read, the rows come from part_o [N, heads, n_slices, K] and part_ml [N,
+// heads, n_slices, 2] as a sliced attention kernel leaves them.
 extern "C" int ei_head_matmul(const void* x, int x_dtype, int nsplit, long long split_stride,
                               long long x_row, int x_head, int x_first, const void* m,
                               int m_dtype, void* y, int y_dtype, long long y_row, int y_head,
                               int y_first, int N, int heads, int K, int J, const void* gate,
                               int gate_dtype, int gate_slices, long long gate_stride,
-                              long long gate_row, hipStream_t stream) {
+                              long long gate_row, const float* part_o, const float* part_ml,
+                              int n_slices, hipStream_t stream) {
   EI_REQUIRE(!gate || (gate_slices >= 1 && gate_row >= static_cast<long long>(heads) * J &&
                        (gate_dtype == EI_F32 || gate_dtype == EI_BF16)),
              "head_matmul: a gate's row holds one column an element");
-  EI_REQUIRE(N > 0 && heads > 0 && K > 0 && J > 0 && nsplit >= 1, "head_matmul: bad sizes");
-  EI_REQUIRE(x && m && y, "head_matmul: null pointer");
-  EI_REQUIRE(x_first >= 0 && y_first >= 0 &&
-                 static_cast<long long>(heads - 1) * x_head + x_first + K <= x_row &&
-                 static_cast<long long>(heads - 1) * y_head + y_first + J <= y_row,
-             "head_matmul: a head's part lies outside its row");
-  EI_REQUIRE(heads <= 65535 && (J + kCols - 1) / kCols <= 65535,
-             "head_matmul: too many heads or columns");
-  dim3 grid((N + kTileRows - 1) / kTileRows, heads, (J + kCols - 1) / kCols);
+  EI_REQUIRE(N > 0 && heads > 0 && K > 0 && J > 0, "head_matmul: bad sizes");
+  EI_REQUIRE(m && y, "head_matmul: null pointer");
+  EI_REQUIRE(n_slices >= 0 && n_slices <= kMaxSlices && (n_slices == 0 || (part_o && part_ml)),
+             "head_matmul: at most 64 slices, with their sums and weights");
+  EI_REQUIRE(n_slices > 0 || (x && nsplit >= 1 && x_first >= 0 &&
+                              static_cast<long long>(heads - 1) * x_head + x_first + K <= x_row),
+             "head_matmul: a head's part lies outside its row of x");
+  EI_REQUIRE(y_first >= 0 && static_cast<long long>(heads - 1) * y_head + y_first + J <= y_row,
+             "head_matmul: a head's part lies outside its row of y");
+  const int col_blocks = (J + ei::kFewCols - 1) / ei::kFewCols;
+  EI_REQUIRE(heads <= 65535 && col_blocks <= 65535, "head_matmul: too many heads or columns");
+  const Slices slices{n_slices > 0 ? part_o : nullptr, part_ml, n_slices};
+  if (n_slices > 0) x_dtype = m_dtype;
   const size_t ss = static_cast<size_t>(split_stride);
-#define EI_HM_CASE_G(TI, TW, TO, TG)                                                            \
-  head_matmul_kernel<TI, TW, TO, TG><<<grid, 256, 0, stream>>>(                                 \
-      static_cast<const TI*>(x), nsplit, ss, x_row, x_head, x_first, static_cast<const TW*>(m), \
-      static_cast<TO*>(y), y_row, y_head, y_first, N, K, J, static_cast<const TG*>(gate),       \
-      gate_slices, static_cast<size_t>(gate_stride), static_cast<size_t>(gate_row))
+  // rows a block takes: all of a decode step's few, more where weights are used by many rows
+  const int rows = N == 1 ? 1 : (N <= 64 ? 8 : 16);
+  const bool deep = K > 4 * ei::kFewK && rows < 16;        // 16 threads a column instead of 4
+  const dim3 grid((N + rows - 1) / rows, heads, col_blocks);
+#define EI_HM_RP(TI, TW, TO, TG, RR, PP)                                                          \
+  head_matmul_kernel<TI, TW, TO, TG, RR, PP><<<grid, ei::kFewCols * PP, 0, stream>>>(             \
+      static_cast<const TI*>(x), nsplit, ss, x_row, x_head, x_first, static_cast<const TW*>(m),   \
+      static_cast<TO*>(y), y_row, y_head, y_first, N, K, J, static_cast<const TG*>(gate),         \
+      gate_slices, static_cast<size_t>(gate_stride), static_cast<size_t>(gate_row), slices)
+#define EI_HM_CASE_G(TI, TW, TO, TG)                              \
+  do {                                                            \
+    if (rows == 1 && deep) EI_HM_RP(TI, TW, TO, TG, 1, 16);       \
+    else if (rows == 1) EI_HM_RP(TI, TW, TO, TG, 1, 4);           \
+    else if (rows == 8 && deep) EI_HM_RP(TI, TW, TO, TG, 8, 16);  \
+    else if (rows == 8) EI_HM_RP(TI, TW, TO, TG, 8, 4);           \
+    else EI_HM_RP(TI, TW, TO, TG, 16, 4);                         \
+  } while (0)
 #define EI_HM_CASE(TI, TW, TO)                                          \
   do {                                                                  \
     if (gate && gate_dtype == EI_BF16) EI_HM_CASE_G(TI, TW, TO, bf16_t); \
@@ -419,6 +439,7 @@ extern "C" int ei_head_matmul(const void* x, int x_dtype, int nsplit, long long 
   else EI_REQUIRE(false, "head_matmul: unsupported dtype combination");
 #undef EI_HM_CASE
 #undef EI_HM_CASE_G
+#undef EI_HM_RP
   EI_LAUNCH_CHECK();
 }
 

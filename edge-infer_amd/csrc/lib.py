@@ -154,7 +154,7 @@ _SIGNATURES = {
         "ei_attention_wide": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                               c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                               c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_float, c_int,
-                              c_int, c_int, c_void_p, c_void_p],
+                              c_int, c_int, c_void_p, c_int, c_void_p],
     },
     "head_ops": {
         "ei_latent_down_store": [c_void_p, c_int, c_int, c_longlong, c_longlong, c_void_p, c_void_p,
@@ -164,7 +164,8 @@ _SIGNATURES = {
                                  c_int, c_void_p],
         "ei_head_matmul": [c_void_p, c_int, c_int, c_longlong, c_longlong, c_int, c_int, c_void_p,
                            c_int, c_void_p, c_int, c_longlong, c_int, c_int, c_int, c_int, c_int,
-                           c_int, c_void_p, c_int, c_int, c_longlong, c_longlong, c_void_p],
+                           c_int, c_void_p, c_int, c_int, c_longlong, c_longlong, c_void_p,
+                           c_void_p, c_int, c_void_p],
         "ei_heads_to_rows": [c_void_p, c_int, c_void_p, c_longlong, c_int, c_int, c_int, c_int,
                              c_void_p, c_longlong, c_void_p, c_longlong, c_int, c_int, c_void_p,
                              c_float, c_void_p, c_void_p],
@@ -805,9 +806,10 @@ def attention_wide_positions(group: int) -> int:
 def attention_wide(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items, row_pos, row_seq,
                    page_table, out, n_heads, n_kv_heads, head_dim, window=None, scale=None,
                    n_splits=1, part_o=None, part_ml=None, value_dim=None, sinks=None, key_heads=1,
-                   values_in_keys=False, gate=None) -> None:
+                   values_in_keys=False, gate=None, merge=True) -> None:
     """bfloat16 attention on the matrix cores for wide keys (see attention_wide.hip); arguments
-    as `attention`'s."""
+    as `attention`'s.  merge False (with n_splits > 1, no gate): `out` is not written, the slices
+    stay in part_o and part_ml for `head_matmul(slices=...)`."""
     lib = library("attention_wide")
     n = q.shape[0]
     value_dim = head_dim if value_dim is None else int(value_dim)
@@ -853,7 +855,7 @@ def attention_wide(q, k_pages, v_pages, item_seq, item_row0, item_npos, n_items,
         n_kv_heads, head_dim, value_dim, int(window or 0),
         None if sinks is None else _gpu(sinks, "sinks", torch.float32), float(scale), n_splits,
         key_heads, int(bool(values_in_keys)),
-        None if gate is None else _gpu(gate, "gate", torch.float32), _stream())
+        None if gate is None else _gpu(gate, "gate", torch.float32), int(bool(merge)), _stream())
     _check(lib, status, "attention_wide")
 
 
@@ -937,12 +939,27 @@ def latent_down_store(proj, q_norm_w, c_norm_w, eps, frequencies, row_pos, row_s
     _check(lib, status, "latent_down_store")
 
 
-def head_matmul(x, matrices, y, heads, x_head, x_first, y_head, y_first, gate=None) -> None:
+def head_matmul(x, matrices, y, heads, x_head, x_first, y_head, y_first, gate=None,
+                slices=None) -> None:
     """y[n, h * y_head + y_first + j] = sum_i x[n, h * x_head + x_first + i] * matrices[h, i, j]
     for matrices [heads, K, J] of the storage type; x [rows, width] or float32 slices of it.
-    gate: `Columns` [heads * J]; the element is multiplied by the sigmoid of its column h * J + j."""
+    gate: `Columns` [heads * J]; the element is multiplied by the sigmoid of its column h * J + j.
+    slices (part_o, part_ml, count), x None: x is the merge of what attention over a key range cut
+    into `count` slices left of every row and head (K elements a head)."""
     lib = library("head_ops")
-    n, x_row, nsplit, stride = _rows_of(x, "x")
+    if slices is None:
+        n, x_row, nsplit, stride = _rows_of(x, "x")
+        x_args = (_gpu(x, "x"), _code(x, "x"), nsplit, stride, x_row)
+        slice_args = (None, None, 0)
+    else:
+        part_o, part_ml, count = slices
+        n = y.shape[0]
+        if part_o.numel() < n * heads * count * matrices.shape[1] or \
+                part_ml.numel() < n * heads * count * 2 or not 1 <= count <= 64:
+            raise KernelError("head_matmul: the slices are too small for these rows")
+        x_args = (None, F32, 1, 0, 0)
+        slice_args = (_gpu(part_o, "part_o", torch.float32), _gpu(part_ml, "part_ml", torch.float32),
+                      int(count))
     if matrices.dim() != 3 or matrices.shape[0] != heads:
         raise KernelError("head_matmul: matrices must be [heads, K, J]")
     if y.dim() != 2 or y.shape[0] != n:
@@ -951,11 +968,10 @@ def head_matmul(x, matrices, y, heads, x_head, x_first, y_head, y_first, gate=No
     gate_args = (None, F32, 1, 0, 0)
     if gate is not None:
         gate_args = _columns(gate, n, heads * j, "gate")
-    status = lib.ei_head_matmul(_gpu(x, "x"), _code(x, "x"), nsplit, stride, x_row, int(x_head),
-                                int(x_first), _gpu(matrices, "matrices"),
+    status = lib.ei_head_matmul(*x_args, int(x_head), int(x_first), _gpu(matrices, "matrices"),
                                 _code(matrices, "matrices"), _gpu(y, "y"), _code(y, "y"),
                                 y.shape[1], int(y_head), int(y_first), n, heads, k, j, *gate_args,
-                                _stream())
+                                *slice_args, _stream())
     _check(lib, status, "head_matmul")
 
 

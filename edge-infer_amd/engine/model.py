@@ -275,6 +275,9 @@ class DecoderModel:
                 if obj.data_ptr() not in seen:
                     seen.add(obj.data_ptr())
                     total += obj.numel() * obj.element_size()
+            elif isinstance(obj, (list, tuple)):
+                for value in obj:
+                    visit(value)
             elif hasattr(obj, "__dict__"):
                 for value in vars(obj).values():
                     visit(value)

@@ -541,18 +541,28 @@ class Attention:
                 self.decode_launch(n_seqs, pages * PAGE_TOKENS)
         return launch
 
+    def input_product(self):
+        """The product of x that a caller may make together with others, or None where this part
+        has to make it itself."""
+        return self.qkv if self.whole_store and self.qkv.bias is None else None
+
+    def use_input_product(self, product):
+        self.qkv = product
+
     bias_later = True      # forward(..., bias_later=True) hands the last product's bias on
 
-    def forward(self, ctx, x, entry, bias_later=False):
+    def forward(self, ctx, x, entry, bias_later=False, projected=None):
         """The mixer's rows; with `bias_later`, (rows, float32 bias of the output projection
-        that is still to be added, or None), for a caller whose next kernel adds it."""
+        that is still to be added, or None), for a caller whose next kernel adds it.  `projected`:
+        the input product's rows, made by the caller."""
         spec = self.spec
         n = x.shape[0]
         meta = ctx.meta
         group_index, k_pages, v_pages = ctx.cache.kv(entry.cache)
         page_table = meta.page_table(group_index)
         # (these store kernels add the projection's bias as well)
-        qkv, bias = (self.qkv.forward(ctx, x, "attn.qkv", bias_later=True)
+        qkv, bias = ((projected, None) if projected is not None
+                     else self.qkv.forward(ctx, x, "attn.qkv", bias_later=True)
                      if self.whole_store or self.general
                      else (self.qkv.forward(ctx, x, "attn.qkv"), None))
         gate, pooled, aside = None, {}, {}
@@ -703,7 +713,7 @@ class Attention:
                               scale=self.scale, **more)
         if spec.output_gate and not self.head_gate and wide_gate is None:
             lib.gate_rows(qkv, self.gate_column, out)
-        ctx.release(qkv, None if isinstance(q, lib.DecodeProjection) else q, part_o, part_ml, gate,
+        ctx.release(None if projected is not None else qkv, None if isinstance(q, lib.DecodeProjection) else q, part_o, part_ml, gate,
                     aside.get("pool_o"), aside.get("pool_ml"))
         delta = self.o.forward(ctx, out, "attn.o", bias_later=bias_later)
         ctx.release(out)

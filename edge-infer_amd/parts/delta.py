@@ -159,11 +159,19 @@ class GatedDelta:
             fused[at[name]:at[name] + weight.shape[0]] = weight
         return fused
 
+    def input_product(self):
+        """The product of x that a caller may make together with others."""
+        return self.proj
+
+    def use_input_product(self, product):
+        self.proj = product
+
     def _convolved(self, ctx, proj, state, renew):
         """The convolved channels (and behind them, with a decay per key channel, the decays) and
         what holds the gate's logits (None: the projection itself)."""
         shape, meta = self.shape, ctx.meta
-        n = proj.shape[-2]
+        rows, first = (proj.rows, proj.first) if isinstance(proj, lib.Columns) else (proj, 0)
+        n = rows.shape[-2]
         conv = ctx.buffer("delta.conv", (n, shape.conv_width), torch.float32)
         where = (meta.row_pos, meta.row_seq, meta.seq_state_in, meta.seq_state_out, meta.seq_start)
         if not shape.low_rank:
@@ -176,12 +184,13 @@ class GatedDelta:
             return conv, gate, gate
         # a bfloat16 step of many rows: decays' and gate's logits as one library product
         both = ctx.buffer("delta.low", (n, shape.decay_width + shape.v_width))
-        torch.matmul(proj[:, shape.low_col:shape.beta_col], self.w_both.t(), out=both)
+        torch.matmul(rows[:, first + shape.low_col:first + shape.beta_col], self.w_both.t(), out=both)
         lib.delta_conv(proj, self.conv_w, state, shape, *where, conv, renew_tail=renew,
                        decay_logits=both, a_log=self.decay_log_rate, dt_bias=self.decay_bias)
         return conv, lib.Columns(both, shape.decay_width, shape.v_width), both
 
-    def forward(self, ctx, x, entry):
+    def forward(self, ctx, x, entry, projected=None):
+        """The mixer's rows; `projected`: the input product's rows, made by the caller."""
         if not entry.writes_cache:
             raise ValueError("gated_delta: a run that only reads another run's state is not "
                              "implemented")
@@ -190,7 +199,7 @@ class GatedDelta:
         state = ctx.cache.state(entry.cache)                 # [2 (slots + 1), state_floats]
         rows_in = meta.seq_state_in                          # a sequence's state, and the row
         rows_out = meta.seq_state_out                        # the step writes
-        proj = self.proj.forward(ctx, x, "delta.proj")
+        proj = self.proj.forward(ctx, x, "delta.proj") if projected is None else projected
         # a decode step (one row a sequence) renews the convolution's tails in the same kernel
         renew = ctx.decode and shape.taps <= lib.DELTA_FEW_TAPS
         conv, gate, held = self._convolved(ctx, proj, state, renew)
@@ -206,7 +215,7 @@ class GatedDelta:
         gated = ctx.buffer("delta.gated", (n, shape.v_width))
         lib.delta_out(o_raw, proj, self.out_norm, self.spec.out_norm_eps, shape, meta.row_seq,
                       gated, sigmoid_gate=self.spec.gate_activation == "sigmoid", gate_logits=gate)
-        ctx.release(o_raw, proj, held)
+        ctx.release(o_raw, proj if projected is None else None, held)
         delta = self.o.forward(ctx, gated, "delta.o")
         ctx.release(gated)
         return delta

@@ -225,30 +225,32 @@ class LatentAttention:
         torch.bmm(taken.transpose(0, 1), matrices, out=made)
         return made
 
-    def _values(self, ctx, mixed, gate_rows):
-        """The heads' values [N, heads * value_dim] from their weighted sums of latents, gated
-        element by element where the spec says so (`gate_rows` holds the logits)."""
+    def _values(self, ctx, mixed, slices, gate_rows):
+        """The heads' values [N, heads * value_dim] from their weighted sums of latents `mixed` (or
+        the slices of them), gated element by element where the spec says so (`gate_rows` holds
+        the logits)."""
         spec = self.spec
-        n = mixed.shape[0]
+        n = gate_rows.shape[-2]
         out = ctx.buffer("latent.out", (n, spec.out_width))
         gate = None
         if spec.output_gate == "element":
             gate = lib.Columns(gate_rows, self.gate_column, spec.out_width)
-        if self._by_library(n, spec.value_dim) and (gate is None or gate.dtype == self.dtype):
+        if slices is None and self._by_library(n, spec.value_dim) and \
+                (gate is None or gate.dtype == self.dtype):
             made = self._batched(ctx, mixed, self.v_up, spec.kv_rank, 0, "latent.v_made")
             lib.heads_to_rows(made, out, spec.value_dim, gate=gate)
             ctx.release(made)
         else:
             lib.head_matmul(mixed, self.v_up, out, spec.n_heads, x_head=spec.kv_rank, x_first=0,
-                            y_head=spec.value_dim, y_first=0, gate=gate)
+                            y_head=spec.value_dim, y_first=0, gate=gate, slices=slices)
         return out
 
     def _attend(self, ctx, q_wide, k_pages, page_table, gate):
-        """The heads' weighted sums of latents [N, heads * kv_rank]."""
+        """(the heads' weighted sums of latents [N, heads * kv_rank], None), or, where the kernel that
+        takes them can merge the slices of the key range itself, (None, (sums, weights, slices))."""
         spec, meta = self.spec, ctx.meta
         H, rank = spec.n_heads, spec.kv_rank
         n = q_wide.shape[0]
-        mixed = ctx.buffer("latent.mixed", (n, H * rank))
         common = dict(window=spec.window, scale=self.scale, value_dim=rank, sinks=self.sinks,
                       values_in_keys=True, gate=gate)
         part_o = part_ml = None
@@ -261,13 +263,23 @@ class LatentAttention:
             common.update(n_splits=splits, part_o=part_o, part_ml=part_ml)
         else:
             section = meta.section(f"latent.items{self.positions_per_item}")
+        slices = None
+        if part_o is not None and self.wide and gate is None:
+            slices = (part_o, part_ml, splits)
+            common["merge"] = False
+        # (the slices stand for it where they are merged later)
+        mixed = ctx.buffer("latent.mixed", (n, H * rank))
         count = section.numel() // 3
         kernel = lib.attention_wide if self.wide else lib.attention
         kernel(q_wide, k_pages, None, section[:count], section[count:2 * count],
                section[2 * count:], count, meta.row_pos, meta.row_seq, page_table, mixed,
                H, 1, spec.cache_width, **common)
-        ctx.release(q_wide, gate, part_o, part_ml)
-        return mixed
+        ctx.release(q_wide, gate)
+        if slices is None:
+            ctx.release(part_o, part_ml)
+            return mixed, None
+        ctx.release(mixed)
+        return None, slices
 
     def forward(self, ctx, x, entry):
         spec, meta = self.spec, ctx.meta
@@ -281,9 +293,9 @@ class LatentAttention:
         q_wide = ctx.buffer("latent.q_wide", (n, spec.n_heads * spec.cache_width))
         store = self._store_with_latent if spec.q_rank else self._store_direct
         gate = store(ctx, down, q_wide, k_pages, page_table, entry)
-        mixed = self._attend(ctx, q_wide, k_pages, page_table, gate)
-        out = self._values(ctx, mixed, down)
-        ctx.release(mixed, down)
+        mixed, slices = self._attend(ctx, q_wide, k_pages, page_table, gate)
+        out = self._values(ctx, mixed, slices, down)
+        ctx.release(mixed, down, *(slices or ())[:2])
         delta = self.o.forward(ctx, out, "latent.o")
         ctx.release(out)
         return delta

@@ -5,7 +5,10 @@ branches' outputs, each first RMS-normed over the model's width with a weight of
 
 The branches are mixers of any registered kind (`spec.branches`); branch b's parameters are
 prefixed `spec.names[b]`, its output norm's weight is `<name>_out.weight`, and what it asks of
-the cache is found under the cache id `(id, name)` of the layer's entry.  Kernel:
+the cache is found under the cache id `(id, name)` of the layer's entry.  Where every branch says
+that another may make its input projection (`input_product()`, the branch's `Linear` of x, and
+`use_input_product()`), the projections are one matrix and one product; a branch is then handed
+its columns (`forward(..., projected=...)`).  Kernel:
 `norm_mean` of `csrc/norms.hip`.
 """
 from __future__ import annotations
@@ -16,6 +19,7 @@ import torch
 
 from ..csrc import lib
 from ..weights.loader import ParamSpec
+from .linear import Linear
 from .registry import lookup
 
 
@@ -94,6 +98,20 @@ class ParallelMixer:
             self.branches.append(owner(branch, hidden, own, dtype, device, positions=positions))
             self.out_norms.append(params[f"{name}_out.weight"].to(
                 device=device, dtype=torch.float32).contiguous())
+        self.proj, self.columns = None, []
+        products = [branch.input_product() if hasattr(branch, "input_product") else None
+                    for branch in self.branches]
+        if len(products) > 1 and all(product is not None for product in products):
+            rows = []
+            for product in products:
+                self.columns.append((sum(matrix.shape[0] for matrix in rows), product.out_features))
+                rows.append(product.weight)
+                spare = -product.out_features % 8       # (every part begins at a 16-byte piece)
+                if spare:
+                    rows.append(product.weight.new_zeros((spare, hidden)))
+            self.proj = Linear(torch.cat(rows, dim=0), dtype, device)
+            for branch in self.branches:
+                branch.use_input_product(self.proj)
 
     def members(self):
         return tuple(self.branches)
@@ -123,10 +141,13 @@ class ParallelMixer:
     def forward(self, ctx, x, entry, join_later=False):
         """The mean of the normed branches; with `join_later`, the `Branches` themselves."""
         outputs = []
-        for name, branch in zip(self.names, self.branches):
+        proj = None if self.proj is None else self.proj.forward(ctx, x, "parallel.proj")
+        for index, (name, branch) in enumerate(zip(self.names, self.branches)):
+            more = {} if proj is None else {"projected": lib.Columns(proj, *self.columns[index])}
             outputs.append(branch.forward(ctx, x, BranchEntry(
                 layer=entry.layer, cache=(entry.cache, name), writes_cache=entry.writes_cache,
-                own_id=(entry.own_id, name))))
+                own_id=(entry.own_id, name)), **more))
+        ctx.release(proj)
         if join_later:
             return Branches(tuple(outputs), tuple(self.out_norms), self.spec.norm_eps)
         out = ctx.buffer("parallel.out", (x.shape[0], self.hidden), torch.float32)
