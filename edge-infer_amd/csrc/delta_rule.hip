@@ -247,6 +247,97 @@ __global__ void delta_conv_vec_kernel(const TI* __restrict__ proj, int nsplit, s
   }
 }
 
+// Prompts (one product, no slices): a thread makes kRun consecutive rows of four channels (or of four
+// decays), so that an input is read once, the filters stay in registers and every row of the run is
+// asked for before the first is used.  J taps (a constant: the window moves through registers).
+constexpr int kRun = 8;
+constexpr int kManyRows = 128;   // from so many rows on there are blocks enough
+
+template <typename TI, int J>
+__global__ void __launch_bounds__(EI_WAVE)
+delta_conv_run_kernel(const TI* __restrict__ proj, int WP, const float* __restrict__ conv_w,
+                      const float* __restrict__ state, size_t state_stride, size_t tail_offset,
+                      const int32_t* __restrict__ row_pos, const int32_t* __restrict__ row_seq,
+                      const int32_t* __restrict__ seq_in, const int32_t* __restrict__ seq_start,
+                      float* __restrict__ out, int OW, int N, int C, Decays decays) {
+  const int row0 = blockIdx.x * kRun;
+  const int c = (blockIdx.y * EI_WAVE + threadIdx.x) * 4;
+  if (c >= C + decays.HD) return;
+  const bool channel = c < C;
+  float in[kRun][4];
+#pragma unroll
+  for (int r = 0; r < kRun; ++r) {
+    const size_t row = static_cast<size_t>(min(row0 + r, N - 1));
+    if (channel)
+      ei::Vec4<TI>::load(proj + row * WP + c, in[r]);
+    else if (decays.z_dtype == EI_BF16)
+      ei::Vec4<bf16_t>::load(static_cast<const bf16_t*>(decays.z) + row * decays.z_row + (c - C), in[r]);
+    else
+      ei::Vec4<float>::load(static_cast<const float*>(decays.z) + row * decays.z_row + (c - C), in[r]);
+  }
+  if (!channel) {
+    float a_log[4], bias[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      a_log[e] = decays.a_log[(c - C + e) / decays.D];
+      bias[e] = decays.dt_bias[c - C + e];
+    }
+#pragma unroll
+    for (int r = 0; r < kRun; ++r) {
+      if (row0 + r >= N || row_seq[row0 + r] < 0) continue;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) in[r][e] = decay_of(in[r][e], a_log[e], bias[e]);
+      ei::Vec4<float>::store(out + static_cast<size_t>(row0 + r) * OW + c, in[r]);
+    }
+    return;
+  }
+  float w[4][J], x[J][4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+#pragma unroll
+    for (int j = 0; j < J; ++j) w[e][j] = conv_w[static_cast<size_t>(c + e) * J + j];
+  int held = -1;                          // the sequence whose inputs x holds
+#pragma unroll
+  for (int r = 0; r < kRun; ++r) {
+    const int row = row0 + r;
+    const int seq = row < N ? row_seq[row] : -1;
+    if (seq < 0) {
+      held = -1;
+      continue;
+    }
+    if (seq == held) {
+#pragma unroll
+      for (int j = 0; j + 1 < J; ++j)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[j][e] = x[j + 1][e];
+    } else {                              // what lies before this row
+      const int pos = row_pos[row], start = seq_start[seq];
+      const float* tail = state + static_cast<size_t>(seq_in[seq]) * state_stride + tail_offset;
+#pragma unroll
+      for (int j = 0; j + 1 < J; ++j) {
+        const int back = J - 1 - j;
+        const int at = pos - back;
+        x[j][0] = x[j][1] = x[j][2] = x[j][3] = 0.f;
+        if (at >= start)
+          ei::Vec4<TI>::load(proj + static_cast<size_t>(row - back) * WP + c, x[j]);
+        else if (at >= 0)
+          ei::Vec4<float>::load(tail + static_cast<size_t>(at - start + J - 1) * C + c, x[j]);
+      }
+      held = seq;
+    }
+    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x[J - 1][e] = in[r][e];
+#pragma unroll
+    for (int j = 0; j < J; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc[e] += w[e][j] * x[j][e];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) acc[e] = silu_f32(acc[e]);
+    ei::Vec4<float>::store(out + static_cast<size_t>(row) * OW + c, acc);
+  }
+}
+
 // The low-rank products of few rows in the convolution's launch.  a_col, g_col: where the two
 // low-rank parts (ra and rg wide) begin in a projection row; wa [ra, HD], wg [rg, GW]: their second
 // matrices, transposed; the decays go behind the convolved channels of `out`, the gate's logits to
@@ -645,6 +736,40 @@ __global__ void delta_out_kernel(const float* __restrict__ o_raw, const TI* __re
   }
 }
 
+// The same with four elements a lane and L lanes a head (a power of two, at least DV / 4): heads and
+// rows in turn, one gate row a row.
+template <typename TI, typename TO, int L>
+__global__ void __launch_bounds__(kThreads)
+delta_out_vec_kernel(const float* __restrict__ o_raw, const TI* __restrict__ proj, int WP,
+                     int gate_col, int sigmoid_gate, const float* __restrict__ norm_w, float eps,
+                     const int32_t* __restrict__ row_seq, TO* __restrict__ out, int N, int H, int DV) {
+  const long long id = static_cast<long long>(blockIdx.x) * (kThreads / L) + threadIdx.x / L;
+  const bool live = id < static_cast<long long>(N) * H;
+  const size_t row = live ? id / H : 0;
+  const int head = live ? static_cast<int>(id % H) : 0;
+  const int j = threadIdx.x % L * 4;
+  const bool mine = live && j < DV;
+  const size_t base = (row * H + head) * DV;
+  float o[4] = {0.f, 0.f, 0.f, 0.f}, gate[4] = {0.f, 0.f, 0.f, 0.f}, w[4] = {0.f, 0.f, 0.f, 0.f};
+  const bool padding = row_seq[row] < 0;      // a defined input for the next product
+  if (mine && !padding) {
+    ei::Vec4<float>::load(o_raw + base + j, o);
+    ei::Vec4<TI>::load(proj + row * WP + gate_col + static_cast<size_t>(head) * DV + j, gate);
+    ei::Vec4<float>::load(norm_w + j, w);
+  }
+  float sq = (o[0] * o[0] + o[1] * o[1]) + (o[2] * o[2] + o[3] * o[3]);
+#pragma unroll
+  for (int step = L / 2; step > 0; step /= 2) sq += __shfl_xor(sq, step, EI_WAVE);
+  if (!mine) return;
+  const float inv = 1.0f / sqrtf(sq / static_cast<float>(DV) + eps);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const float open = 1.0f / (1.0f + expf(-gate[e]));
+    o[e] = padding ? 0.f : (o[e] * inv) * w[e] * (sigmoid_gate ? open : gate[e] * open);
+  }
+  ei::Vec4<TO>::store(out + base + j, o);
+}
+
 int lanes_a_column(int D, int own) {
   int lanes = 1;
   while (lanes * own < D) lanes *= 2;
@@ -687,6 +812,25 @@ extern "C" int ei_delta_conv(const void* proj, int in_dtype, int nsplit, long lo
       static_cast<const TI*>(proj), nsplit, ss, WP, conv_w, J, state,                             \
       static_cast<size_t>(state_stride), static_cast<size_t>(tail_offset), row_pos, row_seq,      \
       seq_in, seq_out, seq_start, out, OW, C, renewed, decays)
+  if (vec && !renewed && nsplit == 1 && N >= kManyRows && (J >= 2 && J <= 4)) {
+    const dim3 rgrid((N + kRun - 1) / kRun, ((C + HD) / 4 + EI_WAVE - 1) / EI_WAVE);
+#define EI_DRUN(TI, JJ)                                                                           \
+  delta_conv_run_kernel<TI, JJ><<<rgrid, EI_WAVE, 0, stream>>>(                                   \
+      static_cast<const TI*>(proj), WP, conv_w, state, static_cast<size_t>(state_stride),         \
+      static_cast<size_t>(tail_offset), row_pos, row_seq, seq_in, seq_start, out, OW, N, C, decays)
+#define EI_DRUN_T(TI)                \
+  do {                               \
+    if (J == 2) EI_DRUN(TI, 2);      \
+    else if (J == 3) EI_DRUN(TI, 3); \
+    else EI_DRUN(TI, 4);             \
+  } while (0)
+    if (in_dtype == EI_F32) EI_DRUN_T(float);
+    else if (in_dtype == EI_BF16) EI_DRUN_T(bf16_t);
+    else EI_REQUIRE(false, "delta_conv: unknown dtype");
+#undef EI_DRUN_T
+#undef EI_DRUN
+    EI_LAUNCH_CHECK();
+  }
   if (vec) {
     const int threads = 64;         // four channels a thread: 256 channels a block
     const dim3 vgrid(N, ((C + HD) / 4 + threads - 1) / threads);
@@ -882,6 +1026,25 @@ extern "C" int ei_delta_out(const float* o_raw, const void* proj, int in_dtype, 
   EI_REQUIRE(eps > 0.f, "delta_out: eps must be positive");
   EI_REQUIRE((H + 3) / 4 <= 65535, "delta_out: too many heads");
   const size_t ss = static_cast<size_t>(split_stride);
+  if (nsplit == 1 && N >= kManyRows && DV % 4 == 0 && DV > 16 && DV <= 256 && WP % 4 == 0 &&
+      gate_col % 4 == 0 && in_dtype == EI_BF16 && out_dtype == EI_BF16 &&
+      (reinterpret_cast<uintptr_t>(proj) | reinterpret_cast<uintptr_t>(out)) % 8 == 0 &&
+      (reinterpret_cast<uintptr_t>(o_raw) | reinterpret_cast<uintptr_t>(norm_w)) % 16 == 0) {
+    const int lanes = DV <= 32 ? 8 : (DV <= 64 ? 16 : (DV <= 128 ? 32 : 64));
+    const long long heads = static_cast<long long>(N) * H;
+    const long long blocks = (heads + kThreads / lanes - 1) / (kThreads / lanes);
+    EI_REQUIRE(blocks < (1ll << 31), "delta_out: too many rows");
+#define EI_DOUT_L(LL)                                                                              \
+  delta_out_vec_kernel<bf16_t, bf16_t, LL><<<static_cast<unsigned>(blocks), kThreads, 0, stream>>>( \
+      o_raw, static_cast<const bf16_t*>(proj), WP, gate_col, sigmoid_gate, norm_w, eps, row_seq,  \
+      static_cast<bf16_t*>(out), N, H, DV)
+    if (lanes == 8) EI_DOUT_L(8);
+    else if (lanes == 16) EI_DOUT_L(16);
+    else if (lanes == 32) EI_DOUT_L(32);
+    else EI_DOUT_L(64);
+#undef EI_DOUT_L
+    EI_LAUNCH_CHECK();
+  }
 #define EI_DOUT(TI, TO)                                                                      \
   delta_out_kernel<TI, TO><<<dim3(N, (H + 3) / 4), kThreads, 0, stream>>>(                   \
       o_raw, static_cast<const TI*>(proj), nsplit, ss, WP, gate_col, sigmoid_gate, norm_w, eps, row_seq, \
